@@ -552,6 +552,17 @@ int sgl_amd_gated_rmsnorm(int is_f32, const void* y, int64_t y_stride, const voi
     float eps, void* stream);
 int sgl_amd_gate_mul(int is_f32, const void* gate, const void* up, void* out, int64_t rows, int d, int64_t in_stride, int64_t out_stride,
     void* stream);
+/* Residual row of pre-norm designs, fp32: x <- table[ids] * scale (+ pos_table[positions]), or x + a + b, each source the sum of
+ * its items [rows x items x width] (times fp32 weight [rows, items] if given) in fp32 or in the activation type; then the copy
+ * `save`, then + extra (rows) + step (vector), then h = RMS norm(x) * weight.  save / extra rows are contiguous. */
+int sgl_amd_residual_rms(int is_f32, const int64_t* ids, const void* table, int64_t vocab, float scale, const int64_t* positions,
+    const void* pos_table, int64_t max_positions, const void* a, int a_f32, int a_items, int64_t a_row_stride,
+    int64_t a_item_stride, const float* a_weight, const void* b, int b_f32, int b_items, int64_t b_row_stride,
+    int64_t b_item_stride, const float* b_weight, float* x, int64_t x_stride, float* save, const float* extra,
+    const float* step, const float* weight, void* h, int64_t h_stride, int64_t rows, int width, float eps, void* stream);
+/* cap * tanh(z / cap) -> fp32 [rows, cols] contiguous; z: `items` addends item_stride apart (split-K partials) */
+int sgl_amd_soft_cap(int is_f32, const void* z, int64_t z_row_stride, int items, int64_t item_stride, float* out, int64_t rows, int cols,
+    float cap, void* stream);
 
 /* ---- recurrent mixers, token by token (recurrent.hip) ---------------------------------------------------------
  * Segments: tokens [seg_start[b], + seg_len[b]) belong to request b, tok_seg[t] names a token's segment; all null = one token
@@ -617,6 +628,37 @@ int sgl_amd_latent_prefill(const void* q, int64_t q_token, const void* latents, 
     const int32_t* blocks, int num_blocks, const int32_t* seg_start, const int32_t* seg_len, const int32_t* key_start,
     const int32_t* key_first, const int64_t* positions, void* out, int64_t o_token, int heads, int dim, int rot,
     int rank, int vdim, int window, float scale, void* stream);
+
+/* ---- grouped-query attention of layers with sizes of their own (grouped_attention.hip) ---------------------------
+ * Cache rows [kv_heads][kd | vd] (kd, vd multiples of 8, one row stride); query head h reads key head h / (heads / kv_heads); position
+ * i sees the `window` positions up to and with itself (window <= 0: all); `sink` joins the softmax denominator as a score without
+ * a value (-inf: none); the output is multiplied by sigmoid(gate) when a gate is given.
+ * sgl_amd_grouped_attention: any token mix; tok_seg null = a decode batch, whose own keys and values may be given as k_new / v_new
+ * (matrix form): they are read from there and stored at `loc`.  part_o fp32 [tokens, heads, splits, vd], part_ml [.., 2] for splits > 1.
+ * sgl_amd_grouped_prefill: stored keys; blocks = [num_blocks, 2] (segment, first of sgl_amd_grouped_prefill_rows() / group tokens). */
+int sgl_amd_grouped_kv_store(int is_f32, const void* k, int64_t k_stride, const void* v, int64_t v_stride, void* cache, int64_t cache_stride,
+    const int64_t* loc, int64_t tokens, int kv_heads, int kd, int vd, void* stream);
+int sgl_amd_grouped_attention_matrix_form(int kd, int vd);
+int sgl_amd_grouped_prefill_supported(int kd, int vd, int group);
+int sgl_amd_grouped_prefill_rows(void);
+int sgl_amd_grouped_attention(int is_f32, const void* q, int64_t q_stride, void* cache, int64_t cache_stride, const void* k_new, int64_t k_stride,
+    const void* v_new, int64_t v_stride, const int64_t* loc, const int32_t* req_to_token, int64_t r2t_stride,
+    const int64_t* req_pool_indices, const int32_t* tok_seg, const int64_t* positions, const void* gate,
+    int64_t gate_stride, void* out, int64_t o_stride, float* part_o, float* part_ml, int64_t tokens, int heads,
+    int kv_heads, int kd, int vd, int window, int splits, float scale, float sink, int plain, void* stream);
+int sgl_amd_grouped_prefill(const void* q, int64_t q_stride, const void* cache, int64_t cache_stride, const int32_t* req_to_token,
+    int64_t r2t_stride, const int64_t* req_pool_indices, const int32_t* blocks, int num_blocks,
+    const int32_t* seg_start, const int32_t* seg_len, const int64_t* positions, const void* gate, int64_t gate_stride,
+    void* out, int64_t o_stride, int heads, int kv_heads, int kd, int vd, int window, float scale, float sink, void* stream);
+
+/* ---- router with a bias, and the plain form of routed experts (moe_route.hip) -------------------------------------
+ * sgl_amd_moe_route: per token the `top` largest of W h + bias (fp32) and the softmax over those -> fp32 weights, int32 ids
+ * [tokens, top].  sgl_amd_experts_plain: pair i = (token i / top, expert ids[i]); up: silu(gate x) * (up x) from w [experts, 2 N, K],
+ * else w x from w [experts, N, K] and x [pairs, K]. */
+int sgl_amd_moe_route(int is_f32, const void* h, int64_t h_stride, const void* w, const float* bias, float* topk_weights, int32_t* topk_ids,
+    int64_t tokens, int K, int experts, int top, void* stream);
+int sgl_amd_experts_plain(int is_f32, int up, const void* x, int64_t x_stride, const void* w, const int32_t* ids, void* out, int64_t o_stride,
+    int64_t pairs, int top, int N, int K, int experts, void* stream);
 
 #ifdef __cplusplus
 }

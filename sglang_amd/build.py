@@ -39,6 +39,8 @@ HIPCC_FLAGS = [
 UNIT_GROUPS = {
     "hybrid": ["api.cpp", "elementwise.hip", "latent_attention.hip", "metadata.hip", "recurrent.hip", "recurrent_chunk.hip", "residual_norm.hip", "sampling.hip",
                "wstream_gemm.hip"],
+    "grouped": ["api.cpp", "elementwise.hip", "grouped_attention.hip", "metadata.hip", "moe.hip", "moe_route.hip", "moe_tiled_gemm.hip", "residual_norm.hip",
+                "sampling.hip", "skinny_gemm.hip", "wstream_gemm.hip"],
 }
 
 

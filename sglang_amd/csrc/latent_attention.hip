@@ -10,13 +10,12 @@
 // A cache row is [rank latents | rot rotated] padded with zeros to a multiple of 32 elements; the pool is created zeroed and
 // only the first rank + rot elements are ever written.
 #include "elem_io.hpp"
+#include "mfma_tiles.hpp"
 #include "sglang_amd.h"
 
 using namespace sgl_amd;
 
 namespace {
-
-__device__ __forceinline__ bf16x8_t as_frag(const U4& v) { return __builtin_bit_cast(bf16x8_t, v); }
 
 struct PrepareParams {
   void* q;                   // [tokens, heads, dim + rot]: the last rot of every head are rotated in place
@@ -326,24 +325,7 @@ void launch_latent_merge(const LatentAttnParams& p, int64_t tokens, hipStream_t 
 //   weights  exp2 in fp32; kept to ~17 bits as a bf16 pair (high, rest), so the sum over values loses nothing to rounding
 //   values   wave w owns a quarter of the latent columns: O^T = V^T P^T, the V^T operand from the row-major tile by
 //            ds_read_b64_tr_b16; a lane's accumulators belong to one head, so the rescale factor is a lane scalar
-typedef short v4s16_t __attribute__((ext_vector_type(4)));
-typedef __attribute__((address_space(3))) v4s16_t* lds_v4_t;
-
-// columns c .. c + 15 (one per lane of a 16-lane group) of rows r0 + 4 g + {0..3} and r0 + 16 + 4 g + {0..3} of a row-major tile
-__device__ __forceinline__ bf16x8_t read_transposed(const uint16_t* tile, int row_elems, int r0, int c, int i16, int g) {
-  const uint16_t* a = tile + (r0 + 4 * g + (i16 >> 2)) * row_elems + c + (i16 & 3) * 4;
-  const v4s16_t lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_v4_t)(a));
-  const v4s16_t hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_v4_t)(a + 16 * row_elems));
-  U4 o;
-  o.x = __builtin_bit_cast(uint2, lo).x; o.y = __builtin_bit_cast(uint2, lo).y;
-  o.z = __builtin_bit_cast(uint2, hi).x; o.w = __builtin_bit_cast(uint2, hi).y;
-  return as_frag(o);
-}
-
-__device__ __forceinline__ f32x4_t mfma_bf16(bf16x8_t a, bf16x8_t b, f32x4_t c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
-
 constexpr int kTile = 64;
-constexpr float kLog2e = 1.4426950408889634f;
 
 template <int KS, int OT, int HG>
 __global__ __launch_bounds__(256 * HG, 2) void latent_attention_mfma_kernel(LatentAttnParams p) {
@@ -575,11 +557,6 @@ __global__ __launch_bounds__(kPfThreads, 2) void latent_prefill_kernel(LatentPre
       j = j < end ? j : end - 1;
       vreg[i] = ld16(kv + (kbase + (j - kfirst)) * p.kv_stride + p.heads * p.dim + h * p.vdim + (e < p.vdim ? e : 0));
     }
-  };
-  auto keep_if = [](U4 v, bool k) __attribute__((always_inline)) {
-    const uint32_t m = k ? 0xffffffffu : 0u;
-    v.x &= m; v.y &= m; v.z &= m; v.w &= m;
-    return v;
   };
   f32x4_t o[2][VT];
   float m[2] = {-INFINITY, -INFINITY}, l[2] = {0.f, 0.f};

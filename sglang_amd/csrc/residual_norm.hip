@@ -3,6 +3,10 @@
 //   residual_norm   one launch between two sublayers:  x <- source  (embedding row, x + LayerNorm(y), or y + vector),
 //                   then optionally h = LayerNorm(x) for the next projection and copies of x in the activation type.
 //                   The residual row lives in fp32 and is in registers for both norms.
+//   residual_rms    the same step of pre-norm designs with RMS norms:  x <- embedding (+ position row), or x + up to two sublayer
+//                   outputs (rows, split-K partials, or weighted expert rows), then a saved copy, then + rows + vector in front
+//                   of a looped pass, then h = RMS norm(x)
+//   soft_cap        cap * tanh(z / cap) on logits, fp32 out
 //   gated_rmsnorm   RMS norm of equal column groups with a silu gate, the gate before the norm (Mamba-2) or behind it
 //                   (gated delta rule).
 //   gate_mul        act(a) * b for activation types / alignments outside silu_and_mul's bf16 form.
@@ -204,6 +208,208 @@ void launch_residual_norm_t(const ResidualNormParams& p, bool vec, hipStream_t s
 }
 
 // ---------------------------------------------------------------------------------------------------------------
+// One addend of a residual row: the sum over i < n of weight[row, i] * data[row * row_stride + i * item_stride + column].
+struct RowSource {
+  const void* data;
+  int f32;                  // element type: fp32, else the activation type
+  int n;
+  int64_t row_stride, item_stride;
+  const float* weight;      // [rows, n], or null: all ones
+};
+
+struct ResidualRmsParams {
+  const int64_t* ids;       // embedding form: x = table[ids] * scale + pos_table[positions]
+  const void* table;
+  int64_t vocab;
+  float scale;
+  const int64_t* positions;
+  const void* pos_table;    // may be null
+  int64_t max_pos;
+  RowSource a, b;           // otherwise x = x + a + b (either may be absent)
+  float* x;                 // [rows, W] fp32
+  int64_t x_stride;
+  float* save;              // optional fp32 copy of x as it is here
+  const float* extra;       // optional fp32 rows, added behind the copy (the stride of `save` / `extra` is W)
+  const float* step;        // optional [W], added last
+  const float* w;           // [W]
+  void* h;                  // RMS norm of the new x (may be null)
+  int64_t h_stride;
+  int64_t rows;
+  int width;
+  float eps;
+};
+
+template <typename T, int VEC>
+__device__ __forceinline__ void add_source(const RowSource& s, int64_t row, int c, float (&v)[VEC]) {
+  const float* wr = s.weight ? s.weight + row * s.n : nullptr;
+  const int64_t base = row * s.row_stride + c;
+  for (int i = 0; i < s.n; i += 4) {                  // four loads in flight, clamped to the last item
+    float u[4][VEC];
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      const int64_t at = base + static_cast<int64_t>(i + q < s.n ? i + q : s.n - 1) * s.item_stride;
+      if (s.f32) ldv<VEC>(static_cast<const float*>(s.data) + at, u[q]);
+      else ldv<VEC>(static_cast<const T*>(s.data) + at, u[q]);
+    }
+#pragma unroll
+    for (int q = 0; q < 4; ++q)
+      if (i + q < s.n) {
+        const float f = wr ? wr[i + q] : 1.0f;
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) v[j] += f * u[q][j];
+      }
+  }
+}
+
+template <typename T, int VEC>
+__device__ __forceinline__ void add_single(const RowSource& s, int64_t row, int c, float (&v)[VEC]) {
+  float u[VEC];
+  if (s.f32) ldv<VEC>(static_cast<const float*>(s.data) + row * s.row_stride + c, u);
+  else ldv<VEC>(static_cast<const T*>(s.data) + row * s.row_stride + c, u);
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) v[j] += u[j];
+}
+
+// kWaveRow: a wave owns a row (many rows: no barrier), else a workgroup does (decode batches: shortest path to one row).
+template <typename T, int VEC, int kItems, bool kWaveRow>
+__global__ __launch_bounds__(kWaveRow ? 256 : 1024) void residual_rms_kernel(ResidualRmsParams p) {
+  __shared__ float scratch[16];
+  const int tpr = kWaveRow ? 64 : static_cast<int>(blockDim.x);
+  const int lane = kWaveRow ? threadIdx.x & 63 : threadIdx.x;
+  const int64_t row = kWaveRow ? static_cast<int64_t>(blockIdx.x) * (blockDim.x >> 6) + (threadIdx.x >> 6) : blockIdx.x;
+  if (row >= p.rows) return;                          // (whole waves, and whole workgroups where barriers follow)
+  const int W = p.width;
+  float v[kItems][VEC];
+  float* xr = p.x + row * p.x_stride;
+  if (p.ids) {
+    int64_t id = p.ids[row];
+    if (id < 0 || id >= p.vocab) id = 0;
+    const T* tr = static_cast<const T*>(p.table) + id * W;
+    const T* pr = nullptr;
+    if (p.pos_table) {
+      int64_t pos = p.positions[row];
+      if (pos < 0 || pos >= p.max_pos) pos = p.max_pos - 1;      // (the host admits no such position)
+      pr = static_cast<const T*>(p.pos_table) + pos * W;
+    }
+#pragma unroll
+    for (int i = 0; i < kItems; ++i) {
+      const int c = (i * tpr + lane) * VEC;
+      if (c < W) {
+        ldv<VEC>(tr + c, v[i]);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) v[i][j] *= p.scale;
+        if (pr) {
+          float u[VEC];
+          ldv<VEC>(pr + c, u);
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) v[i][j] += u[j];
+        }
+      }
+    }
+  } else {
+    const bool simple = p.a.data && p.a.n == 1 && !p.a.weight && !p.b.data;
+#pragma unroll
+    for (int i = 0; i < kItems; ++i) {
+      const int c = (i * tpr + lane) * VEC;
+      if (c < W) ldv<VEC>(xr + c, v[i]);
+    }
+    if (simple) {                                     // rows of a library product: nothing between the loads
+#pragma unroll
+      for (int i = 0; i < kItems; ++i) {
+        const int c = (i * tpr + lane) * VEC;
+        if (c < W) add_single<T, VEC>(p.a, row, c, v[i]);
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < kItems; ++i) {
+        const int c = (i * tpr + lane) * VEC;
+        if (c < W) {
+          if (p.a.data) add_source<T, VEC>(p.a, row, c, v[i]);
+          if (p.b.data) add_source<T, VEC>(p.b, row, c, v[i]);
+        }
+      }
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < kItems; ++i) {
+    const int c = (i * tpr + lane) * VEC;
+    if (c < W) {
+      if (p.save) stv<VEC>(p.save + row * W + c, v[i]);
+      float u[VEC];
+      if (p.extra) {
+        ldv<VEC>(p.extra + row * W + c, u);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) v[i][j] += u[j];
+      }
+      if (p.step) {
+        ldv<VEC>(p.step + c, u);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) v[i][j] += u[j];
+      }
+      stv<VEC>(xr + c, v[i]);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) ss += v[i][j] * v[i][j];
+    }
+  }
+  if (!p.h) return;
+  ss = kWaveRow ? wave_sum(ss) : block_sum(ss, scratch);
+  const float rs = 1.0f / sqrtf(ss / static_cast<float>(W) + p.eps);
+  T* hr = static_cast<T*>(p.h) + row * p.h_stride;
+#pragma unroll
+  for (int i = 0; i < kItems; ++i) {
+    const int c = (i * tpr + lane) * VEC;
+    if (c < W) {
+      float wv[VEC], o[VEC];
+      ldv<VEC>(p.w + c, wv);
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) o[j] = v[i][j] * rs * wv[j];
+      stv<VEC>(hr + c, o);
+    }
+  }
+}
+
+template <typename T>
+void launch_residual_rms(const ResidualRmsParams& p, bool vec, hipStream_t st) {
+  const unsigned by4 = static_cast<unsigned>((p.rows + 3) / 4), one = static_cast<unsigned>(p.rows);
+  const int W = p.width;
+  if (vec && p.rows >= 1024 && W <= 1024) hipLaunchKernelGGL((residual_rms_kernel<T, 4, 4, true>), dim3(by4), dim3(256), 0, st, p);
+  else if (vec && p.rows >= 1024 && W <= 2048) hipLaunchKernelGGL((residual_rms_kernel<T, 4, 8, true>), dim3(by4), dim3(256), 0, st, p);
+  else if (vec && p.rows >= 1024 && W <= 4096) hipLaunchKernelGGL((residual_rms_kernel<T, 4, 16, true>), dim3(by4), dim3(256), 0, st, p);
+  else if (vec && W <= 4096) hipLaunchKernelGGL((residual_rms_kernel<T, 4, 1, false>), dim3(one), dim3((W / 4 + 63) / 64 * 64), 0, st, p);
+  else if (vec) hipLaunchKernelGGL((residual_rms_kernel<T, 4, 4, false>), dim3(one), dim3(1024), 0, st, p);
+  else hipLaunchKernelGGL((residual_rms_kernel<T, 1, 16, false>), dim3(one), dim3(W >= 1024 ? 1024 : (W + 63) / 64 * 64), 0, st, p);
+}
+
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void soft_cap_kernel(const T* __restrict__ z, int64_t z_stride, int n, int64_t item_stride, float* __restrict__ out,
+                                                       int cols, float cap, float inv_cap) {
+  const int64_t row = blockIdx.y;
+  const int c = (blockIdx.x * 256 + threadIdx.x) * VEC;
+  if (c >= cols) return;
+  float v[VEC];
+  ldv<VEC>(z + row * z_stride + c, v);
+  for (int i = 1; i < n; ++i) {
+    float u[VEC];
+    ldv<VEC>(z + i * item_stride + row * z_stride + c, u);
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) v[j] += u[j];
+  }
+#pragma unroll
+  for (int j = 0; j < VEC; ++j) v[j] = cap * tanhf(v[j] * inv_cap);
+  stv<VEC>(out + row * cols + c, v);
+}
+
+template <typename T>
+void launch_soft_cap(const void* z, int64_t z_stride, int n, int64_t item_stride, float* out, int64_t rows, int cols, float cap, hipStream_t st) {
+  const bool vec = cols % 4 == 0 && z_stride % 4 == 0 && item_stride % 4 == 0 && aligned_to(z, sizeof(T) * 4) && aligned_to(out, 16);
+  const int per = vec ? 1024 : 256;
+  const dim3 grid((cols + per - 1) / per, static_cast<unsigned>(rows));
+  if (vec) hipLaunchKernelGGL((soft_cap_kernel<T, 4>), grid, dim3(256), 0, st, static_cast<const T*>(z), z_stride, n, item_stride, out, cols, cap, 1.0f / cap);
+  else hipLaunchKernelGGL((soft_cap_kernel<T, 1>), grid, dim3(256), 0, st, static_cast<const T*>(z), z_stride, n, item_stride, out, cols, cap, 1.0f / cap);
+}
+
+// ---------------------------------------------------------------------------------------------------------------
 struct GatedNormParams {
   const void* y;       // [rows, groups * size]
   int64_t y_stride;
@@ -320,6 +526,43 @@ int sgl_amd_residual_norm(int is_f32, int mode, const int64_t* ids, const void* 
   if (is_f32) launch_residual_norm_t<float>(p, vec, as_stream(stream));
   else launch_residual_norm_t<uint16_t>(p, vec, as_stream(stream));
   SGL_CHECK_LAUNCH("residual_norm");
+  return 0;
+}
+
+int sgl_amd_residual_rms(int is_f32, const int64_t* ids, const void* table, int64_t vocab, float scale, const int64_t* positions,
+                         const void* pos_table, int64_t max_positions, const void* a, int a_f32, int a_items, int64_t a_row_stride,
+                         int64_t a_item_stride, const float* a_weight, const void* b, int b_f32, int b_items, int64_t b_row_stride,
+                         int64_t b_item_stride, const float* b_weight, float* x, int64_t x_stride, float* save, const float* extra,
+                         const float* step, const float* weight, void* h, int64_t h_stride, int64_t rows, int width, float eps, void* stream) {
+  SGL_CLEAR_STALE_ERROR();
+  SGL_CHECK_ARG(width > 0 && width <= 16384, "residual_rms: width %d outside 1..16384", width);
+  SGL_CHECK_ARG(x && (!ids || (table && vocab > 0 && !a && !b)) && (!pos_table || (ids && positions && max_positions > 0)),
+                "residual_rms: missing operand, or an embedding beside sublayer outputs");
+  SGL_CHECK_ARG((!a || a_items >= 1) && (!b || b_items >= 1) && (!h || weight), "residual_rms: empty source, or h without its norm");
+  SGL_CHECK_ARG(rows <= 0x7fffffffLL, "residual_rms: too many rows");
+  if (rows <= 0) return 0;
+  ResidualRmsParams p{ids, table, vocab, scale, positions, pos_table, max_positions, {a, is_f32 || a_f32, a_items, a_row_stride, a_item_stride, a_weight},
+                      {b, is_f32 || b_f32, b_items, b_row_stride, b_item_stride, b_weight}, x, x_stride, save, extra, step, weight, h, h_stride, rows,
+                      width, eps};
+  const size_t al = is_f32 ? 16 : 8;
+  const bool vec = width % 4 == 0 && x_stride % 4 == 0 && h_stride % 4 == 0 && a_row_stride % 4 == 0 && a_item_stride % 4 == 0 &&
+                   b_row_stride % 4 == 0 && b_item_stride % 4 == 0 && aligned_to(table, al) && aligned_to(pos_table, al) &&
+                   aligned_to(a, p.a.f32 ? 16 : 8) && aligned_to(b, p.b.f32 ? 16 : 8) && aligned_to(h, al) && aligned_to(x, 16) &&
+                   aligned_to(save, 16) && aligned_to(extra, 16) && aligned_to(step, 16) && aligned_to(weight, 16);
+  if (is_f32) launch_residual_rms<float>(p, vec, as_stream(stream));
+  else launch_residual_rms<uint16_t>(p, vec, as_stream(stream));
+  SGL_CHECK_LAUNCH("residual_rms");
+  return 0;
+}
+
+int sgl_amd_soft_cap(int is_f32, const void* z, int64_t z_row_stride, int items, int64_t item_stride, float* out, int64_t rows, int cols,
+                     float cap, void* stream) {
+  SGL_CLEAR_STALE_ERROR();
+  SGL_CHECK_ARG(z && out && cols > 0 && items >= 1 && cap > 0.f && rows <= 65535, "soft_cap: %d columns, %d items, cap %g", cols, items, cap);
+  if (rows <= 0) return 0;
+  if (is_f32) launch_soft_cap<float>(z, z_row_stride, items, item_stride, out, rows, cols, cap, as_stream(stream));
+  else launch_soft_cap<uint16_t>(z, z_row_stride, items, item_stride, out, rows, cols, cap, as_stream(stream));
+  SGL_CHECK_LAUNCH("soft_cap");
   return 0;
 }
 

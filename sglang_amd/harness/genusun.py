@@ -6,58 +6,32 @@ The model is a list of layer RUNS.  One launch between two sublayers closes the 
 opens the next (its input norm): kernels.residual_norm; in decode batches it also sums the projection's split-K partials."""
 from __future__ import annotations
 
-from dataclasses import dataclass, field
+from dataclasses import dataclass
 from typing import Any, Dict, List, Optional
 
 import torch
 from torch import nn
 
 from .. import kernels
-from ..layers.activation import SiluAndMul, rows_vectorisable
 from ..layers.attention.hybrid_backend import HybridAttnBackend
+from ..layers.feed_forward import DenseMLP
 from ..layers.mixers import MIXERS
 from ..layers.sampler import LogitsProcessorOutput
 from ..mem_cache.memory_pool import HybridReqToTokenPool, LatentTokenToKVPool
+from .layered import LayeredConfig
 
 BF = torch.bfloat16
 
 
 @dataclass
-class GenusunConfig:
-    name: str
-    vocab_size: int
-    hidden_size: int
-    layers: List[Dict[str, Any]]
-    eps: float
+class GenusunConfig(LayeredConfig):
     embedding_scale: float = 1.0
-    loop: Optional[Dict[str, int]] = None
-    num_local_experts: int = field(default=0, init=False)
 
     @classmethod
     def from_dict(cls, d: Dict[str, Any], name: str = "genusun") -> "GenusunConfig":
-        cfg = cls(name, d["vocab"], d["width"], d["layers"], d["norm"]["eps"], d["embedding"]["scale"], d.get("loop"))
-        for i, lay in enumerate(cfg.layers):
-            if lay["type"] not in MIXERS:
-                raise ValueError(f"layer {i}: unknown mixer {lay['type']!r} (have {sorted(MIXERS)})")
-            if lay.get("mlp") is not None and lay["mlp"]["kind"] != "dense":
-                raise ValueError(f"layer {i}: unknown feed-forward {lay['mlp']['kind']!r}")
-        lp = cfg.loop
-        if lp is not None and not (0 <= lp["start"] < lp["stop"] <= len(cfg.layers) and lp["times"] >= 1):
-            raise ValueError(f"loop {lp} does not fit {len(cfg.layers)} layers")
+        cfg = cls(name, d["vocab"], d["width"], d["layers"], d["norm"]["eps"], d.get("loop"), d["embedding"]["scale"])
+        cfg.check(MIXERS, ("dense",))
         return cfg
-
-    def runs(self):
-        """(layer, number of the pass that begins right before it, or None) in execution order."""
-        n = len(self.layers)
-        if self.loop is None:
-            return [(i, None) for i in range(n)]
-        a, b, times = self.loop["start"], self.loop["stop"], self.loop["times"]
-        body = [(i, t if i == a else None) for t in range(times) for i in range(a, b)]
-        return [(i, None) for i in range(a)] + body + [(i, None) for i in range(b, n)]
-
-    @property
-    def num_hidden_layers(self) -> int:
-        return len(self.runs())
 
 
 def _sizes(name: str, width: int, vocab: int, ff: int, heads: int, mamba_heads: int, delta_heads: int, rank: int, window: int,
@@ -69,7 +43,7 @@ def _sizes(name: str, width: int, vocab: int, ff: int, heads: int, mamba_heads: 
                   mixer=dict(heads=heads, dim=128, rot_dim=64, vdim=128, kv_rank=rank, scale=192 ** -0.5, mask=dict(size=window),
                              rot=dict(base=10000.0, dims=64))),
     }
-    return GenusunConfig(name, vocab, width, [mixers[c] for c in pattern], 1e-6, width ** 0.5, loop)
+    return GenusunConfig(name, vocab, width, [mixers[c] for c in pattern], 1e-6, loop, width ** 0.5)
 
 
 CONFIGS: Dict[str, GenusunConfig] = {
@@ -77,24 +51,6 @@ CONFIGS: Dict[str, GenusunConfig] = {
     "genusun-1b": _sizes("genusun-1b", 2048, 32000, 8192, 16, 64, 16, 512, 1024, "mmamdm", dict(start=1, stop=4, times=2)),
     "genusun-8b": _sizes("genusun-8b", 4096, 32000, 14336, 32, 128, 32, 512, 4096, "mmamdm", dict(start=1, stop=4, times=2)),
 }
-
-
-class _DenseMLP(nn.Module):
-    def __init__(self, width: int, m: dict, get, linear):
-        super().__init__()
-        ff = m["ff"]
-        self.gate_up = linear(torch.cat([get("gate", (ff, width)), get("up", (ff, width))], 0),
-                              torch.cat([get("gate.b", (ff,), "zeros"), get("up.b", (ff,), "zeros")], 0))
-        self.down = linear(get("down", (width, ff)), get("down.b", (width,), "zeros"))
-        self.act = SiluAndMul()
-
-    def forward(self, h: torch.Tensor):
-        if self.gate_up.streams(h):                     # decode: bias, silu and the product in the weight stream's epilogue
-            return self.down.forward_partials(kernels.wstream_gemm(h, self.gate_up.weight.data, self.gate_up.bias.data, epilogue="silu_and_mul"))
-        g = self.gate_up(h)
-        if g.dtype == BF and (g.shape[1] // 2) % 8 == 0 and rows_vectorisable(g, g.shape[1]):
-            return self.down(kernels.silu_and_mul(g, round_intermediate=False))
-        return self.down(kernels.gate_mul(g))
 
 
 class _Norm(nn.Module):
@@ -123,7 +79,7 @@ class _Layer(nn.Module):
         self.mlp = None
         if lay.get("mlp") is not None:
             self.norm2, self.norm2b = _Norm(get, f"l{i}.norm2", W), _Norm(get, f"l{i}.norm2b", W)
-            self.mlp = _DenseMLP(W, lay["mlp"], sub("mlp"), linear)
+            self.mlp = DenseMLP(W, lay["mlp"]["ff"], sub("mlp"), linear)
 
 
 class GenusunForCausalLM(nn.Module):

@@ -5,13 +5,15 @@ import json
 from pathlib import Path
 from typing import Any, Callable, Dict
 
-from . import genusun, models
+from . import genusun, models, mosurax
 
 # config.json "architecture" -> reader of the file
-ARCHITECTURES: Dict[str, Callable[[dict, str], Any]] = {"Genusun": genusun.GenusunConfig.from_dict}
-_MODELS = {models.ModelConfig: models.CausalLM, genusun.GenusunConfig: genusun.GenusunForCausalLM}
+ARCHITECTURES: Dict[str, Callable[[dict, str], Any]] = {"Genusun": genusun.GenusunConfig.from_dict, "Mosurax": mosurax.MosuraxConfig.from_dict}
+_MODELS = {models.ModelConfig: models.CausalLM, genusun.GenusunConfig: genusun.GenusunForCausalLM,
+           mosurax.MosuraxConfig: mosurax.MosuraxForCausalLM}
 # HIP units (sglang_amd/csrc) a model's path needs; a model that is not listed uses the whole library
-_UNITS = {genusun.GenusunConfig: "hybrid"}
+_UNITS = {genusun.GenusunConfig: "hybrid", mosurax.MosuraxConfig: "grouped"}
+_NAMED = (models.CONFIGS, genusun.CONFIGS, mosurax.CONFIGS)
 
 
 def model_class(config):
@@ -36,14 +38,14 @@ def load_config(path):
 
 
 def named_config(name: str):
-    for table in (models.CONFIGS, genusun.CONFIGS):
+    for table in _NAMED:
         if name in table:
             return table[name]
-    raise KeyError(f"unknown model {name!r} (have {sorted(list(models.CONFIGS) + list(genusun.CONFIGS))})")
+    raise KeyError(f"unknown model {name!r} (have {config_names()})")
 
 
 def config_names():
-    return sorted(list(models.CONFIGS) + list(genusun.CONFIGS))
+    return sorted(n for table in _NAMED for n in table)
 
 
 def runner_for(model: str, dtype=None, device=None, **kw):

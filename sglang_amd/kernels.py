@@ -1249,6 +1249,86 @@ def residual_norm(x: torch.Tensor, eps: float, *, embed: Optional[Tuple[torch.Te
                 rows, W, float(eps), _stream())
 
 
+class ExpertRows:
+    """The routed experts' outputs on their way into the launch that sums them: data [tokens, top, W] and fp32 weights [tokens, top]."""
+
+    def __init__(self, data: torch.Tensor, weights: torch.Tensor):
+        self.data, self.weights = data, weights
+
+
+def _row_source(who: str, y, rows: int, W: int):
+    """(data, fp32?, items, row stride, item stride, weights) of one addend: rows [rows, W], Partials or ExpertRows."""
+    if y is None:
+        return None, 0, 0, 0, 0, None
+    if isinstance(y, Partials):
+        _need((y.rows, y.cols) == (rows, W) and y.bias is None, f"{who}: partials are [splits, rows, W] without a bias")
+        return y.data, 1, y.splits, W, rows * W, None
+    if isinstance(y, ExpertRows):
+        d = y.data
+        _need(d.dim() == 3 and (d.shape[0], d.shape[2]) == (rows, W) and d.stride(2) == 1 and tuple(y.weights.shape) == tuple(d.shape[:2]),
+              f"{who}: expert rows are [rows, top, W] with weights [rows, top]")
+        _f32(who, y.weights)
+        return d, int(d.dtype == torch.float32), d.shape[1], d.stride(0), d.stride(1), y.weights
+    _rows(who, y)
+    _need(tuple(y.shape) == (rows, W), f"{who}: row operands are [rows, W]")
+    return y, int(y.dtype == torch.float32), 1, y.stride(0), 0, None
+
+
+def residual_rms(x: torch.Tensor, eps: float, *, embed: Optional[Tuple[torch.Tensor, torch.Tensor, float]] = None,
+                 pos: Optional[Tuple[torch.Tensor, torch.Tensor]] = None, add: tuple = (), save: Optional[torch.Tensor] = None,
+                 extra: Optional[torch.Tensor] = None, step: Optional[torch.Tensor] = None, norm: Optional[torch.Tensor] = None,
+                 h: Optional[torch.Tensor] = None) -> None:
+    """Update the fp32 residual rows `x` -- embed = (ids, table, scale) with pos = (positions, table): embedding row + position row;
+    else x + the addends `add` (at most two: rows, Partials or ExpertRows) -- copy them to `save`, add the rows `extra` and the
+    vector `step`, then h = RMS norm(x) * norm, in one launch."""
+    _need(x.dtype == torch.float32 and x.dim() == 2 and x.stride(1) == 1, "residual_rms: fp32 residual rows")
+    _need(len(add) <= 2 and not (embed is not None and len(add)) and (pos is None or embed is not None), "residual_rms: an embedding, or at most two addends")
+    _need((h is None) == (norm is None), "residual_rms: h and its norm come together")
+    rows, W = x.shape
+    ids = table = positions = pos_table = None
+    scale = 0.0
+    if embed is not None:
+        ids, table, scale = embed
+        _i64("residual_rms", ids)
+        _need(ids.numel() == rows and table.dim() == 2 and table.shape[1] == W and table.is_contiguous(), "residual_rms: table [V, W], ids [rows]")
+        if pos is not None:
+            positions, pos_table = pos
+            _i64("residual_rms", positions)
+            _need(positions.numel() == rows and pos_table.dim() == 2 and pos_table.shape[1] == W and pos_table.is_contiguous()
+                  and pos_table.dtype == table.dtype, "residual_rms: position table [P, W], positions [rows]")
+    a, b = (_row_source("residual_rms", y, rows, W) for y in (tuple(add) + (None, None))[:2])
+    _rows("residual_rms", h)
+    for t in (save, extra):
+        _need(t is None or (t.dtype == torch.float32 and t.is_contiguous() and tuple(t.shape) == (rows, W)), "residual_rms: contiguous fp32 rows")
+    for t in (step, norm):
+        _need(t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == W), "residual_rms: fp32 parameters [W]")
+    _need(h is None or tuple(h.shape) == (rows, W), "residual_rms: h [rows, W]")
+    _dev(x, ids, table, positions, pos_table, a[0], b[0], save, extra, step, norm, h)
+    acts = [t for t in (table, h, *(s[0] for s in (a, b) if s[0] is not None and not s[1])) if t is not None]
+    f32 = _is_f32(*acts) if acts else 1
+    native.call("sgl_amd_residual_rms", f32, _ptr(ids), _ptr(table), table.shape[0] if table is not None else 0, float(scale), _ptr(positions),
+                _ptr(pos_table), pos_table.shape[0] if pos_table is not None else 0, _ptr(a[0]), *a[1:5], _ptr(a[5]), _ptr(b[0]), *b[1:5], _ptr(b[5]),
+                x.data_ptr(), x.stride(0), _ptr(save), _ptr(extra), _ptr(step), _ptr(norm), _ptr(h), h.stride(0) if h is not None else 0, rows, W,
+                float(eps), _stream())
+
+
+def soft_cap(z, cap: float) -> torch.Tensor:
+    """cap * tanh(z / cap) in fp32 of logits [n, V], or of their split-K Partials."""
+    if isinstance(z, Partials):
+        _need(z.bias is None, "soft_cap: partials without a bias")
+        data, f32, n, V, stride, items, item = z.data, 1, z.rows, z.cols, z.cols, z.splits, z.rows * z.cols
+    else:
+        _rows("soft_cap", z)
+        data, f32, (n, V), stride, items, item = z, _is_f32(z), z.shape, z.stride(0), 1, 0
+    _dev(data)
+    out = torch.empty((n, V), dtype=torch.float32, device=data.device)
+    es = data.element_size()
+    for r in range(0, n, 65535):
+        native.call("sgl_amd_soft_cap", f32, data.data_ptr() + r * stride * es, stride, items, item, out.data_ptr() + r * V * 4, min(65535, n - r), V,
+                    float(cap), _stream())
+    return out
+
+
 def gated_rmsnorm(y: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, groups: int, eps: float, gate_first: bool,
                   out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """RMS norm of `groups` equal column groups with a silu gate: before the norm (gate_first) or behind it.  `weight` covers
@@ -1479,3 +1559,141 @@ def latent_prefill(q: torch.Tensor, latents: torch.Tensor, kv: torch.Tensor, key
                 keys.first.data_ptr(), positions.data_ptr(), out.data_ptr(), out.stride(0), heads, dim, rot, rank, vdim, int(window),
                 float(scale), _stream())
     return out
+
+
+# ---------------------------------------------------------------------------- grouped-query attention with sizes of its own
+def grouped_attention_matrix_form(kd: int, vd: int) -> bool:
+    return bool(native.lib().sgl_amd_grouped_attention_matrix_form(kd, vd))
+
+
+def grouped_prefill_supported(kd: int, vd: int, group: int) -> bool:
+    return bool(native.lib().sgl_amd_grouped_prefill_supported(kd, vd, group))
+
+
+class QueryBlocks:
+    """The workgroups of a prefill launch: int32 [n, 2] (segment, first token), `rows` query rows each, the ones with the most
+    visible keys first."""
+
+    def __init__(self, prefix_lens, extend_lens, window: int, group: int, device, rows: Optional[int] = None):
+        rows = native.lib().sgl_amd_grouped_prefill_rows() if rows is None else rows
+        tokens, w = rows // group, window if window > 0 else 1 << 40
+        blocks = sorted(((b, q) for b, n in enumerate(extend_lens) for q in range(0, n, tokens)), key=lambda e: -min(prefix_lens[e[0]] + e[1], w))
+        self.blocks = torch.tensor(blocks, dtype=torch.int32).reshape(-1, 2).to(device, non_blocking=True)
+        self.group = group
+
+
+def _grouped_checks(who: str, q: torch.Tensor, cache: torch.Tensor, out: torch.Tensor, gate: Optional[torch.Tensor], heads: int, kv_heads: int,
+                    kd: int, vd: int, req_to_token: torch.Tensor) -> None:
+    T = q.shape[0]
+    _rows(who, q, cache, out, gate)
+    _need(heads % kv_heads == 0 and q.shape[1] == heads * kd and cache.shape[1] >= kv_heads * (kd + vd) and tuple(out.shape) == (T, heads * vd)
+          and (gate is None or tuple(gate.shape) == (T, heads * vd)) and req_to_token.dtype == torch.int32 and req_to_token.stride(1) == 1,
+          f"{who}: shapes")
+
+
+def grouped_kv_store(k: torch.Tensor, v: torch.Tensor, cache: torch.Tensor, loc: torch.Tensor, kv_heads: int) -> None:
+    """k [T, kv_heads * kd], v [T, kv_heads * vd] into the cache rows `loc`, [kv_heads][kd | vd]."""
+    _dev(k, v, cache, loc)
+    _rows("grouped_kv_store", k, v, cache)
+    _i64("grouped_kv_store", loc)
+    _need(k.shape[0] == v.shape[0] == loc.numel() and k.shape[1] % kv_heads == 0 and v.shape[1] % kv_heads == 0
+          and cache.shape[1] >= k.shape[1] + v.shape[1], "grouped_kv_store: shapes")
+    native.call("sgl_amd_grouped_kv_store", _is_f32(k, v, cache), k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), cache.data_ptr(),
+                cache.stride(0), loc.data_ptr(), k.shape[0], kv_heads, k.shape[1] // kv_heads, v.shape[1] // kv_heads, _stream())
+
+
+def grouped_attention(q: torch.Tensor, cache: torch.Tensor, req_to_token: torch.Tensor, req_pool_indices: torch.Tensor, positions: torch.Tensor,
+                      seg: Segments, heads: int, kv_heads: int, kd: int, vd: int, window: int, scale: float, *, sink: Optional[float] = None,
+                      gate: Optional[torch.Tensor] = None, new: Optional[Tuple[torch.Tensor, torch.Tensor, torch.Tensor]] = None, splits: int = 1,
+                      plain: bool = False) -> torch.Tensor:
+    """q [T, heads * kd] over the cached keys of each token's request -> [T, heads * vd], times sigmoid(gate).  new = (k, v, loc): a
+    decode batch's own keys and values, stored on the way (matrix form).  `plain` forces the form without matrix instructions."""
+    _dev(q, cache, req_to_token, req_pool_indices, positions, gate)
+    T = q.shape[0]
+    _seg_checks("grouped_attention", seg, req_pool_indices, positions, T)
+    out = torch.empty((T, heads * vd), dtype=q.dtype, device=q.device)
+    _grouped_checks("grouped_attention", q, cache, out, gate, heads, kv_heads, kd, vd, req_to_token)
+    k = v = loc = None
+    if new is not None:
+        k, v, loc = new
+        _dev(k, v, loc)
+        _rows("grouped_attention", k, v)
+        _i64("grouped_attention", loc)
+        _need(seg.tok_seg is None and tuple(k.shape) == (T, kv_heads * kd) and tuple(v.shape) == (T, kv_heads * vd) and loc.numel() == T
+              and k.dtype == v.dtype == q.dtype, "grouped_attention: new keys and values belong to a decode batch")
+    po = pml = None
+    if splits > 1:
+        po = torch.empty((T, heads, splits, vd), dtype=torch.float32, device=q.device)
+        pml = torch.empty((T, heads, splits, 2), dtype=torch.float32, device=q.device)
+    native.call("sgl_amd_grouped_attention", _is_f32(q, cache, gate), q.data_ptr(), q.stride(0), cache.data_ptr(), cache.stride(0), _ptr(k),
+                k.stride(0) if k is not None else 0, _ptr(v), v.stride(0) if v is not None else 0, _ptr(loc), req_to_token.data_ptr(),
+                req_to_token.stride(0), req_pool_indices.data_ptr(), _ptr(seg.tok_seg), positions.data_ptr(), _ptr(gate),
+                gate.stride(0) if gate is not None else 0, out.data_ptr(), out.stride(0), _ptr(po), _ptr(pml), T, heads, kv_heads, kd, vd, int(window),
+                splits, float(scale), float("-inf") if sink is None else float(sink), 1 if plain else 0, _stream())
+    return out
+
+
+def grouped_prefill(q: torch.Tensor, cache: torch.Tensor, req_to_token: torch.Tensor, req_pool_indices: torch.Tensor, positions: torch.Tensor,
+                    seg: Segments, blocks: QueryBlocks, heads: int, kv_heads: int, kd: int, vd: int, window: int, scale: float, *,
+                    sink: Optional[float] = None, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """grouped_attention over long extends whose keys are stored (bf16)."""
+    _dev(q, cache, req_to_token, req_pool_indices, positions, gate, blocks.blocks)
+    T = q.shape[0]
+    _seg_checks("grouped_prefill", seg, req_pool_indices, positions, T)
+    out = torch.empty((T, heads * vd), dtype=q.dtype, device=q.device)
+    _grouped_checks("grouped_prefill", q, cache, out, gate, heads, kv_heads, kd, vd, req_to_token)
+    _need(_is_f32(q, cache, gate) == 0 and seg.start is not None and blocks.group == heads // kv_heads, "grouped_prefill: bf16 segments, blocks of this group size")
+    native.call("sgl_amd_grouped_prefill", q.data_ptr(), q.stride(0), cache.data_ptr(), cache.stride(0), req_to_token.data_ptr(),
+                req_to_token.stride(0), req_pool_indices.data_ptr(), blocks.blocks.data_ptr(), blocks.blocks.shape[0], seg.start.data_ptr(),
+                seg.len.data_ptr(), positions.data_ptr(), _ptr(gate), gate.stride(0) if gate is not None else 0, out.data_ptr(), out.stride(0), heads,
+                kv_heads, kd, vd, int(window), float(scale), float("-inf") if sink is None else float(sink), _stream())
+    return out
+
+
+# ---------------------------------------------------------------------------- routed experts behind a biased router
+def moe_route(h: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], top: int) -> Tuple[torch.Tensor, torch.Tensor]:
+    """The `top` largest of w h + bias (fp32) and the softmax over those: fp32 weights, int32 ids [T, top]."""
+    _dev(h, w, bias)
+    _rows("moe_route", h)
+    _f32("moe_route", bias)
+    T, K = h.shape
+    _need(w.dim() == 2 and w.shape[1] == K and w.is_contiguous() and (bias is None or bias.numel() == w.shape[0]), "moe_route: shapes")
+    weights = torch.empty((T, top), dtype=torch.float32, device=h.device)
+    ids = torch.empty((T, top), dtype=torch.int32, device=h.device)
+    native.call("sgl_amd_moe_route", _is_f32(h, w), h.data_ptr(), h.stride(0), w.data_ptr(), _ptr(bias), weights.data_ptr(), ids.data_ptr(), T, K,
+                w.shape[0], top, _stream())
+    return weights, ids
+
+
+def _experts_plain(x: torch.Tensor, w: torch.Tensor, ids: torch.Tensor, up: bool) -> torch.Tensor:
+    E, N, K = w.shape[0], w.shape[1] // (2 if up else 1), w.shape[2]
+    pairs, top = ids.numel(), ids.shape[1]
+    _rows("experts", x)
+    _need(w.is_contiguous() and ids.dtype == torch.int32 and ids.is_contiguous() and x.shape == (ids.shape[0] if up else pairs, K), "experts: shapes")
+    out = torch.empty((pairs, N), dtype=x.dtype, device=x.device)
+    native.call("sgl_amd_experts_plain", _is_f32(x, w), 1 if up else 0, x.data_ptr(), x.stride(0), w.data_ptr(), ids.data_ptr(), out.data_ptr(), N, pairs,
+                top, N, K, E, _stream())
+    return out
+
+
+def routed_experts(h: torch.Tensor, w13: torch.Tensor, w2: torch.Tensor, ids: torch.Tensor, plain: bool = False) -> torch.Tensor:
+    """Every token's chosen experts, silu(gate h) * (up h) and the down projection, unweighted: [T, top, W] in the type of h.  bf16 rows
+    run on the grouped matrix kernels of fused_experts; fp32 rows and sizes they do not take go through a plain form."""
+    _dev(h, w13, w2, ids)
+    (T, W), (E, N2, _), top = h.shape, w13.shape, ids.shape[1]
+    N, numel = N2 // 2, T * top
+    if plain or h.dtype != _BF16 or W % 8 or W < 32 or N % 32:
+        return _experts_plain(_experts_plain(h, w13, ids, True), w2, ids, False).view(T, top, W)
+    inter = torch.empty((numel, N), dtype=_BF16, device=h.device)
+    down = torch.empty((numel, W), dtype=_BF16, device=h.device)
+    if numel // E >= MOE_TILED_MIN_ROWS_PER_EXPERT and W % 64 == 0 and N % 64 == 0:
+        block_m, up_rows, down_rows = moe_tile_plan(numel, E, N, W) if MOE_TILE_OVERRIDE is None else MOE_TILE_OVERRIDE
+        s = moe_align_block_size(ids, block_m, E)
+        moe_tiled_gemm(h, w13, inter, *s, None, False, top, numel, block_m, fuse_silu=True, tile_rows=up_rows)
+        moe_tiled_gemm(inter, w2, down, *s, None, False, 1, numel, block_m, tile_rows=down_rows)
+    else:
+        block_m = choose_moe_block_m(numel, E)
+        s = moe_align_block_size(ids, block_m, E)
+        (moe_wstream_gemm if W % 128 == 0 else moe_grouped_gemm)(h, w13, inter, *s, None, False, top, numel, block_m, fuse_silu=True)
+        (moe_wstream_gemm if W % 16 == 0 and N % 128 == 0 else moe_grouped_gemm)(inter, w2, down, *s, None, False, 1, numel, block_m)
+    return down.view(T, top, W)

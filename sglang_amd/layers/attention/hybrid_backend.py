@@ -1,4 +1,4 @@
-"""Attention backend of models that mix latent attention with recurrent layers.
+"""Attention backend of models that mix latent or grouped-query attention of any sizes with recurrent layers.
 
 Per forward it holds what every mixer needs of the batch: the segments of the packed tokens (none for a decode batch: one
 token per request), the request rows (= state slots) and the positions.  Like HipAttnBackend nothing is gathered on the host
@@ -20,22 +20,25 @@ class HybridAttnBackend(AttentionBackend):
         self.device = model_runner.device
         self.req_to_token_pool = model_runner.req_to_token_pool
         self.token_to_kv_pool = model_runner.token_to_kv_pool
-        self.state_pool = model_runner.req_to_token_pool.state_pool
+        self.state_pool = getattr(model_runner.req_to_token_pool, "state_pool", None)      # (models without recurrent layers)
         self.max_context_len = model_runner.req_to_token_pool.max_context_len
         self.segments = kernels.Segments()
         self._extend = None            # (prefix lengths, extend lengths) of the current extend batch
         self._keys = {}                # window -> kernels.VisibleKeys of the current extend batch
+        self._blocks = {}              # (window, group) -> kernels.QueryBlocks of the current extend batch
         self.latent_form = None        # tests: "absorbed" / "expanded" forces the form of every extend
+        self.grouped_form = None       # tests: "rows" / "prefill" / "plain" forces the form of grouped-query attention
 
     # ------------------------------------------------------------------ per-step metadata
     def init_forward_metadata_out_graph(self, forward_batch, in_capture: bool = False):
         mode = forward_batch.forward_mode
         if getattr(mode, "is_target_verify", lambda: False)():
-            raise NotImplementedError("a tree of draft tokens cannot be verified over recurrent state (one state per request)")
+            raise NotImplementedError("a tree of draft tokens cannot be verified here: recurrent layers hold one state per request, and these "
+                                      "attention kernels take no tree mask")
         if mode.is_decode() or mode.is_idle():
             self.segments = kernels.Segments()
             return
-        self._extend, self._keys = (list(forward_batch.extend_prefix_lens_cpu), list(forward_batch.extend_seq_lens_cpu)), {}
+        self._extend, self._keys, self._blocks = (list(forward_batch.extend_prefix_lens_cpu), list(forward_batch.extend_seq_lens_cpu)), {}, {}
         lens = torch.tensor(forward_batch.extend_seq_lens_cpu, dtype=torch.int64)
         tok_seg = torch.repeat_interleave(torch.arange(len(lens), dtype=torch.int32), lens)
         self.segments = kernels.Segments(tok_seg.to(self.device, non_blocking=True), forward_batch.extend_start_loc.to(torch.int32),
@@ -71,6 +74,38 @@ class HybridAttnBackend(AttentionBackend):
         oc = kernels.latent_attention(qc, q3[:, :, layer.dim:], cache, self.req_to_token_pool.req_to_token, forward_batch.req_pool_indices,
                                       forward_batch.positions, self.segments, layer.window, layer.scale, self._splits(layer, T))
         return kernels.head_gemm(oc, layer.w_value).view(T, layer.heads * layer.vdim)
+
+    # Extends shorter than this go token by token, like decode batches; longer ones as tiles of query rows.
+    PREFILL_MIN_TOKENS = 16
+
+    def grouped_attention(self, layer, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate, run_id: int, forward_batch) -> torch.Tensor:
+        """q [T, heads * kd], k [T, kv_heads * kd], v [T, kv_heads * vd] and the gate [T, heads * vd] as projected -> gated values
+        [T, heads * vd].  A decode step on the matrix form stores its own keys and values on the way."""
+        rows, T = self.token_to_kv_pool.get_kv_rows(run_id), q.shape[0]
+        sizes = (layer.heads, layer.kv_heads, layer.kd, layer.vd, layer.window, layer.scale)
+        where = (rows, self.req_to_token_pool.req_to_token, forward_batch.req_pool_indices, forward_batch.positions, self.segments)
+        matrix, form = layer.matrix and self.grouped_form != "plain", self.grouped_form
+        new = None
+        if matrix and forward_batch.forward_mode.is_decode():
+            new = (k, v, forward_batch.out_cache_loc)
+        else:
+            kernels.grouped_kv_store(k, v, rows, forward_batch.out_cache_loc, layer.kv_heads)
+        if (matrix and layer.prefill and forward_batch.forward_mode.is_extend()
+                and (max(self._extend[1]) >= self.PREFILL_MIN_TOKENS if form is None else form == "prefill")):
+            key = (layer.window, layer.group)
+            if key not in self._blocks:
+                self._blocks[key] = kernels.QueryBlocks(*self._extend, layer.window, layer.group, self.device)
+            return kernels.grouped_prefill(q, *where, self._blocks[key], *sizes, sink=layer.sink, gate=gate)
+        return kernels.grouped_attention(q, *where, *sizes, sink=layer.sink, gate=gate, new=new, splits=self._grouped_splits(layer, T, matrix),
+                                         plain=not matrix)
+
+    def _grouped_splits(self, layer, tokens: int, matrix: bool) -> int:
+        """Workgroups enough for the chip on small batches, never shorter than 128 keys; a function of the batch size and the context
+        bound only (fixed inside a captured graph)."""
+        keys = min(layer.window, self.max_context_len) if layer.window > 0 else self.max_context_len
+        groups = layer.kv_heads * ((layer.group + 15) // 16) if matrix else layer.heads
+        want = (512 + tokens * groups - 1) // (tokens * groups)
+        return max(1, min(want, (keys + 127) // 128, 32))
 
     def _expanded(self, layer) -> bool:
         """Which form of an extend costs less: per (query, key) pair the absorbed form multiplies 2 rank + rot elements, the

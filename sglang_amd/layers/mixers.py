@@ -1,4 +1,5 @@
-"""Token mixers beside RadixAttention: latent attention, the gated delta rule and Mamba-2.  A mixer owns its projections and
+"""Token mixers beside RadixAttention: latent attention, grouped-query attention with sizes of its own, the gated delta rule and
+Mamba-2.  A mixer owns its projections and
 constants; caches, states and kernel dispatch belong to the attention backend (layers/attention/hybrid_backend.py).
 
 Every module takes its tensors from `get(name, shape, init)` (harness/weights.py) and merges the projections that share an
@@ -65,6 +66,53 @@ class LatentAttention(nn.Module):
         p = self.in_proj(h)
         o = fb.attn_backend.latent_attention(self, p[:, :self.q_rows], p[:, self.q_rows:self.q_rows + self.dkv_rows], run_id, fb)
         return self.o_proj.forward_partials(o)
+
+
+def padded_heads(w: torch.Tensor, heads: int, dim: int, to: int, axis: int) -> torch.Tensor:
+    """Zeros behind every head of `dim` rows (axis 0) or columns (axis 1) up to `to`."""
+    if dim == to:
+        return w
+    split = w.unflatten(axis, (heads, dim))
+    out = split.new_zeros(split.shape[:axis] + (heads, to) + split.shape[axis + 2:])
+    out.narrow(axis + 1, 0, dim).copy_(split)
+    return out.flatten(axis, axis + 1)
+
+
+class GroupedAttention(nn.Module):
+    """Grouped-query attention without rotation: own key and value widths, an optional sliding window (mask.size), an optional sink (a
+    score in the softmax denominator that carries no value) and an optional sigmoid gate on the heads' outputs.  Head vectors are
+    padded with zeros to multiples of 8 elements, in the projections and in the cache."""
+
+    def __init__(self, width: int, m: dict, eps: float, get: Callable, linear: Callable, max_positions: int, device, *,
+                 sink: Optional[float] = None, gated: bool = False):
+        super().__init__()
+        self.heads, self.kv_heads, dim, vdim = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        self.window, self.scale, self.sink = (m.get("mask") or {}).get("size", 0), float(m["scale"]), sink
+        H, G = self.heads, self.kv_heads
+        if H % G:
+            raise ValueError(f"grouped attention: {H} query heads over {G} key heads")
+        self.kd, self.vd, self.group = dim + -dim % 8, vdim + -vdim % 8, H // G
+        parts = [padded_heads(get("q", (H * dim, width)), H, dim, self.kd, 0), padded_heads(get("k", (G * dim, width)), G, dim, self.kd, 0),
+                 padded_heads(get("v", (G * vdim, width)), G, vdim, self.vd, 0)]
+        if gated:
+            parts.append(padded_heads(get("g", (H * vdim, width)), H, vdim, self.vd, 0))
+        self.gated = gated
+        self.in_proj = linear(merged_rows(parts))
+        self.o_proj = linear(padded_heads(get("o", (width, H * vdim)), H, vdim, self.vd, 1).contiguous())
+        self.matrix = self.in_proj.weight.dtype == torch.bfloat16 and self.scale > 0 and kernels.grouped_attention_matrix_form(self.kd, self.vd)
+        self.prefill = self.matrix and kernels.grouped_prefill_supported(self.kd, self.vd, self.group)
+
+    @property
+    def cache_spec(self):
+        return self.kv_heads, self.kd, self.vd
+
+    def forward(self, h: torch.Tensor, run_id: int, fb) -> torch.Tensor:
+        p = self.in_proj(h)
+        a = self.heads * self.kd
+        b = a + self.kv_heads * self.kd
+        c = b + self.kv_heads * self.vd
+        gate = p[:, c:c + self.heads * self.vd] if self.gated else None
+        return self.o_proj.forward_partials(fb.attn_backend.grouped_attention(self, p[:, :a], p[:, a:b], p[:, b:c], gate, run_id, fb))
 
 
 class GatedDelta(nn.Module):

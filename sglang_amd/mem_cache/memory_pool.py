@@ -196,6 +196,27 @@ class LatentTokenToKVPool:
         return sum(b.numel() * b.element_size() for b in self.latent_buffer), 0
 
 
+class GroupedTokenToKVPool:
+    """Key / value cache of grouped-query layers with sizes of their own: per attention run one row per token, [kv_heads][key | value],
+    a head's key and value side by side.  Runs may differ in every size (`specs`: kv heads, key and value elements)."""
+
+    is_fp8 = False
+    use_hnd = False
+
+    def __init__(self, size: int, page_size: int, dtype: torch.dtype, specs, device):
+        assert dtype in (torch.bfloat16, torch.float32)
+        self.size, self.page_size, self.dtype, self.device = size, page_size, dtype, device
+        self.layer_num = len(specs)
+        # zero-filled: slot 0's page is the sink of padded batch entries
+        self.kv_rows = [torch.zeros((size + page_size, g * (k + v)), dtype=dtype, device=device) for g, k, v in specs]
+
+    def get_kv_rows(self, run_id: int) -> torch.Tensor:
+        return self.kv_rows[run_id]
+
+    def get_kv_size_bytes(self):
+        return sum(b.numel() * b.element_size() for b in self.kv_rows), 0
+
+
 class RecurrentStatePool:
     """One slot per request row for every recurrent run: the fp32 state [slots, heads, rows, columns] and the ring of past
     convolution inputs [slots, taps, channels] in the activation type.  Slot 0 absorbs padded (graph) batch entries.  A
