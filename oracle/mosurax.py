@@ -56,10 +56,15 @@ def gated_mlp(h, gate, up, down):
     return oh.linear(oh._r(oh.silu(oh.linear(h, gate)) * oh.linear(h, up)), down)
 
 
+margins: List[float] = []      # smallest gap of every route() call between the last expert taken and the first one left out
+
+
 def route(h, w, b, top):
     """The `top` largest of the logits w h + b per token and the softmax over those alone -> (weights, experts) [T, top]."""
-    z, e = torch.topk(h @ w.T + b, top, dim=-1)
-    return torch.softmax(z, -1), e
+    z, e = torch.sort(h @ w.T + b, dim=-1, descending=True)
+    if top < z.shape[1]:
+        margins.append(float((z[:, top - 1] - z[:, top]).min()))
+    return torch.softmax(z[:, :top], -1), e[:, :top]
 
 
 def moe_mlp(h, w, m):
@@ -131,12 +136,17 @@ def tensor_shapes(cfg: dict) -> Dict[str, Tuple[int, ...]]:
     return out
 
 
+CODE_DIMS, CODES = 8, 12
+
+
 def random_weights(cfg: dict, seed: int) -> Dict[str, torch.Tensor]:
-    """bf16 weights whose every branch matters: matrices keep unit variance, norms spread around 1, router logits are far enough
-    apart that no token sits between two experts."""
+    """bf16 weights whose every branch matters: matrices keep unit variance, norms spread around 1.  No token sits between two
+    experts: the first CODE_DIMS columns of the embedding hold one of CODES sign patterns, nothing else writes to those columns of
+    the residual, and the routers read only them, drawn until every pattern's choice is clear."""
     g = torch.Generator().manual_seed(seed)
-    out = {}
-    for name, shape in tensor_shapes(cfg).items():
+    code = torch.randint(0, 2, (CODES, CODE_DIMS), generator=g) * 4.0 - 2.0
+    shapes, out = tensor_shapes(cfg), {}
+    for name, shape in shapes.items():
         r = torch.randn(shape, generator=g)
         last = name.split(".")[-1]
         if last in ("norm1", "norm2", "norm"):
@@ -145,9 +155,27 @@ def random_weights(cfg: dict, seed: int) -> Dict[str, torch.Tensor]:
             t = r
         elif last in ("step", "b"):
             t = r * 0.5
-        elif last == "router":
-            t = r * 3.0 / math.sqrt(shape[1])
         else:
             t = r / math.sqrt(shape[1])
+        if last == "embed":
+            t[:, :CODE_DIMS] = code[torch.arange(shape[0]) % CODES]
+        elif last in ("pos", "step"):
+            t[:, :CODE_DIMS] = 0.0
+        elif last in ("o", "down"):
+            t[:CODE_DIMS] = 0.0
         out[name] = t.to(torch.bfloat16)
+    for name in (n for n in shapes if n.endswith(".router")):
+        top, best = next(lay["mlp"]["router"]["top"] for i, lay in enumerate(cfg["layers"]) if name.startswith(f"l{i}.")), None
+        c = code * out[name.replace("mlp.router", "norm2")][:CODE_DIMS].float()
+        for _ in range(200):
+            w = torch.zeros(shapes[name])
+            w[:, :CODE_DIMS] = torch.randn((shapes[name][0], CODE_DIMS), generator=g)
+            gap = float("inf")
+            for s in (0.3, 0.6, 1.0):
+                z = torch.sort(s * c @ w[:, :CODE_DIMS].T + out[name + ".b"].float(), dim=-1, descending=True).values
+                if top < z.shape[1]:
+                    gap = min(gap, float((z[:, top - 1] - z[:, top]).min()))
+            if best is None or gap > best[0]:
+                best = (gap, w)
+        out[name] = best[1].to(torch.bfloat16)
     return out
