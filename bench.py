@@ -187,8 +187,8 @@ def parse_args():
     ap.add_argument("--no-reference-scheduler", action="store_true", help="skip the leg that runs the job under the reference's Scheduler")
     ap.add_argument("--cpu-budget-s", type=float, default=30.0)
     ap.add_argument("--hybrid", nargs="*", metavar="NAME", default=None,
-                    help="instead of the default workload: throughput and kernel table of hybrid models (default genusun-1b genusun-8b) "
-                         "beside a plain decoder of equal size, on one GPU")
+                    help="instead of the default workload: throughput and kernel table of layered models (default genusun-1b genusun-8b; also "
+                         "mosurax-1b mosurax-8b) beside plain decoders of equal size, on one GPU")
     ap.add_argument("--hybrid-kernels-only", action="store_true", help="with --hybrid: the kernel table alone")
     return ap.parse_args()
 

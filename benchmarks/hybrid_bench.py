@@ -1,8 +1,9 @@
-"""Throughput of the hybrid design (Genusun) beside the closest decoder of this framework at equal size, and every kernel of the
-design against its roofline beside the like kernel of that decoder.  Run through `bench.py --hybrid`; random weights.
+"""Throughput of the layered designs (Genusun here, Mosurax with grouped_bench.py) beside the closest decoders of this framework at
+equal size, and every kernel of a design against its roofline beside the like kernel of such a decoder.  Run through
+`bench.py --hybrid`; random weights.
 
 The decoder beside it has the same width, feed-forward width, vocabulary and number of attention heads and as many layers as the
-hybrid executes layer runs.  One JSON line: prompt tokens / s of cold prefills, tokens / s of graph-replayed decode steps, and a
+design executes layer runs.  One JSON line: prompt tokens / s of cold prefills, tokens / s of graph-replayed decode steps, and a
 kernel table (us, fraction of the roofline: 8 TB/s HBM, 2.5 PFLOP/s bf16, 157 TFLOP/s fp32 matrix)."""
 from __future__ import annotations
 
@@ -233,16 +234,20 @@ def kernel_table(cfg, device, T=8192, segs=4, B=64, ctx=1024):
 
 
 def run(names, device, kernels_only=False):
+    from benchmarks import grouped_bench
+    from sglang_amd.harness.mosurax import MosuraxConfig
     from sglang_amd.harness.registry import named_config
 
     out = {}
     for name in names:
         cfg = named_config(name)
+        grouped = isinstance(cfg, MosuraxConfig)
         shape = dict(prompts=4, length=2048, batch=64, ctx=1024)
-        r = dict(shape=shape, kernels=kernel_table(cfg, device))
+        r = dict(shape=shape, kernels=(grouped_bench.kernel_table if grouped else kernel_table)(cfg, device))
         torch.cuda.empty_cache()
         if not kernels_only:
-            r["hybrid"] = throughput(cfg, device, **shape)
-            r["decoder_beside"] = throughput(_llama_beside(cfg), device, **shape)
+            r["design" if grouped else "hybrid"] = throughput(cfg, device, **shape)
+            for key, beside in (grouped_bench.decoders_beside(cfg) if grouped else {"decoder_beside": _llama_beside(cfg)}).items():
+                r[key] = throughput(beside, device, **shape)
         out[name] = r
     print(json.dumps({"hybrid": out, "dtype": "bf16", "data": "synthetic (random weights and tokens)"}), flush=True)

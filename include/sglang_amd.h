@@ -653,10 +653,11 @@ int sgl_amd_grouped_prefill(const void* q, int64_t q_stride, const void* cache, 
 
 /* ---- router with a bias, and the plain form of routed experts (moe_route.hip) -------------------------------------
  * sgl_amd_moe_route: per token the `top` largest of W h + bias (fp32) and the softmax over those -> fp32 weights, int32 ids
- * [tokens, top].  sgl_amd_experts_plain: pair i = (token i / top, expert ids[i]); up: silu(gate x) * (up x) from w [experts, 2 N, K],
+ * [tokens, top].  partials fp32 [slices, tokens, pad] (pad = 16, 32, .. 256 >= experts): the matrix form, `slices` pieces of the
+ * columns; null: the plain one.  sgl_amd_experts_plain: pair i = (token i / top, expert ids[i]); up: silu(gate x) * (up x) from w [experts, 2 N, K],
  * else w x from w [experts, N, K] and x [pairs, K]. */
 int sgl_amd_moe_route(int is_f32, const void* h, int64_t h_stride, const void* w, const float* bias, float* topk_weights, int32_t* topk_ids,
-    int64_t tokens, int K, int experts, int top, void* stream);
+    float* partials, int slices, int pad, int64_t tokens, int K, int experts, int top, void* stream);
 int sgl_amd_experts_plain(int is_f32, int up, const void* x, int64_t x_stride, const void* w, const int32_t* ids, void* out, int64_t o_stride,
     int64_t pairs, int top, int N, int K, int experts, void* stream);
 

@@ -31,15 +31,36 @@ __device__ __forceinline__ void st4(float* p, const float (&f)[4]) {
   *reinterpret_cast<f32x4_t*>(p) = f32x4_t{f[0], f[1], f[2], f[3]};
 }
 
-// VEC consecutive elements, VEC in {1, 4}
+__device__ __forceinline__ void ld8(const uint16_t* p, float (&f)[8]) {
+  const U4 w = ld16(p);
+  f[0] = bf_lo(w.x); f[1] = bf_hi(w.x); f[2] = bf_lo(w.y); f[3] = bf_hi(w.y);
+  f[4] = bf_lo(w.z); f[5] = bf_hi(w.z); f[6] = bf_lo(w.w); f[7] = bf_hi(w.w);
+}
+__device__ __forceinline__ void ld8(const float* p, float (&f)[8]) {
+  const f32x4_t a = *reinterpret_cast<const f32x4_t*>(p), b = *reinterpret_cast<const f32x4_t*>(p + 4);
+  f[0] = a[0]; f[1] = a[1]; f[2] = a[2]; f[3] = a[3]; f[4] = b[0]; f[5] = b[1]; f[6] = b[2]; f[7] = b[3];
+}
+__device__ __forceinline__ void st8(uint16_t* p, const float (&f)[8]) {
+  U4 w;
+  w.x = pack_bf2(f[0], f[1]); w.y = pack_bf2(f[2], f[3]); w.z = pack_bf2(f[4], f[5]); w.w = pack_bf2(f[6], f[7]);
+  st16(p, w);
+}
+__device__ __forceinline__ void st8(float* p, const float (&f)[8]) {
+  *reinterpret_cast<f32x4_t*>(p) = f32x4_t{f[0], f[1], f[2], f[3]};
+  *reinterpret_cast<f32x4_t*>(p + 4) = f32x4_t{f[4], f[5], f[6], f[7]};
+}
+
+// VEC consecutive elements, VEC in {1, 4, 8}
 template <int VEC, typename T>
 __device__ __forceinline__ void ldv(const T* p, float (&f)[VEC]) {
-  if constexpr (VEC == 4) ld4(p, f);
+  if constexpr (VEC == 8) ld8(p, f);
+  else if constexpr (VEC == 4) ld4(p, f);
   else f[0] = ld1(p);
 }
 template <int VEC, typename T>
 __device__ __forceinline__ void stv(T* p, const float (&f)[VEC]) {
-  if constexpr (VEC == 4) st4(p, f);
+  if constexpr (VEC == 8) st8(p, f);
+  else if constexpr (VEC == 4) st4(p, f);
   else st1(p, f[0]);
 }
 

@@ -383,14 +383,15 @@ __global__ __launch_bounds__(256, 2) void grouped_attention_mfma_kernel(GroupedP
 }
 
 // ---------------------------------------------------------------------------------------------------------------
-// Long extends: a workgroup = 256 rows of one key head, row = (token, query head of the group), a wave = 32 rows; key tiles of 64
-// double-buffered in LDS, the next tile's rows in registers meanwhile.  S^T = K Q^T leaves the weights of a row in the lane that
+// Long extends: a workgroup = 128 rows of one key head, row = (token, query head of the group), a wave = 32 rows; key tiles of 64
+// double-buffered in LDS, the next tile's rows in registers meanwhile; two workgroups a compute unit, so that one multiplies
+// while the other forms weights.  S^T = K Q^T leaves the weights of a row in the lane that
 // needs them for O^T = V^T P^T, so they never touch LDS.
-constexpr int kPfThreads = 512, kPfRows = 256, kPfTile = 64;
+constexpr int kPfThreads = 256, kPfRows = 128, kPfTile = 64, kPfPass = kPfThreads / 8;
 
 template <int KS, int VT>
 __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedParams p) {
-  constexpr int KLS = KS * 32 + 8, VLS = VT * 16 + 8, KP = KS / 2, VP = VT / 4;
+  constexpr int KLS = KS * 32 + 8, VLS = VT * 16 + 8, KP = KS / 2, VP = VT / 4, NP = kPfTile / kPfPass;
   __shared__ __attribute__((aligned(16))) uint16_t kimg[2][kPfTile * KLS];
   __shared__ __attribute__((aligned(16))) uint16_t vimg[2][kPfTile * VLS];
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), i16 = lane & 15, g = lane >> 4;
@@ -424,20 +425,26 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
   const bool wave_live = tok_first <= last;
   const int wave_first = pos0 + tok_first, wave_last = pos0 + (tok_last < last ? tok_last : last);
   const int r_row = threadIdx.x >> 3, r_col = (threadIdx.x & 7) * 8;           // eight threads a key row
-  U4 kreg[KP], vreg[VP];
-  int slot;
+  U4 kreg[NP][KP], vreg[NP][VP];
+  int slot[NP];
   auto next_slot = [&](int j0) __attribute__((always_inline)) {
-    const int j = j0 + r_row;
-    slot = row[j < end ? j : end - 1];
+#pragma unroll
+    for (int w = 0; w < NP; ++w) {
+      const int j = j0 + w * kPfPass + r_row;
+      slot[w] = row[j < end ? j : end - 1];
+    }
   };
   // (addresses are clamped, never predicated: all loads stay in flight; columns behind kd meet zeros of the query, columns behind
   // vd are not stored, keys behind the last are masked)
   auto load = [&]() __attribute__((always_inline)) {
-    const uint16_t* kr = cache + static_cast<int64_t>(slot) * p.cache_stride;
 #pragma unroll
-    for (int i = 0; i < KP; ++i) kreg[i] = ld16(r_col + 64 * i < p.kd ? kr + r_col + 64 * i : kr);
+    for (int w = 0; w < NP; ++w) {
+      const uint16_t* kr = cache + static_cast<int64_t>(slot[w]) * p.cache_stride;
 #pragma unroll
-    for (int i = 0; i < VP; ++i) vreg[i] = ld16(kr + p.kd + (r_col + 64 * i < p.vd ? r_col + 64 * i : 0));
+      for (int i = 0; i < KP; ++i) kreg[w][i] = ld16(r_col + 64 * i < p.kd ? kr + r_col + 64 * i : kr);
+#pragma unroll
+      for (int i = 0; i < VP; ++i) vreg[w][i] = ld16(kr + p.kd + (r_col + 64 * i < p.vd ? r_col + 64 * i : 0));
+    }
   };
   f32x4_t o[2][VT];
   float m[2] = {-INFINITY, -INFINITY}, l[2] = {0.f, 0.f};
@@ -454,9 +461,12 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
     // (the barrier of the tile before this one lies behind every read of this image)
     uint16_t *kt = kimg[image], *vt = vimg[image];
 #pragma unroll
-    for (int i = 0; i < KP; ++i) st16(kt + r_row * KLS + r_col + 64 * i, kreg[i]);
+    for (int w = 0; w < NP; ++w) {
 #pragma unroll
-    for (int i = 0; i < VP; ++i) st16(vt + r_row * VLS + r_col + 64 * i, vreg[i]);
+      for (int i = 0; i < KP; ++i) st16(kt + (w * kPfPass + r_row) * KLS + r_col + 64 * i, kreg[w][i]);
+#pragma unroll
+      for (int i = 0; i < VP; ++i) st16(vt + (w * kPfPass + r_row) * VLS + r_col + 64 * i, vreg[w][i]);
+    }
     __syncthreads();
     if (j0 + kPfTile < end) {
       load();

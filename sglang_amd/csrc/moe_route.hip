@@ -1,7 +1,8 @@
 // Router and the plain form of routed experts.
 //
-//   moe_route     logits W h + b in fp32, the `top` largest per token, softmax over those alone: one launch, so the logits never
-//                 leave the workgroup (bf16 rows on matrix instructions, fp32 rows and odd sizes by plain sums)
+//   moe_route     logits W h + b in fp32, the `top` largest per token, softmax over those alone.  bf16 rows: matrix instructions over
+//                 slices of the columns, one wave each (a compute unit alone streams the router's rows far too slowly), then a
+//                 launch that adds the slices and the bias and picks; fp32 rows and odd sizes: plain sums and the pick in one launch
 //   experts_up / experts_down   silu(gate h) * (up h) and its down projection per (token, expert) pair for fp32 rows and sizes outside
 //                 the grouped matrix kernels' forms: a wave sums one output
 #include "elem_io.hpp"
@@ -19,99 +20,136 @@ struct RouteParams {
   const float* bias;      // [experts], or null
   float* weights;         // [tokens, top]
   int32_t* ids;           // [tokens, top]
+  float* part;            // [slices, tokens, pad] partial logits
   int64_t tokens;
-  int K, experts, top;
+  int K, experts, top, slices, pad;
 };
 
-// A wave picks for one token: z[j] is the logit of expert lane + 64 j (-inf behind the last).
+// A wave picks for one token: z[j] is the logit of expert lane + 64 j.  An expert's place is the number of experts in front of it
+// (larger logit, or the same and a smaller index; what is not a number goes last), so every place has exactly one expert.
 template <int N>
-__device__ __forceinline__ void pick_experts(const RouteParams& p, int64_t t, float (&z)[N], int lane) {
-  float mine = -INFINITY, best = 0.f, sum = 0.f;
-  int my_id = 0;
-  for (int i = 0; i < p.top; ++i) {
-    float bv = -INFINITY;
-    int be = 0x7fffffff;
+__device__ __forceinline__ void pick_experts(const RouteParams& p, int64_t t, float (&z)[N], int lane, float* all) {
+  int place[N];
+  float top = -INFINITY;
 #pragma unroll
-    for (int j = 0; j < N; ++j)
-      if (lane + 64 * j < p.experts && (be == 0x7fffffff || z[j] > bv) && z[j] > -INFINITY) { bv = z[j]; be = lane + 64 * j; }
-    for (int off = 32; off > 0; off >>= 1) {
-      const float ov = __shfl_xor(bv, off, 64);
-      const int oe = __shfl_xor(be, off, 64);
-      if (oe != 0x7fffffff && (be == 0x7fffffff || ov > bv || (ov == bv && oe < be))) { bv = ov; be = oe; }
+  for (int j = 0; j < N; ++j) {
+    place[j] = 0;
+    if (!(z[j] == z[j]) || lane + 64 * j >= p.experts) z[j] = -INFINITY;
+    top = fmaxf(top, z[j]);
+    all[lane + 64 * j] = z[j];                         // (this wave's own array: LDS serves a wave in order)
+  }
+  top = wave_max(top);
+  asm volatile("" ::: "memory");
+  __builtin_amdgcn_wave_barrier();
+#pragma unroll
+  for (int i = 0; i < N; ++i) {
+    const int n = p.experts - 64 * i < 64 ? p.experts - 64 * i : 64;
+#pragma unroll 4
+    for (int l = 0; l < n; l += 4) {                   // (what lies behind the last expert is -inf, in front of nobody)
+      float other[4];
+      ld4(all + 64 * i + l, other);
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+#pragma unroll
+        for (int j = 0; j < N; ++j) place[j] += other[u] > z[j] || (other[u] == z[j] && (i < j || (i == j && l + u < lane))) ? 1 : 0;
     }
-    if (be == 0x7fffffff) { be = i; bv = -INFINITY; }  // (logits that are not numbers: some expert, weight zero or not a number)
+  }
+  float e[N], sum = 0.f;
 #pragma unroll
-    for (int j = 0; j < N; ++j)
-      if (be == lane + 64 * j) z[j] = -INFINITY;
-    if (i == 0) best = bv;
-    if (lane == i) { mine = bv; my_id = be; }
-    sum += expf(bv - best);
+  for (int j = 0; j < N; ++j) {
+    const bool taken = place[j] < p.top && lane + 64 * j < p.experts;
+    e[j] = taken ? expf(z[j] - top) : 0.f;
+    sum += e[j];
   }
-  if (lane < p.top) {
-    p.weights[t * p.top + lane] = expf(mine - best) / sum;
-    p.ids[t * p.top + lane] = my_id;
-  }
+  sum = wave_sum(sum);
+#pragma unroll
+  for (int j = 0; j < N; ++j)
+    if (place[j] < p.top && lane + 64 * j < p.experts) {
+      p.weights[t * p.top + place[j]] = e[j] / sum;
+      p.ids[t * p.top + place[j]] = lane + 64 * j;
+    }
 }
 
-// 16 tokens a workgroup; its kWaves waves share the columns, partial logits meet in LDS, then a wave picks for one token at a time.
-template <int NT, int kWaves>
-__global__ __launch_bounds__(kWaves * 64) void moe_route_mfma_kernel(RouteParams p) {
-  constexpr int LS = NT * 16 + 4;                    // logits of a token, in fp32
-  __shared__ __attribute__((aligned(16))) float part[(kWaves > 4 ? 4 : kWaves)][16][LS];
-  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), i16 = lane & 15, g = lane >> 4;
-  const int64_t t0 = static_cast<int64_t>(blockIdx.x) * 16;
-  const int64_t t = t0 + i16 < p.tokens ? t0 + i16 : p.tokens - 1;
-  const uint16_t* hr = static_cast<const uint16_t*>(p.h) + t * p.h_stride;
-  const uint16_t* wr[NT];
+// One wave: 16 MT tokens, 16 NT experts (all of them), one slice of the columns.
+template <int NT, int MT>
+__global__ __launch_bounds__(64) void moe_route_slice_kernel(RouteParams p) {
+  constexpr int kSteps = NT * MT <= 8 ? 4 : NT * MT <= 16 ? 2 : 1;       // column steps in flight together
+  const int lane = threadIdx.x, i16 = lane & 15, g = lane >> 4;
+  const int64_t t0 = static_cast<int64_t>(blockIdx.x) * (16 * MT);
+  const int chunk = ((p.K + p.slices - 1) / p.slices + 31) / 32 * 32, k_first = blockIdx.y * chunk;
+  const int k_end = k_first + chunk < p.K ? k_first + chunk : p.K;
+  const uint16_t *hr[MT], *wr[NT];
+#pragma unroll
+  for (int m = 0; m < MT; ++m) {
+    const int64_t t = t0 + 16 * m + i16;
+    hr[m] = static_cast<const uint16_t*>(p.h) + (t < p.tokens ? t : p.tokens - 1) * p.h_stride;
+  }
 #pragma unroll
   for (int n = 0; n < NT; ++n) {
     const int e = 16 * n + i16;
     wr[n] = static_cast<const uint16_t*>(p.w) + static_cast<int64_t>(e < p.experts ? e : p.experts - 1) * p.K;
   }
-  f32x4_t acc[NT];
+  f32x4_t acc[NT][MT];
 #pragma unroll
-  for (int n = 0; n < NT; ++n) acc[n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  for (int k0 = wave * 32; k0 < p.K; k0 += kWaves * 32) {
-    const int k = k0 + 8 * g;
-    const bool in = k < p.K;
-    const bf16x8_t x = as_frag(keep_if(ld16(in ? hr + k : hr), in));
+  for (int n = 0; n < NT; ++n)
 #pragma unroll
-    for (int n = 0; n < NT; ++n) acc[n] = mfma_bf16(as_frag(ld16(in ? wr[n] + k : wr[n])), x, acc[n]);
-  }
-  // lane: token i16, experts 16 n + 4 g + r.  Four slabs: with more waves they add up in turn
+    for (int m = 0; m < MT; ++m) acc[n][m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  for (int k0 = k_first; k0 < k_end; k0 += kSteps * 32) {
+    U4 x[kSteps][MT], w[kSteps][NT];
 #pragma unroll
-  for (int turn = 0; turn < (kWaves + 3) / 4; ++turn) {
-    if (wave / 4 == turn) {
+    for (int s = 0; s < kSteps; ++s) {
+      const int k = k0 + 32 * s + 8 * g;
+      const bool in = k < k_end;
 #pragma unroll
-      for (int n = 0; n < NT; ++n) {
-        f32x4_t* dst = reinterpret_cast<f32x4_t*>(&part[wave & 3][i16][16 * n + 4 * g]);
-        *dst = turn == 0 ? acc[n] : *dst + acc[n];
-      }
+      for (int m = 0; m < MT; ++m) x[s][m] = keep_if(ld16(in ? hr[m] + k : hr[m]), in);
+#pragma unroll
+      for (int n = 0; n < NT; ++n) w[s][n] = ld16(in ? wr[n] + k : wr[n]);
     }
-    __syncthreads();
+#pragma unroll
+    for (int s = 0; s < kSteps; ++s)
+#pragma unroll
+      for (int n = 0; n < NT; ++n)
+#pragma unroll
+        for (int m = 0; m < MT; ++m) acc[n][m] = mfma_bf16(as_frag(w[s][n]), as_frag(x[s][m]), acc[n][m]);
   }
-  constexpr int PN = (NT + 3) / 4;
-  for (int tk = wave; tk < 16 && t0 + tk < p.tokens; tk += kWaves) {
-    float z[PN];
+  // lane: token 16 m + i16, experts 16 n + 4 g + r
 #pragma unroll
-    for (int j = 0; j < PN; ++j) {
-      const int e = lane + 64 * j;
-      z[j] = -INFINITY;
-      if (e < p.experts) {
-        float v = p.bias ? p.bias[e] : 0.f;
+  for (int m = 0; m < MT; ++m) {
+    const int64_t t = t0 + 16 * m + i16;
+    if (t >= p.tokens) continue;
+    float* dst = p.part + (blockIdx.y * p.tokens + t) * p.pad + 4 * g;
 #pragma unroll
-        for (int s = 0; s < (kWaves > 4 ? 4 : kWaves); ++s) v += part[s][tk][e];
-        z[j] = v;
-      }
+    for (int n = 0; n < NT; ++n) *reinterpret_cast<f32x4_t*>(dst + 16 * n) = acc[n][m];
+  }
+}
+
+// A wave per token.
+template <int N>
+__global__ __launch_bounds__(256) void moe_route_pick_kernel(RouteParams p) {
+  __shared__ __attribute__((aligned(16))) float all[4][N * 64];
+  const int lane = threadIdx.x & 63;
+  const int64_t t = static_cast<int64_t>(blockIdx.x) * 4 + (threadIdx.x >> 6);
+  if (t >= p.tokens) return;
+  float z[N];
+#pragma unroll
+  for (int j = 0; j < N; ++j) {
+    const int e = lane + 64 * j;
+    z[j] = -INFINITY;
+    if (e < p.experts) {
+      float v = p.bias ? p.bias[e] : 0.f;
+#pragma unroll 4
+      for (int s = 0; s < p.slices; ++s) v += p.part[(s * p.tokens + t) * p.pad + e];
+      z[j] = v;
     }
-    pick_experts<PN>(p, t0 + tk, z, lane);
   }
+  pick_experts<N>(p, t, z, lane, all[threadIdx.x >> 6]);
 }
 
 // One token a workgroup, a wave per expert in turn.
 template <typename T>
 __global__ __launch_bounds__(256) void moe_route_plain_kernel(RouteParams p) {
   __shared__ float logits[256];
+  __shared__ __attribute__((aligned(16))) float all[256];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int64_t t = blockIdx.x;
   const T* hr = static_cast<const T*>(p.h) + t * p.h_stride;
@@ -127,15 +165,17 @@ __global__ __launch_bounds__(256) void moe_route_plain_kernel(RouteParams p) {
     float z[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) z[j] = lane + 64 * j < p.experts ? logits[lane + 64 * j] : -INFINITY;
-    pick_experts<4>(p, t, z, lane);
+    pick_experts<4>(p, t, z, lane, all);
   }
 }
 
 template <int NT>
 void launch_route(const RouteParams& p, hipStream_t st) {
-  const dim3 grid(static_cast<unsigned>((p.tokens + 15) / 16));
-  if (p.tokens <= 2048 && p.K >= 1024) hipLaunchKernelGGL((moe_route_mfma_kernel<NT, 16>), grid, dim3(1024), 0, st, p);
-  else hipLaunchKernelGGL((moe_route_mfma_kernel<NT, 4>), grid, dim3(256), 0, st, p);
+  constexpr int MT = NT <= 8 ? 4 : 2;
+  const dim3 grid(static_cast<unsigned>((p.tokens + 16 * MT - 1) / (16 * MT)), p.slices);
+  if (p.tokens <= 16) hipLaunchKernelGGL((moe_route_slice_kernel<NT, 1>), dim3(1, p.slices), dim3(64), 0, st, p);
+  else hipLaunchKernelGGL((moe_route_slice_kernel<NT, MT>), grid, dim3(64), 0, st, p);
+  hipLaunchKernelGGL((moe_route_pick_kernel<(NT + 3) / 4>), dim3(static_cast<unsigned>((p.tokens + 3) / 4)), dim3(256), 0, st, p);
 }
 
 // ---------------------------------------------------------------------------------------------------------------
@@ -176,19 +216,24 @@ __global__ __launch_bounds__(256) void experts_plain_kernel(ExpertParams p) {
 extern "C" {
 
 int sgl_amd_moe_route(int is_f32, const void* h, int64_t h_stride, const void* w, const float* bias, float* topk_weights, int32_t* topk_ids,
-                      int64_t tokens, int K, int experts, int top, void* stream) {
+                      float* partials, int slices, int pad, int64_t tokens, int K, int experts, int top, void* stream) {
   SGL_CLEAR_STALE_ERROR();
   SGL_CHECK_ARG(h && w && topk_weights && topk_ids && K > 0, "moe_route: null operand");
   SGL_CHECK_ARG(experts >= 1 && experts <= 256 && top >= 1 && top <= experts && top <= 64, "moe_route: %d of %d experts (at most 64 of 256)", top, experts);
   SGL_CHECK_ARG(tokens <= 0x7fffffffLL, "moe_route: too many tokens");
   if (tokens <= 0) return 0;
-  RouteParams p{h, h_stride, w, bias, topk_weights, topk_ids, tokens, K, experts, top};
+  RouteParams p{h, h_stride, w, bias, topk_weights, topk_ids, partials, tokens, K, experts, top, slices, pad};
   hipStream_t st = as_stream(stream);
-  if (!is_f32 && K % 8 == 0 && h_stride % 8 == 0 && aligned_to(h, 16) && aligned_to(w, 16)) {
-    if (experts <= 16) launch_route<1>(p, st);
-    else if (experts <= 32) launch_route<2>(p, st);
-    else if (experts <= 64) launch_route<4>(p, st);
-    else if (experts <= 128) launch_route<8>(p, st);
+  if (partials) {
+    const int nt = pad / 16;
+    SGL_CHECK_ARG(!is_f32 && K % 8 == 0 && h_stride % 8 == 0 && aligned_to(h, 16) && aligned_to(w, 16) && aligned_to(partials, 16),
+                  "moe_route: the matrix form takes bf16 rows of whole 16-byte vectors");
+    SGL_CHECK_ARG(pad % 16 == 0 && (nt & (nt - 1)) == 0 && nt >= 1 && nt <= 16 && pad >= experts && slices >= 1 && slices <= 65535,
+                  "moe_route: %d slices of %d columns for %d experts", slices, pad, experts);
+    if (nt == 1) launch_route<1>(p, st);
+    else if (nt == 2) launch_route<2>(p, st);
+    else if (nt == 4) launch_route<4>(p, st);
+    else if (nt == 8) launch_route<8>(p, st);
     else launch_route<16>(p, st);
   } else {
     const dim3 grid(static_cast<unsigned>(tokens));

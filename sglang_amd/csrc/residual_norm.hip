@@ -261,13 +261,27 @@ __device__ __forceinline__ void add_source(const RowSource& s, int64_t row, int 
   }
 }
 
-template <typename T, int VEC>
-__device__ __forceinline__ void add_single(const RowSource& s, int64_t row, int c, float (&v)[VEC]) {
-  float u[VEC];
-  if (s.f32) ldv<VEC>(static_cast<const float*>(s.data) + row * s.row_stride + c, u);
-  else ldv<VEC>(static_cast<const T*>(s.data) + row * s.row_stride + c, u);
+// The same over all the columns of a thread: one item at a time, its pieces in flight together.
+template <typename T, int VEC, int kItems>
+__device__ __forceinline__ void add_source_row(const RowSource& s, int64_t row, int lane, int tpr, int W, float (&v)[kItems][VEC]) {
+  constexpr int kAhead = kItems <= 4 ? 2 : 1;
+#pragma unroll kAhead
+  for (int q = 0; q < s.n; ++q) {
+    const int64_t base = row * s.row_stride + q * s.item_stride;
+    const float f = s.weight ? s.weight[row * s.n + q] : 1.0f;
+    float u[kItems][VEC];
 #pragma unroll
-  for (int j = 0; j < VEC; ++j) v[j] += u[j];
+    for (int i = 0; i < kItems; ++i) {
+      int c = (i * tpr + lane) * VEC;
+      if (c >= W) c = 0;
+      if (s.f32) ldv<VEC>(static_cast<const float*>(s.data) + base + c, u[i]);
+      else ldv<VEC>(static_cast<const T*>(s.data) + base + c, u[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < kItems; ++i)
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) v[i][j] += f * u[i][j];
+  }
 }
 
 // kWaveRow: a wave owns a row (many rows: no barrier), else a workgroup does (decode batches: shortest path to one row).
@@ -307,27 +321,19 @@ __global__ __launch_bounds__(kWaveRow ? 256 : 1024) void residual_rms_kernel(Res
       }
     }
   } else {
-    const bool simple = p.a.data && p.a.n == 1 && !p.a.weight && !p.b.data;
 #pragma unroll
     for (int i = 0; i < kItems; ++i) {
       const int c = (i * tpr + lane) * VEC;
       if (c < W) ldv<VEC>(xr + c, v[i]);
     }
-    if (simple) {                                     // rows of a library product: nothing between the loads
-#pragma unroll
-      for (int i = 0; i < kItems; ++i) {
-        const int c = (i * tpr + lane) * VEC;
-        if (c < W) add_single<T, VEC>(p.a, row, c, v[i]);
+    if constexpr (kItems == 1) {
+      if (lane * VEC < W) {
+        if (p.a.data) add_source<T, VEC>(p.a, row, lane * VEC, v[0]);
+        if (p.b.data) add_source<T, VEC>(p.b, row, lane * VEC, v[0]);
       }
     } else {
-#pragma unroll
-      for (int i = 0; i < kItems; ++i) {
-        const int c = (i * tpr + lane) * VEC;
-        if (c < W) {
-          if (p.a.data) add_source<T, VEC>(p.a, row, c, v[i]);
-          if (p.b.data) add_source<T, VEC>(p.b, row, c, v[i]);
-        }
-      }
+      if (p.a.data) add_source_row<T, VEC, kItems>(p.a, row, lane, tpr, W, v);
+      if (p.b.data) add_source_row<T, VEC, kItems>(p.b, row, lane, tpr, W, v);
     }
   }
   float ss = 0.f;
@@ -370,12 +376,12 @@ __global__ __launch_bounds__(kWaveRow ? 256 : 1024) void residual_rms_kernel(Res
 }
 
 template <typename T>
-void launch_residual_rms(const ResidualRmsParams& p, bool vec, hipStream_t st) {
+void launch_residual_rms(const ResidualRmsParams& p, bool vec, bool vec8, hipStream_t st) {
   const unsigned by4 = static_cast<unsigned>((p.rows + 3) / 4), one = static_cast<unsigned>(p.rows);
   const int W = p.width;
-  if (vec && p.rows >= 1024 && W <= 1024) hipLaunchKernelGGL((residual_rms_kernel<T, 4, 4, true>), dim3(by4), dim3(256), 0, st, p);
-  else if (vec && p.rows >= 1024 && W <= 2048) hipLaunchKernelGGL((residual_rms_kernel<T, 4, 8, true>), dim3(by4), dim3(256), 0, st, p);
-  else if (vec && p.rows >= 1024 && W <= 4096) hipLaunchKernelGGL((residual_rms_kernel<T, 4, 16, true>), dim3(by4), dim3(256), 0, st, p);
+  if (vec8 && p.rows >= 1024 && W <= 1024) hipLaunchKernelGGL((residual_rms_kernel<T, 8, 2, true>), dim3(by4), dim3(256), 0, st, p);
+  else if (vec8 && p.rows >= 1024 && W <= 2048) hipLaunchKernelGGL((residual_rms_kernel<T, 8, 4, true>), dim3(by4), dim3(256), 0, st, p);
+  else if (vec8 && p.rows >= 1024 && W <= 4096) hipLaunchKernelGGL((residual_rms_kernel<T, 8, 8, true>), dim3(by4), dim3(256), 0, st, p);
   else if (vec && W <= 4096) hipLaunchKernelGGL((residual_rms_kernel<T, 4, 1, false>), dim3(one), dim3((W / 4 + 63) / 64 * 64), 0, st, p);
   else if (vec) hipLaunchKernelGGL((residual_rms_kernel<T, 4, 4, false>), dim3(one), dim3(1024), 0, st, p);
   else hipLaunchKernelGGL((residual_rms_kernel<T, 1, 16, false>), dim3(one), dim3(W >= 1024 ? 1024 : (W + 63) / 64 * 64), 0, st, p);
@@ -549,8 +555,10 @@ int sgl_amd_residual_rms(int is_f32, const int64_t* ids, const void* table, int6
                    b_row_stride % 4 == 0 && b_item_stride % 4 == 0 && aligned_to(table, al) && aligned_to(pos_table, al) &&
                    aligned_to(a, p.a.f32 ? 16 : 8) && aligned_to(b, p.b.f32 ? 16 : 8) && aligned_to(h, al) && aligned_to(x, 16) &&
                    aligned_to(save, 16) && aligned_to(extra, 16) && aligned_to(step, 16) && aligned_to(weight, 16);
-  if (is_f32) launch_residual_rms<float>(p, vec, as_stream(stream));
-  else launch_residual_rms<uint16_t>(p, vec, as_stream(stream));
+  const bool vec8 = vec && width % 8 == 0 && h_stride % 8 == 0 && a_row_stride % 8 == 0 && a_item_stride % 8 == 0 && b_row_stride % 8 == 0 &&
+                    b_item_stride % 8 == 0 && aligned_to(table, 16) && aligned_to(pos_table, 16) && aligned_to(a, 16) && aligned_to(b, 16) && aligned_to(h, 16);
+  if (is_f32) launch_residual_rms<float>(p, vec, vec8, as_stream(stream));
+  else launch_residual_rms<uint16_t>(p, vec, vec8, as_stream(stream));
   SGL_CHECK_LAUNCH("residual_rms");
   return 0;
 }

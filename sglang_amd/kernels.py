@@ -1660,8 +1660,15 @@ def moe_route(h: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], to
     _need(w.dim() == 2 and w.shape[1] == K and w.is_contiguous() and (bias is None or bias.numel() == w.shape[0]), "moe_route: shapes")
     weights = torch.empty((T, top), dtype=torch.float32, device=h.device)
     ids = torch.empty((T, top), dtype=torch.int32, device=h.device)
-    native.call("sgl_amd_moe_route", _is_f32(h, w), h.data_ptr(), h.stride(0), w.data_ptr(), _ptr(bias), weights.data_ptr(), ids.data_ptr(), T, K,
-                w.shape[0], top, _stream())
+    f32, E, part, slices, pad = _is_f32(h, w), w.shape[0], None, 0, 0
+    if not f32 and T and E <= 256 and K % 8 == 0 and h.stride(0) % 8 == 0 and h.data_ptr() % 16 == 0:
+        # one wave per 64 (32 at most experts, 16 at few) tokens and slice: waves enough for the chip, slices of 64 columns at least
+        pad = next(16 << i for i in range(5) if E <= 16 << i)
+        blocks = -(-T // (16 if T <= 16 else 64 if pad <= 128 else 32))
+        slices = max(1, min(-(-1024 // blocks), K // 64, 32))
+        part = torch.empty((slices, T, pad), dtype=torch.float32, device=h.device)
+    native.call("sgl_amd_moe_route", f32, h.data_ptr(), h.stride(0), w.data_ptr(), _ptr(bias), weights.data_ptr(), ids.data_ptr(), _ptr(part), slices,
+                pad, T, K, E, top, _stream())
     return weights, ids
 
 
