@@ -119,3 +119,24 @@ def test_hybrid_kernels_keep_their_state_in_registers(tmp_path):
         assert len(inst) == n, sorted(usage)
         for name, u in inst.items():
             assert u["vgpr_spill_count"] == 0 and u["vgpr_count"] <= 256, (name, u)
+
+
+@pytest.mark.skipif(not Path(HIPCC).exists(), reason="hipcc not installed")
+def test_grouped_attention_kernels_keep_their_sums_in_registers(tmp_path):
+    """Queries, sums and the next tile's rows live in registers through the key loop.  Only the widest decode instance (keys and values
+    both above 128 elements) goes over, by 20 values.  Two prefill workgroups share a compute unit up to 128 / 128."""
+    usage = _resource_usage("grouped_attention.hip", tmp_path)
+    decode = {k: v for k, v in usage.items() if "grouped_attention_mfma_kernel" in k}
+    prefill = {k: v for k, v in usage.items() if "grouped_prefill_kernel" in k}
+    assert len(decode) == 9 and len(prefill) == 6, sorted(usage)
+    for name, u in decode.items():
+        assert u["vgpr_spill_count"] <= (20 if "ILi8ELi16E" in name else 0) and u["vgpr_count"] <= 256, (name, u)
+    for name, u in prefill.items():
+        assert u["vgpr_spill_count"] == 0 and u["sgpr_spill_count"] == 0, (name, u)
+        if "ILi8E" not in name:
+            assert u["vgpr_count"] <= 256 and u["group_segment_fixed_size"] <= 80 * 1024, (name, u)
+    for name, u in _resource_usage("moe_route.hip", tmp_path).items():
+        assert u["vgpr_spill_count"] == 0, (name, u)
+    for name, u in _resource_usage("residual_norm.hip", tmp_path).items():
+        if "residual_rms_kernel" in name:
+            assert u["vgpr_spill_count"] == 0, (name, u)
