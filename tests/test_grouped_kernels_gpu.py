@@ -96,7 +96,7 @@ class _Case:
 
 
 LENS = [(0, 100), (77, 3), (150, 1), (5, 70), (64, 64), (0, 1)]
-SIZES = [(6, 2, 48, 80), (3, 1, 16, 24), (4, 4, 64, 128), (20, 1, 136, 136), (16, 4, 128, 64), (2, 1, 200, 256)]
+SIZES = [(6, 2, 40, 72), (3, 1, 16, 24), (4, 4, 64, 128), (20, 1, 136, 136), (16, 4, 128, 64), (2, 1, 200, 256)]
 
 
 @pytest.mark.parametrize("window", [1, 33, 64, 65, 0])
@@ -163,7 +163,7 @@ def test_the_sink_takes_everything_or_nothing(device, dtype):
                 assert _rel(got, c2.want(30, 1.0, 0.0, False)) < (4e-3 if dtype == BF else 3e-5)
 
 
-@pytest.mark.parametrize("sizes", [(6, 2, 48, 80), (20, 1, 136, 136), (16, 16, 64, 64)])
+@pytest.mark.parametrize("sizes", [(6, 2, 40, 72), (20, 1, 136, 136), (16, 16, 64, 64)])
 @pytest.mark.parametrize("splits", [1, 3])
 def test_a_decode_batch_brings_its_own_keys(device, sizes, splits):
     """New keys and values read from the projection and stored on the way equal stored-first ones, and land in their rows."""
@@ -198,7 +198,7 @@ def test_store_writes_exactly_its_rows(device, dtype):
 
 # ---------------------------------------------------------------------------------------------- router and experts
 @pytest.mark.parametrize("dtype", [BF, F32])
-@pytest.mark.parametrize("T,K,E,top", [(1, 64, 1, 1), (37, 320, 16, 2), (5, 102, 7, 4), (64, 2048, 64, 8), (19, 136, 20, 20), (3, 72, 200, 5),
+@pytest.mark.parametrize("T,K,E,top", [(1, 64, 1, 1), (37, 288, 24, 3), (5, 102, 7, 4), (64, 2048, 64, 8), (19, 136, 20, 20), (3, 72, 200, 5),
                                        (2100, 256, 33, 3), (70, 4096, 128, 6)])
 def test_router_picks_and_weighs(device, dtype, T, K, E, top):
     from sglang_amd import kernels as Kn
@@ -220,7 +220,7 @@ def test_router_picks_and_weighs(device, dtype, T, K, E, top):
     assert E == top or not torch.equal(Kn.moe_route(h.to(device), w.to(device), None, top)[1].long().cpu(), ge) or T == 1
 
 
-@pytest.mark.parametrize("T,W,ff,E,top", [(3, 320, 64, 16, 2), (70, 256, 128, 4, 2), (40, 136, 64, 9, 3), (900, 256, 64, 4, 2), (500, 320, 128, 3, 3)])
+@pytest.mark.parametrize("T,W,ff,E,top", [(3, 288, 64, 12, 3), (70, 256, 128, 4, 2), (40, 136, 64, 9, 3), (900, 256, 64, 4, 2), (500, 384, 128, 3, 3)])
 def test_routed_experts_forms(device, T, W, ff, E, top):
     from sglang_amd import kernels as K
 
@@ -240,7 +240,7 @@ def test_routed_experts_forms(device, T, W, ff, E, top):
 
 # ---------------------------------------------------------------------------------------------- residual rows
 @pytest.mark.parametrize("dtype", [BF, F32])
-@pytest.mark.parametrize("rows,W", [(3, 102), (5, 320), (64, 2048), (1100, 320), (1030, 2048), (1025, 4096), (9, 5120), (2, 6001)])
+@pytest.mark.parametrize("rows,W", [(3, 102), (5, 336), (64, 2048), (1100, 336), (1030, 2048), (1025, 4096), (9, 5120), (2, 6001)])
 def test_residual_rms_sources_and_order(device, dtype, rows, W):
     from sglang_amd import kernels as K
 
@@ -282,7 +282,7 @@ def test_residual_rms_sources_and_order(device, dtype, rows, W):
     check(x, h, now)
 
 
-@pytest.mark.parametrize("rows,V", [(1, 97), (7, 320), (64, 32000)])
+@pytest.mark.parametrize("rows,V", [(1, 97), (7, 352), (64, 32000)])
 def test_soft_cap(device, rows, V):
     from sglang_amd import kernels as K
 
