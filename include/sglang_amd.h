@@ -65,6 +65,10 @@ int sgl_amd_fused_add_rmsnorm(void* x, void* residual, const void* weight, int64
  * bf16 rounding of silu(x) before the multiply; 0 keeps the product in fp32. */
 int sgl_amd_silu_and_mul(const void* in, void* out, int64_t num_rows, int d, int64_t in_row_stride,
                          int64_t out_row_stride, int round_intermediate, void* stream);
+/* The same with any gated activation, in fp32.  glu_kind: 1 = silu(g) u; 2 = gelu_tanh(g) u; 3 = g' sigmoid(glu_alpha g') (u' + 1) with
+ * g' = min(g, glu_limit) and u' = u clamped to +- glu_limit.  Every function with these three parameters uses them so. */
+int sgl_amd_glu_and_mul(const void* in, void* out, int64_t num_rows, int d, int64_t in_row_stride, int64_t out_row_stride, int glu_kind,
+                        float glu_limit, float glu_alpha, void* stream);
 
 /* ---- Rotary embedding (reference: srt/layers/rotary_embedding/base.py:236-276,
  *      utils.py:36-63; sgl_kernel.rotary_embedding, common_extension_rocm.cc:236-240) */
@@ -328,6 +332,11 @@ int sgl_amd_wstream_gemm(const void* x, const void* w, const void* bias, void* y
                          int64_t y_row_stride, int64_t y_chunk_stride, int epilogue, void* residual,
                          int64_t residual_row_stride, const void* norm_weight, float eps, int waves_per_group,
                          int tiles_per_wave, int num_k_splits, void* ws_partials, void* stream);
+/* epilogue 1 with another activation of the [gate | up] columns (kinds 2, 3: in fp32 up to the final rounding) */
+int sgl_amd_wstream_glu_gemm(const void* x, const void* w, const void* bias, void* y, int64_t M, int64_t N, int64_t K,
+                             int64_t x_row_stride, int64_t x_chunk_stride, int64_t w_row_stride, int64_t y_row_stride,
+                             int64_t y_chunk_stride, int glu_kind, float glu_limit, float glu_alpha, int waves_per_group,
+                             int tiles_per_wave, int num_k_splits, void* ws_partials, void* stream);
 /* qkv_proj + neox rotary embedding + KV-pool store for a decode batch, as one GEMM + combine pair:
  * q_out[M, Hq*D] = rope(x . w_q^T + b), k_cache[cache_loc[m]] = rope(x . w_k^T + b), v_cache[...] = x . w_v^T + b,
  * with the rounding points of QKVParallelLinear -> RotaryEmbedding.forward_native -> set_kv_buffer
@@ -346,16 +355,16 @@ int sgl_amd_wstream_qkv_rope(const void* x, const void* w_qkv, const void* bias,
                              int num_k_splits, void* ws_partials, void* stream);
 /* Grouped (mixture-of-experts) form of the weight-streaming GEMM, same contract as sgl_amd_moe_grouped_gemm
  * (fused_moe_triton_kernels.py:324,771) for shapes with N % 16 == 0 and K % 128 == 0, without split-K: one
- * workgroup per (row block of moe_align_block_size, group of weight tiles of that block's expert).  fuse_silu=1:
- * w is [E, 2N, K] and c[id, :N] = silu_and_mul; otherwise c[id, :] = a[id / top_k_div] . w[e]^T, optionally
+ * workgroup per (row block of moe_align_block_size, group of weight tiles of that block's expert).  glu_kind > 0:
+ * w is [E, 2N, K] and c[id, :N] = the activation of gate and up; otherwise c[id, :] = a[id / top_k_div] . w[e]^T, optionally
  * rounded to bf16 and scaled by topk_weights[id], written bf16 or fp32 (out_f32). */
 int sgl_amd_wstream_moe_gemm(const void* a, const void* w, void* c, const int32_t* sorted_token_ids,
                              const int32_t* expert_ids, const int32_t* num_tokens_post_padded,
                              const float* topk_weights, int mul_routed_weight, int round_before_scale,
                              int top_k_div, int64_t num_valid_ids, int64_t N, int64_t K,
                              int64_t a_row_stride, int64_t w_row_stride, int64_t w_expert_stride,
-                             int64_t c_row_stride, int block_m, int64_t max_m_blocks, int fuse_silu,
-                             int out_f32, int waves_per_group, void* stream);
+                             int64_t c_row_stride, int block_m, int64_t max_m_blocks, int glu_kind,
+                             float glu_limit, float glu_alpha, int out_f32, int waves_per_group, void* stream);
 int sgl_amd_wstream_gemm_max_rows(void);
 int64_t sgl_amd_wstream_gemm_workspace_floats(int64_t M, int64_t N, int num_k_splits);
 /* Grouped GEMM over moe_align_block_size output: for every row block b < num_tokens_post_padded/block_m
@@ -370,7 +379,7 @@ int sgl_amd_moe_grouped_gemm(const void* a, const void* w, void* c, const int32_
                              int top_k_div, int64_t num_valid_ids, int64_t N, int64_t K,
                              int64_t num_experts, int64_t a_row_stride, int64_t w_row_stride,
                              int64_t w_expert_stride, int64_t c_row_stride, int block_m,
-                             int64_t max_m_blocks, int fuse_silu, int out_f32, int tiles_per_wave,
+                             int64_t max_m_blocks, int glu_kind, float glu_limit, float glu_alpha, int out_f32, int tiles_per_wave,
                              int num_k_splits, void* ws_slabs, void* stream);
 
 /* ---- MoE routing / bookkeeping (reference: sgl_kernel.topk_softmax / moe_align_block_size /
@@ -533,7 +542,8 @@ int sgl_amd_moe_tiled_gemm_ex(const void* a, const void* w, void* c, const int32
                               const int32_t* num_tokens_post_padded, const float* topk_weights, int mul_routed_weight,
                               int round_before_scale, int top_k_div, int64_t num_valid_ids, int64_t N, int64_t K,
                               int64_t a_row_stride, int64_t w_row_stride, int64_t w_expert_stride, int64_t c_row_stride,
-                              int64_t max_m_blocks, int fuse_silu, int out_f32, int align_block_m, int tile_rows, void* stream);
+                              int64_t max_m_blocks, int glu_kind, float glu_limit, float glu_alpha, int out_f32, int align_block_m, int tile_rows,
+                              void* stream);
 
 /* ---- fp32 residual stream and gated norms (residual_norm.hip) -----------------------------------------------
  * sgl_amd_residual_norm: one launch between two sublayers.  mode 0: x = table[ids] * scale; 1: x += LayerNorm(y; w1, b1);
@@ -542,7 +552,7 @@ int sgl_amd_moe_tiled_gemm_ex(const void* a, const void* w, void* c, const int32
  * type.  x and all norm parameters are fp32; y, h, table and the copies are bf16, or fp32 with is_f32.
  * sgl_amd_gated_rmsnorm: per (row, group of group_size columns): gate_first ? rms(y * silu(gate)) * w : rms(y) * w * silu(gate);
  * w is [groups * group_size], or [group_size] with shared_weight.
- * sgl_amd_gate_mul: out = silu(gate) * up, rows of `d` at the given strides. */
+ * sgl_amd_gate_mul: out = activation(gate, up), rows of `d` at the given strides. */
 int sgl_amd_residual_norm(int is_f32, int mode, const int64_t* ids, const void* table, int64_t vocab, float scale, const void* y,
     int64_t y_stride, const float* partials, int splits, const void* partials_bias, const float* step, const float* w1, const float* b1, float* x, int64_t x_stride,
     const float* w2, const float* b2, void* h, int64_t h_stride, void* copy0, void* copy1, int64_t copy_stride,
@@ -551,15 +561,17 @@ int sgl_amd_gated_rmsnorm(int is_f32, const void* y, int64_t y_stride, const voi
     void* out, int64_t out_stride, int64_t rows, int groups, int group_size, int gate_first, int shared_weight,
     float eps, void* stream);
 int sgl_amd_gate_mul(int is_f32, const void* gate, const void* up, void* out, int64_t rows, int d, int64_t in_stride, int64_t out_stride,
-    void* stream);
+    int glu_kind, float glu_limit, float glu_alpha, void* stream);
 /* Residual row of pre-norm designs, fp32: x <- table[ids] * scale (+ pos_table[positions]), or x + a + b, each source the sum of
  * its items [rows x items x width] (times fp32 weight [rows, items] if given) in fp32 or in the activation type; then the copy
- * `save`, then + extra (rows) + step (vector), then h = RMS norm(x) * weight.  save / extra rows are contiguous. */
+ * `save`, then + extra (rows) + step (vector), then h = RMS norm(x) * weight (null: h = x).  With `post` (designs that norm a sublayer's
+ * output) x <- x + mult * (RMS norm(a + b) * post).  save / extra rows are contiguous. */
 int sgl_amd_residual_rms(int is_f32, const int64_t* ids, const void* table, int64_t vocab, float scale, const int64_t* positions,
     const void* pos_table, int64_t max_positions, const void* a, int a_f32, int a_items, int64_t a_row_stride,
     int64_t a_item_stride, const float* a_weight, const void* b, int b_f32, int b_items, int64_t b_row_stride,
     int64_t b_item_stride, const float* b_weight, float* x, int64_t x_stride, float* save, const float* extra,
-    const float* step, const float* weight, void* h, int64_t h_stride, int64_t rows, int width, float eps, void* stream);
+    const float* step, const float* post, float mult, const float* weight, void* h, int64_t h_stride, int64_t rows, int width, float eps,
+    void* stream);
 /* cap * tanh(z / cap) -> fp32 [rows, cols] contiguous; z: `items` addends item_stride apart (split-K partials) */
 int sgl_amd_soft_cap(int is_f32, const void* z, int64_t z_row_stride, int items, int64_t item_stride, float* out, int64_t rows, int cols,
     float cap, void* stream);
@@ -615,7 +627,7 @@ int sgl_amd_latent_attention(int is_f32, const void* qc, int64_t qc_token, int64
     int64_t qr_head, const void* cache, int64_t cache_stride, const int32_t* req_to_token, int64_t r2t_stride,
     const int64_t* req_pool_indices, const int32_t* tok_seg, const int64_t* positions, void* out, int64_t o_token,
     int64_t o_head, float* part_o, float* part_ml, int64_t tokens, int heads, int rank, int rot, int window,
-    int splits, float scale, int plain, void* stream);
+    int splits, float scale, const float* sinks, int plain, void* stream);
 /* Prefill form (bf16): sgl_amd_latent_gather packs the rows of every segment's visible keys (segment b: positions key_first[b] ..,
  * at key_start[b] of the packed rows; key_seg names a packed key's segment); the caller expands them per head into
  * kv = [heads * dim keys | heads * vdim values]; sgl_amd_latent_prefill attends: blocks = [num_blocks, 2] (segment, first of 256
@@ -627,12 +639,37 @@ int sgl_amd_latent_gather(const void* cache, int64_t cache_stride, const int32_t
 int sgl_amd_latent_prefill(const void* q, int64_t q_token, const void* latents, int64_t latents_stride, const void* kv, int64_t kv_stride,
     const int32_t* blocks, int num_blocks, const int32_t* seg_start, const int32_t* seg_len, const int32_t* key_start,
     const int32_t* key_first, const int64_t* positions, void* out, int64_t o_token, int heads, int dim, int rot,
-    int rank, int vdim, int window, float scale, void* stream);
+    int rank, int vdim, int window, float scale, const float* sinks, void* stream);
+
+/* ---- between a projection and attention (projection_rows.hip) ------------------------------------------------------
+ * The source is rows in the activation type, or the fp32 split-K partials of a decode projection (`items` of them item_stride apart, rows
+ * row_stride apart, plus `bias` in the activation type).  cos_sin fp32 [max_positions, rot_dims] = cos | sin; dimension i of the rotated
+ * part turns with i + rot_dims / 2.
+ * sgl_amd_head_prepare: columns [heads * kd queries | kv_heads * kd keys | kv_heads * vd values | gate].  norm_order 1: RMS norm over `dim`
+ * elements with q_norm / k_norm, then rotation of [rot_off, rot_off + rot_dims); 2: rotation, then the norm without weights; 0: rotation alone.
+ * Queries go to `out` (which may be the source rows), the gate columns behind them (gate_cols > 0), keys and values to cache rows
+ * `loc`, [kv_heads][kd | vd].  `plain` forces the form for any sizes.
+ * sgl_amd_latent_down: columns [q_rank query latent | rank latent | rot rotated key part] -> cq = RMS norm of the first, cache row `loc` =
+ * [RMS norm of the second | rotated third].
+ * sgl_amd_bigram_rows: rows[t] = (prev * mul_prev + ids[t] * mul_cur) mod buckets, `buckets` at position 0; prev is the token in front of t
+ * in its segment, or the one its request left at position - 1: slot_ids[req_to_token[..]].  Leaves ids[t] at slot_ids[loc[t]]. */
+int sgl_amd_head_prepare(int is_f32, const void* rows, int64_t row_stride, const float* partials, int items, int64_t item_stride, const void* bias,
+    void* out, int64_t o_stride, const float* q_norm, const float* k_norm, int norm_order, float eps, const float* cos_sin,
+    int64_t max_positions, const int64_t* positions, int rot_off, int rot_dims, void* cache, int64_t cache_stride,
+    const int64_t* loc, int64_t tokens, int heads, int kv_heads, int kd, int vd, int dim, int gate_cols, int plain, void* stream);
+int sgl_amd_latent_down(int is_f32, const void* rows, int64_t row_stride, const float* partials, int items, int64_t item_stride,
+    const float* q_norm, const float* norm, float eps, const float* cos_sin, int64_t max_positions, const int64_t* positions, int rot_dims,
+    void* cq, int64_t cq_stride, void* cache, int64_t cache_stride, const int64_t* loc, int64_t tokens, int q_rank, int rank, int rot,
+    void* stream);
+int sgl_amd_bigram_rows(const int64_t* ids, const int64_t* positions, const int64_t* loc, const int32_t* req_to_token, int64_t r2t_stride,
+    const int64_t* req_pool_indices, const int32_t* tok_seg, int32_t* slot_ids, int64_t* rows, int64_t tokens, int64_t mul_prev,
+    int64_t mul_cur, int64_t buckets, void* stream);
 
 /* ---- grouped-query attention of layers with sizes of their own (grouped_attention.hip) ---------------------------
  * Cache rows [kv_heads][kd | vd] (kd, vd multiples of 8, one row stride); query head h reads key head h / (heads / kv_heads); position
  * i sees the `window` positions up to and with itself (window <= 0: all); `sink` joins the softmax denominator as a score without
- * a value (-inf: none); the output is multiplied by sigmoid(gate) when a gate is given.
+ * a value (-inf: none), `sinks` [heads] instead of it one a head; cap > 0 makes scores cap * tanh(score / cap); the output is multiplied by
+ * sigmoid(gate) when a gate is given: [tokens, heads * vd], or [tokens, heads] with gate_per_head.
  * sgl_amd_grouped_attention: any token mix; tok_seg null = a decode batch, whose own keys and values may be given as k_new / v_new
  * (matrix form): they are read from there and stored at `loc`.  part_o fp32 [tokens, heads, splits, vd], part_ml [.., 2] for splits > 1.
  * sgl_amd_grouped_prefill: stored keys; blocks = [num_blocks, 2] (segment, first of sgl_amd_grouped_prefill_rows() / group tokens). */
@@ -645,21 +682,25 @@ int sgl_amd_grouped_attention(int is_f32, const void* q, int64_t q_stride, void*
     const void* v_new, int64_t v_stride, const int64_t* loc, const int32_t* req_to_token, int64_t r2t_stride,
     const int64_t* req_pool_indices, const int32_t* tok_seg, const int64_t* positions, const void* gate,
     int64_t gate_stride, void* out, int64_t o_stride, float* part_o, float* part_ml, int64_t tokens, int heads,
-    int kv_heads, int kd, int vd, int window, int splits, float scale, float sink, int plain, void* stream);
+    int kv_heads, int kd, int vd, int window, int splits, float scale, float sink, const float* sinks, float cap, int gate_per_head,
+    int plain, void* stream);
 int sgl_amd_grouped_prefill(const void* q, int64_t q_stride, const void* cache, int64_t cache_stride, const int32_t* req_to_token,
     int64_t r2t_stride, const int64_t* req_pool_indices, const int32_t* blocks, int num_blocks,
     const int32_t* seg_start, const int32_t* seg_len, const int64_t* positions, const void* gate, int64_t gate_stride,
-    void* out, int64_t o_stride, int heads, int kv_heads, int kd, int vd, int window, float scale, float sink, void* stream);
+    void* out, int64_t o_stride, int heads, int kv_heads, int kd, int vd, int window, float scale, float sink,
+    const float* sinks, float cap, int gate_per_head, void* stream);
 
 /* ---- router with a bias, and the plain form of routed experts (moe_route.hip) -------------------------------------
  * sgl_amd_moe_route: per token the `top` largest of W h + bias (fp32) and the softmax over those -> fp32 weights, int32 ids
- * [tokens, top].  partials fp32 [slices, tokens, pad] (pad = 16, 32, .. 256 >= experts): the matrix form, `slices` pieces of the
- * columns; null: the plain one.  sgl_amd_experts_plain: pair i = (token i / top, expert ids[i]); up: silu(gate x) * (up x) from w [experts, 2 N, K],
+ * [tokens, top].  sigmoid = 1: scores sigmoid(W h + bias), the choice by score + correction among the experts of the best `keep` of `groups`
+ * equal groups (a group counts by the sum of its two largest), weights score * scale.  partials fp32 [slices, tokens, pad] (pad = 16, 32, .. 256 >= experts): the matrix form, `slices` pieces of the
+ * columns; null: the plain one.  sgl_amd_experts_plain: pair i = (token i / top, expert ids[i]); up: activation(gate x, up x) from w [experts, 2 N, K],
  * else w x from w [experts, N, K] and x [pairs, K]. */
 int sgl_amd_moe_route(int is_f32, const void* h, int64_t h_stride, const void* w, const float* bias, float* topk_weights, int32_t* topk_ids,
-    float* partials, int slices, int pad, int64_t tokens, int K, int experts, int top, void* stream);
+    float* partials, int slices, int pad, int64_t tokens, int K, int experts, int top, int sigmoid, const float* correction, int groups,
+    int keep, float scale, void* stream);
 int sgl_amd_experts_plain(int is_f32, int up, const void* x, int64_t x_stride, const void* w, const int32_t* ids, void* out, int64_t o_stride,
-    int64_t pairs, int top, int N, int K, int experts, void* stream);
+    int64_t pairs, int top, int N, int K, int experts, int glu_kind, float glu_limit, float glu_alpha, void* stream);
 
 #ifdef __cplusplus
 }

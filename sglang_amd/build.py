@@ -41,6 +41,8 @@ UNIT_GROUPS = {
                "wstream_gemm.hip"],
     "grouped": ["api.cpp", "elementwise.hip", "grouped_attention.hip", "metadata.hip", "moe.hip", "moe_route.hip", "moe_tiled_gemm.hip", "residual_norm.hip",
                 "sampling.hip", "skinny_gemm.hip", "wstream_gemm.hip"],
+    "layered": ["api.cpp", "elementwise.hip", "grouped_attention.hip", "latent_attention.hip", "metadata.hip", "moe.hip", "moe_route.hip",
+                "moe_tiled_gemm.hip", "projection_rows.hip", "residual_norm.hip", "sampling.hip", "skinny_gemm.hip", "wstream_gemm.hip"],
 }
 
 

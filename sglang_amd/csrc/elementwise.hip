@@ -13,6 +13,7 @@
 // bf16 rounding points reproduced so results are bit-comparable with the
 // torch-native path.
 #include "common.hpp"
+#include "glu.hpp"
 #include "kv_format.hpp"
 #include "sglang_amd.h"
 
@@ -147,9 +148,9 @@ __device__ __forceinline__ U4 ld16_once(const uint16_t* p) {
   return __builtin_bit_cast(U4, __builtin_nontemporal_load(reinterpret_cast<const u32x4_t*>(p)));
 }
 
-template <bool ROUND_MID>
+template <bool ROUND_MID, int KIND>
 __global__ __launch_bounds__(256) void silu_and_mul_kernel(const uint16_t* __restrict__ in, uint16_t* __restrict__ out,
-                                                           int d, int64_t in_stride, int64_t out_stride) {
+                                                           int d, int64_t in_stride, int64_t out_stride, float limit, float alpha) {
   const int64_t row = blockIdx.y;
   const uint16_t* g = in + row * in_stride;
   const uint16_t* u = g + d;
@@ -178,9 +179,16 @@ __global__ __launch_bounds__(256) void silu_and_mul_kernel(const uint16_t* __res
     for (int j = 0; j < 8; ++j) {
       // hardware exp2 / rcp (1 ulp each): the result is rounded to bf16 right after, 2^-15 of the outputs can land on
       // the other side of a rounding boundary; the IEEE expf + division made this kernel VALU-bound at 4.5 TB/s
-      float sl = gs[j] * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(gs[j] * -1.4426950408889634f));
+      float gv = gs[j], uv = us[j], arg = gs[j];
+      if (KIND == kGluGeluTanh) arg = 1.5957691216057308f * (gv + 0.044715f * gv * gv * gv);
+      if (KIND == kGluClampedSwish) {
+        gv = fminf(gv, limit);
+        uv = fminf(fmaxf(uv, -limit), limit) + 1.0f;
+        arg = alpha * gv;
+      }
+      float sl = gv * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(arg * -1.4426950408889634f));
       if (ROUND_MID) sl = rbf(sl);
-      r[j] = sl * us[j];
+      r[j] = sl * uv;
     }
     st16(o + (static_cast<int64_t>(v) << 3), pack8(r));
   }
@@ -420,13 +428,36 @@ int sgl_amd_silu_and_mul(const void* in, void* out, int64_t num_rows, int d, int
     const uint16_t* ip = static_cast<const uint16_t*>(in) + r0 * in_row_stride;
     uint16_t* op = static_cast<uint16_t*>(out) + r0 * out_row_stride;
     if (round_intermediate)
-      hipLaunchKernelGGL(silu_and_mul_kernel<true>, dim3(bx, nr), dim3(threads), 0, as_stream(stream),
-                         ip, op, d, in_row_stride, out_row_stride);
+      hipLaunchKernelGGL((silu_and_mul_kernel<true, kGluSilu>), dim3(bx, nr), dim3(threads), 0, as_stream(stream),
+                         ip, op, d, in_row_stride, out_row_stride, 0.f, 0.f);
     else
-      hipLaunchKernelGGL(silu_and_mul_kernel<false>, dim3(bx, nr), dim3(threads), 0, as_stream(stream),
-                         ip, op, d, in_row_stride, out_row_stride);
+      hipLaunchKernelGGL((silu_and_mul_kernel<false, kGluSilu>), dim3(bx, nr), dim3(threads), 0, as_stream(stream),
+                         ip, op, d, in_row_stride, out_row_stride, 0.f, 0.f);
   }
   SGL_CHECK_LAUNCH("silu_and_mul");
+  return 0;
+}
+
+int sgl_amd_glu_and_mul(const void* in, void* out, int64_t num_rows, int d, int64_t in_row_stride, int64_t out_row_stride, int glu_kind,
+                        float glu_limit, float glu_alpha, void* stream) {
+  if (glu_kind == kGluSilu) return sgl_amd_silu_and_mul(in, out, num_rows, d, in_row_stride, out_row_stride, 0, stream);
+  SGL_CLEAR_STALE_ERROR();
+  SGL_CHECK_ARG(glu_kind > kGluSilu && glu_kind < kGluKinds, "glu_and_mul: no activation %d", glu_kind);
+  SGL_CHECK_ARG(d > 0 && d % 8 == 0 && in_row_stride % 8 == 0 && out_row_stride % 8 == 0 && aligned16(in) && aligned16(out),
+                "glu_and_mul: rows of whole 16-byte vectors (d = %d)", d);
+  SGL_CHECK_ARG(num_rows <= 65535LL * 65535LL, "glu_and_mul: too many rows");
+  const int bx = ((d >> 3) + 256 * kSiluVecPerThread - 1) / (256 * kSiluVecPerThread);
+  for (int64_t r0 = 0; r0 < num_rows; r0 += 65535) {
+    const dim3 grid(bx, static_cast<unsigned>(num_rows - r0 < 65535 ? num_rows - r0 : 65535));
+    const uint16_t* ip = static_cast<const uint16_t*>(in) + r0 * in_row_stride;
+    uint16_t* op = static_cast<uint16_t*>(out) + r0 * out_row_stride;
+    if (glu_kind == kGluGeluTanh)
+      hipLaunchKernelGGL((silu_and_mul_kernel<false, kGluGeluTanh>), grid, dim3(256), 0, as_stream(stream), ip, op, d, in_row_stride, out_row_stride, 0.f, 0.f);
+    else
+      hipLaunchKernelGGL((silu_and_mul_kernel<false, kGluClampedSwish>), grid, dim3(256), 0, as_stream(stream), ip, op, d, in_row_stride, out_row_stride,
+                         glu_limit, glu_alpha);
+  }
+  SGL_CHECK_LAUNCH("glu_and_mul");
   return 0;
 }
 

@@ -1,6 +1,6 @@
 // Grouped-query attention over a paged pool for layers with sizes of their own: keys and values of different width, an optional
-// sliding window, an optional sink (a score in the softmax denominator that carries no value) and an optional sigmoid gate on
-// the output, all fused into one pass.
+// sliding window, an optional sink (a score in the softmax denominator that carries no value, one for all heads or one a head), an
+// optional soft cap of the scores and an optional sigmoid gate on the output (a number an element or a head), all fused into one pass.
 //
 //   grouped_kv_store   the keys and values of new tokens into their cache rows
 //   grouped_attention  any token mix, split along the keys; matrix form (bf16) and a plain form (every size, bf16 and fp32).  In a
@@ -30,7 +30,7 @@ struct GroupedParams {
   const int64_t* req;        // [segments] row of req_to_token
   const int32_t* tok_seg;    // [tokens] (null: token index)
   const int64_t* positions;  // [tokens]
-  const void* gate;          // [tokens, heads * vd], or null
+  const void* gate;          // [tokens, heads * vd], [tokens, heads] (gate_per_head), or null
   int64_t gate_stride;
   void* out;                 // [tokens, heads * vd]
   int64_t o_stride;
@@ -41,7 +41,20 @@ struct GroupedParams {
   int64_t tokens;
   int heads, kv_heads, group, kd, vd, window, splits, block_tokens;
   float scale, sink;         // sink = -inf: none
+  const float* sinks;        // [heads], instead of `sink`
+  float cap;                 // > 0: scores become cap * tanh(score / cap)
+  float softmax_scale, cap_in, cap_out;      // matrix forms: factor in front of 2^x, and of a cap's argument and result
+  int gate_per_head;
 };
+
+__device__ __forceinline__ float sink_of(const GroupedParams& p, int head) { return p.sinks ? p.sinks[head] : p.sink; }
+
+// Products of the matrix form -> what the softmax takes, times `softmax_scale`: log2(e) cap tanh(scale product / cap), with
+// tanh x = 1 - 2 / (1 + e^2x): absolute error of a few 2^-24, which is what a score needs.
+__device__ __forceinline__ void cap_scores(const GroupedParams& p, f32x4_t& s) {
+#pragma unroll
+  for (int r = 0; r < 4; ++r) s[r] = p.cap_out - 2.0f * p.cap_out * __builtin_amdgcn_rcpf(1.0f + fast_exp2(s[r] * p.cap_in));
+}
 
 __device__ __forceinline__ void key_range(const GroupedParams& p, int64_t pos, int split, int& lo, int& hi) {
   const int end = static_cast<int>(pos) + 1;
@@ -60,7 +73,11 @@ __device__ __forceinline__ float inverse_sum(float m, float l, float sink) {
 
 template <int VEC, typename T>
 __device__ __forceinline__ void store_gated(const GroupedParams& p, int64_t t, int col, float (&v)[VEC]) {
-  if (p.gate) {
+  if (p.gate && p.gate_per_head) {
+    const float g = sigmoid_f(ld1(static_cast<const T*>(p.gate) + t * p.gate_stride + col / p.vd));
+#pragma unroll
+    for (int j = 0; j < VEC; ++j) v[j] *= g;
+  } else if (p.gate) {
     float g[VEC];
     ldv<VEC>(static_cast<const T*>(p.gate) + t * p.gate_stride + col, g);
 #pragma unroll
@@ -119,6 +136,7 @@ __global__ __launch_bounds__(256) void grouped_attention_plain_kernel(GroupedPar
         for (int u = 0; u < 4; ++u) d += q[c + u] * e[u];
       }
       s = d * p.scale;
+      if (p.cap > 0.f) s = p.cap * tanhf(s / p.cap);
       kp[threadIdx.x] = k;
     }
     const float mn = fmaxf(m, block_max(s, scratch));
@@ -137,8 +155,8 @@ __global__ __launch_bounds__(256) void grouped_attention_plain_kernel(GroupedPar
     __syncthreads();
   }
   if (p.splits == 1) {
-    const float top = fmaxf(m, p.sink), f = expf(m - top);
-    const float inv = f / (l * f + expf(p.sink - top));
+    const float sink = sink_of(p, h), top = fmaxf(m, sink), f = expf(m - top);
+    const float inv = f / (l * f + expf(sink - top));
     for (int c = threadIdx.x; c < p.vd; c += 256) {
       float v[1] = {acc[c] * inv};
       store_gated<1, T>(p, t, h * p.vd + c, v);
@@ -173,7 +191,7 @@ __global__ __launch_bounds__(256) void grouped_merge_kernel(GroupedParams p) {
 #pragma unroll
     for (int j = 0; j < 4; ++j) a[j] += w * v[j];
   }
-  const float inv = inverse_sum(m, l, p.sink);
+  const float inv = inverse_sum(m, l, sink_of(p, h));
 #pragma unroll
   for (int j = 0; j < 4; ++j) a[j] *= inv;
   store_gated<4, T>(p, t, h * p.vd + c, a);
@@ -264,7 +282,6 @@ __global__ __launch_bounds__(256, 2) void grouped_attention_mfma_kernel(GroupedP
 #pragma unroll
   for (int n = 0; n < VT; ++n) o[n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   float m = -INFINITY, l = 0.f;
-  const float sc = p.scale * kLog2e;
   const int first = lo + 32 * wave;
   int slot[2];
   U4 kreg[2][KS], vreg[4][VP];
@@ -318,6 +335,10 @@ __global__ __launch_bounds__(256, 2) void grouped_attention_mfma_kernel(GroupedP
       load(j0 + 128);
       slots(j0 + 256);
     }
+    if (p.cap > 0.f) {
+#pragma unroll
+      for (int n = 0; n < 2; ++n) cap_scores(p, s[n]);
+    }
     if (j0 + 32 > hi) {
 #pragma unroll
       for (int n = 0; n < 2; ++n)
@@ -326,7 +347,7 @@ __global__ __launch_bounds__(256, 2) void grouped_attention_mfma_kernel(GroupedP
           if (j0 + 16 * n + 4 * g + r >= hi) s[n][r] = -INFINITY;
     }
     bf16x8_t pf[1][2];
-    online_softmax<2, VT>(s, sc, m, l, o, pf);
+    online_softmax<2, VT>(s, p.softmax_scale, m, l, o, pf);
     asm volatile("" ::: "memory");                     // (the tile is this wave's own; LDS serves a wave in order)
     __builtin_amdgcn_wave_barrier();
 #pragma unroll
@@ -370,7 +391,7 @@ __global__ __launch_bounds__(256, 2) void grouped_attention_mfma_kernel(GroupedP
     }
     const int head = kvh * p.group + h0 + hd;
     if (p.splits == 1) {
-      const float inv = inverse_sum(mt, lt, p.sink);
+      const float inv = inverse_sum(mt, lt, sink_of(p, head));
 #pragma unroll
       for (int j = 0; j < 4; ++j) a[j] *= inv;
       store_gated<4, uint16_t>(p, t, head * p.vd + c, a);
@@ -452,7 +473,6 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
   for (int c = 0; c < 2; ++c)
 #pragma unroll
     for (int n = 0; n < VT; ++n) o[c][n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  const float sc = p.scale * kLog2e;
   next_slot(lo);
   load();
   next_slot(lo + kPfTile);
@@ -485,6 +505,13 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
         s[1][n] = mfma_bf16(a, q[1][k], s[1][n]);
       }
     }
+    if (p.cap > 0.f) {
+#pragma unroll
+      for (int n = 0; n < 4; ++n) {
+        cap_scores(p, s[0][n]);
+        cap_scores(p, s[1][n]);
+      }
+    }
     if (j0 + kPfTile - 1 > wave_first || (p.window > 0 && j0 <= wave_last - p.window)) {
 #pragma unroll
       for (int c = 0; c < 2; ++c) {
@@ -500,7 +527,7 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
     }
     bf16x8_t pf[2][2][2];
 #pragma unroll
-    for (int c = 0; c < 2; ++c) online_softmax<4, VT>(s[c], sc, m[c], l[c], o[c], pf[c]);
+    for (int c = 0; c < 2; ++c) online_softmax<4, VT>(s[c], p.softmax_scale, m[c], l[c], o[c], pf[c]);
 #pragma unroll
     for (int n = 0; n < VT; ++n)
 #pragma unroll
@@ -518,8 +545,8 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
     float sum = l[c];
     sum += __shfl_xor(sum, 16, 64);
     sum += __shfl_xor(sum, 32, 64);
-    const float inv = inverse_sum(m[c], sum, p.sink);
     if (qtok[c] > last) continue;
+    const float inv = inverse_sum(m[c], sum, sink_of(p, kvh * p.group + qhead[c]));
 #pragma unroll
     for (int n = 0; n < VT; ++n) {
       const int e = 16 * n + 4 * g;
@@ -545,10 +572,17 @@ void launch_prefill(const GroupedParams& p, const dim3& grid, hipStream_t st) {
   else hipLaunchKernelGGL((grouped_prefill_kernel<KS, 8>), grid, dim3(kPfThreads), 0, st, p);
 }
 
+void set_scores(GroupedParams& p, float scale, float cap) {
+  p.scale = scale; p.cap = cap;
+  p.softmax_scale = cap > 0.f ? 1.0f : scale * kLog2e;
+  p.cap_in = cap > 0.f ? 2.0f * kLog2e * scale / cap : 0.f;
+  p.cap_out = kLog2e * cap;
+}
+
 bool whole_vectors(const GroupedParams& p) {
-  return p.kd % 8 == 0 && p.vd % 8 == 0 && p.q_stride % 8 == 0 && p.cache_stride % 8 == 0 && p.o_stride % 4 == 0 && p.gate_stride % 4 == 0 &&
+  return p.kd % 8 == 0 && p.vd % 8 == 0 && p.q_stride % 8 == 0 && p.cache_stride % 8 == 0 && p.o_stride % 4 == 0 && (p.gate_per_head || (p.gate_stride % 4 == 0 && aligned_to(p.gate, 8))) &&
          p.k_stride % 8 == 0 && p.v_stride % 8 == 0 && aligned_to(p.q, 16) && aligned_to(p.cache, 16) && aligned_to(p.k_new, 16) &&
-         aligned_to(p.v_new, 16) && aligned_to(p.gate, 8) && aligned_to(p.out, 8) && aligned_to(p.part_o, 16);
+         aligned_to(p.v_new, 16) && aligned_to(p.out, 8) && aligned_to(p.part_o, 16);
 }
 
 }  // namespace
@@ -583,7 +617,8 @@ int sgl_amd_grouped_attention(int is_f32, const void* q, int64_t q_stride, void*
                               const void* v_new, int64_t v_stride, const int64_t* loc, const int32_t* req_to_token, int64_t r2t_stride,
                               const int64_t* req_pool_indices, const int32_t* tok_seg, const int64_t* positions, const void* gate,
                               int64_t gate_stride, void* out, int64_t o_stride, float* part_o, float* part_ml, int64_t tokens, int heads,
-                              int kv_heads, int kd, int vd, int window, int splits, float scale, float sink, int plain, void* stream) {
+                              int kv_heads, int kd, int vd, int window, int splits, float scale, float sink, const float* sinks, float cap,
+                              int gate_per_head, int plain, void* stream) {
   SGL_CLEAR_STALE_ERROR();
   SGL_CHECK_ARG(q && cache && req_to_token && req_pool_indices && positions && out, "grouped_attention: null operand");
   SGL_CHECK_ARG(heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && heads <= 65535 && kd > 0 && vd > 0 && kd % 4 == 0 && vd % 4 == 0 &&
@@ -596,7 +631,8 @@ int sgl_amd_grouped_attention(int is_f32, const void* q, int64_t q_stride, void*
   p.v_stride = v_stride; p.loc = loc; p.req_to_token = req_to_token; p.r2t_stride = r2t_stride; p.req = req_pool_indices; p.tok_seg = tok_seg;
   p.positions = positions; p.gate = gate; p.gate_stride = gate_stride; p.out = out; p.o_stride = o_stride; p.part_o = part_o; p.part_ml = part_ml;
   p.tokens = tokens; p.heads = heads; p.kv_heads = kv_heads; p.group = heads / kv_heads; p.kd = kd; p.vd = vd; p.window = window;
-  p.splits = splits; p.scale = scale; p.sink = sink;
+  p.splits = splits; p.sink = sink; p.sinks = sinks; p.gate_per_head = gate_per_head;
+  set_scores(p, scale, cap);
   hipStream_t st = as_stream(stream);
   const bool matrix = !is_f32 && !plain && sgl_amd_grouped_attention_matrix_form(kd, vd) && whole_vectors(p) && scale > 0.f;
   SGL_CHECK_ARG(!k_new || (matrix && v_new && loc && !tok_seg), "grouped_attention: only the matrix form of a decode batch takes keys and values that are not stored yet");
@@ -610,7 +646,8 @@ int sgl_amd_grouped_attention(int is_f32, const void* q, int64_t q_stride, void*
     const size_t lds = (static_cast<size_t>(kd) + vd + 256) * 4 + 256 * 8;
     SGL_CHECK_ARG(lds <= 64 * 1024 - 256, "grouped_attention: head sizes %d + %d need %zu bytes of LDS", kd, vd, lds);
     const size_t al = is_f32 ? 16 : 8;
-    SGL_CHECK_ARG(cache_stride % 4 == 0 && aligned_to(cache, al) && o_stride % 4 == 0 && gate_stride % 4 == 0 && aligned_to(out, al) && aligned_to(gate, al),
+    SGL_CHECK_ARG(cache_stride % 4 == 0 && aligned_to(cache, al) && o_stride % 4 == 0 && aligned_to(out, al) &&
+                      (gate_per_head || (gate_stride % 4 == 0 && aligned_to(gate, al))),
                   "grouped_attention: rows of whole 4-element pieces");
     if (is_f32) hipLaunchKernelGGL((grouped_attention_plain_kernel<float>), grid, dim3(256), lds, st, p);
     else hipLaunchKernelGGL((grouped_attention_plain_kernel<uint16_t>), grid, dim3(256), lds, st, p);
@@ -629,7 +666,7 @@ int sgl_amd_grouped_prefill(const void* q, int64_t q_stride, const void* cache, 
                             int64_t r2t_stride, const int64_t* req_pool_indices, const int32_t* blocks, int num_blocks,
                             const int32_t* seg_start, const int32_t* seg_len, const int64_t* positions, const void* gate, int64_t gate_stride,
                             void* out, int64_t o_stride, int heads, int kv_heads, int kd, int vd, int window, float scale, float sink,
-                            void* stream) {
+                            const float* sinks, float cap, int gate_per_head, void* stream) {
   SGL_CLEAR_STALE_ERROR();
   SGL_CHECK_ARG(q && cache && req_to_token && req_pool_indices && blocks && seg_start && seg_len && positions && out, "grouped_prefill: null operand");
   SGL_CHECK_ARG(heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && sgl_amd_grouped_prefill_supported(kd, vd, heads / kv_heads) &&
@@ -640,7 +677,9 @@ int sgl_amd_grouped_prefill(const void* q, int64_t q_stride, const void* cache, 
   p.q = q; p.q_stride = q_stride; p.cache = const_cast<void*>(cache); p.cache_stride = cache_stride; p.req_to_token = req_to_token;
   p.r2t_stride = r2t_stride; p.req = req_pool_indices; p.positions = positions; p.gate = gate; p.gate_stride = gate_stride; p.out = out;
   p.o_stride = o_stride; p.blocks = blocks; p.seg_start = seg_start; p.seg_len = seg_len; p.heads = heads; p.kv_heads = kv_heads;
-  p.group = heads / kv_heads; p.kd = kd; p.vd = vd; p.window = window; p.splits = 1; p.block_tokens = kPfRows / p.group; p.scale = scale; p.sink = sink;
+  p.group = heads / kv_heads; p.kd = kd; p.vd = vd; p.window = window; p.splits = 1; p.block_tokens = kPfRows / p.group; p.sink = sink;
+  p.sinks = sinks; p.gate_per_head = gate_per_head;
+  set_scores(p, scale, cap);
   SGL_CHECK_ARG(whole_vectors(p), "grouped_prefill: rows of whole 16-byte vectors");
   const dim3 grid(kv_heads, num_blocks);
   hipStream_t st = as_stream(stream);

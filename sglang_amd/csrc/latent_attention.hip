@@ -204,7 +204,15 @@ struct LatentAttnParams {
   float* part_ml;            // [tokens, heads, splits, 2]
   int heads, rank, rot, window, splits;
   float scale;
+  const float* sinks;        // [heads] scores in the softmax denominator that carry no value, or null
 };
+
+// 1 / denominator in units of e^m, for the sum l taken relative to the maximum m: a sink joins here
+__device__ __forceinline__ float inverse_sum(float m, float l, const float* sinks, int head) {
+  if (!sinks) return l > 0.f ? 1.0f / l : 0.f;
+  const float s = sinks[head], top = fmaxf(m, s), f = expf(m - top);
+  return f / (l * f + expf(s - top));
+}
 
 __device__ __forceinline__ void key_range(const LatentAttnParams& p, int64_t pos, int split, int& lo, int& hi) {
   const int first = p.window > 0 && pos + 1 > p.window ? static_cast<int>(pos + 1 - p.window) : 0;
@@ -265,7 +273,7 @@ __global__ __launch_bounds__(256) void latent_attention_plain_kernel(LatentAttnP
     __syncthreads();
   }
   if (p.splits == 1) {
-    const float inv = l > 0.f ? 1.0f / l : 0.f;
+    const float inv = inverse_sum(m, l, p.sinks, h);
     T* o = static_cast<T*>(p.out) + t * p.o_token + h * p.o_head;
     for (int c = threadIdx.x; c < p.rank; c += 256) st1(o + c, acc[c] * inv);
   } else {
@@ -297,7 +305,7 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(LatentAttnParams p) {
 #pragma unroll
       for (int j = 0; j < VEC; ++j) a[j] += w * v[j];
     }
-    const float inv = 1.0f / l;
+    const float inv = inverse_sum(m, l, p.sinks, h);
 #pragma unroll
     for (int j = 0; j < VEC; ++j) a[j] *= inv;
     stv<VEC>(static_cast<T*>(p.out) + t * p.o_token + h * p.o_head + c, a);
@@ -459,7 +467,7 @@ __global__ __launch_bounds__(256 * HG, 2) void latent_attention_mfma_kernel(Late
   l = (wmax[i16] + wmax[16 + i16]) + (wmax[32 + i16] + wmax[48 + i16]);
   if (head >= p.heads) return;
   const int64_t part = (t * p.heads + head) * p.splits + split;
-  const float inv = p.splits == 1 ? 1.0f / l : 1.0f;
+  const float inv = p.splits == 1 ? inverse_sum(m / kLog2e, l, p.sinks, head) : 1.0f;
 #pragma unroll
   for (int i = 0; i < OT; ++i) {
     const int c = (wave * OT + i) * 16 + 4 * g;
@@ -493,6 +501,7 @@ struct LatentPrefillParams {
   int64_t o_token;
   int heads, dim, rot, rank, vdim, window;
   float scale;
+  const float* sinks;        // [heads], or null
 };
 
 constexpr int kPfThreads = 512;
@@ -660,7 +669,7 @@ __global__ __launch_bounds__(kPfThreads, 2) void latent_prefill_kernel(LatentPre
     float sum = l[c];
     sum += __shfl_xor(sum, 16, 64);
     sum += __shfl_xor(sum, 32, 64);
-    const float inv = 1.0f / sum;
+    const float inv = inverse_sum(m[c] / kLog2e, sum, p.sinks, h);
     const int qi = q0 + 32 * wave + 16 * c + i16;
     if (qi >= len) continue;
     uint16_t* orow = static_cast<uint16_t*>(p.out) + (t0 + qi) * p.o_token + static_cast<int64_t>(h) * p.vdim;
@@ -759,7 +768,7 @@ int sgl_amd_latent_attention(int is_f32, const void* qc, int64_t qc_token, int64
                              int64_t qr_head, const void* cache, int64_t cache_stride, const int32_t* req_to_token, int64_t r2t_stride,
                              const int64_t* req_pool_indices, const int32_t* tok_seg, const int64_t* positions, void* out, int64_t o_token,
                              int64_t o_head, float* part_o, float* part_ml, int64_t tokens, int heads, int rank, int rot, int window,
-                             int splits, float scale, int plain, void* stream) {
+                             int splits, float scale, const float* sinks, int plain, void* stream) {
   SGL_CLEAR_STALE_ERROR();
   SGL_CHECK_ARG(qc && qr && cache && req_to_token && req_pool_indices && positions && out, "latent_attention: null operand");
   SGL_CHECK_ARG(heads > 0 && heads <= 65535 && rank > 0 && rot >= 0 && cache_stride >= rank + rot && splits >= 1 && splits <= 64,
@@ -767,7 +776,7 @@ int sgl_amd_latent_attention(int is_f32, const void* qc, int64_t qc_token, int64
   SGL_CHECK_ARG(splits == 1 || (part_o && part_ml), "latent_attention: split launches need their workspaces");
   if (tokens <= 0) return 0;
   LatentAttnParams p{qc, qc_token, qc_head, qr, qr_token, qr_head, cache, cache_stride, req_to_token, r2t_stride, req_pool_indices, tok_seg,
-                     positions, out, o_token, o_head, part_o, part_ml, heads, rank, rot, window, splits, scale};
+                     positions, out, o_token, o_head, part_o, part_ml, heads, rank, rot, window, splits, scale, sinks};
   // queries in whole 16-byte pieces
   const bool vecq = rank % 8 == 0 && rot % 8 == 0 && qc_token % 8 == 0 && qc_head % 8 == 0 && qr_token % 8 == 0 && qr_head % 8 == 0 &&
            aligned_to(qc, 16) && aligned_to(qr, 16) && o_token % 4 == 0 && o_head % 4 == 0 && aligned_to(out, 8) && aligned_to(part_o, 16);
@@ -820,7 +829,7 @@ int sgl_amd_latent_gather(const void* cache, int64_t cache_stride, const int32_t
 int sgl_amd_latent_prefill(const void* q, int64_t q_token, const void* latents, int64_t latents_stride, const void* kv, int64_t kv_stride,
                            const int32_t* blocks, int num_blocks, const int32_t* seg_start, const int32_t* seg_len, const int32_t* key_start,
                            const int32_t* key_first, const int64_t* positions, void* out, int64_t o_token, int heads, int dim, int rot,
-                           int rank, int vdim, int window, float scale, void* stream) {
+                           int rank, int vdim, int window, float scale, const float* sinks, void* stream) {
   SGL_CLEAR_STALE_ERROR();
   SGL_CHECK_ARG(q && latents && kv && blocks && seg_start && seg_len && key_start && key_first && positions && out, "latent_prefill: null operand");
   SGL_CHECK_ARG(sgl_amd_latent_prefill_supported(dim, rot, vdim) && heads > 0 && rank % 8 == 0 && num_blocks <= 65535,
@@ -831,7 +840,7 @@ int sgl_amd_latent_prefill(const void* q, int64_t q_token, const void* latents, 
                 "latent_prefill: rows of whole 16-byte vectors");
   if (num_blocks <= 0) return 0;
   LatentPrefillParams p{q, q_token, latents, latents_stride, kv, kv_stride, blocks, seg_start, seg_len, key_start, key_first, positions, out, o_token,
-                        heads, dim, rot, rank, vdim, window, scale};
+                        heads, dim, rot, rank, vdim, window, scale, sinks};
   const dim3 grid(heads, num_blocks);
   hipStream_t st = as_stream(stream);
   const int dk = dim + rot;

@@ -181,6 +181,25 @@ __global__ void alloc_decode_kernel(const int64_t* __restrict__ seq_lens,
   else out_indices[pid] = free_pages[page_start] * ps;
 }
 
+// Row of the bigram table per token.  The token in front of a portion's first one is found by its cache slot, so it follows
+// the slots through shared prefixes, portions and reuse; slots written here belong to this batch's tokens and are never read in it.
+__global__ __launch_bounds__(256) void bigram_rows_kernel(const int64_t* __restrict__ ids, const int64_t* __restrict__ positions,
+                                                          const int64_t* __restrict__ loc, const int32_t* __restrict__ req_to_token,
+                                                          int64_t r2t_stride, const int64_t* __restrict__ req, const int32_t* __restrict__ tok_seg,
+                                                          int32_t* slot_ids, int64_t* __restrict__ rows, int64_t tokens, int64_t mul_prev,
+                                                          int64_t mul_cur, int64_t buckets) {
+  const int64_t t = static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x;
+  if (t >= tokens) return;
+  const int64_t b = tok_seg ? tok_seg[t] : t, pos = positions[t], id = ids[t];
+  int64_t row = buckets;
+  if (pos > 0) {
+    const int64_t prev = tok_seg && t > 0 && tok_seg[t - 1] == b ? ids[t - 1] : slot_ids[req_to_token[req[b] * r2t_stride + pos - 1]];
+    row = (prev % buckets * mul_prev + id % buckets * mul_cur) % buckets;
+  }
+  rows[t] = row;
+  slot_ids[loc[t]] = static_cast<int32_t>(id);
+}
+
 }  // namespace
 
 extern "C" {
@@ -280,6 +299,20 @@ int sgl_amd_clamp_position(const void* seq_lens, int lens_are_i64, int64_t* posi
     hipLaunchKernelGGL(clamp_position_kernel<int32_t>, grid, dim3(256), 0, as_stream(stream),
                        static_cast<const int32_t*>(seq_lens), positions, batch);
   SGL_CHECK_LAUNCH("clamp_position");
+  return 0;
+}
+
+int sgl_amd_bigram_rows(const int64_t* ids, const int64_t* positions, const int64_t* loc, const int32_t* req_to_token, int64_t r2t_stride,
+                        const int64_t* req_pool_indices, const int32_t* tok_seg, int32_t* slot_ids, int64_t* rows, int64_t tokens,
+                        int64_t mul_prev, int64_t mul_cur, int64_t buckets, void* stream) {
+  SGL_CLEAR_STALE_ERROR();
+  SGL_CHECK_ARG(ids && positions && loc && req_to_token && req_pool_indices && slot_ids && rows, "bigram_rows: null operand");
+  SGL_CHECK_ARG(buckets >= 1 && buckets < (int64_t{1} << 31) && mul_prev >= 0 && mul_prev < buckets && mul_cur >= 0 && mul_cur < buckets,
+                "bigram_rows: factors %lld, %lld modulo %lld", (long long)mul_prev, (long long)mul_cur, (long long)buckets);
+  if (tokens <= 0) return 0;
+  hipLaunchKernelGGL(bigram_rows_kernel, dim3(static_cast<unsigned>((tokens + 255) / 256)), dim3(256), 0, as_stream(stream), ids, positions, loc,
+                     req_to_token, r2t_stride, req_pool_indices, tok_seg, slot_ids, rows, tokens, mul_prev, mul_cur, buckets);
+  SGL_CHECK_LAUNCH("bigram_rows");
   return 0;
 }
 

@@ -1,11 +1,13 @@
 // Router and the plain form of routed experts.
 //
-//   moe_route     logits W h + b in fp32, the `top` largest per token, softmax over those alone.  bf16 rows: matrix instructions over
+//   moe_route     logits W h + b in fp32, the `top` largest per token, softmax over those alone; or sigmoid scores, chosen by score +
+//                 correction among the groups of experts whose two best sum highest, weighted by score * scale.  bf16 rows: matrix instructions over
 //                 slices of the columns, one wave each (a compute unit alone streams the router's rows far too slowly), then a
 //                 launch that adds the slices and the bias and picks; fp32 rows and odd sizes: plain sums and the pick in one launch
 //   experts_up / experts_down   silu(gate h) * (up h) and its down projection per (token, expert) pair for fp32 rows and sizes outside
 //                 the grouped matrix kernels' forms: a wave sums one output
 #include "elem_io.hpp"
+#include "glu.hpp"
 #include "mfma_tiles.hpp"
 #include "sglang_amd.h"
 
@@ -23,24 +25,69 @@ struct RouteParams {
   float* part;            // [slices, tokens, pad] partial logits
   int64_t tokens;
   int K, experts, top, slices, pad;
+  int sigmoid;            // 0: softmax over the chosen logits
+  const float* correction;// sigmoid: [experts] added to the scores for the choice alone, or null
+  int group_size, groups, keep;   // sigmoid: equal groups of neighbours, experts of the best `keep` can be chosen
+  float scale;
 };
+
+__device__ __forceinline__ void wave_lds_fence() {     // (a wave's own array: LDS serves a wave in order)
+  asm volatile("" ::: "memory");
+  __builtin_amdgcn_wave_barrier();
+}
+
+// Sigmoid scores: s[j] of expert lane + 64 j, z[j] what it is chosen by (-inf: not at all).  all, group: [64 N] of this wave.
+template <int N>
+__device__ __forceinline__ void score_experts(const RouteParams& p, float (&z)[N], float (&s)[N], int lane, float* all, float* group) {
+#pragma unroll
+  for (int j = 0; j < N; ++j) {
+    const int e = lane + 64 * j;
+    s[j] = sigmoid_f(z[j]);
+    z[j] = e < p.experts ? s[j] + (p.correction ? p.correction[e] : 0.f) : -INFINITY;
+    if (!(z[j] == z[j])) z[j] = -INFINITY;
+    all[e] = z[j];
+  }
+  if (p.keep >= p.groups) return;
+  wave_lds_fence();
+  for (int g = lane; g < p.groups; g += 64) {
+    float a = -INFINITY, b = -INFINITY;                // the two largest
+    for (int i = 0; i < p.group_size; ++i) {
+      const float v = all[g * p.group_size + i];
+      b = fmaxf(b, fminf(a, v));
+      a = fmaxf(a, v);
+    }
+    group[g] = p.group_size > 1 ? a + b : a;
+  }
+  wave_lds_fence();
+#pragma unroll
+  for (int j = 0; j < N; ++j) {
+    const int e = lane + 64 * j;
+    if (e >= p.experts) continue;
+    const int g = e / p.group_size;
+    const float mine = group[g];
+    int ahead = 0;
+    for (int i = 0; i < p.groups; ++i) ahead += group[i] > mine || (group[i] == mine && i < g) ? 1 : 0;
+    if (ahead >= p.keep) z[j] = -INFINITY;
+  }
+  wave_lds_fence();
+}
 
 // A wave picks for one token: z[j] is the logit of expert lane + 64 j.  An expert's place is the number of experts in front of it
 // (larger logit, or the same and a smaller index; what is not a number goes last), so every place has exactly one expert.
 template <int N>
 __device__ __forceinline__ void pick_experts(const RouteParams& p, int64_t t, float (&z)[N], int lane, float* all) {
   int place[N];
-  float top = -INFINITY;
+  float top = -INFINITY, score[N];
+  if (p.sigmoid) score_experts<N>(p, z, score, lane, all, all + 64 * N);
 #pragma unroll
   for (int j = 0; j < N; ++j) {
     place[j] = 0;
     if (!(z[j] == z[j]) || lane + 64 * j >= p.experts) z[j] = -INFINITY;
     top = fmaxf(top, z[j]);
-    all[lane + 64 * j] = z[j];                         // (this wave's own array: LDS serves a wave in order)
+    all[lane + 64 * j] = z[j];
   }
   top = wave_max(top);
-  asm volatile("" ::: "memory");
-  __builtin_amdgcn_wave_barrier();
+  wave_lds_fence();
 #pragma unroll
   for (int i = 0; i < N; ++i) {
     const int n = p.experts - 64 * i < 64 ? p.experts - 64 * i : 64;
@@ -58,10 +105,10 @@ __device__ __forceinline__ void pick_experts(const RouteParams& p, int64_t t, fl
 #pragma unroll
   for (int j = 0; j < N; ++j) {
     const bool taken = place[j] < p.top && lane + 64 * j < p.experts;
-    e[j] = taken ? expf(z[j] - top) : 0.f;
+    e[j] = taken ? (p.sigmoid ? score[j] * p.scale : expf(z[j] - top)) : 0.f;
     sum += e[j];
   }
-  sum = wave_sum(sum);
+  sum = p.sigmoid ? 1.0f : wave_sum(sum);
 #pragma unroll
   for (int j = 0; j < N; ++j)
     if (place[j] < p.top && lane + 64 * j < p.experts) {
@@ -126,7 +173,7 @@ __global__ __launch_bounds__(64) void moe_route_slice_kernel(RouteParams p) {
 // A wave per token.
 template <int N>
 __global__ __launch_bounds__(256) void moe_route_pick_kernel(RouteParams p) {
-  __shared__ __attribute__((aligned(16))) float all[4][N * 64];
+  __shared__ __attribute__((aligned(16))) float all[4][2 * N * 64];
   const int lane = threadIdx.x & 63;
   const int64_t t = static_cast<int64_t>(blockIdx.x) * 4 + (threadIdx.x >> 6);
   if (t >= p.tokens) return;
@@ -149,7 +196,7 @@ __global__ __launch_bounds__(256) void moe_route_pick_kernel(RouteParams p) {
 template <typename T>
 __global__ __launch_bounds__(256) void moe_route_plain_kernel(RouteParams p) {
   __shared__ float logits[256];
-  __shared__ __attribute__((aligned(16))) float all[256];
+  __shared__ __attribute__((aligned(16))) float all[512];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int64_t t = blockIdx.x;
   const T* hr = static_cast<const T*>(p.h) + t * p.h_stride;
@@ -187,6 +234,7 @@ struct ExpertParams {
   void* out;              // [pairs, N]
   int64_t o_stride;
   int N, K, experts, div;
+  GluParams glu;
 };
 
 template <typename T, bool kUp>
@@ -206,7 +254,7 @@ __global__ __launch_bounds__(256) void experts_plain_kernel(ExpertParams p) {
       if (kUp) u += v * ld1(w1 + k);
     }
     a = wave_sum(a);
-    if (kUp) a = silu_f(a) * wave_sum(u);
+    if (kUp) a = glu<false>(p.glu, a, wave_sum(u));
     if (lane == 0) st1(static_cast<T*>(p.out) + i * p.o_stride + n, a);
   }
 }
@@ -216,13 +264,17 @@ __global__ __launch_bounds__(256) void experts_plain_kernel(ExpertParams p) {
 extern "C" {
 
 int sgl_amd_moe_route(int is_f32, const void* h, int64_t h_stride, const void* w, const float* bias, float* topk_weights, int32_t* topk_ids,
-                      float* partials, int slices, int pad, int64_t tokens, int K, int experts, int top, void* stream) {
+                      float* partials, int slices, int pad, int64_t tokens, int K, int experts, int top, int sigmoid, const float* correction,
+                      int groups, int keep, float scale, void* stream) {
   SGL_CLEAR_STALE_ERROR();
   SGL_CHECK_ARG(h && w && topk_weights && topk_ids && K > 0, "moe_route: null operand");
   SGL_CHECK_ARG(experts >= 1 && experts <= 256 && top >= 1 && top <= experts && top <= 64, "moe_route: %d of %d experts (at most 64 of 256)", top, experts);
   SGL_CHECK_ARG(tokens <= 0x7fffffffLL, "moe_route: too many tokens");
+  SGL_CHECK_ARG(!sigmoid || (groups >= 1 && experts % groups == 0 && keep >= 1 && keep <= groups && top <= keep * (experts / groups)),
+                "moe_route: %d of %d experts from %d of %d groups", top, experts, keep, groups);
   if (tokens <= 0) return 0;
-  RouteParams p{h, h_stride, w, bias, topk_weights, topk_ids, partials, tokens, K, experts, top, slices, pad};
+  RouteParams p{h, h_stride, w, bias, topk_weights, topk_ids, partials, tokens, K, experts, top, slices, pad,
+                sigmoid, correction, sigmoid ? experts / groups : experts, sigmoid ? groups : 1, sigmoid ? keep : 1, scale};
   hipStream_t st = as_stream(stream);
   if (partials) {
     const int nt = pad / 16;
@@ -245,12 +297,13 @@ int sgl_amd_moe_route(int is_f32, const void* h, int64_t h_stride, const void* w
 }
 
 int sgl_amd_experts_plain(int is_f32, int up, const void* x, int64_t x_stride, const void* w, const int32_t* ids, void* out, int64_t o_stride,
-                          int64_t pairs, int top, int N, int K, int experts, void* stream) {
+                          int64_t pairs, int top, int N, int K, int experts, int glu_kind, float glu_limit, float glu_alpha, void* stream) {
   SGL_CLEAR_STALE_ERROR();
+  SGL_CHECK_ARG(!up || (glu_kind > kGluNone && glu_kind < kGluKinds), "experts_plain: no activation %d", glu_kind);
   SGL_CHECK_ARG(x && w && ids && out && N > 0 && K > 0 && experts > 0 && top > 0 && pairs <= 0x7fffffffLL && (N + 31) / 32 <= 65535,
                 "experts_plain: %d experts of %d x %d", experts, N, K);
   if (pairs <= 0) return 0;
-  ExpertParams p{x, x_stride, w, ids, out, o_stride, N, K, experts, up ? top : 1};
+  ExpertParams p{x, x_stride, w, ids, out, o_stride, N, K, experts, up ? top : 1, GluParams{glu_kind, glu_limit, glu_alpha}};
   const dim3 grid(static_cast<unsigned>(pairs), (N + 31) / 32);
   hipStream_t st = as_stream(stream);
   if (is_f32) {

@@ -30,6 +30,7 @@
 // keeps the 32 workgroups an XCD runs at a time on a 4 (row blocks) x 8 (column tiles) patch of the output, so that its
 // L2 fetches 12 operand tiles per step for 32 workgroups.  Same contract, same rounding points, same epilogues.
 #include "common.hpp"
+#include "glu.hpp"
 #include "sglang_amd.h"
 
 using namespace sgl_amd;
@@ -57,7 +58,8 @@ struct TiledParams {
   const float* row_scale;       // optional [num_valid_ids]
   int64_t a_stride, w_row_stride, w_expert_stride, c_stride;
   int num_valid, N, K, topk_div;
-  int fuse_silu, out_f32, round_before_scale;
+  int fuse_silu, out_f32, round_before_scale;      // (fuse_silu: any gated activation, `glu`)
+  GluParams glu;
   int eid_shift;                // expert_ids is indexed by (row block >> eid_shift): 128-row tiles over a 256-row alignment
   int n_tiles;                  // 256-form: output-column tiles (its grid is one-dimensional)
 };
@@ -184,9 +186,7 @@ __global__ __launch_bounds__(kThreads, 2) void moe_tiled_gemm_kernel(TiledParams
         float o[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const float gb = rbf(acc[i][j][r]);
-          const float sl = rbf(gb / (1.0f + expf(-gb)));
-          o[r] = sl * rbf(acc[i + 2][j][r]);
+          o[r] = glu<true>(p.glu, acc[i][j][r], acc[i + 2][j][r]);
         }
         uint2 w2;
         w2.x = pack_bf2(o[0], o[1]); w2.y = pack_bf2(o[2], o[3]);
@@ -504,9 +504,7 @@ __global__ __launch_bounds__(kThreads2, 1) void moe_gemm256_kernel(TiledParams p
         float o[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const float gb = rbf(acc[i][j][r]);
-          const float sl = rbf(gb / (1.0f + expf(-gb)));
-          o[r] = sl * rbf(acc[i + 4][j][r]);
+          o[r] = glu<true>(p.glu, acc[i][j][r], acc[i + 4][j][r]);
         }
         uint2 w2;
         w2.x = pack_bf2(o[0], o[1]); w2.y = pack_bf2(o[2], o[3]);
@@ -548,15 +546,17 @@ int sgl_amd_moe_tiled_gemm(const void* a, const void* w, void* c, const int32_t*
                            int64_t max_m_blocks, int fuse_silu, int out_f32, void* stream) {
   return sgl_amd_moe_tiled_gemm_ex(a, w, c, sorted_token_ids, expert_ids, num_tokens_post_padded, topk_weights, mul_routed_weight,
                                    round_before_scale, top_k_div, num_valid_ids, N, K, a_row_stride, w_row_stride, w_expert_stride,
-                                   c_row_stride, max_m_blocks, fuse_silu, out_f32, kBM, kBM, stream);
+                                   c_row_stride, max_m_blocks, fuse_silu ? kGluSilu : kGluNone, 0.f, 0.f, out_f32, kBM, kBM, stream);
 }
 
 int sgl_amd_moe_tiled_gemm_ex(const void* a, const void* w, void* c, const int32_t* sorted_token_ids, const int32_t* expert_ids,
                               const int32_t* num_tokens_post_padded, const float* topk_weights, int mul_routed_weight,
                               int round_before_scale, int top_k_div, int64_t num_valid_ids, int64_t N, int64_t K,
                               int64_t a_row_stride, int64_t w_row_stride, int64_t w_expert_stride, int64_t c_row_stride,
-                              int64_t max_m_blocks, int fuse_silu, int out_f32, int align_block_m, int tile_rows, void* stream) {
+                              int64_t max_m_blocks, int glu_kind, float glu_limit, float glu_alpha, int out_f32, int align_block_m, int tile_rows, void* stream) {
   SGL_CLEAR_STALE_ERROR();
+  SGL_CHECK_ARG(glu_kind >= kGluNone && glu_kind < kGluKinds, "moe_tiled_gemm: no activation %d", glu_kind);
+  const int fuse_silu = glu_kind != kGluNone;
   SGL_CHECK_ARG((align_block_m == 128 || align_block_m == 256) && (tile_rows == 128 || tile_rows == 256) && tile_rows <= align_block_m,
                 "moe_tiled_gemm: align_block_m / tile_rows must be 128 or 256, tile_rows <= align_block_m (got %d / %d)", align_block_m, tile_rows);
   SGL_CHECK_ARG(N > 0 && N % 4 == 0 && K >= kBK && K % kBK == 0, "moe_tiled_gemm: need N %% 4 == 0 and K %% %d == 0 (got N=%lld K=%lld)",
@@ -574,7 +574,7 @@ int sgl_amd_moe_tiled_gemm_ex(const void* a, const void* w, void* c, const int32
   p.row_scale = mul_routed_weight ? topk_weights : nullptr;
   p.a_stride = a_row_stride; p.w_row_stride = w_row_stride; p.w_expert_stride = w_expert_stride; p.c_stride = c_row_stride;
   p.num_valid = static_cast<int>(num_valid_ids); p.N = static_cast<int>(N); p.K = static_cast<int>(K); p.topk_div = top_k_div;
-  p.fuse_silu = fuse_silu; p.out_f32 = out_f32; p.round_before_scale = round_before_scale;
+  p.fuse_silu = fuse_silu; p.glu = GluParams{glu_kind, glu_limit, glu_alpha}; p.out_f32 = out_f32; p.round_before_scale = round_before_scale;
   if (tile_rows == 256) {
     // one-dimensional grid of patches: 4 row blocks x 8 column tiles each, eight patches (one per XCD) per 256 workgroups
     const int cols = fuse_silu ? 128 : 256;

@@ -5,12 +5,13 @@
 //                   The residual row lives in fp32 and is in registers for both norms.
 //   residual_rms    the same step of pre-norm designs with RMS norms:  x <- embedding (+ position row), or x + up to two sublayer
 //                   outputs (rows, split-K partials, or weighted expert rows), then a saved copy, then + rows + vector in front
-//                   of a looped pass, then h = RMS norm(x)
+//                   of a looped pass, then h = RMS norm(x).  Post-norm designs: x + mult * RMS norm(sum of the outputs), h = x
 //   soft_cap        cap * tanh(z / cap) on logits, fp32 out
 //   gated_rmsnorm   RMS norm of equal column groups with a silu gate, the gate before the norm (Mamba-2) or behind it
 //                   (gated delta rule).
 //   gate_mul        act(a) * b for activation types / alignments outside silu_and_mul's bf16 form.
 #include "elem_io.hpp"
+#include "glu.hpp"
 #include "sglang_amd.h"
 
 using namespace sgl_amd;
@@ -231,7 +232,9 @@ struct ResidualRmsParams {
   float* save;              // optional fp32 copy of x as it is here
   const float* extra;       // optional fp32 rows, added behind the copy (the stride of `save` / `extra` is W)
   const float* step;        // optional [W], added last
-  const float* w;           // [W]
+  const float* post;        // optional [W]: x = x + mult * (RMS norm(a + b) * post)
+  float mult;
+  const float* w;           // [W]; null: h is the new x itself
   void* h;                  // RMS norm of the new x (may be null)
   int64_t h_stride;
   int64_t rows;
@@ -324,7 +327,12 @@ __global__ __launch_bounds__(kWaveRow ? 256 : 1024) void residual_rms_kernel(Res
 #pragma unroll
     for (int i = 0; i < kItems; ++i) {
       const int c = (i * tpr + lane) * VEC;
-      if (c < W) ldv<VEC>(xr + c, v[i]);
+      if (p.post) {
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) v[i][j] = 0.f;
+      } else if (c < W) {
+        ldv<VEC>(xr + c, v[i]);
+      }
     }
     if constexpr (kItems == 1) {
       if (lane * VEC < W) {
@@ -334,6 +342,28 @@ __global__ __launch_bounds__(kWaveRow ? 256 : 1024) void residual_rms_kernel(Res
     } else {
       if (p.a.data) add_source_row<T, VEC, kItems>(p.a, row, lane, tpr, W, v);
       if (p.b.data) add_source_row<T, VEC, kItems>(p.b, row, lane, tpr, W, v);
+    }
+    if (p.post) {
+      float sq = 0.f;
+#pragma unroll
+      for (int i = 0; i < kItems; ++i)
+        if ((i * tpr + lane) * VEC < W) {
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) sq += v[i][j] * v[i][j];
+        }
+      sq = kWaveRow ? wave_sum(sq) : block_sum(sq, scratch);
+      const float f = p.mult / sqrtf(sq / static_cast<float>(W) + p.eps);
+#pragma unroll
+      for (int i = 0; i < kItems; ++i) {
+        const int c = (i * tpr + lane) * VEC;
+        if (c < W) {
+          float wv[VEC], old[VEC];
+          ldv<VEC>(p.post + c, wv);
+          ldv<VEC>(xr + c, old);
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) v[i][j] = old[j] + v[i][j] * f * wv[j];
+        }
+      }
     }
   }
   float ss = 0.f;
@@ -359,9 +389,17 @@ __global__ __launch_bounds__(kWaveRow ? 256 : 1024) void residual_rms_kernel(Res
     }
   }
   if (!p.h) return;
+  T* hr = static_cast<T*>(p.h) + row * p.h_stride;
+  if (!p.w) {
+#pragma unroll
+    for (int i = 0; i < kItems; ++i) {
+      const int c = (i * tpr + lane) * VEC;
+      if (c < W) stv<VEC>(hr + c, v[i]);
+    }
+    return;
+  }
   ss = kWaveRow ? wave_sum(ss) : block_sum(ss, scratch);
   const float rs = 1.0f / sqrtf(ss / static_cast<float>(W) + p.eps);
-  T* hr = static_cast<T*>(p.h) + row * p.h_stride;
 #pragma unroll
   for (int i = 0; i < kItems; ++i) {
     const int c = (i * tpr + lane) * VEC;
@@ -501,10 +539,10 @@ void launch_gated(const GatedNormParams& p, hipStream_t st) {
 // ---------------------------------------------------------------------------------------------------------------
 template <typename T>
 __global__ __launch_bounds__(256) void gate_mul_kernel(const T* __restrict__ a, const T* __restrict__ b, T* __restrict__ out, int d,
-                                                       int64_t in_stride, int64_t out_stride) {
+                                                       int64_t in_stride, int64_t out_stride, GluParams act) {
   const int64_t row = blockIdx.y;
   const int c = blockIdx.x * 256 + threadIdx.x;
-  if (c < d) st1(out + row * out_stride + c, silu_f(ld1(a + row * in_stride + c)) * ld1(b + row * in_stride + c));
+  if (c < d) st1(out + row * out_stride + c, glu<false>(act, ld1(a + row * in_stride + c), ld1(b + row * in_stride + c)));
 }
 
 }  // namespace
@@ -539,22 +577,23 @@ int sgl_amd_residual_rms(int is_f32, const int64_t* ids, const void* table, int6
                          const void* pos_table, int64_t max_positions, const void* a, int a_f32, int a_items, int64_t a_row_stride,
                          int64_t a_item_stride, const float* a_weight, const void* b, int b_f32, int b_items, int64_t b_row_stride,
                          int64_t b_item_stride, const float* b_weight, float* x, int64_t x_stride, float* save, const float* extra,
-                         const float* step, const float* weight, void* h, int64_t h_stride, int64_t rows, int width, float eps, void* stream) {
+                         const float* step, const float* post, float mult, const float* weight, void* h, int64_t h_stride, int64_t rows, int width,
+                         float eps, void* stream) {
   SGL_CLEAR_STALE_ERROR();
   SGL_CHECK_ARG(width > 0 && width <= 16384, "residual_rms: width %d outside 1..16384", width);
   SGL_CHECK_ARG(x && (!ids || (table && vocab > 0 && !a && !b)) && (!pos_table || (ids && positions && max_positions > 0)),
                 "residual_rms: missing operand, or an embedding beside sublayer outputs");
-  SGL_CHECK_ARG((!a || a_items >= 1) && (!b || b_items >= 1) && (!h || weight), "residual_rms: empty source, or h without its norm");
+  SGL_CHECK_ARG((!a || a_items >= 1) && (!b || b_items >= 1) && (!post || a), "residual_rms: empty source, or a norm behind none");
   SGL_CHECK_ARG(rows <= 0x7fffffffLL, "residual_rms: too many rows");
   if (rows <= 0) return 0;
   ResidualRmsParams p{ids, table, vocab, scale, positions, pos_table, max_positions, {a, is_f32 || a_f32, a_items, a_row_stride, a_item_stride, a_weight},
-                      {b, is_f32 || b_f32, b_items, b_row_stride, b_item_stride, b_weight}, x, x_stride, save, extra, step, weight, h, h_stride, rows,
+                      {b, is_f32 || b_f32, b_items, b_row_stride, b_item_stride, b_weight}, x, x_stride, save, extra, step, post, mult, weight, h, h_stride, rows,
                       width, eps};
   const size_t al = is_f32 ? 16 : 8;
   const bool vec = width % 4 == 0 && x_stride % 4 == 0 && h_stride % 4 == 0 && a_row_stride % 4 == 0 && a_item_stride % 4 == 0 &&
                    b_row_stride % 4 == 0 && b_item_stride % 4 == 0 && aligned_to(table, al) && aligned_to(pos_table, al) &&
                    aligned_to(a, p.a.f32 ? 16 : 8) && aligned_to(b, p.b.f32 ? 16 : 8) && aligned_to(h, al) && aligned_to(x, 16) &&
-                   aligned_to(save, 16) && aligned_to(extra, 16) && aligned_to(step, 16) && aligned_to(weight, 16);
+                   aligned_to(save, 16) && aligned_to(extra, 16) && aligned_to(step, 16) && aligned_to(post, 16) && aligned_to(weight, 16);
   const bool vec8 = vec && width % 8 == 0 && h_stride % 8 == 0 && a_row_stride % 8 == 0 && a_item_stride % 8 == 0 && b_row_stride % 8 == 0 &&
                     b_item_stride % 8 == 0 && aligned_to(table, 16) && aligned_to(pos_table, 16) && aligned_to(a, 16) && aligned_to(b, 16) && aligned_to(h, 16);
   if (is_f32) launch_residual_rms<float>(p, vec, vec8, as_stream(stream));
@@ -593,18 +632,20 @@ int sgl_amd_gated_rmsnorm(int is_f32, const void* y, int64_t y_stride, const voi
 }
 
 int sgl_amd_gate_mul(int is_f32, const void* gate, const void* up, void* out, int64_t rows, int d, int64_t in_stride, int64_t out_stride,
-                     void* stream) {
+                     int glu_kind, float glu_limit, float glu_alpha, void* stream) {
   SGL_CLEAR_STALE_ERROR();
+  SGL_CHECK_ARG(glu_kind > kGluNone && glu_kind < kGluKinds, "gate_mul: no activation %d", glu_kind);
+  const GluParams act{glu_kind, glu_limit, glu_alpha};
   SGL_CHECK_ARG(gate && up && out && d > 0, "gate_mul: null operand or empty rows");
   SGL_CHECK_ARG(rows <= 65535, "gate_mul: at most 65535 rows per call (got %lld)", (long long)rows);
   if (rows <= 0) return 0;
   const dim3 grid((d + 255) / 256, static_cast<unsigned>(rows));
   if (is_f32)
     hipLaunchKernelGGL((gate_mul_kernel<float>), grid, dim3(256), 0, as_stream(stream), static_cast<const float*>(gate),
-                       static_cast<const float*>(up), static_cast<float*>(out), d, in_stride, out_stride);
+                       static_cast<const float*>(up), static_cast<float*>(out), d, in_stride, out_stride, act);
   else
     hipLaunchKernelGGL((gate_mul_kernel<uint16_t>), grid, dim3(256), 0, as_stream(stream), static_cast<const uint16_t*>(gate),
-                       static_cast<const uint16_t*>(up), static_cast<uint16_t*>(out), d, in_stride, out_stride);
+                       static_cast<const uint16_t*>(up), static_cast<uint16_t*>(out), d, in_stride, out_stride, act);
   SGL_CHECK_LAUNCH("gate_mul");
   return 0;
 }

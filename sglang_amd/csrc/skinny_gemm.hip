@@ -29,6 +29,7 @@
 //     epilogue with the same bf16 rounding points as the unfused torch ops.
 #include <cstdlib>
 #include "common.hpp"
+#include "glu.hpp"
 #include "sglang_amd.h"
 
 using namespace sgl_amd;
@@ -65,6 +66,7 @@ struct SkinnyParams {
   int splits;
   int out_f32;
   int round_before_scale;       // grouped: round the accumulator to bf16 before the router weight
+  GluParams glu;                // FUSE: what becomes of a gate and an up column
 };
 
 // Columns per workgroup: each of the 4 waves owns NTW 16-column tiles (FUSE: one gate + one up tile).
@@ -112,11 +114,8 @@ __device__ __forceinline__ void epilogue(const SkinnyParams& p, f32x4_t (&acc)[N
       for (int r = 0; r < 4; ++r) {
         float v;
         if (FUSE) {
-          // torch: gate_up = linear(x) (bf16) -> silu(gate) (bf16) -> * up (bf16)
-          const float gt = rbf(acc[0][mt][r]);
-          const float up = rbf(acc[NTW - 1][mt][r]);
-          const float sl = rbf(gt / (1.0f + expf(-gt)));
-          v = sl * up;
+          // silu as torch rounds it: gate_up = linear(x) (bf16) -> silu(gate) (bf16) -> * up (bf16)
+          v = glu<true>(p.glu, acc[0][mt][r], acc[NTW - 1][mt][r]);
         } else {
           v = acc[nt][mt][r] + bias4[r];
         }
@@ -400,6 +399,7 @@ int sgl_amd_skinny_gemm(const void* x, const void* w, const void* bias, void* y,
   p.x_stride = x_row_stride; p.w_stride = w_row_stride; p.w_expert_stride = 0; p.y_stride = y_row_stride;
   p.M = static_cast<int>(M); p.N = static_cast<int>(N); p.K = static_cast<int>(K);
   p.topk_div = 1; p.splits = num_k_splits; p.out_f32 = 0; p.round_before_scale = 0;
+  p.glu.kind = kGluSilu;
   dispatch<false>(p, static_cast<int>((M + 15) / 16), 1, fuse_silu, tiles_per_wave, as_stream(stream));
   SGL_CHECK_LAUNCH("skinny_gemm");
   return 0;
@@ -410,7 +410,7 @@ int sgl_amd_moe_grouped_gemm(const void* a, const void* w, void* c, const int32_
                              const float* topk_weights, int mul_routed_weight, int round_before_scale,
                              int top_k_div, int64_t num_valid_ids, int64_t N, int64_t K, int64_t num_experts,
                              int64_t a_row_stride, int64_t w_row_stride, int64_t w_expert_stride,
-                             int64_t c_row_stride, int block_m, int64_t max_m_blocks, int fuse_silu, int out_f32,
+                             int64_t c_row_stride, int block_m, int64_t max_m_blocks, int glu_kind, float glu_limit, float glu_alpha, int out_f32,
                              int tiles_per_wave, int num_k_splits, void* ws_slabs, void* stream) {
   SGL_CLEAR_STALE_ERROR();
   SGL_CHECK_ARG(block_m == 16 || block_m == 32 || block_m == 48 || block_m == 64,
@@ -419,6 +419,7 @@ int sgl_amd_moe_grouped_gemm(const void* a, const void* w, void* c, const int32_
   SGL_CHECK_ARG(top_k_div >= 1 && num_experts >= 1, "moe_grouped_gemm: bad top_k_div / num_experts");
   SGL_CHECK_ARG(!mul_routed_weight || topk_weights, "moe_grouped_gemm: mul_routed_weight needs topk_weights");
   SGL_CHECK_ARG(max_m_blocks <= 65535, "moe_grouped_gemm: too many row blocks (%lld)", (long long)max_m_blocks);
+  SGL_CHECK_ARG(glu_kind >= kGluNone && glu_kind < kGluKinds, "moe_grouped_gemm: no activation %d", glu_kind);
   if (max_m_blocks == 0 || num_valid_ids == 0) return 0;
   SkinnyParams p{};
   p.x = static_cast<const uint16_t*>(a);
@@ -431,7 +432,8 @@ int sgl_amd_moe_grouped_gemm(const void* a, const void* w, void* c, const int32_
   p.x_stride = a_row_stride; p.w_stride = w_row_stride; p.w_expert_stride = w_expert_stride; p.y_stride = c_row_stride;
   p.M = static_cast<int>(num_valid_ids); p.N = static_cast<int>(N); p.K = static_cast<int>(K);
   p.topk_div = top_k_div; p.splits = num_k_splits; p.out_f32 = out_f32; p.round_before_scale = round_before_scale;
-  dispatch<true>(p, block_m / 16, static_cast<int>(max_m_blocks), fuse_silu, tiles_per_wave, as_stream(stream));
+  p.glu = GluParams{glu_kind, glu_limit, glu_alpha};
+  dispatch<true>(p, block_m / 16, static_cast<int>(max_m_blocks), glu_kind, tiles_per_wave, as_stream(stream));
   SGL_CHECK_LAUNCH("moe_grouped_gemm");
   return 0;
 }

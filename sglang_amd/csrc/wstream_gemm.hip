@@ -24,6 +24,7 @@
 //     split order (deterministic) and applies the epilogue the next operator would have been:
 //     bias, silu(gate)*up, or residual-add + RMSNorm, with the torch-native bf16 rounding points.
 #include "common.hpp"
+#include "glu.hpp"
 #include "kv_format.hpp"
 #include "sglang_amd.h"
 
@@ -205,6 +206,7 @@ struct WsParams {
                                 // 2 GiB and more (32-bit buffer offsets)
   int pair_silu;                // 1: two-tile waves, y[:, 16 t ..] = silu(tile t) * tile (t + ntiles/2) instead of two outputs;
                                 // 2: one-tile waves whose 16 weight rows are [8 gate rows | 8 up rows] of output columns 8 t .. 8 t + 7
+  GluParams glu;                // the activation of the paired forms (silu in their names, or another kind)
 };
 
 // ---- LDS-DMA plumbing ------------------------------------------------------------------------
@@ -513,9 +515,7 @@ __global__ __launch_bounds__(64 * NW, 1) void wstream_gemm_kernel(WsParams p) {
           gv += bf2f(p.bias[c]);
           uv += bf2f(p.bias[p.N / 2 + c]);
         }
-        const float gb = rbf(gv);
-        const float sl = rbf(gb / (1.0f + expf(-gb)));
-        o[r] = sl * rbf(uv);
+        o[r] = glu<true>(p.glu, gv, uv);
       }
       if (g < 2) put(o, tile * 8 + g * 4, false);
       continue;
@@ -530,9 +530,7 @@ __global__ __launch_bounds__(64 * NW, 1) void wstream_gemm_kernel(WsParams p) {
           gv += bf2f(p.bias[n0 + r]);
           uv += bf2f(p.bias[p.N / 2 + n0 + r]);
         }
-        const float gb = rbf(gv);
-        const float sl = rbf(gb / (1.0f + expf(-gb)));
-        o[r] = sl * rbf(uv);
+        o[r] = glu<true>(p.glu, gv, uv);
       }
       put(o, n0, false);
       continue;
@@ -577,6 +575,7 @@ struct CombineParams {
   int64_t y_stride, y_cstride, res_stride;
   int M, N, splits;
   float eps;
+  GluParams glu;
 };
 
 __global__ __launch_bounds__(256) void wstream_combine_kernel(CombineParams p) {
@@ -607,9 +606,7 @@ __global__ __launch_bounds__(256) void wstream_combine_silu_kernel(CombineParams
   float o[4];
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
-    const float gb = rbf(p.bias ? gt[r] + bf2f(p.bias[j0 + r]) : gt[r]);
-    const float sl = rbf(gb / (1.0f + expf(-gb)));
-    o[r] = sl * rbf(p.bias ? up[r] + bf2f(p.bias[half + j0 + r]) : up[r]);
+    o[r] = glu<true>(p.glu, p.bias ? gt[r] + bf2f(p.bias[j0 + r]) : gt[r], p.bias ? up[r] + bf2f(p.bias[half + j0 + r]) : up[r]);
   }
   uint2 w2;
   w2.x = pack_bf2(o[0], o[1]);
@@ -773,7 +770,8 @@ int64_t sgl_amd_wstream_gemm_workspace_floats(int64_t M, int64_t N, int num_k_sp
 static int wstream_launch_main(const char* who, const void* x, const void* w, const void* bias, void* y, int64_t M, int64_t N,
                                int64_t K, int64_t x_row_stride, int64_t x_chunk_stride, int64_t w_row_stride,
                                int64_t y_row_stride, int64_t y_chunk_stride, bool fused_silu, int tiles_per_wave,
-                               bool to_partials, int waves_per_group, int num_k_splits, void* ws_partials, hipStream_t st) {
+                               bool to_partials, int waves_per_group, int num_k_splits, void* ws_partials, hipStream_t st,
+                               GluParams act = GluParams{kGluSilu, 0.f, 0.f}) {
   SGL_CHECK_ARG(M >= 1 && M <= 128, "%s: M=%lld rows (supported: 1..128)", who, (long long)M);
   SGL_CHECK_ARG(N > 0 && N % 16 == 0 && K >= kKC && K % kKC == 0,
                 "%s: need N %% 16 == 0 and K %% %d == 0 (got N=%lld K=%lld)", who, kKC, (long long)N, (long long)K);
@@ -802,6 +800,7 @@ static int wstream_launch_main(const char* who, const void* x, const void* w, co
   p.M = static_cast<int>(M); p.N = static_cast<int>(N); p.K = static_cast<int>(K);
   p.splits = num_k_splits; p.ntiles = static_cast<int>(N / 16);
   p.pair_silu = fused_silu ? (two_tiles ? 1 : 2) : 0;
+  p.glu = act;
   p.dbg = g_ws_debug_flags;
   if (static_cast<int64_t>(num_k_splits) * M * N * 4 >= (int64_t{1} << 31)) p.dbg |= 2;
   int rc;
@@ -817,11 +816,11 @@ static int wstream_launch_main(const char* who, const void* x, const void* w, co
   return 0;
 }
 
-int sgl_amd_wstream_gemm(const void* x, const void* w, const void* bias, void* y, int64_t M, int64_t N, int64_t K,
-                         int64_t x_row_stride, int64_t x_chunk_stride, int64_t w_row_stride, int64_t y_row_stride,
-                         int64_t y_chunk_stride, int epilogue, void* residual, int64_t residual_row_stride,
-                         const void* norm_weight, float eps, int waves_per_group, int tiles_per_wave, int num_k_splits,
-                         void* ws_partials, void* stream) {
+static int wstream_gemm_impl(const void* x, const void* w, const void* bias, void* y, int64_t M, int64_t N, int64_t K,
+                             int64_t x_row_stride, int64_t x_chunk_stride, int64_t w_row_stride, int64_t y_row_stride,
+                             int64_t y_chunk_stride, int epilogue, GluParams act, void* residual, int64_t residual_row_stride,
+                             const void* norm_weight, float eps, int waves_per_group, int tiles_per_wave, int num_k_splits,
+                             void* ws_partials, void* stream) {
   SGL_CLEAR_STALE_ERROR();
   if (M == 0) return 0;
   SGL_CHECK_ARG(epilogue >= 0 && epilogue <= 3, "wstream_gemm: epilogue must be 0 (bias), 1 (silu_and_mul), 2 (add_rmsnorm) or 3 (partials)");
@@ -835,7 +834,7 @@ int sgl_amd_wstream_gemm(const void* x, const void* w, const void* bias, void* y
   SGL_CHECK_ARG(y_chunk_stride == 0 || (epilogue == 1 ? N % 256 == 0 : N % 128 == 0),
                 "wstream_gemm: a chunk-major y needs whole 128-column blocks");
   if (int rc = wstream_launch_main("wstream_gemm", x, w, bias, y, M, N, K, x_row_stride, x_chunk_stride, w_row_stride, y_row_stride,
-                                   y_chunk_stride, fused_silu, tiles_per_wave, combine, waves_per_group, num_k_splits, ws_partials, st))
+                                   y_chunk_stride, fused_silu, tiles_per_wave, combine, waves_per_group, num_k_splits, ws_partials, st, act))
     return rc;
   if (combine && epilogue != 3) {
     CombineParams c{};
@@ -843,6 +842,7 @@ int sgl_amd_wstream_gemm(const void* x, const void* w, const void* bias, void* y
     c.residual = static_cast<uint16_t*>(residual); c.norm_w = static_cast<const uint16_t*>(norm_weight);
     c.y_stride = y_row_stride; c.y_cstride = y_chunk_stride ? y_chunk_stride : 128; c.res_stride = residual_row_stride;
     c.M = static_cast<int>(M); c.N = static_cast<int>(N); c.splits = num_k_splits; c.eps = eps;
+    c.glu = act;
     if (epilogue == 0) {
       hipLaunchKernelGGL(wstream_combine_kernel, dim3((c.N / 4 + 255) / 256, c.M), dim3(256), 0, st, c);
     } else if (epilogue == 1) {
@@ -855,13 +855,35 @@ int sgl_amd_wstream_gemm(const void* x, const void* w, const void* bias, void* y
   return 0;
 }
 
+int sgl_amd_wstream_gemm(const void* x, const void* w, const void* bias, void* y, int64_t M, int64_t N, int64_t K,
+                         int64_t x_row_stride, int64_t x_chunk_stride, int64_t w_row_stride, int64_t y_row_stride,
+                         int64_t y_chunk_stride, int epilogue, void* residual, int64_t residual_row_stride,
+                         const void* norm_weight, float eps, int waves_per_group, int tiles_per_wave, int num_k_splits,
+                         void* ws_partials, void* stream) {
+  return wstream_gemm_impl(x, w, bias, y, M, N, K, x_row_stride, x_chunk_stride, w_row_stride, y_row_stride, y_chunk_stride, epilogue,
+                           GluParams{kGluSilu, 0.f, 0.f}, residual, residual_row_stride, norm_weight, eps, waves_per_group, tiles_per_wave,
+                           num_k_splits, ws_partials, stream);
+}
+
+int sgl_amd_wstream_glu_gemm(const void* x, const void* w, const void* bias, void* y, int64_t M, int64_t N, int64_t K, int64_t x_row_stride,
+                             int64_t x_chunk_stride, int64_t w_row_stride, int64_t y_row_stride, int64_t y_chunk_stride, int glu_kind,
+                             float glu_limit, float glu_alpha, int waves_per_group, int tiles_per_wave, int num_k_splits,
+                             void* ws_partials, void* stream) {
+  SGL_CHECK_ARG(glu_kind > kGluNone && glu_kind < kGluKinds, "wstream_glu_gemm: no activation %d", glu_kind);
+  return wstream_gemm_impl(x, w, bias, y, M, N, K, x_row_stride, x_chunk_stride, w_row_stride, y_row_stride, y_chunk_stride, 1,
+                           GluParams{glu_kind, glu_limit, glu_alpha}, nullptr, 0, nullptr, 0.f, waves_per_group, tiles_per_wave,
+                           num_k_splits, ws_partials, stream);
+}
+
 int sgl_amd_wstream_moe_gemm(const void* a, const void* w, void* c, const int32_t* sorted_token_ids,
                              const int32_t* expert_ids, const int32_t* num_tokens_post_padded,
                              const float* topk_weights, int mul_routed_weight, int round_before_scale, int top_k_div,
                              int64_t num_valid_ids, int64_t N, int64_t K, int64_t a_row_stride, int64_t w_row_stride,
                              int64_t w_expert_stride, int64_t c_row_stride, int block_m, int64_t max_m_blocks,
-                             int fuse_silu, int out_f32, int waves_per_group, void* stream) {
+                             int glu_kind, float glu_limit, float glu_alpha, int out_f32, int waves_per_group, void* stream) {
   SGL_CLEAR_STALE_ERROR();
+  SGL_CHECK_ARG(glu_kind >= kGluNone && glu_kind < kGluKinds, "wstream_moe_gemm: no activation %d", glu_kind);
+  const int fuse_silu = glu_kind != kGluNone;
   SGL_CHECK_ARG(block_m == 16 || block_m == 32 || block_m == 48 || block_m == 64,
                 "wstream_moe_gemm: block_m=%d (supported: 16/32/48/64, must equal the moe_align block size)", block_m);
   const int64_t wn = fuse_silu ? 2 * N : N;             // weight rows per expert
@@ -887,6 +909,7 @@ int sgl_amd_wstream_moe_gemm(const void* a, const void* w, void* c, const int32_
   p.row_scale = mul_routed_weight ? topk_weights : nullptr;
   p.topk_div = top_k_div; p.out_f32 = out_f32; p.round_before_scale = round_before_scale;
   p.pair_silu = fuse_silu ? 1 : 0;
+  p.glu = GluParams{glu_kind, glu_limit, glu_alpha};
   hipStream_t st = as_stream(stream);
   const int blocks = static_cast<int>(max_m_blocks);
   int rc;

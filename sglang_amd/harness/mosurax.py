@@ -23,7 +23,7 @@ from ..mem_cache.memory_pool import GroupedTokenToKVPool, ReqToTokenPool
 from .layered import LayeredConfig
 
 BF = torch.bfloat16
-MIXERS = {"attention": partial(GroupedAttention, sink=0.0, gated=True)}
+MIXERS = {"attention": partial(GroupedAttention, sink=0.0, gate="elements")}
 
 
 @dataclass

@@ -5,15 +5,16 @@ import json
 from pathlib import Path
 from typing import Any, Callable, Dict
 
-from . import genusun, models, mosurax
+from . import bulodra, genusun, models, mosurax
 
 # config.json "architecture" -> reader of the file
-ARCHITECTURES: Dict[str, Callable[[dict, str], Any]] = {"Genusun": genusun.GenusunConfig.from_dict, "Mosurax": mosurax.MosuraxConfig.from_dict}
+ARCHITECTURES: Dict[str, Callable[[dict, str], Any]] = {"Genusun": genusun.GenusunConfig.from_dict, "Mosurax": mosurax.MosuraxConfig.from_dict,
+                                                        "Bulodra": bulodra.BulodraConfig.from_dict}
 _MODELS = {models.ModelConfig: models.CausalLM, genusun.GenusunConfig: genusun.GenusunForCausalLM,
-           mosurax.MosuraxConfig: mosurax.MosuraxForCausalLM}
+           mosurax.MosuraxConfig: mosurax.MosuraxForCausalLM, bulodra.BulodraConfig: bulodra.BulodraForCausalLM}
 # HIP units (sglang_amd/csrc) a model's path needs; a model that is not listed uses the whole library
-_UNITS = {genusun.GenusunConfig: "hybrid", mosurax.MosuraxConfig: "grouped"}
-_NAMED = (models.CONFIGS, genusun.CONFIGS, mosurax.CONFIGS)
+_UNITS = {genusun.GenusunConfig: "hybrid", mosurax.MosuraxConfig: "grouped", bulodra.BulodraConfig: "layered"}
+_NAMED = (models.CONFIGS, genusun.CONFIGS, mosurax.CONFIGS, bulodra.CONFIGS)
 
 
 def model_class(config):

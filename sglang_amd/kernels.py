@@ -105,6 +105,30 @@ def silu_and_mul(x: torch.Tensor, out: Optional[torch.Tensor] = None, round_inte
 
 
 # --------------------------------------------------------------------------- rope
+class Glu:
+    """A gated activation of (gate, up) columns: 'silu' g sigmoid(g) u, 'gelu_tanh' gelu_tanh(g) u, or 'clamped_swish' g' sigmoid(alpha g')
+    (u' + 1) with g' = min(g, limit) and u' = u clamped to +- limit."""
+
+    KINDS = {"silu": 1, "gelu_tanh": 2, "clamped_swish": 3}
+
+    def __init__(self, kind: str = "silu", limit: float = 0.0, alpha: float = 0.0):
+        self.kind, self.args = kind, (self.KINDS[kind], float(limit), float(alpha))
+
+
+SILU = Glu()
+NO_GLU = (0, 0.0, 0.0)
+
+
+def glu_and_mul(x: torch.Tensor, act: Glu) -> torch.Tensor:
+    """act(x[:, :d], x[:, d:]) of bf16 rows, in fp32 up to the result."""
+    _dev(x)
+    d = x.shape[1] // 2
+    _need(x.dtype == _BF16 and x.dim() == 2 and x.stride(1) == 1, "glu_and_mul: bf16 rows")
+    out = torch.empty((x.shape[0], d), dtype=_BF16, device=x.device)
+    native.call("sgl_amd_glu_and_mul", x.data_ptr(), out.data_ptr(), x.shape[0], d, x.stride(0), d, *act.args, _stream())
+    return out
+
+
 def rotary_embedding(positions: torch.Tensor, query: torch.Tensor, key: torch.Tensor, head_size: int,
                      cos_sin_cache: torch.Tensor, is_neox: bool = True,
                      value: Optional[torch.Tensor] = None, k_cache: Optional[torch.Tensor] = None,
@@ -232,6 +256,24 @@ def clamp_position(seq_lens: torch.Tensor, out: Optional[torch.Tensor] = None) -
     native.call("sgl_amd_clamp_position", seq_lens.data_ptr(), 1 if seq_lens.dtype == torch.int64 else 0,
                 out.data_ptr(), seq_lens.numel(), _stream())
     return out
+
+
+def bigram_rows(ids: torch.Tensor, positions: torch.Tensor, loc: torch.Tensor, req_to_token: torch.Tensor, req_pool_indices: torch.Tensor,
+                tok_seg: Optional[torch.Tensor], slot_ids: torch.Tensor, mul_prev: int, mul_cur: int, buckets: int) -> torch.Tensor:
+    """int64 [T]: (previous token * mul_prev + token * mul_cur) mod buckets, `buckets` for a sequence's first token.  slot_ids int32 [slots]
+    holds the token of every cache slot: read in front of a portion, written for the batch's own tokens."""
+    _dev(ids, positions, loc, req_to_token, req_pool_indices, tok_seg, slot_ids)
+    T = ids.numel()
+    for t in (ids, positions, loc, req_pool_indices):
+        _need(t.dtype == torch.int64 and t.is_contiguous(), "bigram_rows: contiguous int64 indices")
+    _need(positions.numel() == T and loc.numel() == T and req_to_token.dtype == torch.int32 and req_to_token.stride(1) == 1
+          and slot_ids.dtype == torch.int32 and slot_ids.is_contiguous()
+          and (req_pool_indices.numel() == T if tok_seg is None else tok_seg.dtype == torch.int32 and tok_seg.numel() == T), "bigram_rows: shapes")
+    rows = torch.empty(T, dtype=torch.int64, device=ids.device)
+    native.call("sgl_amd_bigram_rows", ids.data_ptr(), positions.data_ptr(), loc.data_ptr(), req_to_token.data_ptr(), req_to_token.stride(0),
+                req_pool_indices.data_ptr(), _ptr(tok_seg), slot_ids.data_ptr(), rows.data_ptr(), T, mul_prev % buckets, mul_cur % buckets,
+                buckets, _stream())
+    return rows
 
 
 def alloc_extend(prefix_lens: torch.Tensor, seq_lens: torch.Tensor, last_loc: torch.Tensor, free_pages: torch.Tensor,
@@ -840,10 +882,10 @@ def choose_wstream_decomposition(M: int, N: int, K: int, need_combine: bool = Fa
 def wstream_gemm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] = None, epilogue: str = "none",
                  residual: Optional[torch.Tensor] = None, norm_weight: Optional[torch.Tensor] = None, eps: float = 0.0,
                  out: Optional[torch.Tensor] = None, waves_per_group: Optional[int] = None,
-                 splits: Optional[int] = None, out_blocked: bool = False, tiles_per_wave: Optional[int] = None) -> torch.Tensor:
+                 splits: Optional[int] = None, out_blocked: bool = False, tiles_per_wave: Optional[int] = None, act: Glu = SILU) -> torch.Tensor:
     """Decode-batch F.linear(x, w, bias) on the weight-streaming kernel, optionally followed (in the
     split-K combine kernel) by silu_and_mul or by fused_add_rmsnorm(out, residual, norm_weight, eps).
-    x may be chunk-major (see _x_layout); out_blocked=True returns the result chunk-major."""
+    x may be chunk-major (see _x_layout); out_blocked=True returns the result chunk-major.  `act` replaces silu in silu_and_mul."""
     _dev(x, w)
     _need(x.dtype == _BF16 and w.dtype == _BF16 and w.dim() == 2, "wstream_gemm: bf16 x / 2-D bf16 w")
     M, K, x_rs, x_cs = _x_layout(x, "wstream_gemm")
@@ -876,6 +918,10 @@ def wstream_gemm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] 
     # multiple of 16 but not of 32 runs the interleaved one-pass form when the automatic decomposition says one tile per wave
     one_pass = ep == 1 and s == 1 and (N % 16 == 0 if tpw == 1 else N % 32 == 0)
     ws = _gemm_workspace(x.device, native.lib().sgl_amd_wstream_gemm_workspace_floats(M, N, s)) if ((s > 1 or ep) and not one_pass) else None
+    if ep == 1 and act.kind != "silu":
+        native.call("sgl_amd_wstream_glu_gemm", x.data_ptr(), w.data_ptr(), _ptr(bias), out.data_ptr(), M, N, K, x_rs, x_cs, w.stride(0), y_rs, y_cs,
+                    *act.args, nw, tpw, s, _ptr(ws), _stream())
+        return out
     native.call("sgl_amd_wstream_gemm", x.data_ptr(), w.data_ptr(), _ptr(bias), out.data_ptr(), M, N, K, x_rs, x_cs,
                 w.stride(0), y_rs, y_cs, ep, _ptr(residual), residual.stride(0) if residual is not None else 0,
                 _ptr(norm_weight), float(eps), nw, tpw, s, _ptr(ws), _stream())
@@ -949,7 +995,7 @@ def moe_wstream_gemm(a: torch.Tensor, w: torch.Tensor, c: torch.Tensor, sorted_t
                      expert_ids: torch.Tensor, num_tokens_post_padded: torch.Tensor,
                      topk_weights: Optional[torch.Tensor], mul_routed_weight: bool, top_k_div: int, num_valid_ids: int,
                      block_m: int, fuse_silu: bool = False, round_before_scale: bool = False,
-                     waves_per_group: Optional[int] = None) -> torch.Tensor:
+                     waves_per_group: Optional[int] = None, act: Glu = SILU) -> torch.Tensor:
     """moe_grouped_gemm on the weight-streaming kernel (no split-K): a [rows, K] bf16, w [E, N(or 2N), K] bf16,
     c [num_valid_ids, N] bf16 or fp32; needs N % 16 == 0 and K % 128 == 0."""
     _dev(a, w, c, sorted_token_ids, expert_ids, num_tokens_post_padded)
@@ -975,7 +1021,7 @@ def moe_wstream_gemm(a: torch.Tensor, w: torch.Tensor, c: torch.Tensor, sorted_t
     native.call("sgl_amd_wstream_moe_gemm", a.data_ptr(), w.data_ptr(), c.data_ptr(), sorted_token_ids.data_ptr(),
                 expert_ids.data_ptr(), num_tokens_post_padded.data_ptr(), _ptr(topk_weights),
                 1 if mul_routed_weight else 0, 1 if round_before_scale else 0, top_k_div, num_valid_ids, N, K,
-                a.stride(0), w.stride(1), w.stride(0), c.stride(0), block_m, max_m_blocks, 1 if fuse_silu else 0,
+                a.stride(0), w.stride(1), w.stride(0), c.stride(0), block_m, max_m_blocks, *(act.args if fuse_silu else NO_GLU),
                 1 if c.dtype == torch.float32 else 0, waves_per_group, _stream())
     return c
 
@@ -987,7 +1033,7 @@ def moe_tiled_gemm_block_m() -> int:
 def moe_tiled_gemm(a: torch.Tensor, w: torch.Tensor, c: torch.Tensor, sorted_token_ids: torch.Tensor,
                    expert_ids: torch.Tensor, num_tokens_post_padded: torch.Tensor, topk_weights: Optional[torch.Tensor],
                    mul_routed_weight: bool, top_k_div: int, num_valid_ids: int, block_m: int, fuse_silu: bool = False,
-                   round_before_scale: bool = False, tile_rows: Optional[int] = None) -> torch.Tensor:
+                   round_before_scale: bool = False, tile_rows: Optional[int] = None, act: Glu = SILU) -> torch.Tensor:
     """moe_grouped_gemm on the row-tiled MFMA kernels (prefill-sized batches): block_m = the align block size (128 or
     256), tile_rows = rows of an expert per workgroup tile (128, or 256 over a 256 alignment: the 256 x 256 x 64 form);
     a [rows, K] bf16, w [E, N(or 2N), K] bf16, c [num_valid_ids, N] bf16 or fp32."""
@@ -1010,7 +1056,7 @@ def moe_tiled_gemm(a: torch.Tensor, w: torch.Tensor, c: torch.Tensor, sorted_tok
     native.call("sgl_amd_moe_tiled_gemm_ex", a.data_ptr(), w.data_ptr(), c.data_ptr(), sorted_token_ids.data_ptr(),
                 expert_ids.data_ptr(), num_tokens_post_padded.data_ptr(), _ptr(topk_weights), 1 if mul_routed_weight else 0,
                 1 if round_before_scale else 0, top_k_div, num_valid_ids, N, K, a.stride(0), w.stride(1), w.stride(0),
-                c.stride(0), max_m_blocks, 1 if fuse_silu else 0, 1 if c.dtype == torch.float32 else 0, int(block_m), int(tile_rows),
+                c.stride(0), max_m_blocks, *(act.args if fuse_silu else NO_GLU), 1 if c.dtype == torch.float32 else 0, int(block_m), int(tile_rows),
                 _stream())
     return c
 
@@ -1037,7 +1083,7 @@ def moe_grouped_gemm(a: torch.Tensor, w: torch.Tensor, c: torch.Tensor, sorted_t
                      expert_ids: torch.Tensor, num_tokens_post_padded: torch.Tensor,
                      topk_weights: Optional[torch.Tensor], mul_routed_weight: bool, top_k_div: int, num_valid_ids: int,
                      block_m: int, fuse_silu: bool = False, round_before_scale: bool = False,
-                     splits: Optional[int] = None, tiles_per_wave: Optional[int] = None) -> torch.Tensor:
+                     splits: Optional[int] = None, tiles_per_wave: Optional[int] = None, act: Glu = SILU) -> torch.Tensor:
     """invoke_fused_moe_kernel equivalent (fused_moe_triton_kernels.py:771): a [rows, K] bf16,
     w [E, N(or 2N), K] bf16, c [num_valid_ids, N] bf16 or fp32."""
     _dev(a, w, c, sorted_token_ids, expert_ids, num_tokens_post_padded)
@@ -1067,7 +1113,7 @@ def moe_grouped_gemm(a: torch.Tensor, w: torch.Tensor, c: torch.Tensor, sorted_t
     native.call("sgl_amd_moe_grouped_gemm", a.data_ptr(), w.data_ptr(), c.data_ptr(), sorted_token_ids.data_ptr(),
                 expert_ids.data_ptr(), num_tokens_post_padded.data_ptr(), _ptr(topk_weights),
                 1 if mul_routed_weight else 0, 1 if round_before_scale else 0, top_k_div, num_valid_ids, N, K, E,
-                a.stride(0), w.stride(1), w.stride(0), c.stride(0), block_m, max_m_blocks, 1 if fuse_silu else 0,
+                a.stride(0), w.stride(1), w.stride(0), c.stride(0), block_m, max_m_blocks, *(act.args if fuse_silu else NO_GLU),
                 1 if c.dtype == torch.float32 else 0, ntw, splits, _ptr(slabs), _stream())
     return c
 
@@ -1277,15 +1323,18 @@ def _row_source(who: str, y, rows: int, W: int):
 def residual_rms(x: torch.Tensor, eps: float, *, embed: Optional[Tuple[torch.Tensor, torch.Tensor, float]] = None,
                  pos: Optional[Tuple[torch.Tensor, torch.Tensor]] = None, add: tuple = (), save: Optional[torch.Tensor] = None,
                  extra: Optional[torch.Tensor] = None, step: Optional[torch.Tensor] = None, norm: Optional[torch.Tensor] = None,
-                 h: Optional[torch.Tensor] = None) -> None:
+                 h: Optional[torch.Tensor] = None, post: Optional[Tuple[torch.Tensor, float]] = None) -> None:
     """Update the fp32 residual rows `x` -- embed = (ids, table, scale) with pos = (positions, table): embedding row + position row;
     else x + the addends `add` (at most two: rows, Partials or ExpertRows) -- copy them to `save`, add the rows `extra` and the
-    vector `step`, then h = RMS norm(x) * norm, in one launch."""
+    vector `step`, then h = RMS norm(x) * norm (no norm: h = x), in one launch.  post = (weight, factor): x + factor * (RMS norm of the
+    addends' sum * weight)."""
     _need(x.dtype == torch.float32 and x.dim() == 2 and x.stride(1) == 1, "residual_rms: fp32 residual rows")
     _need(len(add) <= 2 and not (embed is not None and len(add)) and (pos is None or embed is not None), "residual_rms: an embedding, or at most two addends")
-    _need((h is None) == (norm is None), "residual_rms: h and its norm come together")
+    _need(h is not None or norm is None, "residual_rms: a norm without h")
+    _need(post is None or len(add) >= 1, "residual_rms: a norm behind no sublayer")
     rows, W = x.shape
     ids = table = positions = pos_table = None
+    post_w, mult = post if post is not None else (None, 0.0)
     scale = 0.0
     if embed is not None:
         ids, table, scale = embed
@@ -1300,15 +1349,15 @@ def residual_rms(x: torch.Tensor, eps: float, *, embed: Optional[Tuple[torch.Ten
     _rows("residual_rms", h)
     for t in (save, extra):
         _need(t is None or (t.dtype == torch.float32 and t.is_contiguous() and tuple(t.shape) == (rows, W)), "residual_rms: contiguous fp32 rows")
-    for t in (step, norm):
+    for t in (step, norm, post_w):
         _need(t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == W), "residual_rms: fp32 parameters [W]")
     _need(h is None or tuple(h.shape) == (rows, W), "residual_rms: h [rows, W]")
-    _dev(x, ids, table, positions, pos_table, a[0], b[0], save, extra, step, norm, h)
+    _dev(x, ids, table, positions, pos_table, a[0], b[0], save, extra, step, norm, post_w, h)
     acts = [t for t in (table, h, *(s[0] for s in (a, b) if s[0] is not None and not s[1])) if t is not None]
     f32 = _is_f32(*acts) if acts else 1
     native.call("sgl_amd_residual_rms", f32, _ptr(ids), _ptr(table), table.shape[0] if table is not None else 0, float(scale), _ptr(positions),
                 _ptr(pos_table), pos_table.shape[0] if pos_table is not None else 0, _ptr(a[0]), *a[1:5], _ptr(a[5]), _ptr(b[0]), *b[1:5], _ptr(b[5]),
-                x.data_ptr(), x.stride(0), _ptr(save), _ptr(extra), _ptr(step), _ptr(norm), _ptr(h), h.stride(0) if h is not None else 0, rows, W,
+                x.data_ptr(), x.stride(0), _ptr(save), _ptr(extra), _ptr(step), _ptr(post_w), float(mult), _ptr(norm), _ptr(h), h.stride(0) if h is not None else 0, rows, W,
                 float(eps), _stream())
 
 
@@ -1347,8 +1396,8 @@ def gated_rmsnorm(y: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, gro
     return out
 
 
-def gate_mul(x: torch.Tensor) -> torch.Tensor:
-    """silu(x[:, :d]) * x[:, d:] for fp32 rows, or bf16 rows silu_and_mul's vector form does not take."""
+def gate_mul(x: torch.Tensor, act: Glu = SILU) -> torch.Tensor:
+    """act(x[:, :d], x[:, d:]) for fp32 rows, or bf16 rows the vector form (silu_and_mul, glu_and_mul) does not take."""
     _dev(x)
     _rows("gate_mul", x)
     rows, d = x.shape[0], x.shape[1] // 2
@@ -1357,7 +1406,7 @@ def gate_mul(x: torch.Tensor) -> torch.Tensor:
     for r in range(0, rows, 65535):
         n = min(65535, rows - r)
         base = x.data_ptr() + r * x.stride(0) * es
-        native.call("sgl_amd_gate_mul", f32, base, base + d * es, out.data_ptr() + r * d * es, n, d, x.stride(0), out.stride(0), _stream())
+        native.call("sgl_amd_gate_mul", f32, base, base + d * es, out.data_ptr() + r * d * es, n, d, x.stride(0), out.stride(0), *act.args, _stream())
     return out
 
 
@@ -1480,8 +1529,10 @@ def head_gemm(x: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor] = No
 
 
 def latent_attention(qc: torch.Tensor, qr: torch.Tensor, cache: torch.Tensor, req_to_token: torch.Tensor, req_pool_indices: torch.Tensor,
-                     positions: torch.Tensor, seg: Segments, window: int, scale: float, splits: int = 1, plain: bool = False) -> torch.Tensor:
-    """Absorbed latent attention: qc [T, H, rank], qr [T, H, rot] over the cached rows -> attended latents [T, H, rank].
+                     positions: torch.Tensor, seg: Segments, window: int, scale: float, splits: int = 1, plain: bool = False,
+                     sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """Absorbed latent attention: qc [T, H, rank], qr [T, H, rot] over the cached rows -> attended latents [T, H, rank].  sinks fp32 [H] join
+    the softmax denominators.
     bf16 rows run on matrix instructions where the sizes allow (`plain` forces the other form)."""
     _dev(qc, qr, cache, req_to_token, req_pool_indices, positions)
     T, H, rank = qc.shape
@@ -1489,6 +1540,8 @@ def latent_attention(qc: torch.Tensor, qr: torch.Tensor, cache: torch.Tensor, re
     _rows("latent_attention", cache)
     _need(qr.shape[:2] == (T, H) and qc.stride(2) == 1 and qr.stride(2) == 1 and cache.shape[1] >= rank + qr.shape[2]
           and req_to_token.dtype == torch.int32 and req_to_token.stride(1) == 1, "latent_attention: shapes")
+    _f32("latent_attention", sinks)
+    _need(sinks is None or sinks.numel() == H, "latent_attention: one sink a head")
     out = torch.empty((T, H, rank), dtype=qc.dtype, device=qc.device)
     po = pml = None
     if splits > 1:
@@ -1497,7 +1550,7 @@ def latent_attention(qc: torch.Tensor, qr: torch.Tensor, cache: torch.Tensor, re
     native.call("sgl_amd_latent_attention", _is_f32(qc, qr, cache), qc.data_ptr(), qc.stride(0), qc.stride(1), qr.data_ptr(), qr.stride(0),
                 qr.stride(1), cache.data_ptr(), cache.stride(0), req_to_token.data_ptr(), req_to_token.stride(0), req_pool_indices.data_ptr(),
                 _ptr(seg.tok_seg), positions.data_ptr(), out.data_ptr(), out.stride(0), out.stride(1), _ptr(po), _ptr(pml), T, H, rank,
-                qr.shape[2], int(window), splits, float(scale), 1 if plain else 0, _stream())
+                qr.shape[2], int(window), splits, float(scale), _ptr(sinks), 1 if plain else 0, _stream())
     return out
 
 
@@ -1544,7 +1597,8 @@ def latent_gather(cache: torch.Tensor, req_to_token: torch.Tensor, req_pool_indi
 
 
 def latent_prefill(q: torch.Tensor, latents: torch.Tensor, kv: torch.Tensor, keys: VisibleKeys, positions: torch.Tensor, seg: Segments,
-                   heads: int, dim: int, rot: int, rank: int, vdim: int, window: int, scale: float) -> torch.Tensor:
+                   heads: int, dim: int, rot: int, rank: int, vdim: int, window: int, scale: float,
+                   sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Flash attention of q [T, heads * (dim + rot)] over expanded keys / values kv [keys, heads * dim | heads * vdim] and the
     rotated key parts in latents[:, rank:rank + rot] -> [T, heads * vdim]."""
     _dev(q, latents, kv, positions)
@@ -1553,12 +1607,74 @@ def latent_prefill(q: torch.Tensor, latents: torch.Tensor, kv: torch.Tensor, key
           and latents.shape[0] == keys.total and latents.shape[1] >= rank + rot and seg.start is not None, "latent_prefill: shapes")
     _i64("latent_prefill", positions)
     _need(positions.numel() == q.shape[0] and seg.start.numel() == keys.start.numel(), "latent_prefill: one position per token, one key range per segment")
+    _f32("latent_prefill", sinks)
+    _need(sinks is None or sinks.numel() == heads, "latent_prefill: one sink a head")
     out = torch.empty((q.shape[0], heads * vdim), dtype=q.dtype, device=q.device)
     native.call("sgl_amd_latent_prefill", q.data_ptr(), q.stride(0), latents.data_ptr(), latents.stride(0), kv.data_ptr(), kv.stride(0),
                 keys.blocks.data_ptr(), keys.blocks.shape[0], seg.start.data_ptr(), seg.len.data_ptr(), keys.start.data_ptr(),
                 keys.first.data_ptr(), positions.data_ptr(), out.data_ptr(), out.stride(0), heads, dim, rot, rank, vdim, int(window),
-                float(scale), _stream())
+                float(scale), _ptr(sinks), _stream())
     return out
+
+
+# ---------------------------------------------------------------------------- between a projection and attention
+def _projection(who: str, p, cols: int):
+    """(rows, row stride, partials, items, item stride, bias) of a projection's rows [T, >= cols] or Partials."""
+    if isinstance(p, Partials):
+        _need(p.cols >= cols, f"{who}: {p.cols} columns, needs {cols}")
+        return None, p.cols, p.data.data_ptr(), p.splits, p.rows * p.cols, p.bias
+    _rows(who, p)
+    _need(p.shape[1] >= cols, f"{who}: {p.shape[1]} columns, needs {cols}")
+    return p.data_ptr(), p.stride(0), None, 0, 0, None
+
+
+def head_prepare(p, heads: int, dim: int, kd: int, positions: torch.Tensor, cos_sin: Optional[torch.Tensor], eps: float, *, rot_off: int = 0,
+                 norms: Optional[Tuple[torch.Tensor, torch.Tensor]] = None, norm_after: bool = False, gate_cols: int = 0,
+                 kv: Optional[Tuple[int, int, torch.Tensor, torch.Tensor]] = None, plain: bool = False):
+    """Query heads [T, heads * kd] (and the gate columns [T, gate_cols], or None) of a projection p -- rows, changed in place, or Partials --
+    behind an RMS norm a head over `dim` elements (norms = (query weight, key weight): in front of the rotation; norm_after: behind it,
+    without weights) and the rotation by halves of [rot_off, + cos_sin.shape[1]).  kv = (kv_heads, vd, cache, loc): keys, treated alike, and
+    values go to the cache rows."""
+    G, vd, cache, loc = kv if kv is not None else (0, 0, None, None)
+    cols = heads * kd + G * (kd + vd)
+    rows, stride, part, items, item_stride, bias = _projection("head_prepare", p, cols + gate_cols)
+    T = p.rows if part is not None else p.shape[0]
+    f32 = 0 if part is not None else _is_f32(p)
+    _dev(positions, cos_sin, cache, loc, *(norms or ()))
+    _i64("head_prepare", positions, loc)
+    _f32("head_prepare", cos_sin, *(norms or ()))
+    _need(positions.numel() == T and (loc is None or loc.numel() == T) and all(w.numel() == dim for w in norms or ()), "head_prepare: shapes")
+    _need(cache is None or (_is_f32(cache) == f32 and cache.shape[1] >= G * (kd + vd) and cache.stride(1) == 1), "head_prepare: cache rows")
+    _need(bias is None or bias.dtype == _BF16, "head_prepare: the partials' bias is bf16")
+    out = p if part is None else torch.empty((T, heads * kd + gate_cols), dtype=_BF16, device=positions.device)
+    native.call("sgl_amd_head_prepare", f32, rows, stride, part, items, item_stride, _ptr(bias), out.data_ptr(), out.stride(0),
+                _ptr(norms[0]) if norms else None, _ptr(norms[1]) if norms else None, 1 if norms else 2 if norm_after else 0, float(eps), _ptr(cos_sin),
+                cos_sin.shape[0] if cos_sin is not None else 0, positions.data_ptr(), rot_off, cos_sin.shape[1] if cos_sin is not None else 0,
+                _ptr(cache), cache.stride(0) if cache is not None else 0, _ptr(loc), T, heads, G, kd, vd, dim, gate_cols if part is not None else 0,
+                1 if plain else 0, _stream())
+    g0 = heads * kd if part is not None else cols
+    return out[:, :heads * kd], out[:, g0:g0 + gate_cols] if gate_cols else None
+
+
+def latent_down(p, q_norm: Optional[torch.Tensor], norm: torch.Tensor, cos_sin: torch.Tensor, positions: torch.Tensor, loc: torch.Tensor,
+                cache: torch.Tensor, rot: int, eps: float) -> torch.Tensor:
+    """p: rows or Partials [T, query latent | latent | rotated key part] -> RMS norm of the query latent [T, q_rank]; the normed latent and
+    the key part, rotated by halves, go to the cache rows `loc`."""
+    q_rank, rank = q_norm.numel() if q_norm is not None else 0, norm.numel()
+    rows, stride, part, items, item_stride, bias = _projection("latent_down", p, q_rank + rank + rot)
+    T = p.rows if part is not None else p.shape[0]
+    _dev(positions, loc, cache, cos_sin, q_norm, norm)
+    _i64("latent_down", positions, loc)
+    _f32("latent_down", q_norm, norm, cos_sin)
+    _rows("latent_down", cache)
+    f32 = _is_f32(cache) if part is not None else _is_f32(p, cache)
+    _need(bias is None and not (part is not None and f32) and positions.numel() == T and loc.numel() == T and cache.shape[1] >= rank + rot
+          and cos_sin.shape[1] <= rot, "latent_down: shapes")
+    cq = torch.empty((T, q_rank), dtype=cache.dtype, device=cache.device)
+    native.call("sgl_amd_latent_down", f32, rows, stride, part, items, item_stride, _ptr(q_norm), norm.data_ptr(), float(eps), cos_sin.data_ptr(),
+                cos_sin.shape[0], positions.data_ptr(), cos_sin.shape[1], cq.data_ptr() if q_rank else None, cq.stride(0), cache.data_ptr(),
+                cache.stride(0), loc.data_ptr(), T, q_rank, rank, rot, _stream())
+    return cq
 
 
 # ---------------------------------------------------------------------------- grouped-query attention with sizes of its own
@@ -1587,7 +1703,7 @@ def _grouped_checks(who: str, q: torch.Tensor, cache: torch.Tensor, out: torch.T
     T = q.shape[0]
     _rows(who, q, cache, out, gate)
     _need(heads % kv_heads == 0 and q.shape[1] == heads * kd and cache.shape[1] >= kv_heads * (kd + vd) and tuple(out.shape) == (T, heads * vd)
-          and (gate is None or tuple(gate.shape) == (T, heads * vd)) and req_to_token.dtype == torch.int32 and req_to_token.stride(1) == 1,
+          and (gate is None or tuple(gate.shape) in ((T, heads * vd), (T, heads))) and req_to_token.dtype == torch.int32 and req_to_token.stride(1) == 1,
           f"{who}: shapes")
 
 
@@ -1602,11 +1718,23 @@ def grouped_kv_store(k: torch.Tensor, v: torch.Tensor, cache: torch.Tensor, loc:
                 cache.stride(0), loc.data_ptr(), k.shape[0], kv_heads, k.shape[1] // kv_heads, v.shape[1] // kv_heads, _stream())
 
 
+def _sink_args(who: str, sink, cap: Optional[float], gate: Optional[torch.Tensor], heads: int):
+    """(scalar sink, sink of every head, cap, gate a head?) of a launch."""
+    per_head = isinstance(sink, torch.Tensor)
+    if per_head:
+        _dev(sink)
+        _f32(who, sink)
+        _need(sink.numel() == heads, f"{who}: one sink a head")
+    return (float("-inf") if sink is None or per_head else float(sink), sink.data_ptr() if per_head else None, float(cap or 0.0),
+            1 if gate is not None and gate.shape[1] == heads else 0)
+
+
 def grouped_attention(q: torch.Tensor, cache: torch.Tensor, req_to_token: torch.Tensor, req_pool_indices: torch.Tensor, positions: torch.Tensor,
-                      seg: Segments, heads: int, kv_heads: int, kd: int, vd: int, window: int, scale: float, *, sink: Optional[float] = None,
+                      seg: Segments, heads: int, kv_heads: int, kd: int, vd: int, window: int, scale: float, *, sink=None,
                       gate: Optional[torch.Tensor] = None, new: Optional[Tuple[torch.Tensor, torch.Tensor, torch.Tensor]] = None, splits: int = 1,
-                      plain: bool = False) -> torch.Tensor:
-    """q [T, heads * kd] over the cached keys of each token's request -> [T, heads * vd], times sigmoid(gate).  new = (k, v, loc): a
+                      plain: bool = False, cap: Optional[float] = None) -> torch.Tensor:
+    """q [T, heads * kd] over the cached keys of each token's request -> [T, heads * vd], times sigmoid(gate) (one an element, or one a head).
+    sink: a float, or fp32 [heads]; cap: scores become cap * tanh(score / cap).  new = (k, v, loc): a
     decode batch's own keys and values, stored on the way (matrix form).  `plain` forces the form without matrix instructions."""
     _dev(q, cache, req_to_token, req_pool_indices, positions, gate)
     T = q.shape[0]
@@ -1629,13 +1757,13 @@ def grouped_attention(q: torch.Tensor, cache: torch.Tensor, req_to_token: torch.
                 k.stride(0) if k is not None else 0, _ptr(v), v.stride(0) if v is not None else 0, _ptr(loc), req_to_token.data_ptr(),
                 req_to_token.stride(0), req_pool_indices.data_ptr(), _ptr(seg.tok_seg), positions.data_ptr(), _ptr(gate),
                 gate.stride(0) if gate is not None else 0, out.data_ptr(), out.stride(0), _ptr(po), _ptr(pml), T, heads, kv_heads, kd, vd, int(window),
-                splits, float(scale), float("-inf") if sink is None else float(sink), 1 if plain else 0, _stream())
+                splits, float(scale), *_sink_args("grouped_attention", sink, cap, gate, heads), 1 if plain else 0, _stream())
     return out
 
 
 def grouped_prefill(q: torch.Tensor, cache: torch.Tensor, req_to_token: torch.Tensor, req_pool_indices: torch.Tensor, positions: torch.Tensor,
                     seg: Segments, blocks: QueryBlocks, heads: int, kv_heads: int, kd: int, vd: int, window: int, scale: float, *,
-                    sink: Optional[float] = None, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+                    sink=None, gate: Optional[torch.Tensor] = None, cap: Optional[float] = None) -> torch.Tensor:
     """grouped_attention over long extends whose keys are stored (bf16)."""
     _dev(q, cache, req_to_token, req_pool_indices, positions, gate, blocks.blocks)
     T = q.shape[0]
@@ -1646,16 +1774,27 @@ def grouped_prefill(q: torch.Tensor, cache: torch.Tensor, req_to_token: torch.Te
     native.call("sgl_amd_grouped_prefill", q.data_ptr(), q.stride(0), cache.data_ptr(), cache.stride(0), req_to_token.data_ptr(),
                 req_to_token.stride(0), req_pool_indices.data_ptr(), blocks.blocks.data_ptr(), blocks.blocks.shape[0], seg.start.data_ptr(),
                 seg.len.data_ptr(), positions.data_ptr(), _ptr(gate), gate.stride(0) if gate is not None else 0, out.data_ptr(), out.stride(0), heads,
-                kv_heads, kd, vd, int(window), float(scale), float("-inf") if sink is None else float(sink), _stream())
+                kv_heads, kd, vd, int(window), float(scale), *_sink_args("grouped_prefill", sink, cap, gate, heads), _stream())
     return out
 
 
 # ---------------------------------------------------------------------------- routed experts behind a biased router
-def moe_route(h: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], top: int) -> Tuple[torch.Tensor, torch.Tensor]:
-    """The `top` largest of w h + bias (fp32) and the softmax over those: fp32 weights, int32 ids [T, top]."""
-    _dev(h, w, bias)
+class SigmoidScores:
+    """A router of sigmoid scores: `top` experts by score + correction (fp32 [experts]) out of the best `keep` of `groups` equal groups of
+    neighbours -- a group counts by the sum of its two best -- weighted by score * scale."""
+
+    def __init__(self, correction: Optional[torch.Tensor], groups: int = 1, keep: int = 1, scale: float = 1.0):
+        self.correction, self.groups, self.keep, self.scale = correction, groups, keep, scale
+
+
+def moe_route(h: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], top: int, scores: Optional[SigmoidScores] = None
+              ) -> Tuple[torch.Tensor, torch.Tensor]:
+    """The `top` largest of w h + bias (fp32) and the softmax over those, or what `scores` picks: fp32 weights, int32 ids [T, top]."""
+    c = scores.correction if scores is not None else None
+    _dev(h, w, bias, c)
     _rows("moe_route", h)
-    _f32("moe_route", bias)
+    _f32("moe_route", bias, c)
+    _need(c is None or c.numel() == w.shape[0], "moe_route: one correction an expert")
     T, K = h.shape
     _need(w.dim() == 2 and w.shape[1] == K and w.is_contiguous() and (bias is None or bias.numel() == w.shape[0]), "moe_route: shapes")
     weights = torch.empty((T, top), dtype=torch.float32, device=h.device)
@@ -1668,39 +1807,39 @@ def moe_route(h: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], to
         slices = max(1, min(-(-1024 // blocks), K // 64, 32))
         part = torch.empty((slices, T, pad), dtype=torch.float32, device=h.device)
     native.call("sgl_amd_moe_route", f32, h.data_ptr(), h.stride(0), w.data_ptr(), _ptr(bias), weights.data_ptr(), ids.data_ptr(), _ptr(part), slices,
-                pad, T, K, E, top, _stream())
+                pad, T, K, E, top, *((1, _ptr(c), scores.groups, scores.keep, float(scores.scale)) if scores is not None else (0, None, 1, 1, 1.0)), _stream())
     return weights, ids
 
 
-def _experts_plain(x: torch.Tensor, w: torch.Tensor, ids: torch.Tensor, up: bool) -> torch.Tensor:
+def _experts_plain(x: torch.Tensor, w: torch.Tensor, ids: torch.Tensor, up: bool, act: Glu = SILU) -> torch.Tensor:
     E, N, K = w.shape[0], w.shape[1] // (2 if up else 1), w.shape[2]
     pairs, top = ids.numel(), ids.shape[1]
     _rows("experts", x)
     _need(w.is_contiguous() and ids.dtype == torch.int32 and ids.is_contiguous() and x.shape == (ids.shape[0] if up else pairs, K), "experts: shapes")
     out = torch.empty((pairs, N), dtype=x.dtype, device=x.device)
     native.call("sgl_amd_experts_plain", _is_f32(x, w), 1 if up else 0, x.data_ptr(), x.stride(0), w.data_ptr(), ids.data_ptr(), out.data_ptr(), N, pairs,
-                top, N, K, E, _stream())
+                top, N, K, E, *act.args, _stream())
     return out
 
 
-def routed_experts(h: torch.Tensor, w13: torch.Tensor, w2: torch.Tensor, ids: torch.Tensor, plain: bool = False) -> torch.Tensor:
-    """Every token's chosen experts, silu(gate h) * (up h) and the down projection, unweighted: [T, top, W] in the type of h.  bf16 rows
+def routed_experts(h: torch.Tensor, w13: torch.Tensor, w2: torch.Tensor, ids: torch.Tensor, plain: bool = False, act: Glu = SILU) -> torch.Tensor:
+    """Every token's chosen experts, act(gate h, up h) and the down projection, unweighted: [T, top, W] in the type of h.  bf16 rows
     run on the grouped matrix kernels of fused_experts; fp32 rows and sizes they do not take go through a plain form."""
     _dev(h, w13, w2, ids)
     (T, W), (E, N2, _), top = h.shape, w13.shape, ids.shape[1]
     N, numel = N2 // 2, T * top
     if plain or h.dtype != _BF16 or W % 8 or W < 32 or N % 32:
-        return _experts_plain(_experts_plain(h, w13, ids, True), w2, ids, False).view(T, top, W)
+        return _experts_plain(_experts_plain(h, w13, ids, True, act), w2, ids, False).view(T, top, W)
     inter = torch.empty((numel, N), dtype=_BF16, device=h.device)
     down = torch.empty((numel, W), dtype=_BF16, device=h.device)
     if numel // E >= MOE_TILED_MIN_ROWS_PER_EXPERT and W % 64 == 0 and N % 64 == 0:
         block_m, up_rows, down_rows = moe_tile_plan(numel, E, N, W) if MOE_TILE_OVERRIDE is None else MOE_TILE_OVERRIDE
         s = moe_align_block_size(ids, block_m, E)
-        moe_tiled_gemm(h, w13, inter, *s, None, False, top, numel, block_m, fuse_silu=True, tile_rows=up_rows)
+        moe_tiled_gemm(h, w13, inter, *s, None, False, top, numel, block_m, fuse_silu=True, tile_rows=up_rows, act=act)
         moe_tiled_gemm(inter, w2, down, *s, None, False, 1, numel, block_m, tile_rows=down_rows)
     else:
         block_m = choose_moe_block_m(numel, E)
         s = moe_align_block_size(ids, block_m, E)
-        (moe_wstream_gemm if W % 128 == 0 else moe_grouped_gemm)(h, w13, inter, *s, None, False, top, numel, block_m, fuse_silu=True)
+        (moe_wstream_gemm if W % 128 == 0 else moe_grouped_gemm)(h, w13, inter, *s, None, False, top, numel, block_m, fuse_silu=True, act=act)
         (moe_wstream_gemm if W % 16 == 0 and N % 128 == 0 else moe_grouped_gemm)(inter, w2, down, *s, None, False, 1, numel, block_m)
     return down.view(T, top, W)

@@ -60,6 +60,18 @@ class HybridAttnBackend(AttentionBackend):
         cache = self.token_to_kv_pool.get_latent_buffer(run_id)
         kernels.latent_prepare(q, dkv, layer.norm_weight, layer.cos_sin, forward_batch.positions, forward_batch.out_cache_loc, cache,
                                layer.heads, layer.dim, layer.rot_dim, layer.eps)
+        return self._latent(layer, q, cache, forward_batch)
+
+    def query_latent_attention(self, layer, p, run_id: int, forward_batch) -> torch.Tensor:
+        """p: the projection [query latent | latent | rotated key part], rows or Partials -> values [T, heads * vdim]."""
+        cache, pos = self.token_to_kv_pool.get_latent_buffer(run_id), forward_batch.positions
+        cq = kernels.latent_down(p, layer.q_norm, layer.norm_weight, layer.cos_sin, pos, forward_batch.out_cache_loc, cache, layer.rot_dim, layer.eps)
+        dk = layer.dim + layer.rot_dim
+        q, _ = kernels.head_prepare(layer.up_proj.forward_partials(cq), layer.heads, dk, dk, pos, layer.cos_sin, layer.eps, rot_off=layer.dim)
+        return self._latent(layer, q, cache, forward_batch)
+
+    def _latent(self, layer, q: torch.Tensor, cache: torch.Tensor, forward_batch) -> torch.Tensor:
+        """Turned queries [T, heads * (dim + rot)] over the stored rows -> values [T, heads * vdim]."""
         if forward_batch.forward_mode.is_extend() and self._expanded(layer):
             keys = self._keys.get(layer.window)
             if keys is None:
@@ -67,12 +79,12 @@ class HybridAttnBackend(AttentionBackend):
             lat = kernels.latent_gather(cache, self.req_to_token_pool.req_to_token, forward_batch.req_pool_indices, keys)
             kv = torch.nn.functional.linear(lat[:, :layer.rank], layer.w_expand)
             return kernels.latent_prefill(q, lat, kv, keys, forward_batch.positions, self.segments, layer.heads, layer.dim, layer.rot_dim,
-                                          layer.rank, layer.vdim, layer.window, layer.scale)
+                                          layer.rank, layer.vdim, layer.window, layer.scale, sinks=layer.sinks)
         T = q.shape[0]
         q3 = q.view(T, layer.heads, layer.dim + layer.rot_dim) if q.is_contiguous() else q.unflatten(1, (layer.heads, layer.dim + layer.rot_dim))
         qc = kernels.head_gemm(q3[:, :, :layer.dim], layer.w_absorb)
         oc = kernels.latent_attention(qc, q3[:, :, layer.dim:], cache, self.req_to_token_pool.req_to_token, forward_batch.req_pool_indices,
-                                      forward_batch.positions, self.segments, layer.window, layer.scale, self._splits(layer, T))
+                                      forward_batch.positions, self.segments, layer.window, layer.scale, self._splits(layer, T), sinks=layer.sinks)
         return kernels.head_gemm(oc, layer.w_value).view(T, layer.heads * layer.vdim)
 
     # Extends shorter than this go token by token, like decode batches; longer ones as tiles of query rows.
@@ -81,23 +93,35 @@ class HybridAttnBackend(AttentionBackend):
     def grouped_attention(self, layer, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate, run_id: int, forward_batch) -> torch.Tensor:
         """q [T, heads * kd], k [T, kv_heads * kd], v [T, kv_heads * vd] and the gate [T, heads * vd] as projected -> gated values
         [T, heads * vd].  A decode step on the matrix form stores its own keys and values on the way."""
-        rows, T = self.token_to_kv_pool.get_kv_rows(run_id), q.shape[0]
+        rows = self.token_to_kv_pool.get_kv_rows(run_id)
+        if layer.matrix and self.grouped_form != "plain" and forward_batch.forward_mode.is_decode():
+            return self._grouped(layer, q, gate, rows, (k, v, forward_batch.out_cache_loc), forward_batch)
+        kernels.grouped_kv_store(k, v, rows, forward_batch.out_cache_loc, layer.kv_heads)
+        return self._grouped(layer, q, gate, rows, None, forward_batch)
+
+    def prepared_attention(self, layer, p, run_id: int, forward_batch) -> torch.Tensor:
+        """p: the projection [queries | keys | values | gate], rows or Partials -> gated values [T, heads * vd]; one launch norms, turns and
+        stores in front of attention."""
+        rows = self.token_to_kv_pool.get_kv_rows(run_id)
+        q, gate = kernels.head_prepare(p, layer.heads, layer.dim, layer.kd, forward_batch.positions, layer.cos_sin, layer.eps, norms=layer.norms,
+                                       norm_after=layer.norm_after, gate_cols=(layer.gate_cols + 7) // 8 * 8,
+                                       kv=(layer.kv_heads, layer.vd, rows, forward_batch.out_cache_loc))
+        return self._grouped(layer, q, gate[:, :layer.gate_cols] if gate is not None else None, rows, None, forward_batch)
+
+    def _grouped(self, layer, q: torch.Tensor, gate, rows: torch.Tensor, new, forward_batch) -> torch.Tensor:
+        """Queries over the stored rows, and over the step's own keys and values `new` of a decode batch that are not stored yet."""
+        T, form = q.shape[0], self.grouped_form
+        matrix = layer.matrix and form != "plain"
         sizes = (layer.heads, layer.kv_heads, layer.kd, layer.vd, layer.window, layer.scale)
         where = (rows, self.req_to_token_pool.req_to_token, forward_batch.req_pool_indices, forward_batch.positions, self.segments)
-        matrix, form = layer.matrix and self.grouped_form != "plain", self.grouped_form
-        new = None
-        if matrix and forward_batch.forward_mode.is_decode():
-            new = (k, v, forward_batch.out_cache_loc)
-        else:
-            kernels.grouped_kv_store(k, v, rows, forward_batch.out_cache_loc, layer.kv_heads)
         if (matrix and layer.prefill and forward_batch.forward_mode.is_extend()
                 and (max(self._extend[1]) >= self.PREFILL_MIN_TOKENS if form is None else form == "prefill")):
             key = (layer.window, layer.group)
             if key not in self._blocks:
                 self._blocks[key] = kernels.QueryBlocks(*self._extend, layer.window, layer.group, self.device)
-            return kernels.grouped_prefill(q, *where, self._blocks[key], *sizes, sink=layer.sink, gate=gate)
+            return kernels.grouped_prefill(q, *where, self._blocks[key], *sizes, sink=layer.sink, gate=gate, cap=layer.cap)
         return kernels.grouped_attention(q, *where, *sizes, sink=layer.sink, gate=gate, new=new, splits=self._grouped_splits(layer, T, matrix),
-                                         plain=not matrix)
+                                         plain=not matrix, cap=layer.cap)
 
     def _grouped_splits(self, layer, tokens: int, matrix: bool) -> int:
         """Workgroups enough for the chip on small batches, never shorter than 128 keys; a function of the batch size and the context

@@ -6,7 +6,8 @@ Every module takes its tensors from `get(name, shape, init)` (harness/weights.py
 input into one product, its rows padded to a multiple of 16."""
 from __future__ import annotations
 
-from typing import Callable, List, Optional
+import math
+from typing import Callable, List, Optional, Union
 
 import torch
 from torch import nn
@@ -28,24 +29,50 @@ def conv_taps(w: torch.Tensor) -> torch.Tensor:
     return w.float().flip(1).t().contiguous()
 
 
-def rotary_table(positions: int, dims: int, base: float, device) -> torch.Tensor:
-    """fp32 cos | sin of p * base^(-2i / dims), evaluated in double so that far positions keep their angle."""
-    f = float(base) ** (-2.0 * torch.arange(dims // 2, dtype=torch.float64) / dims)
+def yarn_frequencies(f: torch.Tensor, dims: int, base: float, s: dict):
+    """The frequencies f [dims / 2] with the slow ones divided by s['factor'] (YaRN), and the factor on cos and sin.  Pairs that turn more
+    than s['fast'] times over s['original'] positions keep theirs, those below s['slow'] turns are divided, a ramp lies between."""
+    def pair(turns: float) -> float:
+        return dims * math.log(s["original"] / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+
+    lo, hi = max(math.floor(pair(s["fast"])), 0), min(math.ceil(pair(s["slow"])), dims - 1)
+    ramp = ((torch.arange(dims // 2, dtype=torch.float64) - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    return f / s["factor"] * ramp + f * (1.0 - ramp), 0.1 * math.log(s["factor"]) + 1.0
+
+
+def rotary_table(positions: int, dims: int, base: float, device, scaling: Optional[dict] = None) -> torch.Tensor:
+    """fp32 cos | sin of p * base^(-2i / dims), evaluated in double so that far positions keep their angle; `scaling` as in
+    yarn_frequencies."""
+    f, factor = float(base) ** (-2.0 * torch.arange(dims // 2, dtype=torch.float64) / dims), 1.0
+    if scaling is not None:
+        f, factor = yarn_frequencies(f, dims, float(base), scaling)
     a = torch.arange(positions, dtype=torch.float64)[:, None] * f[None, :]
-    return torch.cat([a.cos(), a.sin()], 1).to(torch.float32).contiguous().to(device)
+    return (torch.cat([a.cos(), a.sin()], 1) * factor).to(torch.float32).contiguous().to(device)
 
 
 class LatentAttention(nn.Module):
-    def __init__(self, width: int, m: dict, eps: float, get: Callable, linear: Callable, max_positions: int, device):
+    """Latent attention.  Queries come from the input and turn in neighbouring pairs, or (q_latent) through a normed latent of their own
+    (q_rank) and turn by halves; `sink`: a learned score a head in the softmax denominator."""
+
+    def __init__(self, width: int, m: dict, eps: float, get: Callable, linear: Callable, max_positions: int, device, *, q_latent: bool = False,
+                 sink: bool = False):
         super().__init__()
         self.heads, self.dim, self.rot_dim, self.vdim, self.rank = m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"]
-        self.window, self.scale, self.eps = m["mask"]["size"], float(m["scale"]), eps
+        self.window, self.scale, self.eps = (m.get("mask") or {}).get("size", 0), float(m["scale"]), eps
         dims = m["rot"]["dims"]
         if dims % 2 or dims > self.rot_dim:
             raise ValueError(f"latent attention: {dims} rotated dimensions in a rotated part of {self.rot_dim}")
         H = self.heads
         self.q_rows, self.dkv_rows = H * (self.dim + self.rot_dim), self.rank + self.rot_dim
-        self.in_proj = linear(merged_rows([get("q", (self.q_rows, width)), get("dkv", (self.dkv_rows, width))]))
+        self.q_norm = self.up_proj = None
+        if q_latent:
+            q_rank = m["q_rank"]
+            self.in_proj = linear(merged_rows([get("dq", (q_rank, width)), get("dkv", (self.dkv_rows, width))]))
+            self.q_norm = get("dq.norm", (q_rank,), "ones").float()
+            self.up_proj = linear(merged_rows([get("uq", (self.q_rows, q_rank))]))
+        else:
+            self.in_proj = linear(merged_rows([get("q", (self.q_rows, width)), get("dkv", (self.dkv_rows, width))]))
+        self.sinks = get("sink", (H,)).float() if sink else None
         self.norm_weight = get("dkv.norm", (self.rank,), "ones").float()
         uk = get("uk", (H * self.dim, self.rank))
         self.w_absorb = uk.view(H, self.dim, self.rank).transpose(1, 2).contiguous()       # [H, rank, dim]
@@ -56,13 +83,15 @@ class LatentAttention(nn.Module):
         if uv.dtype == torch.bfloat16 and self.rank % 8 == 0 and kernels.latent_prefill_supported(self.dim, self.rot_dim, self.vdim):
             self.w_expand = torch.cat([uk, uv], 0).contiguous()
         self.o_proj = linear(get("o", (width, H * self.vdim)))
-        self.cos_sin = rotary_table(max_positions, dims, m["rot"]["base"], device)
+        self.cos_sin = rotary_table(max_positions, dims, m["rot"]["base"], device, m["rot"].get("scaling"))
 
     @property
     def cache_dim(self) -> int:
         return self.rank + self.rot_dim
 
     def forward(self, h: torch.Tensor, run_id: int, fb) -> torch.Tensor:
+        if self.up_proj is not None:
+            return self.o_proj.forward_partials(fb.attn_backend.query_latent_attention(self, self.in_proj.forward_partials(h), run_id, fb))
         p = self.in_proj(h)
         o = fb.attn_backend.latent_attention(self, p[:, :self.q_rows], p[:, self.q_rows:self.q_rows + self.dkv_rows], run_id, fb)
         return self.o_proj.forward_partials(o)
@@ -79,25 +108,43 @@ def padded_heads(w: torch.Tensor, heads: int, dim: int, to: int, axis: int) -> t
 
 
 class GroupedAttention(nn.Module):
-    """Grouped-query attention without rotation: own key and value widths, an optional sliding window (mask.size), an optional sink (a
-    score in the softmax denominator that carries no value) and an optional sigmoid gate on the heads' outputs.  Head vectors are
-    padded with zeros to multiples of 8 elements, in the projections and in the cache."""
+    """Grouped-query attention: own key and value widths, an optional sliding window (mask.size), an optional soft cap of the scores
+    (softcap), an optional sink (a score in the softmax denominator that carries no value: a constant, or "learned", one a head), an
+    optional sigmoid gate on the heads' outputs ("elements", or "heads": one number each), biases on queries, keys and values,
+    rotation by halves (rot), and an RMS norm a head on queries and keys: "before" the rotation, with weights, or "after" it, without.
+    Head vectors are padded with zeros to multiples of 8 elements, in the projections and in the cache."""
 
     def __init__(self, width: int, m: dict, eps: float, get: Callable, linear: Callable, max_positions: int, device, *,
-                 sink: Optional[float] = None, gated: bool = False):
+                 sink: Union[None, float, str] = None, gate: Optional[str] = None, bias: bool = False, rotary: bool = False,
+                 qk_norm: Optional[str] = None):
         super().__init__()
         self.heads, self.kv_heads, dim, vdim = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
-        self.window, self.scale, self.sink = (m.get("mask") or {}).get("size", 0), float(m["scale"]), sink
+        self.window, self.scale, self.cap, self.eps = (m.get("mask") or {}).get("size", 0), float(m["scale"]), m.get("softcap"), eps
         H, G = self.heads, self.kv_heads
         if H % G:
             raise ValueError(f"grouped attention: {H} query heads over {G} key heads")
         self.kd, self.vd, self.group = dim + -dim % 8, vdim + -vdim % 8, H // G
-        parts = [padded_heads(get("q", (H * dim, width)), H, dim, self.kd, 0), padded_heads(get("k", (G * dim, width)), G, dim, self.kd, 0),
-                 padded_heads(get("v", (G * vdim, width)), G, vdim, self.vd, 0)]
-        if gated:
+        self.sink = get("sink", (H,)).float() if sink == "learned" else sink
+        heads = (("q", H, dim, self.kd), ("k", G, dim, self.kd), ("v", G, vdim, self.vd))
+        parts = [padded_heads(get(n, (c * d, width)), c, d, to, 0) for n, c, d, to in heads]
+        biases = [padded_heads(get(n + ".b", (c * d,), "zeros")[:, None], c, d, to, 0) for n, c, d, to in heads] if bias else []
+        self.gate_cols = {None: 0, "heads": H, "elements": H * self.vd}[gate]
+        if gate == "heads":
+            parts.append(get("g", (H, width)))
+        elif gate == "elements":
             parts.append(padded_heads(get("g", (H * vdim, width)), H, vdim, self.vd, 0))
-        self.gated = gated
-        self.in_proj = linear(merged_rows(parts))
+        if bias and gate is not None:
+            biases.append(torch.zeros_like(parts[-1][:, :1]))
+        self.in_proj = linear(merged_rows(parts), merged_rows(biases)[:, 0].contiguous()) if bias else linear(merged_rows(parts))
+        self.dim, self.cos_sin, self.norms, self.norm_after = dim, None, None, qk_norm == "after"
+        if rotary:
+            rot = m["rot"]
+            if rot["dims"] % 2 or rot["dims"] > dim:
+                raise ValueError(f"grouped attention: {rot['dims']} rotated dimensions in heads of {dim}")
+            self.cos_sin = rotary_table(max_positions, rot["dims"], rot["base"], device, rot.get("scaling"))
+        if qk_norm == "before":
+            self.norms = get("q.norm", (dim,), "ones").float(), get("k.norm", (dim,), "ones").float()
+        self.prepared = rotary or qk_norm is not None      # a launch between the projection and attention
         self.o_proj = linear(padded_heads(get("o", (width, H * vdim)), H, vdim, self.vd, 1).contiguous())
         self.matrix = self.in_proj.weight.dtype == torch.bfloat16 and self.scale > 0 and kernels.grouped_attention_matrix_form(self.kd, self.vd)
         self.prefill = self.matrix and kernels.grouped_prefill_supported(self.kd, self.vd, self.group)
@@ -107,11 +154,13 @@ class GroupedAttention(nn.Module):
         return self.kv_heads, self.kd, self.vd
 
     def forward(self, h: torch.Tensor, run_id: int, fb) -> torch.Tensor:
+        if self.prepared:
+            return self.o_proj.forward_partials(fb.attn_backend.prepared_attention(self, self.in_proj.forward_partials(h), run_id, fb))
         p = self.in_proj(h)
         a = self.heads * self.kd
         b = a + self.kv_heads * self.kd
         c = b + self.kv_heads * self.vd
-        gate = p[:, c:c + self.heads * self.vd] if self.gated else None
+        gate = p[:, c:c + self.gate_cols] if self.gate_cols else None
         return self.o_proj.forward_partials(fb.attn_backend.grouped_attention(self, p[:, :a], p[:, a:b], p[:, b:c], gate, run_id, fb))
 
 

@@ -217,6 +217,26 @@ class GroupedTokenToKVPool:
         return sum(b.numel() * b.element_size() for b in self.kv_rows), 0
 
 
+class LayeredTokenToKVPool:
+    """Cache of models whose layers keep grouped keys and values or latents, each kind with run numbers of its own, and -- for embeddings
+    that look at the token in front -- the token of every slot.  Everything is found by the slot, so it follows shared prefixes."""
+
+    is_fp8 = False
+    use_hnd = False
+
+    def __init__(self, size: int, page_size: int, dtype: torch.dtype, grouped_specs, latent_dims: List[int], device, keep_tokens: bool = False):
+        self.size, self.page_size, self.dtype, self.device = size, page_size, dtype, device
+        self.grouped = GroupedTokenToKVPool(size, page_size, dtype, grouped_specs, device)
+        self.latent = LatentTokenToKVPool(size, page_size, dtype, latent_dims, device)
+        self.layer_num = self.grouped.layer_num + self.latent.layer_num
+        self.get_kv_rows, self.get_latent_buffer = self.grouped.get_kv_rows, self.latent.get_latent_buffer
+        self.slot_ids = torch.zeros(size + page_size, dtype=torch.int32, device=device) if keep_tokens else None
+
+    def get_kv_size_bytes(self):
+        ids = self.slot_ids.numel() * 4 if self.slot_ids is not None else 0
+        return self.grouped.get_kv_size_bytes()[0] + self.latent.get_kv_size_bytes()[0] + ids, 0
+
+
 class RecurrentStatePool:
     """One slot per request row for every recurrent run: the fp32 state [slots, heads, rows, columns] and the ring of past
     convolution inputs [slots, taps, channels] in the activation type.  Slot 0 absorbs padded (graph) batch entries.  A
