@@ -1,4 +1,4 @@
-"""Throughput of the layered designs (Genusun here, Mosurax with grouped_bench.py) beside the closest decoders of this framework at
+"""Throughput of the layered designs (Genusun here, Mosurax with grouped_bench.py, Bulodra with layered_bench.py) beside the closest decoders of this framework at
 equal size, and every kernel of a design against its roofline beside the like kernel of such a decoder.  Run through
 `bench.py --hybrid`; random weights.
 
@@ -8,6 +8,7 @@ kernel table (us, fraction of the roofline: 8 TB/s HBM, 2.5 PFLOP/s bf16, 157 TF
 from __future__ import annotations
 
 import json
+import sys
 import time
 
 import torch
@@ -234,20 +235,24 @@ def kernel_table(cfg, device, T=8192, segs=4, B=64, ctx=1024):
 
 
 def run(names, device, kernels_only=False):
-    from benchmarks import grouped_bench
+    from benchmarks import grouped_bench, layered_bench
+    from sglang_amd.harness.bulodra import BulodraConfig
     from sglang_amd.harness.mosurax import MosuraxConfig
     from sglang_amd.harness.registry import named_config
 
     out = {}
     for name in names:
         cfg = named_config(name)
-        grouped = isinstance(cfg, MosuraxConfig)
+        key, table, beside = (("design", layered_bench.kernel_table, layered_bench.models_beside) if isinstance(cfg, BulodraConfig) else
+                              ("design", grouped_bench.kernel_table, grouped_bench.decoders_beside) if isinstance(cfg, MosuraxConfig) else
+                              ("hybrid", kernel_table, lambda c: {"decoder_beside": _llama_beside(c)}))
         shape = dict(prompts=4, length=2048, batch=64, ctx=1024)
-        r = dict(shape=shape, kernels=(grouped_bench.kernel_table if grouped else kernel_table)(cfg, device))
+        r = dict(shape=shape, kernels=table(cfg, device))
         torch.cuda.empty_cache()
+        print(f"{name}: kernel table done", file=sys.stderr, flush=True)
         if not kernels_only:
-            r["design" if grouped else "hybrid"] = throughput(cfg, device, **shape)
-            for key, beside in (grouped_bench.decoders_beside(cfg) if grouped else {"decoder_beside": _llama_beside(cfg)}).items():
-                r[key] = throughput(beside, device, **shape)
+            for other, c in {key: cfg, **beside(cfg)}.items():
+                r[other] = throughput(c, device, **shape)
+                print(f"{name}: throughput of {other} done", file=sys.stderr, flush=True)
         out[name] = r
     print(json.dumps({"hybrid": out, "dtype": "bf16", "data": "synthetic (random weights and tokens)"}), flush=True)

@@ -646,7 +646,7 @@ int sgl_amd_latent_prefill(const void* q, int64_t q_token, const void* latents, 
  * row_stride apart, plus `bias` in the activation type).  cos_sin fp32 [max_positions, rot_dims] = cos | sin; dimension i of the rotated
  * part turns with i + rot_dims / 2.
  * sgl_amd_head_prepare: columns [heads * kd queries | kv_heads * kd keys | kv_heads * vd values | gate].  norm_order 1: RMS norm over `dim`
- * elements with q_norm / k_norm, then rotation of [rot_off, rot_off + rot_dims); 2: rotation, then the norm without weights; 0: rotation alone.
+ * elements with q_norm / k_norm [kd], then rotation of [rot_off, rot_off + rot_dims); 2: rotation, then the norm without weights; 0: rotation alone.
  * Queries go to `out` (which may be the source rows), the gate columns behind them (gate_cols > 0), keys and values to cache rows
  * `loc`, [kv_heads][kd | vd].  `plain` forces the form for any sizes.
  * sgl_amd_latent_down: columns [q_rank query latent | rank latent | rot rotated key part] -> cq = RMS norm of the first, cache row `loc` =

@@ -192,3 +192,92 @@ def forward(cfg: dict, weights: Dict[str, torch.Tensor], tokens: List[int], dtyp
             x = x + m * oh.rms_norm(moe_mlp(h, sub, f) if f["kind"] == "moe" else gelu_mlp(h, sub), w[p + "norm2"], eps)
         trace.append(x)
     return oh.linear(oh._r(oh.rms_norm(x, w["final.norm"], eps)), w["head"]) * cfg["logit_scale"], trace
+
+
+# ---------------------------------------------------------------------------------------------- random models
+def tensor_shapes(cfg: dict) -> Dict[str, Tuple[int, ...]]:
+    W = cfg["width"]
+    out: Dict[str, Tuple[int, ...]] = {"embed": (cfg["vocab"], W), "bigram": (cfg["embedding"]["bigram"]["buckets"] + 1, W), "head": (cfg["vocab"], W),
+                                       "final.norm": (W,)}
+
+    def mlp(prefix, ff):
+        out.update({prefix + "gate": (ff, W), prefix + "up": (ff, W), prefix + "down": (W, ff)})
+
+    for i, lay in enumerate(cfg["layers"]):
+        m, f, p = lay["mixer"], lay["mlp"], f"l{i}."
+        H, D, V = m["heads"], m["dim"], m["vdim"]
+        out[p + "norm1"] = (W,)
+        mix = {"o": (W, H * V)}
+        if lay["type"] == "latent_attention":
+            R, K, Q = m["rot_dim"], m["kv_rank"], m["q_rank"]
+            mix.update({"dq": (Q, W), "dq.norm": (Q,), "uq": (H * (D + R), Q), "dkv": (K + R, W), "dkv.norm": (K,), "uk": (H * D, K), "uv": (H * V, K), "sink": (H,)})
+        else:
+            G = m["kv_heads"]
+            mix.update({"q": (H * D, W), "k": (G * D, W), "v": (G * V, W)})
+            if lay["type"] == "attention":
+                mix.update({"q.b": (H * D,), "k.b": (G * D,), "v.b": (G * V,), "q.norm": (D,), "k.norm": (D,), "sink": (H,)})
+            else:
+                mix["g"] = (H, W)
+        out.update({p + "mix." + n: s for n, s in mix.items()})
+        if f is None:
+            continue
+        out[p + "norm2"] = (W,)
+        if f["kind"] == "dense":
+            mlp(p + "mlp.", f["ff"])
+            continue
+        for e in range(f["router"]["experts"]):
+            mlp(f"{p}mlp.e{e}.", f["expert"]["ff"])
+        out[p + "mlp.router"], out[p + "mlp.correction"] = (f["router"]["experts"], W), (f["router"]["experts"],)
+        if f.get("shared"):
+            mlp(p + "mlp.shared.", f["shared"]["ff"])
+    return out
+
+
+CODE_DIMS, CODES = 8, 12
+
+
+def random_weights(cfg: dict, seed: int) -> Dict[str, torch.Tensor]:
+    """bf16 weights whose every branch matters: matrices keep unit variance, norms spread around 1, sinks and biases are of the size of
+    scores and activations, corrections reach below zero.  No token sits between two experts: the first CODE_DIMS columns of the
+    embedding hold one of CODES sign patterns, nothing else writes to those columns of the residual, and the routers read only
+    them, drawn until every pattern's choice of groups and experts is clear."""
+    g = torch.Generator().manual_seed(seed)
+    code = torch.randint(0, 2, (CODES, CODE_DIMS), generator=g) * 4.0 - 2.0
+    shapes, out = tensor_shapes(cfg), {}
+    for name, shape in shapes.items():
+        r = torch.randn(shape, generator=g)
+        last = name.split(".")[-1]
+        if last in ("norm1", "norm2", "norm"):
+            t = 1.0 + 0.2 * r
+        elif last in ("embed", "bigram", "sink"):
+            t = r
+        elif last in ("b", "correction"):
+            t = r * 0.5
+        else:
+            t = r / math.sqrt(shape[1])
+        if last == "embed":
+            t[:, :CODE_DIMS] = code[torch.arange(shape[0]) % CODES]
+        elif last == "bigram":
+            t[:, :CODE_DIMS] = 0.0
+        elif last in ("norm1", "norm2"):
+            t[:CODE_DIMS] = 0.0
+        out[name] = t.to(torch.bfloat16)
+    saved = list(margins)
+    for i, lay in enumerate(cfg["layers"]):
+        if lay["mlp"] is None or lay["mlp"]["kind"] != "moe":
+            continue
+        name, best = f"l{i}.mlp.router", None
+        for _ in range(200):
+            w = torch.zeros(shapes[name])
+            w[:, :CODE_DIMS] = torch.randn((shapes[name][0], CODE_DIMS), generator=g) * 0.3
+            w = w.to(torch.bfloat16)
+            margins.clear()
+            route(code.double(), w[:, :CODE_DIMS].double(), out[f"l{i}.mlp.correction"].double(), lay["mlp"]["router"])
+            gap = min(margins, default=1.0)
+            if best is None or gap > best[0]:
+                best = (gap, w)
+            if gap > 0.02:
+                break
+        out[name] = best[1]
+    margins[:] = saved
+    return out

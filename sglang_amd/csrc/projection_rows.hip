@@ -54,7 +54,7 @@ struct HeadPrepareParams {
   ProjRows src;
   void* out;                 // [tokens, heads * kd (| gate columns of partials)]; may be the source's rows
   int64_t o_stride;
-  const float *q_norm, *k_norm;      // [dim], order 1
+  const float *q_norm, *k_norm;      // [kd], order 1
   const float* cos_sin;      // [positions, rot_dims]: cos | sin, or null
   int64_t max_pos;
   const int64_t* positions;
@@ -63,6 +63,7 @@ struct HeadPrepareParams {
   const int64_t* loc;
   int64_t tokens;
   int heads, kv_heads, kd, vd, dim, rot_off, rot_dims, norm_order, gate_cols, units, in_place;
+  int q_off, q_width;        // the columns of a query head this launch touches
   float eps;
 };
 
@@ -73,7 +74,7 @@ struct HeadUnit {
 
 __device__ __forceinline__ HeadUnit head_unit(const HeadPrepareParams& p, int u, int gate_piece) {
   const int H = p.heads, G = p.kv_heads;
-  if (u < H) return {0, p.kd, static_cast<int64_t>(u) * p.kd, static_cast<int64_t>(u) * p.kd};
+  if (u < H) return {0, p.q_width, static_cast<int64_t>(u) * p.kd + p.q_off, static_cast<int64_t>(u) * p.kd + p.q_off};
   const int64_t k0 = static_cast<int64_t>(H) * p.kd, v0 = k0 + static_cast<int64_t>(G) * p.kd, g0 = v0 + static_cast<int64_t>(G) * p.vd;
   u -= H;
   if (u < G) return {1, p.kd, k0 + static_cast<int64_t>(u) * p.kd, static_cast<int64_t>(u) * (p.kd + p.vd)};
@@ -105,7 +106,7 @@ __global__ __launch_bounds__(256) void head_prepare_kernel(HeadPrepareParams p) 
   const int lane = threadIdx.x & 63, c = static_cast<int>(threadIdx.x % TPH) * 8;
   const int half = p.rot_dims >> 1, r = c - p.rot_off;
   const bool head = u.kind < 2, turns = head && p.cos_sin && r >= 0 && r < p.rot_dims;
-  const bool active = live && c < u.width && !(p.in_place && u.kind == 0 && !p.norm_order && !turns);
+  const bool active = live && c < u.width;
   float v[8];
 #pragma unroll
   for (int j = 0; j < 8; ++j) v[j] = 0.f;
@@ -122,8 +123,10 @@ __global__ __launch_bounds__(256) void head_prepare_kernel(HeadPrepareParams p) 
     const float rs = unit_scale();
     if (head) {
       const float* w = u.kind == 0 ? p.q_norm : p.k_norm;
+      float wv[8];
+      ldv<8>(w + (active ? c : 0), wv);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) v[j] *= c + j < p.dim ? rs * w[c + j] : 0.f;
+      for (int j = 0; j < 8; ++j) v[j] *= rs * wv[j];
     }
   }
   if (p.cos_sin) {
@@ -176,7 +179,7 @@ __global__ __launch_bounds__(256) void head_prepare_plain_kernel(HeadPreparePara
   const float* w = u.kind == 0 ? p.q_norm : p.k_norm;
   const float* cs = p.cos_sin && head ? rotation(p, t) : nullptr;
   const int half = p.rot_dims >> 1;
-  auto at = [&](int c) { return head && p.norm_order == 1 ? (c < p.dim ? x[c] * before * w[c] : 0.f) : x[c]; };
+  auto at = [&](int c) { return head && p.norm_order == 1 ? x[c] * before * w[c] : x[c]; };
   auto turned = [&](int c) {
     const int r = c - p.rot_off;
     if (!cs || r < 0 || r >= p.rot_dims) return at(c);
@@ -261,7 +264,12 @@ bool source_vec(const ProjRows& s, int vec, size_t bytes) {
 template <typename T>
 void launch_head_prepare(const HeadPrepareParams& p0, bool vec, hipStream_t st) {
   HeadPrepareParams p = p0;
-  const int widest = p.kv_heads && p.vd > p.kd ? p.vd : p.kd, plain_units = p.heads + 2 * p.kv_heads;
+  p.q_off = 0; p.q_width = p.kd;
+  if (p.in_place && !p.norm_order && !p.kv_heads && !p.gate_cols) {            // nothing but the turned columns changes
+    if (!p.rot_dims) return;
+    p.q_off = p.rot_off; p.q_width = p.rot_dims; p.rot_off = 0;
+  }
+  const int widest = p.kv_heads && p.vd > p.q_width ? p.vd : p.q_width, plain_units = p.heads + 2 * p.kv_heads;
   if (vec && widest <= 512) {
     const int tph = widest <= 64 ? 8 : widest <= 128 ? 16 : widest <= 256 ? 32 : 64;
     p.units = plain_units + (p.gate_cols + tph * 8 - 1) / (tph * 8);
@@ -303,7 +311,8 @@ int sgl_amd_head_prepare(int is_f32, const void* rows, int64_t row_stride, const
   p.in_place = !partials && out == rows; p.eps = eps;
   SGL_CHECK_ARG(!p.in_place || o_stride == row_stride, "head_prepare: in place with another row stride");
   const bool vec = !plain && kd % 8 == 0 && (!kv_heads || vd % 8 == 0) && gate_cols % 8 == 0 && p.rot_dims % 16 == 0 && rot_off % 8 == 0 &&
-                   source_vec(p.src, 8, 16) && o_stride % 8 == 0 && cache_stride % 8 == 0 && aligned_to(out, 16) && aligned_to(cache, 16) && aligned_to(cos_sin, 16);
+                   source_vec(p.src, 8, 16) && o_stride % 8 == 0 && cache_stride % 8 == 0 && aligned_to(out, 16) && aligned_to(cache, 16) && aligned_to(cos_sin, 16) &&
+                   aligned_to(q_norm, 16) && aligned_to(k_norm, 16);
   if (is_f32) launch_head_prepare<float>(p, vec, as_stream(stream));
   else launch_head_prepare<uint16_t>(p, vec, as_stream(stream));
   SGL_CHECK_LAUNCH("head_prepare");

@@ -1632,7 +1632,7 @@ def head_prepare(p, heads: int, dim: int, kd: int, positions: torch.Tensor, cos_
                  norms: Optional[Tuple[torch.Tensor, torch.Tensor]] = None, norm_after: bool = False, gate_cols: int = 0,
                  kv: Optional[Tuple[int, int, torch.Tensor, torch.Tensor]] = None, plain: bool = False):
     """Query heads [T, heads * kd] (and the gate columns [T, gate_cols], or None) of a projection p -- rows, changed in place, or Partials --
-    behind an RMS norm a head over `dim` elements (norms = (query weight, key weight): in front of the rotation; norm_after: behind it,
+    behind an RMS norm a head over `dim` elements (norms = (query weight, key weight) [kd]: in front of the rotation; norm_after: behind it,
     without weights) and the rotation by halves of [rot_off, + cos_sin.shape[1]).  kv = (kv_heads, vd, cache, loc): keys, treated alike, and
     values go to the cache rows."""
     G, vd, cache, loc = kv if kv is not None else (0, 0, None, None)
@@ -1643,7 +1643,7 @@ def head_prepare(p, heads: int, dim: int, kd: int, positions: torch.Tensor, cos_
     _dev(positions, cos_sin, cache, loc, *(norms or ()))
     _i64("head_prepare", positions, loc)
     _f32("head_prepare", cos_sin, *(norms or ()))
-    _need(positions.numel() == T and (loc is None or loc.numel() == T) and all(w.numel() == dim for w in norms or ()), "head_prepare: shapes")
+    _need(positions.numel() == T and (loc is None or loc.numel() == T) and all(w.numel() == kd for w in norms or ()), "head_prepare: shapes")
     _need(cache is None or (_is_f32(cache) == f32 and cache.shape[1] >= G * (kd + vd) and cache.stride(1) == 1), "head_prepare: cache rows")
     _need(bias is None or bias.dtype == _BF16, "head_prepare: the partials' bias is bf16")
     out = p if part is None else torch.empty((T, heads * kd + gate_cols), dtype=_BF16, device=positions.device)

@@ -143,7 +143,7 @@ class GroupedAttention(nn.Module):
                 raise ValueError(f"grouped attention: {rot['dims']} rotated dimensions in heads of {dim}")
             self.cos_sin = rotary_table(max_positions, rot["dims"], rot["base"], device, rot.get("scaling"))
         if qk_norm == "before":
-            self.norms = get("q.norm", (dim,), "ones").float(), get("k.norm", (dim,), "ones").float()
+            self.norms = tuple(padded_heads(get(n, (dim,), "ones").float(), 1, dim, self.kd, 0) for n in ("q.norm", "k.norm"))
         self.prepared = rotary or qk_norm is not None      # a launch between the projection and attention
         self.o_proj = linear(padded_heads(get("o", (width, H * vdim)), H, vdim, self.vd, 1).contiguous())
         self.matrix = self.in_proj.weight.dtype == torch.bfloat16 and self.scale > 0 and kernels.grouped_attention_matrix_form(self.kd, self.vd)

@@ -21,15 +21,17 @@ def _rel(got, want):
 
 
 # ---------------------------------------------------------------------------------------------- attention
-def _attend(q, k, v, pos, window, scale, sink, gate):
-    """q [n, H, D] at positions pos over k [L, G, D], v [L, G, V] in float64; gate [n, H, V] or None."""
+def _attend(q, k, v, pos, window, scale, sink, gate, cap=None):
+    """q [n, H, D] at positions pos over k [L, G, D], v [L, G, V] in float64; gate [n, H, V], [n, H, 1] or None; sink a number, [H] or None."""
     per = q.shape[1] // k.shape[1]
     s = torch.einsum("nhd,lhd->hnl", q, k.repeat_interleave(per, 1)) * scale
     j = torch.arange(k.shape[0])[None, :]
     seen = (j <= pos[:, None]) & ((pos[:, None] - j < window) if window > 0 else True)
+    if cap is not None:
+        s = cap * torch.tanh(s / cap)
     s = s.masked_fill(~seen[None], float("-inf"))
     if sink is not None:
-        s = torch.cat([torch.full_like(s[..., :1], sink), s], -1)
+        s = torch.cat([torch.as_tensor(sink, dtype=s.dtype).reshape(-1, 1, 1).expand_as(s[..., :1]), s], -1)
     p = torch.softmax(s, -1)[..., (0 if sink is None else 1):]
     o = torch.einsum("hnl,lhv->nhv", p, v.repeat_interleave(per, 1))
     return o if gate is None else o * torch.sigmoid(gate)
@@ -79,16 +81,19 @@ class _Case:
         self.seg = K.Segments(torch.repeat_interleave(torch.arange(len(lens), dtype=torch.int32), n.long()).to(device),
                               (torch.cumsum(n, 0) - n).int().to(device), n.to(device), int(n.max()))
 
-    def want(self, window, scale, sink, gated):
-        return torch.cat([_attend(q.double(), k.double(), v.double(), pos, window, scale, sink, g.double() if gated else None)
+    def want(self, window, scale, sink, gated, cap=None):
+        """gated: True, False, or "heads" (the first column of every head's gates is the head's)."""
+        return torch.cat([_attend(q.double(), k.double(), v.double(), pos, window, scale, sink,
+                                  None if not gated else g.double()[..., :1] if gated == "heads" else g.double(), cap)
                           for q, k, v, pos, g in zip(self.qs, self.ks, self.vs, self.pos_list, self.gates)]).flatten(1)
 
-    def run(self, form, window, scale, sink, gated, splits=1):
+    def run(self, form, window, scale, sink, gated, splits=1, cap=None):
         from sglang_amd import kernels as K
 
         sizes = (self.H, self.G, self.D, self.V, window, scale)
         where = (self.rows, self.r2t, self.req, self.pos, self.seg)
-        kw = dict(sink=sink, gate=self.gate if gated else None)
+        gate = self.gate.view(-1, self.H, self.V)[:, :, 0].contiguous() if gated == "heads" else self.gate if gated else None
+        kw = dict(sink=sink.float().to(self.q.device) if isinstance(sink, torch.Tensor) else sink, gate=gate, cap=cap)
         if form == "prefill":
             blocks = K.QueryBlocks([p for p, _ in self.lens], [n for _, n in self.lens], window, self.H // self.G, self.q.device)
             return K.grouped_prefill(self.q, *where, blocks, *sizes, **kw)
