@@ -140,3 +140,12 @@ def test_grouped_attention_kernels_keep_their_sums_in_registers(tmp_path):
     for name, u in _resource_usage("residual_norm.hip", tmp_path).items():
         if "residual_rms_kernel" in name:
             assert u["vgpr_spill_count"] == 0, (name, u)
+
+
+@pytest.mark.skipif(not Path(HIPCC).exists(), reason="hipcc not installed")
+def test_projection_row_kernels_do_not_spill(tmp_path):
+    """Rows, rotation partners and four partials in flight stay in registers; none of these launches asks for scratch."""
+    usage = _resource_usage("projection_rows.hip", tmp_path)
+    assert sum("head_prepare_kernel" in k for k in usage) == 8 and sum("latent_down_kernel" in k for k in usage) == 4, sorted(usage)
+    for name, u in usage.items():
+        assert u["vgpr_spill_count"] == 0 and u["sgpr_spill_count"] == 0 and u["vgpr_count"] <= 128, (name, u)
