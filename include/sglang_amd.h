@@ -66,7 +66,8 @@ int sgl_amd_fused_add_rmsnorm(void* x, void* residual, const void* weight, int64
 int sgl_amd_silu_and_mul(const void* in, void* out, int64_t num_rows, int d, int64_t in_row_stride,
                          int64_t out_row_stride, int round_intermediate, void* stream);
 /* The same with any gated activation, in fp32.  glu_kind: 1 = silu(g) u; 2 = gelu_tanh(g) u; 3 = g' sigmoid(glu_alpha g') (u' + 1) with
- * g' = min(g, glu_limit) and u' = u clamped to +- glu_limit.  Every function with these three parameters uses them so. */
+ * g' = min(g, glu_limit) and u' = u clamped to +- glu_limit.  Every function with these three parameters uses them so; the products also take
+ * 4 = relu(u)^2, which has no gate: their weights then are plain rows. */
 int sgl_amd_glu_and_mul(const void* in, void* out, int64_t num_rows, int d, int64_t in_row_stride, int64_t out_row_stride, int glu_kind,
                         float glu_limit, float glu_alpha, void* stream);
 
@@ -332,7 +333,8 @@ int sgl_amd_wstream_gemm(const void* x, const void* w, const void* bias, void* y
                          int64_t y_row_stride, int64_t y_chunk_stride, int epilogue, void* residual,
                          int64_t residual_row_stride, const void* norm_weight, float eps, int waves_per_group,
                          int tiles_per_wave, int num_k_splits, void* ws_partials, void* stream);
-/* epilogue 1 with another activation of the [gate | up] columns (kinds 2, 3: in fp32 up to the final rounding) */
+/* epilogue 1 with another activation of the [gate | up] columns (kinds 2, 3: in fp32 up to the final rounding); kind 4: epilogue 0 with
+ * the activation of y's own columns */
 int sgl_amd_wstream_glu_gemm(const void* x, const void* w, const void* bias, void* y, int64_t M, int64_t N, int64_t K,
                              int64_t x_row_stride, int64_t x_chunk_stride, int64_t w_row_stride, int64_t y_row_stride,
                              int64_t y_chunk_stride, int glu_kind, float glu_limit, float glu_alpha, int waves_per_group,
@@ -355,8 +357,8 @@ int sgl_amd_wstream_qkv_rope(const void* x, const void* w_qkv, const void* bias,
                              int num_k_splits, void* ws_partials, void* stream);
 /* Grouped (mixture-of-experts) form of the weight-streaming GEMM, same contract as sgl_amd_moe_grouped_gemm
  * (fused_moe_triton_kernels.py:324,771) for shapes with N % 16 == 0 and K % 128 == 0, without split-K: one
- * workgroup per (row block of moe_align_block_size, group of weight tiles of that block's expert).  glu_kind > 0:
- * w is [E, 2N, K] and c[id, :N] = the activation of gate and up; otherwise c[id, :] = a[id / top_k_div] . w[e]^T, optionally
+ * workgroup per (row block of moe_align_block_size, group of weight tiles of that block's expert).  glu_kind 1 .. 3:
+ * w is [E, 2N, K] and c[id, :N] = the activation of gate and up; otherwise (4: through the activation) c[id, :] = a[id / top_k_div] . w[e]^T, optionally
  * rounded to bf16 and scaled by topk_weights[id], written bf16 or fp32 (out_f32). */
 int sgl_amd_wstream_moe_gemm(const void* a, const void* w, void* c, const int32_t* sorted_token_ids,
                              const int32_t* expert_ids, const int32_t* num_tokens_post_padded,
@@ -551,27 +553,32 @@ int sgl_amd_moe_tiled_gemm_ex(const void* a, const void* w, void* c, const int32
  * sgl_amd_wstream_gemm) instead of rows.  Then, when `h` is given, h = LayerNorm(x; w2, b2); copy0 / copy1 (optional) receive x in the activation
  * type.  x and all norm parameters are fp32; y, h, table and the copies are bf16, or fp32 with is_f32.
  * sgl_amd_gated_rmsnorm: per (row, group of group_size columns): gate_first ? rms(y * silu(gate)) * w : rms(y) * w * silu(gate);
- * w is [groups * group_size], or [group_size] with shared_weight.
- * sgl_amd_gate_mul: out = activation(gate, up), rows of `d` at the given strides. */
+ * w is [groups * group_size], or [group_size] with shared_weight; gate_sigmoid: sigmoid(gate) in the place of silu(gate).
+ * sgl_amd_gate_mul: out = activation(gate, up), rows of `d` at the given strides.  sgl_amd_squared_relu: out = relu(in)^2, may be in place. */
 int sgl_amd_residual_norm(int is_f32, int mode, const int64_t* ids, const void* table, int64_t vocab, float scale, const void* y,
     int64_t y_stride, const float* partials, int splits, const void* partials_bias, const float* step, const float* w1, const float* b1, float* x, int64_t x_stride,
     const float* w2, const float* b2, void* h, int64_t h_stride, void* copy0, void* copy1, int64_t copy_stride,
     int64_t rows, int width, float eps, void* stream);
 int sgl_amd_gated_rmsnorm(int is_f32, const void* y, int64_t y_stride, const void* gate, int64_t gate_stride, const float* weight,
     void* out, int64_t out_stride, int64_t rows, int groups, int group_size, int gate_first, int shared_weight,
-    float eps, void* stream);
+    int gate_sigmoid, float eps, void* stream);
 int sgl_amd_gate_mul(int is_f32, const void* gate, const void* up, void* out, int64_t rows, int d, int64_t in_stride, int64_t out_stride,
     int glu_kind, float glu_limit, float glu_alpha, void* stream);
+int sgl_amd_squared_relu(int is_f32, const void* in, void* out, int64_t rows, int d, int64_t in_stride, int64_t out_stride, void* stream);
 /* Residual row of pre-norm designs, fp32: x <- table[ids] * scale (+ pos_table[positions]), or x + a + b, each source the sum of
- * its items [rows x items x width] (times fp32 weight [rows, items] if given) in fp32 or in the activation type; then the copy
+ * its items [rows x items x width] (times the fp32 weight at row * weight_row + item * weight_item if given) in fp32 or in the activation
+ * type (an item of a with a negative id in a_ids [rows, items] is the row of a_alt instead), plus bias [width] if given; then the copy
  * `save`, then + extra (rows) + step (vector), then h = RMS norm(x) * weight (null: h = x).  With `post` (designs that norm a sublayer's
- * output) x <- x + mult * (RMS norm(a + b) * post).  save / extra rows are contiguous. */
+ * output) x <- x + mult * (RMS norm(a + b) * post).  save / extra rows are contiguous.  shift [width]: h blends with what its slot of
+ * shift_state [slots, width] (activation type) holds (position 0: zeros), h + (left - h) * shift, and leaves the norm there. */
 int sgl_amd_residual_rms(int is_f32, const int64_t* ids, const void* table, int64_t vocab, float scale, const int64_t* positions,
     const void* pos_table, int64_t max_positions, const void* a, int a_f32, int a_items, int64_t a_row_stride,
     int64_t a_item_stride, const float* a_weight, const void* b, int b_f32, int b_items, int64_t b_row_stride,
     int64_t b_item_stride, const float* b_weight, float* x, int64_t x_stride, float* save, const float* extra,
     const float* step, const float* post, float mult, const float* weight, void* h, int64_t h_stride, int64_t rows, int width, float eps,
-    void* stream);
+    int64_t a_weight_row, int64_t a_weight_item, const int32_t* a_ids, const void* a_alt, int64_t a_alt_stride, int64_t b_weight_row,
+    int64_t b_weight_item, const float* bias, const float* shift, void* shift_state, const int64_t* shift_slots,
+    const int64_t* shift_positions, void* stream);
 /* cap * tanh(z / cap) -> fp32 [rows, cols] contiguous; z: `items` addends item_stride apart (split-K partials) */
 int sgl_amd_soft_cap(int is_f32, const void* z, int64_t z_row_stride, int items, int64_t item_stride, float* out, int64_t rows, int cols,
     float cap, void* stream);
@@ -584,7 +591,11 @@ int sgl_amd_soft_cap(int is_f32, const void* z, int64_t z_row_stride, int items,
  * sgl_amd_mamba2_step: xbc = convolved [x: heads * head_dim | B: groups * state_dim | C: groups * state_dim]; state fp32
  * [slots, heads, state_dim, head_dim]; y includes the D * x term.
  * sgl_amd_delta_step: qkv = convolved [q: kv_heads * key_dim | k | v: heads * value_dim]; state fp32
- * [slots, heads, key_dim, value_dim]; q and k are made unit vectors inside, q times q_scale. */
+ * [slots, heads, key_dim, value_dim]; q and k are made unit vectors inside, q times q_scale.
+ * sgl_amd_memory_step: q, k, v and the gates are columns of one row (one stride).  Log gates i = cap tanh((gate_i + bias_i) / cap) and
+ * f = log sigmoid(cap tanh((gate_f + bias_f) / cap)); state fp32 [slots, heads, key_dim, value_dim] and norm fp32 [slots, heads,
+ * ceil(value_dim / 16), key_dim + 1] (the sum of the keys and the running maximum, a copy per 16 value columns); q times q_scale.
+ * sgl_amd_token_shift: out[t] = h[t] + (h one token ago - h[t]) * mu; state [slots, width] holds every request's last row. */
 int sgl_amd_causal_conv_silu(int is_f32, const void* x, int64_t x_stride, const float* weight, const float* bias, void* state,
     const int64_t* slots, const int64_t* positions, const int32_t* tok_seg, const int32_t* seg_start,
     const int32_t* seg_len, void* out, int64_t out_stride, int64_t tokens, int segments, int channels,
@@ -597,6 +608,13 @@ int sgl_amd_delta_step(int is_f32, const void* qkv, int64_t qkv_stride, const vo
     const float* A_log, const float* dt_bias, float* state, const int64_t* slots, const int64_t* positions,
     const int32_t* seg_start, const int32_t* seg_len, void* o, int64_t o_stride, int segments, int heads, int kv_heads,
     int key_dim, int value_dim, float q_scale, void* stream);
+int sgl_amd_memory_step(int is_f32, const void* q, const void* k, const void* v, const void* gate_i, const void* gate_f, int64_t stride,
+    const float* bias_i, const float* bias_f, float* state, float* norm, const int64_t* slots, const int64_t* positions,
+    const int32_t* seg_start, const int32_t* seg_len, void* o, int64_t o_stride, int segments, int heads, int key_dim,
+    int value_dim, float gate_cap, float q_scale, void* stream);
+int sgl_amd_token_shift(int is_f32, const void* h, int64_t h_stride, const float* mu, void* state, const int64_t* slots, const int64_t* positions,
+    const int32_t* tok_seg, const int32_t* seg_start, const int32_t* seg_len, void* out, int64_t out_stride, int64_t tokens,
+    int width, void* stream);
 
 /* ---- the same recurrences in chunks of 32 tokens on fp32 matrix instructions (recurrent_chunk.hip) -----------------
  * Operands as in the token-by-token forms; segments are required, state_dim / key_dim up to sgl_amd_recurrent_chunk_max_state().
@@ -606,6 +624,10 @@ int sgl_amd_mamba2_chunk(int is_f32, const void* xbc, int64_t xbc_stride, const 
     const float* dt_bias, const float* D, float* state, const int64_t* slots, const int64_t* positions,
     const int32_t* seg_start, const int32_t* seg_len, void* y, int64_t y_stride, int segments, int heads, int head_dim,
     int state_dim, int groups, void* stream);
+int sgl_amd_memory_chunk(int is_f32, const void* q, const void* k, const void* v, const void* gate_i, const void* gate_f, int64_t stride,
+    const float* bias_i, const float* bias_f, float* state, float* norm, const int64_t* slots, const int64_t* positions,
+    const int32_t* seg_start, const int32_t* seg_len, void* o, int64_t o_stride, int segments, int heads, int key_dim,
+    int value_dim, float gate_cap, float q_scale, void* stream);
 int sgl_amd_delta_chunk(int is_f32, const void* qkv, int64_t qkv_stride, const void* b, const void* a, int64_t ba_stride,
     const float* A_log, const float* dt_bias, float* state, const int64_t* slots, const int64_t* positions,
     const int32_t* seg_start, const int32_t* seg_len, void* o, int64_t o_stride, int segments, int heads, int kv_heads,
@@ -648,7 +670,8 @@ int sgl_amd_latent_prefill(const void* q, int64_t q_token, const void* latents, 
  * sgl_amd_head_prepare: columns [heads * kd queries | kv_heads * kd keys | kv_heads * vd values | gate].  norm_order 1: RMS norm over `dim`
  * elements with q_norm / k_norm [kd], then rotation of [rot_off, rot_off + rot_dims); 2: rotation, then the norm without weights; 0: rotation alone.
  * Queries go to `out` (which may be the source rows), the gate columns behind them (gate_cols > 0), keys and values to cache rows
- * `loc`, [kv_heads][kd | vd].  `plain` forces the form for any sizes.
+ * `loc`, [kv_heads][kd | vd].  value_is_key: no value columns, the cached values are the key columns as they are in the source.  `plain`
+ * forces the form for any sizes.
  * sgl_amd_latent_down: columns [q_rank query latent | rank latent | rot rotated key part] -> cq = RMS norm of the first, cache row `loc` =
  * [RMS norm of the second | rotated third].
  * sgl_amd_bigram_rows: rows[t] = (prev * mul_prev + ids[t] * mul_cur) mod buckets, `buckets` at position 0; prev is the token in front of t
@@ -656,7 +679,7 @@ int sgl_amd_latent_prefill(const void* q, int64_t q_token, const void* latents, 
 int sgl_amd_head_prepare(int is_f32, const void* rows, int64_t row_stride, const float* partials, int items, int64_t item_stride, const void* bias,
     void* out, int64_t o_stride, const float* q_norm, const float* k_norm, int norm_order, float eps, const float* cos_sin,
     int64_t max_positions, const int64_t* positions, int rot_off, int rot_dims, void* cache, int64_t cache_stride,
-    const int64_t* loc, int64_t tokens, int heads, int kv_heads, int kd, int vd, int dim, int gate_cols, int plain, void* stream);
+    const int64_t* loc, int64_t tokens, int heads, int kv_heads, int kd, int vd, int dim, int gate_cols, int value_is_key, int plain, void* stream);
 int sgl_amd_latent_down(int is_f32, const void* rows, int64_t row_stride, const float* partials, int items, int64_t item_stride,
     const float* q_norm, const float* norm, float eps, const float* cos_sin, int64_t max_positions, const int64_t* positions, int rot_dims,
     void* cq, int64_t cq_stride, void* cache, int64_t cache_stride, const int64_t* loc, int64_t tokens, int q_rank, int rank, int rot,
@@ -669,7 +692,8 @@ int sgl_amd_bigram_rows(const int64_t* ids, const int64_t* positions, const int6
  * Cache rows [kv_heads][kd | vd] (kd, vd multiples of 8, one row stride); query head h reads key head h / (heads / kv_heads); position
  * i sees the `window` positions up to and with itself (window <= 0: all); `sink` joins the softmax denominator as a score without
  * a value (-inf: none), `sinks` [heads] instead of it one a head; cap > 0 makes scores cap * tanh(score / cap); the output is multiplied by
- * sigmoid(gate) when a gate is given: [tokens, heads * vd], or [tokens, heads] with gate_per_head.
+ * sigmoid(gate) when a gate is given: [tokens, heads * vd], or [tokens, heads] with gate_per_head, and by out_scale.  With a window the first
+ * `keep` positions stay visible.  offsets [heads]: no softmax, a key's weight is sigmoid(score + offset) (no sink, no cap).
  * sgl_amd_grouped_attention: any token mix; tok_seg null = a decode batch, whose own keys and values may be given as k_new / v_new
  * (matrix form): they are read from there and stored at `loc`.  part_o fp32 [tokens, heads, splits, vd], part_ml [.., 2] for splits > 1.
  * sgl_amd_grouped_prefill: stored keys; blocks = [num_blocks, 2] (segment, first of sgl_amd_grouped_prefill_rows() / group tokens). */
@@ -683,22 +707,25 @@ int sgl_amd_grouped_attention(int is_f32, const void* q, int64_t q_stride, void*
     const int64_t* req_pool_indices, const int32_t* tok_seg, const int64_t* positions, const void* gate,
     int64_t gate_stride, void* out, int64_t o_stride, float* part_o, float* part_ml, int64_t tokens, int heads,
     int kv_heads, int kd, int vd, int window, int splits, float scale, float sink, const float* sinks, float cap, int gate_per_head,
-    int plain, void* stream);
+    int plain, int keep, const float* offsets, float out_scale, void* stream);
 int sgl_amd_grouped_prefill(const void* q, int64_t q_stride, const void* cache, int64_t cache_stride, const int32_t* req_to_token,
     int64_t r2t_stride, const int64_t* req_pool_indices, const int32_t* blocks, int num_blocks,
     const int32_t* seg_start, const int32_t* seg_len, const int64_t* positions, const void* gate, int64_t gate_stride,
     void* out, int64_t o_stride, int heads, int kv_heads, int kd, int vd, int window, float scale, float sink,
-    const float* sinks, float cap, int gate_per_head, void* stream);
+    const float* sinks, float cap, int gate_per_head, int keep, const float* offsets, float out_scale, void* stream);
 
 /* ---- router with a bias, and the plain form of routed experts (moe_route.hip) -------------------------------------
  * sgl_amd_moe_route: per token the `top` largest of W h + bias (fp32) and the softmax over those -> fp32 weights, int32 ids
- * [tokens, top].  sigmoid = 1: scores sigmoid(W h + bias), the choice by score + correction among the experts of the best `keep` of `groups`
- * equal groups (a group counts by the sum of its two largest), weights score * scale.  partials fp32 [slices, tokens, pad] (pad = 16, 32, .. 256 >= experts): the matrix form, `slices` pieces of the
- * columns; null: the plain one.  sgl_amd_experts_plain: pair i = (token i / top, expert ids[i]); up: activation(gate x, up x) from w [experts, 2 N, K],
+ * [tokens, top].  kind 1: scores sigmoid(W h + bias), 2: the softmax over all experts; the choice by score + correction among the experts of
+ * the best `keep` of `groups` equal groups (a group counts by its largest with group_best = 1, by the sum of its two largest with 2), weights
+ * score * scale.  Experts from `real` on get the id -1.  gate_row: W has one more row, whose sigmoid goes behind the weights, [tokens,
+ * top + 1].  partials fp32 [slices, tokens, pad] (pad = 16, 32, .. 256 >= rows of W): the matrix form, `slices` pieces of the
+ * columns; null: the plain one.  sgl_amd_experts_plain: pair i = (token i / top, expert ids[i], negative: left out); up: activation(gate x,
+ * up x) from w [experts, 2 N, K] or activation(up x) from w [experts, N, K],
  * else w x from w [experts, N, K] and x [pairs, K]. */
 int sgl_amd_moe_route(int is_f32, const void* h, int64_t h_stride, const void* w, const float* bias, float* topk_weights, int32_t* topk_ids,
-    float* partials, int slices, int pad, int64_t tokens, int K, int experts, int top, int sigmoid, const float* correction, int groups,
-    int keep, float scale, void* stream);
+    float* partials, int slices, int pad, int64_t tokens, int K, int experts, int top, int kind, const float* correction, int groups,
+    int keep, int group_best, float scale, int real, int gate_row, void* stream);
 int sgl_amd_experts_plain(int is_f32, int up, const void* x, int64_t x_stride, const void* w, const int32_t* ids, void* out, int64_t o_stride,
     int64_t pairs, int top, int N, int K, int experts, int glu_kind, float glu_limit, float glu_alpha, void* stream);
 

@@ -43,6 +43,9 @@ UNIT_GROUPS = {
                 "sampling.hip", "skinny_gemm.hip", "wstream_gemm.hip"],
     "layered": ["api.cpp", "elementwise.hip", "grouped_attention.hip", "latent_attention.hip", "metadata.hip", "moe.hip", "moe_route.hip",
                 "moe_tiled_gemm.hip", "projection_rows.hip", "residual_norm.hip", "sampling.hip", "skinny_gemm.hip", "wstream_gemm.hip"],
+    "shifted": ["api.cpp", "elementwise.hip", "grouped_attention.hip", "metadata.hip", "moe.hip", "moe_route.hip", "moe_tiled_gemm.hip",
+                "projection_rows.hip", "recurrent.hip", "recurrent_chunk.hip", "residual_norm.hip", "sampling.hip", "skinny_gemm.hip",
+                "wstream_gemm.hip"],
 }
 
 

@@ -1,11 +1,12 @@
-// Gated activations: what a feed-forward makes of its gate and up columns.  The kind is the same for a whole launch.
+// Activations: what a feed-forward makes of its gate and up columns, or (kinds from kGluKinds on) of its up columns alone.  The kind is
+// the same for a whole launch.
 #pragma once
 
 #include "common.hpp"
 
 namespace sgl_amd {
 
-enum : int { kGluNone = 0, kGluSilu = 1, kGluGeluTanh = 2, kGluClampedSwish = 3, kGluKinds = 4 };
+enum : int { kGluNone = 0, kGluSilu = 1, kGluGeluTanh = 2, kGluClampedSwish = 3, kGluKinds = 4, kActSquaredRelu = 4, kActKinds = 5 };
 
 struct GluParams {
   int kind;
@@ -22,6 +23,15 @@ __device__ __forceinline__ float clamped_swish_glu(const GluParams& p, float g, 
   g = fminf(g, p.limit);
   u = fminf(fmaxf(u, -p.limit), p.limit);
   return g / (1.0f + expf(-p.alpha * g)) * (u + 1.0f);
+}
+
+__device__ __host__ __forceinline__ bool act_gated(int kind) { return kind > kGluNone && kind < kGluKinds; }
+__device__ __host__ __forceinline__ bool act_pointwise(int kind) { return kind >= kGluKinds; }
+
+// the one activation without a gate: relu(v)^2
+__device__ __forceinline__ float squared_relu(float v) {
+  v = fmaxf(v, 0.f);
+  return v * v;
 }
 
 // kRound: silu keeps the rounding points of 16-bit activations (projection -> bf16, silu -> bf16); the other kinds stay in fp32

@@ -1,6 +1,8 @@
 // Grouped-query attention over a paged pool for layers with sizes of their own: keys and values of different width, an optional
-// sliding window, an optional sink (a score in the softmax denominator that carries no value, one for all heads or one a head), an
-// optional soft cap of the scores and an optional sigmoid gate on the output (a number an element or a head), all fused into one pass.
+// sliding window (with or without the first tokens of the sequence kept beside it), an optional sink (a score in the softmax denominator
+// that carries no value, one for all heads or one a head), an optional soft cap of the scores and an optional sigmoid gate on the output
+// (a number an element or a head), all fused into one pass.  Or, instead of the softmax, every key weighted by the sigmoid of its
+// score plus an offset a head.
 //
 //   grouped_kv_store   the keys and values of new tokens into their cache rows
 //   grouped_attention  any token mix, split along the keys; matrix form (bf16) and a plain form (every size, bf16 and fp32).  In a
@@ -45,6 +47,9 @@ struct GroupedParams {
   float cap;                 // > 0: scores become cap * tanh(score / cap)
   float softmax_scale, cap_in, cap_out;      // matrix forms: factor in front of 2^x, and of a cap's argument and result
   int gate_per_head;
+  int keep;                  // with a window: the first `keep` positions stay visible
+  const float* offsets;      // [heads]: weights are sigmoid(score + offset), not normalized; null: softmax
+  float out_scale;           // factor on the output
 };
 
 __device__ __forceinline__ float sink_of(const GroupedParams& p, int head) { return p.sinks ? p.sinks[head] : p.sink; }
@@ -56,12 +61,22 @@ __device__ __forceinline__ void cap_scores(const GroupedParams& p, f32x4_t& s) {
   for (int r = 0; r < 4; ++r) s[r] = p.cap_out - 2.0f * p.cap_out * __builtin_amdgcn_rcpf(1.0f + fast_exp2(s[r] * p.cap_in));
 }
 
-__device__ __forceinline__ void key_range(const GroupedParams& p, int64_t pos, int split, int& lo, int& hi) {
-  const int end = static_cast<int>(pos) + 1;
-  const int first = p.window > 0 && end > p.window ? end - p.window : 0;
-  const int per = (end - first + p.splits - 1) / p.splits;
-  lo = first + split * per;
-  hi = lo + per < end ? lo + per : end;
+// Visible keys are numbered through: the first `kept` positions, then the window's, `gap` further on.
+struct KeyMap {
+  int kept, gap;
+  __device__ __forceinline__ KeyMap(const GroupedParams& p, int window_first) {
+    kept = p.keep < window_first ? p.keep : window_first;
+    gap = window_first - kept;
+  }
+  __device__ __forceinline__ int operator()(int i) const { return i < kept ? i : i + gap; }
+};
+
+__device__ __forceinline__ int window_first(const GroupedParams& p, int pos) { return p.window > 0 && pos + 1 > p.window ? pos + 1 - p.window : 0; }
+
+__device__ __forceinline__ void key_range(const GroupedParams& p, const KeyMap& key, int pos, int split, int& lo, int& hi) {
+  const int n = pos + 1 - key.gap, per = (n + p.splits - 1) / p.splits;
+  lo = split * per;
+  hi = lo + per < n ? lo + per : n;
 }
 
 // 1 / denominator in units of 2^m, for sums taken relative to the maximum m (both in log2): the sink joins here
@@ -69,6 +84,11 @@ __device__ __forceinline__ float inverse_sum(float m, float l, float sink) {
   const float s2 = sink * kLog2e;
   const float top = fmaxf(m, s2), f = exp2f(m - top);
   return f / (l * f + exp2f(s2 - top));
+}
+
+// what the sums are multiplied with: sigmoid weights are what they are (and come with m = 0)
+__device__ __forceinline__ float output_factor(const GroupedParams& p, float m, float l, int head) {
+  return p.out_scale * (p.offsets ? 1.0f : inverse_sum(m, l, sink_of(p, head)));
 }
 
 template <int VEC, typename T>
@@ -116,18 +136,20 @@ __global__ __launch_bounds__(256) void grouped_attention_plain_kernel(GroupedPar
   const int32_t* row = p.req_to_token + p.req[b] * p.r2t_stride;
   const T* cache = static_cast<const T*>(p.cache) + static_cast<int64_t>(kvh) * row_len;
   const int64_t pos = p.positions[t];
+  const KeyMap key(p, window_first(p, static_cast<int>(pos)));
   int lo, hi;
-  key_range(p, pos, split, lo, hi);
+  key_range(p, key, static_cast<int>(pos), split, lo, hi);
+  const float offset = p.offsets ? p.offsets[h] : 0.f;
   const T* qp = static_cast<const T*>(p.q) + t * p.q_stride + static_cast<int64_t>(h) * p.kd;
   for (int c = threadIdx.x; c < p.kd; c += 256) q[c] = ld1(qp + c);
   for (int c = threadIdx.x; c < p.vd; c += 256) acc[c] = 0.f;
   __syncthreads();
-  float m = -INFINITY, l = 0.f;
+  float m = p.offsets ? 0.f : -INFINITY, l = 0.f;
   for (int j0 = lo; j0 < hi; j0 += 256) {
     const int j = j0 + threadIdx.x;
     float s = -INFINITY;
     if (j < hi) {
-      const T* k = cache + static_cast<int64_t>(row[j]) * p.cache_stride;
+      const T* k = cache + static_cast<int64_t>(row[key(j)]) * p.cache_stride;
       float d = 0.f;
       for (int c = 0; c < p.kd; c += 4) {
         float e[4];
@@ -139,11 +161,16 @@ __global__ __launch_bounds__(256) void grouped_attention_plain_kernel(GroupedPar
       if (p.cap > 0.f) s = p.cap * tanhf(s / p.cap);
       kp[threadIdx.x] = k;
     }
-    const float mn = fmaxf(m, block_max(s, scratch));
-    const float e = j < hi ? expf(s - mn) : 0.f;
-    const float fix = expf(m - mn);
-    l = l * fix + block_sum(e, scratch);
-    m = mn;
+    float e, fix = 1.0f;
+    if (p.offsets) {
+      e = j < hi ? sigmoid_f(s + offset) : 0.f;
+    } else {
+      const float mn = fmaxf(m, block_max(s, scratch));
+      e = j < hi ? expf(s - mn) : 0.f;
+      fix = expf(m - mn);
+      l = l * fix + block_sum(e, scratch);
+      m = mn;
+    }
     sc[threadIdx.x] = e;
     __syncthreads();
     const int n = hi - j0 < 256 ? hi - j0 : 256;
@@ -156,7 +183,7 @@ __global__ __launch_bounds__(256) void grouped_attention_plain_kernel(GroupedPar
   }
   if (p.splits == 1) {
     const float sink = sink_of(p, h), top = fmaxf(m, sink), f = expf(m - top);
-    const float inv = f / (l * f + expf(sink - top));
+    const float inv = p.out_scale * (p.offsets ? 1.0f : f / (l * f + expf(sink - top)));
     for (int c = threadIdx.x; c < p.vd; c += 256) {
       float v[1] = {acc[c] * inv};
       store_gated<1, T>(p, t, h * p.vd + c, v);
@@ -191,7 +218,7 @@ __global__ __launch_bounds__(256) void grouped_merge_kernel(GroupedParams p) {
 #pragma unroll
     for (int j = 0; j < 4; ++j) a[j] += w * v[j];
   }
-  const float inv = inverse_sum(m, l, sink_of(p, h));
+  const float inv = output_factor(p, m, l, h);
 #pragma unroll
   for (int j = 0; j < 4; ++j) a[j] *= inv;
   store_gated<4, T>(p, t, h * p.vd + c, a);
@@ -237,11 +264,29 @@ __device__ __forceinline__ void online_softmax(f32x4_t (&s)[N], float sc, float&
   m = mn;
 }
 
+// The same with sigmoid weights: `offset` in log2, nothing to normalize.
+template <int N>
+__device__ __forceinline__ void sigmoid_weights(f32x4_t (&s)[N], float sc, float offset, bf16x8_t (&pf)[N / 2][2]) {
+#pragma unroll
+  for (int kk = 0; kk < N / 2; ++kk) {
+    uint32_t wh[4], wl[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const float e0 = __builtin_amdgcn_rcpf(1.0f + fast_exp2(-(s[2 * kk + (j >> 1)][2 * (j & 1)] * sc + offset)));
+      const float e1 = __builtin_amdgcn_rcpf(1.0f + fast_exp2(-(s[2 * kk + (j >> 1)][2 * (j & 1) + 1] * sc + offset)));
+      wh[j] = pack_bf2(e0, e1);
+      wl[j] = pack_bf2(e0 - bf_lo(wh[j]), e1 - bf_hi(wh[j]));
+    }
+    pf[kk][0] = as_frag(U4{wh[0], wh[1], wh[2], wh[3]});
+    pf[kk][1] = as_frag(U4{wl[0], wl[1], wl[2], wl[3]});
+  }
+}
+
 // Matrix form for few queries a token: a workgroup = one token, 16 query heads of one key head, one split; its four waves take
 // 32-key tiles in turn, each with its own running sums (no barrier in the loop), merged at the end.  S^T = K Q^T with the keys
 // straight from the cache as operands, O^T = V^T P^T with V^T read transposed from the wave's own LDS tile; a tile's keys and
 // values are in flight while the tile before it is multiplied.
-template <int KS, int VT>
+template <int KS, int VT, bool kSigmoid>
 __global__ __launch_bounds__(256, 2) void grouped_attention_mfma_kernel(GroupedParams p) {
   constexpr int VLS = VT * 16 + 8, kRegion = VT * 512 + 256, VP = VT / 4;      // (a region also holds [16][VT * 16] fp32 sums)
   __shared__ __attribute__((aligned(16))) uint16_t smem[4 * kRegion];
@@ -256,8 +301,10 @@ __global__ __launch_bounds__(256, 2) void grouped_attention_mfma_kernel(GroupedP
   const int64_t head_off = static_cast<int64_t>(kvh) * (p.kd + p.vd);
   const uint16_t* cache = static_cast<const uint16_t*>(p.cache) + head_off;
   const int pos = static_cast<int>(p.positions[t]);
+  const KeyMap key(p, window_first(p, pos));
+  const int newest = pos - key.gap;                    // number of the token itself
   int lo, hi;
-  key_range(p, pos, split, lo, hi);
+  key_range(p, key, pos, split, lo, hi);
   const uint16_t *kn = nullptr, *vn = nullptr;
   if (p.k_new) {
     kn = static_cast<const uint16_t*>(p.k_new) + t * p.k_stride + static_cast<int64_t>(kvh) * p.kd;
@@ -281,7 +328,8 @@ __global__ __launch_bounds__(256, 2) void grouped_attention_mfma_kernel(GroupedP
   f32x4_t o[VT];
 #pragma unroll
   for (int n = 0; n < VT; ++n) o[n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  float m = -INFINITY, l = 0.f;
+  float m = kSigmoid ? 0.f : -INFINITY, l = 0.f;
+  const float offset = kSigmoid ? p.offsets[kvh * p.group + h0 + (i16 < head_n ? i16 : head_n - 1)] * kLog2e : 0.f;
   const int first = lo + 32 * wave;
   int slot[2];
   U4 kreg[2][KS], vreg[4][VP];
@@ -289,7 +337,7 @@ __global__ __launch_bounds__(256, 2) void grouped_attention_mfma_kernel(GroupedP
 #pragma unroll
     for (int n = 0; n < 2; ++n) {
       const int j = j0 + 16 * n + i16;
-      slot[n] = row[j < hi ? j : hi - 1];
+      slot[n] = row[key(j < hi ? j : hi - 1)];
     }
   };
   auto load = [&](int j0) __attribute__((always_inline)) {
@@ -297,7 +345,7 @@ __global__ __launch_bounds__(256, 2) void grouped_attention_mfma_kernel(GroupedP
     for (int n = 0; n < 2; ++n) {
       int j = j0 + 16 * n + i16;
       j = j < hi ? j : hi - 1;
-      const uint16_t* kr = kn && j == pos ? kn : cache + static_cast<int64_t>(slot[n]) * p.cache_stride;
+      const uint16_t* kr = kn && j == newest ? kn : cache + static_cast<int64_t>(slot[n]) * p.cache_stride;
 #pragma unroll
       for (int k = 0; k < KS; ++k) kreg[n][k] = ld16(32 * k + 8 * g < p.kd ? kr + 32 * k + 8 * g : kr);
     }
@@ -306,7 +354,7 @@ __global__ __launch_bounds__(256, 2) void grouped_attention_mfma_kernel(GroupedP
       int j = j0 + 8 * w + (lane >> 3);
       j = j < hi ? j : hi - 1;
       const int sl = __shfl(slot[w >> 1], (w & 1) * 8 + (lane >> 3), 64);
-      const uint16_t* vr = vn && j == pos ? vn : cache + static_cast<int64_t>(sl) * p.cache_stride + p.kd;
+      const uint16_t* vr = vn && j == newest ? vn : cache + static_cast<int64_t>(sl) * p.cache_stride + p.kd;
 #pragma unroll
       for (int i = 0; i < VP; ++i) {
         const int e = (lane & 7) * 8 + 64 * i;
@@ -347,7 +395,8 @@ __global__ __launch_bounds__(256, 2) void grouped_attention_mfma_kernel(GroupedP
           if (j0 + 16 * n + 4 * g + r >= hi) s[n][r] = -INFINITY;
     }
     bf16x8_t pf[1][2];
-    online_softmax<2, VT>(s, p.softmax_scale, m, l, o, pf);
+    if constexpr (kSigmoid) sigmoid_weights<2>(s, p.softmax_scale, offset, pf);
+    else online_softmax<2, VT>(s, p.softmax_scale, m, l, o, pf);
     asm volatile("" ::: "memory");                     // (the tile is this wave's own; LDS serves a wave in order)
     __builtin_amdgcn_wave_barrier();
 #pragma unroll
@@ -391,7 +440,7 @@ __global__ __launch_bounds__(256, 2) void grouped_attention_mfma_kernel(GroupedP
     }
     const int head = kvh * p.group + h0 + hd;
     if (p.splits == 1) {
-      const float inv = inverse_sum(mt, lt, sink_of(p, head));
+      const float inv = output_factor(p, mt, lt, head);
 #pragma unroll
       for (int j = 0; j < 4; ++j) a[j] *= inv;
       store_gated<4, uint16_t>(p, t, head * p.vd + c, a);
@@ -410,7 +459,7 @@ __global__ __launch_bounds__(256, 2) void grouped_attention_mfma_kernel(GroupedP
 // needs them for O^T = V^T P^T, so they never touch LDS.
 constexpr int kPfThreads = 256, kPfRows = 128, kPfTile = 64, kPfPass = kPfThreads / 8;
 
-template <int KS, int VT>
+template <int KS, int VT, bool kSigmoid>
 __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedParams p) {
   constexpr int KLS = KS * 32 + 8, VLS = VT * 16 + 8, KP = KS / 2, VP = VT / 4, NP = kPfTile / kPfPass;
   __shared__ __attribute__((aligned(16))) uint16_t kimg[2][kPfTile * KLS];
@@ -422,8 +471,8 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
   const int left = p.seg_len[b] - q0;
   const int last = (left < p.block_tokens ? left : p.block_tokens) - 1;        // last token of the block, from its first
   const int pos0 = static_cast<int>(p.positions[t0]);
-  const int lo = p.window > 0 && pos0 + 1 > p.window ? pos0 + 1 - p.window : 0;
-  const int end = pos0 + last + 1;
+  const KeyMap key(p, window_first(p, pos0));
+  const int end = pos0 + last + 1 - key.gap;           // keys the block sees
   const int32_t* row = p.req_to_token + p.req[b] * p.r2t_stride;
   const uint16_t* cache = static_cast<const uint16_t*>(p.cache) + static_cast<int64_t>(kvh) * (p.kd + p.vd);
 
@@ -452,7 +501,7 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
 #pragma unroll
     for (int w = 0; w < NP; ++w) {
       const int j = j0 + w * kPfPass + r_row;
-      slot[w] = row[j < end ? j : end - 1];
+      slot[w] = row[key(j < end ? j : end - 1)];
     }
   };
   // (addresses are clamped, never predicated: all loads stay in flight; columns behind kd meet zeros of the query, columns behind
@@ -469,15 +518,23 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
   };
   f32x4_t o[2][VT];
   float m[2] = {-INFINITY, -INFINITY}, l[2] = {0.f, 0.f};
+  float offset[2] = {0.f, 0.f};
+  if constexpr (kSigmoid) {
+#pragma unroll
+    for (int c = 0; c < 2; ++c) {
+      m[c] = 0.f;
+      offset[c] = p.offsets[kvh * p.group + qhead[c]] * kLog2e;
+    }
+  }
 #pragma unroll
   for (int c = 0; c < 2; ++c)
 #pragma unroll
     for (int n = 0; n < VT; ++n) o[c][n] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  next_slot(lo);
+  next_slot(0);
   load();
-  next_slot(lo + kPfTile);
+  next_slot(kPfTile);
   int image = 0;
-  for (int j0 = lo; j0 < end; j0 += kPfTile, image ^= 1) {
+  for (int j0 = 0; j0 < end; j0 += kPfTile, image ^= 1) {
     // (the barrier of the tile before this one lies behind every read of this image)
     uint16_t *kt = kimg[image], *vt = vimg[image];
 #pragma unroll
@@ -493,7 +550,8 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
       next_slot(j0 + 2 * kPfTile);
     }
     // a wave leaves out tiles none of its rows sees
-    if (!wave_live || j0 > wave_last || (p.window > 0 && j0 + kPfTile - 1 <= wave_first - p.window)) continue;
+    const int key0 = key(j0), key1 = key(j0 + kPfTile - 1);
+    if (!wave_live || key0 > wave_last || (p.window > 0 && key1 <= wave_first - p.window && key0 >= p.keep)) continue;
     f32x4_t s[2][4];
 #pragma unroll
     for (int n = 0; n < 4; ++n) {
@@ -512,7 +570,7 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
         cap_scores(p, s[1][n]);
       }
     }
-    if (j0 + kPfTile - 1 > wave_first || (p.window > 0 && j0 <= wave_last - p.window)) {
+    if (key1 > wave_first || (p.window > 0 && key0 <= wave_last - p.window)) {
 #pragma unroll
       for (int c = 0; c < 2; ++c) {
         const int qpos = pos0 + qtok[c];
@@ -520,14 +578,17 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
         for (int n = 0; n < 4; ++n)
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
-            const int j = j0 + 16 * n + 4 * g + r;
-            if (j > qpos || (p.window > 0 && j <= qpos - p.window)) s[c][n][r] = -INFINITY;
+            const int j = key(j0 + 16 * n + 4 * g + r);
+            if (j > qpos || (p.window > 0 && j <= qpos - p.window && j >= p.keep)) s[c][n][r] = -INFINITY;
           }
       }
     }
     bf16x8_t pf[2][2][2];
 #pragma unroll
-    for (int c = 0; c < 2; ++c) online_softmax<4, VT>(s[c], p.softmax_scale, m[c], l[c], o[c], pf[c]);
+    for (int c = 0; c < 2; ++c) {
+      if constexpr (kSigmoid) sigmoid_weights<4>(s[c], p.softmax_scale, offset[c], pf[c]);
+      else online_softmax<4, VT>(s[c], p.softmax_scale, m[c], l[c], o[c], pf[c]);
+    }
 #pragma unroll
     for (int n = 0; n < VT; ++n)
 #pragma unroll
@@ -546,7 +607,7 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
     sum += __shfl_xor(sum, 16, 64);
     sum += __shfl_xor(sum, 32, 64);
     if (qtok[c] > last) continue;
-    const float inv = inverse_sum(m[c], sum, sink_of(p, kvh * p.group + qhead[c]));
+    const float inv = output_factor(p, m[c], sum, kvh * p.group + qhead[c]);
 #pragma unroll
     for (int n = 0; n < VT; ++n) {
       const int e = 16 * n + 4 * g;
@@ -559,17 +620,37 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
 }
 
 // ---------------------------------------------------------------------------------------------------------------
-template <int KS>
+template <int KS, bool kSigmoid>
 void launch_mfma(const GroupedParams& p, const dim3& grid, hipStream_t st) {
-  if (p.vd <= 64) hipLaunchKernelGGL((grouped_attention_mfma_kernel<KS, 4>), grid, dim3(256), 0, st, p);
-  else if (p.vd <= 128) hipLaunchKernelGGL((grouped_attention_mfma_kernel<KS, 8>), grid, dim3(256), 0, st, p);
-  else hipLaunchKernelGGL((grouped_attention_mfma_kernel<KS, 16>), grid, dim3(256), 0, st, p);
+  if (p.vd <= 64) hipLaunchKernelGGL((grouped_attention_mfma_kernel<KS, 4, kSigmoid>), grid, dim3(256), 0, st, p);
+  else if (p.vd <= 128) hipLaunchKernelGGL((grouped_attention_mfma_kernel<KS, 8, kSigmoid>), grid, dim3(256), 0, st, p);
+  else hipLaunchKernelGGL((grouped_attention_mfma_kernel<KS, 16, kSigmoid>), grid, dim3(256), 0, st, p);
 }
 
-template <int KS>
+template <bool kSigmoid>
+void launch_mfma(const GroupedParams& p, const dim3& grid, hipStream_t st) {
+  if (p.kd <= 64) launch_mfma<2, kSigmoid>(p, grid, st);
+  else if (p.kd <= 128) launch_mfma<4, kSigmoid>(p, grid, st);
+  else launch_mfma<8, kSigmoid>(p, grid, st);
+}
+
+template <int KS, bool kSigmoid>
 void launch_prefill(const GroupedParams& p, const dim3& grid, hipStream_t st) {
-  if (p.vd <= 64) hipLaunchKernelGGL((grouped_prefill_kernel<KS, 4>), grid, dim3(kPfThreads), 0, st, p);
-  else hipLaunchKernelGGL((grouped_prefill_kernel<KS, 8>), grid, dim3(kPfThreads), 0, st, p);
+  if (p.vd <= 64) hipLaunchKernelGGL((grouped_prefill_kernel<KS, 4, kSigmoid>), grid, dim3(kPfThreads), 0, st, p);
+  else hipLaunchKernelGGL((grouped_prefill_kernel<KS, 8, kSigmoid>), grid, dim3(kPfThreads), 0, st, p);
+}
+
+template <bool kSigmoid>
+void launch_prefill(const GroupedParams& p, const dim3& grid, hipStream_t st) {
+  if (p.kd <= 64) launch_prefill<2, kSigmoid>(p, grid, st);
+  else if (p.kd <= 128) launch_prefill<4, kSigmoid>(p, grid, st);
+  else launch_prefill<8, kSigmoid>(p, grid, st);
+}
+
+// keys the window keeps, weights that are sigmoids, factor on the output
+bool set_variants(GroupedParams& p, int keep, const float* offsets, float out_scale) {
+  p.keep = p.window > 0 ? keep : 0; p.offsets = offsets; p.out_scale = out_scale;
+  return keep >= 0 && !(offsets && (p.cap > 0.f || p.sinks || p.sink > -INFINITY));
 }
 
 void set_scores(GroupedParams& p, float scale, float cap) {
@@ -618,7 +699,7 @@ int sgl_amd_grouped_attention(int is_f32, const void* q, int64_t q_stride, void*
                               const int64_t* req_pool_indices, const int32_t* tok_seg, const int64_t* positions, const void* gate,
                               int64_t gate_stride, void* out, int64_t o_stride, float* part_o, float* part_ml, int64_t tokens, int heads,
                               int kv_heads, int kd, int vd, int window, int splits, float scale, float sink, const float* sinks, float cap,
-                              int gate_per_head, int plain, void* stream) {
+                              int gate_per_head, int plain, int keep, const float* offsets, float out_scale, void* stream) {
   SGL_CLEAR_STALE_ERROR();
   SGL_CHECK_ARG(q && cache && req_to_token && req_pool_indices && positions && out, "grouped_attention: null operand");
   SGL_CHECK_ARG(heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && heads <= 65535 && kd > 0 && vd > 0 && kd % 4 == 0 && vd % 4 == 0 &&
@@ -633,14 +714,14 @@ int sgl_amd_grouped_attention(int is_f32, const void* q, int64_t q_stride, void*
   p.tokens = tokens; p.heads = heads; p.kv_heads = kv_heads; p.group = heads / kv_heads; p.kd = kd; p.vd = vd; p.window = window;
   p.splits = splits; p.sink = sink; p.sinks = sinks; p.gate_per_head = gate_per_head;
   set_scores(p, scale, cap);
+  SGL_CHECK_ARG(set_variants(p, keep, offsets, out_scale), "grouped_attention: %d kept keys; sigmoid weights take no cap and no sink", keep);
   hipStream_t st = as_stream(stream);
   const bool matrix = !is_f32 && !plain && sgl_amd_grouped_attention_matrix_form(kd, vd) && whole_vectors(p) && scale > 0.f;
   SGL_CHECK_ARG(!k_new || (matrix && v_new && loc && !tok_seg), "grouped_attention: only the matrix form of a decode batch takes keys and values that are not stored yet");
   if (matrix) {
     const dim3 grid(static_cast<unsigned>(tokens), kv_heads * ((p.group + 15) / 16), splits);
-    if (kd <= 64) launch_mfma<2>(p, grid, st);
-    else if (kd <= 128) launch_mfma<4>(p, grid, st);
-    else launch_mfma<8>(p, grid, st);
+    if (offsets) launch_mfma<true>(p, grid, st);
+    else launch_mfma<false>(p, grid, st);
   } else {
     const dim3 grid(static_cast<unsigned>(tokens), heads, splits);
     const size_t lds = (static_cast<size_t>(kd) + vd + 256) * 4 + 256 * 8;
@@ -666,7 +747,7 @@ int sgl_amd_grouped_prefill(const void* q, int64_t q_stride, const void* cache, 
                             int64_t r2t_stride, const int64_t* req_pool_indices, const int32_t* blocks, int num_blocks,
                             const int32_t* seg_start, const int32_t* seg_len, const int64_t* positions, const void* gate, int64_t gate_stride,
                             void* out, int64_t o_stride, int heads, int kv_heads, int kd, int vd, int window, float scale, float sink,
-                            const float* sinks, float cap, int gate_per_head, void* stream) {
+                            const float* sinks, float cap, int gate_per_head, int keep, const float* offsets, float out_scale, void* stream) {
   SGL_CLEAR_STALE_ERROR();
   SGL_CHECK_ARG(q && cache && req_to_token && req_pool_indices && blocks && seg_start && seg_len && positions && out, "grouped_prefill: null operand");
   SGL_CHECK_ARG(heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && sgl_amd_grouped_prefill_supported(kd, vd, heads / kv_heads) &&
@@ -680,12 +761,12 @@ int sgl_amd_grouped_prefill(const void* q, int64_t q_stride, const void* cache, 
   p.group = heads / kv_heads; p.kd = kd; p.vd = vd; p.window = window; p.splits = 1; p.block_tokens = kPfRows / p.group; p.sink = sink;
   p.sinks = sinks; p.gate_per_head = gate_per_head;
   set_scores(p, scale, cap);
+  SGL_CHECK_ARG(set_variants(p, keep, offsets, out_scale), "grouped_prefill: %d kept keys; sigmoid weights take no cap and no sink", keep);
   SGL_CHECK_ARG(whole_vectors(p), "grouped_prefill: rows of whole 16-byte vectors");
   const dim3 grid(kv_heads, num_blocks);
   hipStream_t st = as_stream(stream);
-  if (kd <= 64) launch_prefill<2>(p, grid, st);
-  else if (kd <= 128) launch_prefill<4>(p, grid, st);
-  else launch_prefill<8>(p, grid, st);
+  if (offsets) launch_prefill<true>(p, grid, st);
+  else launch_prefill<false>(p, grid, st);
   SGL_CHECK_LAUNCH("grouped_prefill");
   return 0;
 }

@@ -58,7 +58,7 @@ struct TiledParams {
   const float* row_scale;       // optional [num_valid_ids]
   int64_t a_stride, w_row_stride, w_expert_stride, c_stride;
   int num_valid, N, K, topk_div;
-  int fuse_silu, out_f32, round_before_scale;      // (fuse_silu: any gated activation, `glu`)
+  int fuse_silu, out_f32, round_before_scale;      // (fuse_silu: any gated activation, `glu`, which may also be one without a gate)
   GluParams glu;
   int eid_shift;                // expert_ids is indexed by (row block >> eid_shift): 128-row tiles over a 256-row alignment
   int n_tiles;                  // 256-form: output-column tiles (its grid is one-dimensional)
@@ -200,7 +200,7 @@ __global__ __launch_bounds__(kThreads, 2) void moe_tiled_gemm_kernel(TiledParams
         float o[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const float v = acc[i][j][r];
+          const float v = act_pointwise(p.glu.kind) ? squared_relu(acc[i][j][r]) : acc[i][j][r];
           o[r] = p.row_scale ? (p.round_before_scale ? rbf(v) : v) * scale : v;
         }
         if (p.out_f32) {
@@ -518,7 +518,7 @@ __global__ __launch_bounds__(kThreads2, 1) void moe_gemm256_kernel(TiledParams p
         float o[4];
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          const float v = acc[i][j][r];
+          const float v = act_pointwise(p.glu.kind) ? squared_relu(acc[i][j][r]) : acc[i][j][r];
           o[r] = p.row_scale ? (p.round_before_scale ? rbf(v) : v) * scale : v;
         }
         if (p.out_f32) {
@@ -555,8 +555,8 @@ int sgl_amd_moe_tiled_gemm_ex(const void* a, const void* w, void* c, const int32
                               int64_t a_row_stride, int64_t w_row_stride, int64_t w_expert_stride, int64_t c_row_stride,
                               int64_t max_m_blocks, int glu_kind, float glu_limit, float glu_alpha, int out_f32, int align_block_m, int tile_rows, void* stream) {
   SGL_CLEAR_STALE_ERROR();
-  SGL_CHECK_ARG(glu_kind >= kGluNone && glu_kind < kGluKinds, "moe_tiled_gemm: no activation %d", glu_kind);
-  const int fuse_silu = glu_kind != kGluNone;
+  SGL_CHECK_ARG(glu_kind >= kGluNone && glu_kind < kActKinds, "moe_tiled_gemm: no activation %d", glu_kind);
+  const int fuse_silu = act_gated(glu_kind);
   SGL_CHECK_ARG((align_block_m == 128 || align_block_m == 256) && (tile_rows == 128 || tile_rows == 256) && tile_rows <= align_block_m,
                 "moe_tiled_gemm: align_block_m / tile_rows must be 128 or 256, tile_rows <= align_block_m (got %d / %d)", align_block_m, tile_rows);
   SGL_CHECK_ARG(N > 0 && N % 4 == 0 && K >= kBK && K % kBK == 0, "moe_tiled_gemm: need N %% 4 == 0 and K %% %d == 0 (got N=%lld K=%lld)",

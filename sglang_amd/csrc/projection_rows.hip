@@ -1,7 +1,8 @@
 // What stands between a projection and attention, one launch each: split-K sums and biases, norms, rotation by halves, the cache rows.
 //
 //   head_prepare   rows [query heads | key heads | value heads | gate]: an RMS norm a head in front of the rotation (with weights) or behind
-//                  it (without), rotation of dimension i with i + dims / 2; queries to their rows, keys and values to the cache
+//                  it (without), rotation of dimension i with i + dims / 2; queries to their rows, keys and values to the cache.  Where a
+//                  design's values are its keys, there are no value columns: they are the key columns as projected
 //   latent_down    rows [query latent | latent | rotated key part]: RMS norms of both latents, rotation of the key part, the cache row
 //
 // Sources are rows in the activation type or the fp32 split-K partials of a decode projection; everything up to the store is fp32.
@@ -63,6 +64,7 @@ struct HeadPrepareParams {
   const int64_t* loc;
   int64_t tokens;
   int heads, kv_heads, kd, vd, dim, rot_off, rot_dims, norm_order, gate_cols, units, in_place;
+  int value_is_key;          // the values are the keys in front of norm and rotation (vd == kd)
   int q_off, q_width;        // the columns of a query head this launch touches
   float eps;
 };
@@ -75,7 +77,8 @@ struct HeadUnit {
 __device__ __forceinline__ HeadUnit head_unit(const HeadPrepareParams& p, int u, int gate_piece) {
   const int H = p.heads, G = p.kv_heads;
   if (u < H) return {0, p.q_width, static_cast<int64_t>(u) * p.kd + p.q_off, static_cast<int64_t>(u) * p.kd + p.q_off};
-  const int64_t k0 = static_cast<int64_t>(H) * p.kd, v0 = k0 + static_cast<int64_t>(G) * p.kd, g0 = v0 + static_cast<int64_t>(G) * p.vd;
+  const int64_t k0 = static_cast<int64_t>(H) * p.kd, k1 = k0 + static_cast<int64_t>(G) * p.kd;
+  const int64_t v0 = p.value_is_key ? k0 : k1, g0 = p.value_is_key ? k1 : k1 + static_cast<int64_t>(G) * p.vd;
   u -= H;
   if (u < G) return {1, p.kd, k0 + static_cast<int64_t>(u) * p.kd, static_cast<int64_t>(u) * (p.kd + p.vd)};
   u -= G;
@@ -292,7 +295,7 @@ extern "C" {
 int sgl_amd_head_prepare(int is_f32, const void* rows, int64_t row_stride, const float* partials, int items, int64_t item_stride, const void* bias,
                          void* out, int64_t o_stride, const float* q_norm, const float* k_norm, int norm_order, float eps, const float* cos_sin,
                          int64_t max_positions, const int64_t* positions, int rot_off, int rot_dims, void* cache, int64_t cache_stride,
-                         const int64_t* loc, int64_t tokens, int heads, int kv_heads, int kd, int vd, int dim, int gate_cols, int plain,
+                         const int64_t* loc, int64_t tokens, int heads, int kv_heads, int kd, int vd, int dim, int gate_cols, int value_is_key, int plain,
                          void* stream) {
   SGL_CLEAR_STALE_ERROR();
   HeadPrepareParams p{};
@@ -304,7 +307,9 @@ int sgl_amd_head_prepare(int is_f32, const void* rows, int64_t row_stride, const
                 "head_prepare: %d rotated dimensions from %d of %d", rot_dims, rot_off, dim);
   SGL_CHECK_ARG(kd <= 2048 && vd <= 2048 && cache_stride >= static_cast<int64_t>(kv_heads) * (kd + vd) && gate_cols >= 0 && tokens <= (1 << 24),
                 "head_prepare: heads of %d + %d in rows of %lld", kd, vd, (long long)cache_stride);
+  SGL_CHECK_ARG(!value_is_key || (kv_heads && vd == kd), "head_prepare: values of %d that are keys of %d", vd, kd);
   if (tokens <= 0) return 0;
+  p.value_is_key = value_is_key;
   p.out = out; p.o_stride = o_stride; p.q_norm = q_norm; p.k_norm = k_norm; p.cos_sin = cos_sin; p.max_pos = max_positions; p.positions = positions;
   p.cache = cache; p.cache_stride = cache_stride; p.loc = loc; p.tokens = tokens; p.heads = heads; p.kv_heads = kv_heads; p.kd = kd; p.vd = vd;
   p.dim = dim; p.rot_off = rot_off; p.rot_dims = cos_sin ? rot_dims : 0; p.norm_order = norm_order; p.gate_cols = gate_cols;

@@ -1,5 +1,6 @@
-// Recurrent mixers over a ragged batch: the short causal convolution in front of them, and the Mamba-2 and gated-delta-rule
-// state updates in their token-by-token form (decode steps and short portions; prefill-sized portions: recurrent_chunk.hip).
+// Recurrent mixers over a ragged batch: the short causal convolution in front of them, and the Mamba-2, gated-delta-rule and
+// matrix-memory state updates in their token-by-token form (decode steps and short portions; prefill-sized portions:
+// recurrent_chunk.hip).  And the token shift of ragged batches, whose state is one row a request.
 //
 // A batch is a list of segments (one per request): tokens [seg_start[b], seg_start[b] + seg_len[b]) of the packed rows; both
 // pointers null = one token per request.  Request b's state lives in slot slots[b].  A segment that begins at position 0
@@ -348,6 +349,170 @@ __global__ __launch_bounds__(256) void delta_step_kernel(DeltaParams p) {
   }
 }
 
+struct MemoryParams {
+  const void *q, *k, *v;     // [tokens, heads * D], [.., heads * D], [.., heads * V], columns of one row
+  const void *gi, *gf;       // [tokens, heads] gates as projected
+  int64_t stride;            // of all five
+  const float *bi, *bf;      // [heads]
+  float* state;              // [slots, heads, D, V], relative to e^m
+  float* norm;               // [slots, heads, ceil(V / 16), D + 1]: the sum of the keys, then m; one copy per 16 value columns
+  const int64_t* slots;
+  const int64_t* positions;
+  const int32_t *seg_start, *seg_len;
+  void* o;                   // [tokens, heads * V]
+  int64_t o_stride;
+  int heads, D, V, blocks;
+  float cap, q_scale;
+};
+
+// One token, with log gates i = cap tanh((gi + bi) / cap), f = log sigmoid(cap tanh((gf + bf) / cap)) and a running maximum m:
+//   m' = max(f + m, i);  S <- e^(f + m - m') S + e^(i - m') k v^T, n alike with k alone;  o = S^T q / (max(|n.q|, e^-m') + 1e-6)
+// n and m belong to the whole head: every workgroup keeps them for itself, in the copies of its own columns, so that none reads
+// what another one writes.
+template <typename T, int NR>
+__global__ __launch_bounds__(256) void memory_step_kernel(MemoryParams p) {
+  __shared__ float red[2][4 * 5 * 16];
+  const int b = blockIdx.x, h = blockIdx.y;
+  const int cl = threadIdx.x & 15, rg = threadIdx.x >> 4;
+  const int col = blockIdx.z * kStepCols + cl * 4;
+  const int ncol = p.V - col < 0 ? 0 : (p.V - col > 4 ? 4 : p.V - col);
+  const bool vec = ncol == 4 && (p.V & 3) == 0;
+  const int64_t t0 = p.seg_start ? p.seg_start[b] : b;
+  const int len = p.seg_len ? p.seg_len[b] : 1;
+  if (len <= 0) return;
+  const int64_t pos0 = p.positions[t0], head = p.slots[b] * p.heads + h;
+  const int block = blockIdx.z * (kStepCols / 16);
+  float* S = p.state + head * p.D * p.V + col;
+  float* norm = p.norm + (head * p.blocks + block) * (p.D + 1);
+  float s[NR][4], n[NR];
+#pragma unroll
+  for (int i = 0; i < NR; ++i) {
+    const int r = rg + 16 * i;
+    n[i] = pos0 > 0 && r < p.D ? norm[r] : 0.f;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) s[i][j] = 0.f;
+    if (pos0 > 0 && r < p.D && ncol > 0) load_state4(S + static_cast<int64_t>(r) * p.V, ncol, vec, s[i]);
+  }
+  float m = pos0 > 0 ? norm[p.D] : 0.f;
+  const float bi = p.bi[h], bf = p.bf[h];
+  for (int u = 0; u < len; ++u) {
+    const int64_t t = t0 + u, row = t * p.stride;
+    const T* qr = static_cast<const T*>(p.q) + row + h * p.D;
+    const T* kr = static_cast<const T*>(p.k) + row + h * p.D;
+    const T* vr = static_cast<const T*>(p.v) + row + h * p.V + col;
+    const float gi = p.cap * tanhf((ld1(static_cast<const T*>(p.gi) + row + h) + bi) / p.cap);
+    const float gf = -softplus_f(-p.cap * tanhf((ld1(static_cast<const T*>(p.gf) + row + h) + bf) / p.cap));
+    const float top = fmaxf(gf + m, gi), keep = expf(gf + m - top), add = expf(gi - top);
+    m = top;
+    float v[4], acc[5] = {0.f, 0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < 4; ++j) v[j] = j < ncol ? ld1(vr + j) : 0.f;
+#pragma unroll
+    for (int i = 0; i < NR; ++i) {
+      const int r = rg + 16 * i;
+      if (r < p.D) {
+        const float k = ld1(kr + r) * add, q = ld1(qr + r) * p.q_scale;
+        n[i] = n[i] * keep + k;
+        acc[4] += n[i] * q;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          s[i][j] = s[i][j] * keep + k * v[j];
+          acc[j] += s[i][j] * q;
+        }
+      }
+    }
+    reduce_rows<5>(acc, red[u & 1]);
+    if (rg == 0) {
+      const float inv = 1.0f / (fmaxf(fabsf(acc[4]), expf(-m)) + 1e-6f);
+      T* o = static_cast<T*>(p.o) + t * p.o_stride + h * p.V + col;
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (j < ncol) st1(o + j, acc[j] * inv);
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < NR; ++i) {
+    const int r = rg + 16 * i;
+    if (r >= p.D) continue;
+    if (ncol > 0) store_state4(S + static_cast<int64_t>(r) * p.V, ncol, vec, s[i]);
+    if (cl < kStepCols / 16 && block + cl < p.blocks) norm[cl * (p.D + 1) + r] = n[i];
+  }
+  if (rg == 0 && cl < kStepCols / 16 && block + cl < p.blocks) norm[cl * (p.D + 1) + p.D] = m;
+}
+
+template <typename T>
+void launch_memory(const MemoryParams& p, int segs, hipStream_t st) {
+  const dim3 grid(segs, p.heads, (p.V + kStepCols - 1) / kStepCols);
+  const int nr = (p.D + 15) / 16;
+  if (nr <= 2) hipLaunchKernelGGL((memory_step_kernel<T, 2>), grid, dim3(256), 0, st, p);
+  else if (nr <= 4) hipLaunchKernelGGL((memory_step_kernel<T, 4>), grid, dim3(256), 0, st, p);
+  else if (nr <= 8) hipLaunchKernelGGL((memory_step_kernel<T, 8>), grid, dim3(256), 0, st, p);
+  else if (nr <= 16) hipLaunchKernelGGL((memory_step_kernel<T, 16>), grid, dim3(256), 0, st, p);
+  else hipLaunchKernelGGL((memory_step_kernel<T, 32>), grid, dim3(256), 0, st, p);
+}
+
+// ---------------------------------------------------------------------------------------------------------------
+struct ShiftParams {
+  const void* h;             // [tokens, width]
+  int64_t h_stride;
+  const float* mu;           // [width]
+  void* state;               // [slots, width]: the last row of every request
+  const int64_t* slots;
+  const int64_t* positions;
+  const int32_t *tok_seg, *seg_start, *seg_len;
+  void* out;                 // not h
+  int64_t out_stride;
+  int64_t tokens;
+  int width;
+};
+
+constexpr int kShiftTokens = 4;
+
+// out[t] = h[t] + (h in front of t - h[t]) * mu.  A thread owns VEC columns of a few tokens; the one that owns a segment's first token
+// reads what the request left and then leaves the segment's last row, so nothing is read behind its own replacement.
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void token_shift_kernel(ShiftParams p) {
+  const int c = (blockIdx.x * 256 + threadIdx.x) * VEC;
+  if (c >= p.width) return;
+  const T* h = static_cast<const T*>(p.h) + c;
+  const int64_t t0 = static_cast<int64_t>(blockIdx.y) * kShiftTokens;
+  float mu[VEC], v[kShiftTokens + 1][VEC];
+  ldv<VEC>(p.mu + c, mu);
+#pragma unroll
+  for (int i = 0; i <= kShiftTokens; ++i) {            // (rows outside the batch are not used)
+    int64_t t = t0 + i - 1;
+    t = t < 0 ? 0 : t >= p.tokens ? p.tokens - 1 : t;
+    ldv<VEC>(h + t * p.h_stride, v[i]);
+  }
+#pragma unroll
+  for (int i = 0; i < kShiftTokens; ++i) {
+    const int64_t t = t0 + i;
+    if (t >= p.tokens) return;
+    const int64_t b = p.tok_seg[t], start = p.seg_start[b];
+    float o[VEC];
+    if (t == start) {
+      T* left = static_cast<T*>(p.state) + p.slots[b] * p.width + c;
+      float front[VEC], last[VEC];
+      ldv<VEC>(left, front);
+      ldv<VEC>(h + (start + p.seg_len[b] - 1) * p.h_stride, last);
+      const bool fresh = p.positions[t] <= 0;
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) o[j] = v[i + 1][j] + ((fresh ? 0.f : front[j]) - v[i + 1][j]) * mu[j];
+      stv<VEC>(left, last);
+    } else {
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) o[j] = v[i + 1][j] + (v[i][j] - v[i + 1][j]) * mu[j];
+    }
+    stv<VEC>(static_cast<T*>(p.out) + t * p.out_stride + c, o);
+  }
+}
+
+template <typename T, int VEC>
+void launch_shift(const ShiftParams& p, hipStream_t st) {
+  const dim3 grid((p.width + 256 * VEC - 1) / (256 * VEC), static_cast<unsigned>((p.tokens + kShiftTokens - 1) / kShiftTokens));
+  hipLaunchKernelGGL((token_shift_kernel<T, VEC>), grid, dim3(256), 0, st, p);
+}
+
 template <typename T>
 int launch_mamba2(const Mamba2Params& p, int segs, hipStream_t st) {
   const dim3 grid(segs, p.heads, (p.P + kStepCols - 1) / kStepCols);
@@ -436,6 +601,41 @@ int sgl_amd_delta_step(int is_f32, const void* qkv, int64_t qkv_stride, const vo
   if (is_f32) launch_delta<float>(p, segments, as_stream(stream));
   else launch_delta<uint16_t>(p, segments, as_stream(stream));
   SGL_CHECK_LAUNCH("delta_step");
+  return 0;
+}
+
+int sgl_amd_memory_step(int is_f32, const void* q, const void* k, const void* v, const void* gate_i, const void* gate_f, int64_t stride,
+                        const float* bias_i, const float* bias_f, float* state, float* norm, const int64_t* slots, const int64_t* positions,
+                        const int32_t* seg_start, const int32_t* seg_len, void* o, int64_t o_stride, int segments, int heads, int key_dim,
+                        int value_dim, float gate_cap, float q_scale, void* stream) {
+  SGL_CLEAR_STALE_ERROR();
+  SGL_CHECK_ARG(q && k && v && gate_i && gate_f && bias_i && bias_f && state && norm && slots && positions && o, "memory_step: null operand");
+  SGL_CHECK_ARG(heads > 0 && heads <= 65535 && value_dim > 0 && key_dim > 0 && key_dim <= 512 && gate_cap > 0.f,
+                "memory_step: %d heads of %d x %d (keys at most 512), gate cap %g", heads, key_dim, value_dim, gate_cap);
+  SGL_CHECK_ARG((seg_start == nullptr) == (seg_len == nullptr), "memory_step: segment arrays come together");
+  if (segments <= 0) return 0;
+  MemoryParams p{q, k, v, gate_i, gate_f, stride, bias_i, bias_f, state, norm, slots, positions, seg_start, seg_len, o, o_stride,
+                 heads, key_dim, value_dim, (value_dim + 15) / 16, gate_cap, q_scale};
+  if (is_f32) launch_memory<float>(p, segments, as_stream(stream));
+  else launch_memory<uint16_t>(p, segments, as_stream(stream));
+  SGL_CHECK_LAUNCH("memory_step");
+  return 0;
+}
+
+int sgl_amd_token_shift(int is_f32, const void* h, int64_t h_stride, const float* mu, void* state, const int64_t* slots, const int64_t* positions,
+                        const int32_t* tok_seg, const int32_t* seg_start, const int32_t* seg_len, void* out, int64_t out_stride, int64_t tokens,
+                        int width, void* stream) {
+  SGL_CLEAR_STALE_ERROR();
+  SGL_CHECK_ARG(h && mu && state && slots && positions && tok_seg && seg_start && seg_len && out && h != out && width > 0, "token_shift: null operand, or in place");
+  if (tokens <= 0) return 0;
+  SGL_CHECK_ARG((tokens + kShiftTokens - 1) / kShiftTokens <= 65535, "token_shift: %lld tokens", (long long)tokens);
+  ShiftParams p{h, h_stride, mu, state, slots, positions, tok_seg, seg_start, seg_len, out, out_stride, tokens, width};
+  const bool vec = width % 8 == 0 && h_stride % 8 == 0 && out_stride % 8 == 0 && aligned_to(h, 16) && aligned_to(out, 16) && aligned_to(state, 16) &&
+                   aligned_to(mu, 16);
+  hipStream_t st = as_stream(stream);
+  if (is_f32) vec ? launch_shift<float, 8>(p, st) : launch_shift<float, 1>(p, st);
+  else vec ? launch_shift<uint16_t, 8>(p, st) : launch_shift<uint16_t, 1>(p, st);
+  SGL_CHECK_LAUNCH("token_shift");
   return 0;
 }
 

@@ -1,4 +1,4 @@
-// Mamba-2 and gated-delta-rule state updates in chunks of 32 tokens, for prefill-sized segments.
+// Mamba-2, gated-delta-rule and matrix-memory state updates in chunks of 32 tokens, for prefill-sized segments.
 //
 // A workgroup owns one (segment, head) and up to 64 value columns (a wave = 16 of them) and walks the segment; the state tile
 // stays in the accumulators of v_mfma_f32_16x16x4_f32 for the whole walk.  Everything is fp32: operands are widened when they
@@ -15,6 +15,9 @@
 //   delta:    (I + A) U = beta (v - e^{c_i} S0^T k_i),  A_ij = beta_i e^{c_i-c_j} (k_i.k_j) for j < i
 //             o_i = e^{c_i} S0^T q_i + sum_{j<=i} e^{c_i-c_j} (q_i.k_j) u_j
 //             S   = e^{c_n} S0 + sum_j e^{c_n-c_j} k_j u_j^T
+//   memory:   with a_j = i_j - c_j and g_i = max(m0, a_1 .. a_i), so that c_i + g_i is the running maximum behind token i,
+//             (y | d)_i = e^{m0-g_i} (S0 | n0)^T q_i + sum_{j<=i} e^{a_j-g_i} (q_i.k_j) (v_j | 1),  o_i = y_i / (max(|d_i|, e^{-c_i-g_i}) + 1e-6)
+//             (S | n) = e^{m0-g_n} (S0 | n0) + sum_j e^{a_j-g_n} k_j (v_j | 1)^T,  m = c_n + g_n
 // (I + A)^-1 is formed by forward substitution in 16-token blocks, which stays accurate for repeated keys.
 #include "elem_io.hpp"
 #include "sglang_amd.h"
@@ -482,6 +485,194 @@ __global__ __launch_bounds__(256, NT <= 8 ? 2 : 1) void delta_chunk_kernel(Delta
     }
 }
 
+struct MemoryChunkParams {
+  const void *q, *k, *v, *gi, *gf;
+  int64_t stride;
+  const float *bi, *bf;
+  float *state, *norm;       // norm: [slots, heads, blocks, D + 1], one copy per 16 value columns (recurrent.hip)
+  const int64_t* slots;
+  const int64_t* positions;
+  const int32_t *seg_start, *seg_len;
+  void* o;
+  int64_t o_stride;
+  int heads, D, V, blocks, vec, col_waves;
+  float cap, q_scale;
+};
+
+template <typename T, int NT>
+__global__ __launch_bounds__(256, NT <= 8 ? 2 : 1) void memory_chunk_kernel(MemoryChunkParams p) {
+  constexpr int NP = NT * 16, LS = NP + 4;
+  __shared__ __attribute__((aligned(16))) float Ks[kQ * LS];
+  __shared__ __attribute__((aligned(16))) float Qs[kQ * LS];
+  __shared__ __attribute__((aligned(16))) float Gs[kQ * kSq];
+  __shared__ __attribute__((aligned(16))) float ns[NP];
+  __shared__ double cum[kQ], as[kQ], gs[kQ];
+  __shared__ float inv[kQ];
+  const int b = blockIdx.y, h = blockIdx.x;
+  constexpr int waves = 4;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int i16 = lane & 15, g = lane >> 4;
+  const int block = blockIdx.z * p.col_waves, col = (block + wave) * 16 + i16;
+  const bool live = wave < p.col_waves && col < p.V;           // waves without columns only help with the shared matrices
+  const int64_t t0 = p.seg_start[b];
+  const int total = p.seg_len[b];
+  if (total <= 0) return;
+  const int64_t pos0 = p.positions[t0], head = p.slots[b] * p.heads + h;
+  float* S = p.state + head * p.D * p.V + col;
+  float* norm = p.norm + (head * p.blocks + block) * (p.D + 1);
+  f32x4_t s[NT];
+#pragma unroll
+  for (int t = 0; t < NT; ++t)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int n = 16 * t + 4 * g + r;
+      s[t][r] = pos0 > 0 && live && n < p.D ? S[static_cast<int64_t>(n) * p.V] : 0.f;
+    }
+  if (threadIdx.x < NP) ns[threadIdx.x] = pos0 > 0 && static_cast<int>(threadIdx.x) < p.D ? norm[threadIdx.x] : 0.f;
+  double m0 = pos0 > 0 ? norm[p.D] : 0.f;
+  const float bi = p.bi[h], bf = p.bf[h];
+  const T* qp = static_cast<const T*>(p.q) + t0 * p.stride + h * p.D;
+  const T* kp = static_cast<const T*>(p.k) + t0 * p.stride + h * p.D;
+  const T* vp = static_cast<const T*>(p.v) + t0 * p.stride + h * p.V + col;
+  const T* ip = static_cast<const T*>(p.gi) + t0 * p.stride + h;
+  const T* fp = static_cast<const T*>(p.gf) + t0 * p.stride + h;
+  T* op = static_cast<T*>(p.o) + t0 * p.o_stride + h * p.V + col;
+
+  RowTile<T, NP> qt, kt;
+  T vr[2][4], ir = T{}, fr = T{};
+  auto fetch = [&](int c0) __attribute__((always_inline)) {
+    const int len = total - c0 < kQ ? total - c0 : kQ;
+    const int64_t row = static_cast<int64_t>(c0) * p.stride;
+    qt.fetch(qp + row, p.stride, len, p.D, p.vec);
+    kt.fetch(kp + row, p.stride, len, p.D, p.vec);
+#pragma unroll
+    for (int tj = 0; tj < 2; ++tj)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int j = 16 * tj + 4 * g + r;
+        vr[tj][r] = live && j < len ? vp[row + j * p.stride] : T{};
+      }
+    if (wave == 0 && lane < len) {
+      ir = ip[row + lane * p.stride];
+      fr = fp[row + lane * p.stride];
+    }
+  };
+  fetch(0);
+  for (int c0 = 0; c0 < total; c0 += kQ) {
+    const int len = total - c0 < kQ ? total - c0 : kQ;
+    qt.commit(Qs, LS);
+    kt.commit(Ks, LS);
+    if (wave == 0) {
+      const float gi = p.cap * tanhf((ld1(&ir) + bi) / p.cap), gf = -softplus_f(-p.cap * tanhf((ld1(&fr) + bf) / p.cap));
+      const double c = scan32(lane < len ? static_cast<double>(gf) : 0.0, lane);
+      const double a = lane < len ? static_cast<double>(gi) - c : -INFINITY;
+      double top = a > m0 ? a : m0;
+#pragma unroll
+      for (int off = 1; off < kQ; off <<= 1) {
+        const double u = __shfl_up(top, off, 64);
+        if (lane >= off && u > top) top = u;
+      }
+      if (lane < kQ) { cum[lane] = c; as[lane] = a; gs[lane] = top; }
+    }
+    float x[2][4];
+#pragma unroll
+    for (int tj = 0; tj < 2; ++tj)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) x[tj][r] = ld1(&vr[tj][r]);
+    __syncthreads();
+    if (c0 + kQ < total) fetch(c0 + kQ);
+    for (int tile = wave; tile < 3; tile += waves) {
+      const int ti = tile > 0, tj = tile > 1;
+      const f32x4_t gm = gram_tile(Qs + 16 * ti * LS, Ks + 16 * tj * LS, NP, LS, i16, g);
+      const int j = 16 * tj + i16;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int i = 16 * ti + 4 * g + r;
+        Gs[i * kSq + j] = j <= i ? gm[r] * p.q_scale * expf(static_cast<float>(as[j] - gs[i])) : 0.f;
+      }
+    }
+    f32x4_t y[2];
+#pragma unroll
+    for (int ti = 0; ti < 2; ++ti) {
+      y[ti] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int t = 0; t < NT; ++t) {
+        const f32x4_t q = *reinterpret_cast<const f32x4_t*>(Qs + (16 * ti + i16) * LS + 16 * t + 4 * g);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) y[ti] = mfma4(q[r], s[t][r], y[ti]);
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) y[ti][r] *= p.q_scale * expf(static_cast<float>(m0 - gs[16 * ti + 4 * g + r]));
+    }
+    __syncthreads();
+    {                                                  // denominators: eight lanes a token
+      const int i = threadIdx.x >> 3, e = (threadIdx.x & 7) * 4;
+      float d = 0.f;
+      for (int c = e; c < NP; c += 32) {
+        const f32x4_t q = *reinterpret_cast<const f32x4_t*>(Qs + i * LS + c), n = *reinterpret_cast<const f32x4_t*>(ns + c);
+        d += q[0] * n[0] + q[1] * n[1] + q[2] * n[2] + q[3] * n[3];
+      }
+      d *= p.q_scale * expf(static_cast<float>(m0 - gs[i]));
+      if (e < 16 || i >= 16) {                         // (the block above the diagonal is not formed)
+        const f32x4_t w = *reinterpret_cast<const f32x4_t*>(Gs + i * kSq + e);
+        d += w[0] + w[1] + w[2] + w[3];
+      }
+      d += __shfl_xor(d, 1, 64);
+      d += __shfl_xor(d, 2, 64);
+      d += __shfl_xor(d, 4, 64);
+      if (e == 0) inv[i] = 1.0f / (fmaxf(fabsf(d), expf(static_cast<float>(-(cum[i] + gs[i])))) + 1e-6f);
+    }
+#pragma unroll
+    for (int ti = 0; ti < 2; ++ti)
+#pragma unroll
+      for (int tj = 0; tj <= ti; ++tj) {
+        const f32x4_t w = *reinterpret_cast<const f32x4_t*>(Gs + (16 * ti + i16) * kSq + 16 * tj + 4 * g);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) y[ti] = mfma4(w[r], x[tj][r], y[ti]);
+      }
+    const double gn = gs[kQ - 1];
+    const float fix = expf(static_cast<float>(m0 - gn));
+#pragma unroll
+    for (int tj = 0; tj < 2; ++tj)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) x[tj][r] *= expf(static_cast<float>(as[16 * tj + 4 * g + r] - gn));
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+      s[t] *= fix;
+#pragma unroll
+      for (int tj = 0; tj < 2; ++tj)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) s[t] = mfma4(Ks[(16 * tj + 4 * g + r) * LS + 16 * t + i16], x[tj][r], s[t]);
+    }
+    __syncthreads();
+#pragma unroll
+    for (int ti = 0; ti < 2; ++ti)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int i = 16 * ti + 4 * g + r;
+        if (live && i < len) st1(op + static_cast<int64_t>(c0 + i) * p.o_stride, y[ti][r] * inv[i]);
+      }
+    if (threadIdx.x < NP) {
+      float n = ns[threadIdx.x] * fix;
+      for (int j = 0; j < len; ++j) n += Ks[j * LS + threadIdx.x] * expf(static_cast<float>(as[j] - gn));
+      ns[threadIdx.x] = n;
+    }
+    m0 = static_cast<float>(cum[kQ - 1] + gn);         // (what a state of its own would hold)
+    __syncthreads();
+  }
+#pragma unroll
+  for (int t = 0; t < NT; ++t)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int n = 16 * t + 4 * g + r;
+      if (live && n < p.D) S[static_cast<int64_t>(n) * p.V] = s[t][r];
+    }
+  for (int w = 0; w < p.col_waves && block + w < p.blocks; ++w) {
+    if (static_cast<int>(threadIdx.x) < p.D) norm[w * (p.D + 1) + threadIdx.x] = ns[threadIdx.x];
+    if (threadIdx.x == 0) norm[w * (p.D + 1) + p.D] = static_cast<float>(m0);
+  }
+}
+
 // Columns per workgroup in waves of 16: up to 64, fewer while the launch would leave compute units empty.
 int column_waves(int cols, int64_t segs_heads) {
   int w = (cols + 15) / 16;
@@ -510,6 +701,17 @@ void launch_delta_chunk(DeltaChunkParams p, int segs, hipStream_t st) {
   else if (nt <= 4) hipLaunchKernelGGL((delta_chunk_kernel<T, 4>), grid, block, 0, st, p);
   else if (nt <= 8) hipLaunchKernelGGL((delta_chunk_kernel<T, 8>), grid, block, 0, st, p);
   else hipLaunchKernelGGL((delta_chunk_kernel<T, 12>), grid, block, 0, st, p);
+}
+
+template <typename T>
+void launch_memory_chunk(MemoryChunkParams p, int segs, hipStream_t st) {
+  const int w = p.col_waves = column_waves(p.V, static_cast<int64_t>(segs) * p.heads);
+  const dim3 grid(p.heads, segs, (p.V + 16 * w - 1) / (16 * w)), block(256);
+  const int nt = (p.D + 15) / 16;
+  if (nt <= 2) hipLaunchKernelGGL((memory_chunk_kernel<T, 2>), grid, block, 0, st, p);
+  else if (nt <= 4) hipLaunchKernelGGL((memory_chunk_kernel<T, 4>), grid, block, 0, st, p);
+  else if (nt <= 8) hipLaunchKernelGGL((memory_chunk_kernel<T, 8>), grid, block, 0, st, p);
+  else hipLaunchKernelGGL((memory_chunk_kernel<T, 12>), grid, block, 0, st, p);
 }
 
 }  // namespace
@@ -553,6 +755,26 @@ int sgl_amd_delta_chunk(int is_f32, const void* qkv, int64_t qkv_stride, const v
   if (is_f32) launch_delta_chunk<float>(p, segments, as_stream(stream));
   else launch_delta_chunk<uint16_t>(p, segments, as_stream(stream));
   SGL_CHECK_LAUNCH("delta_chunk");
+  return 0;
+}
+
+int sgl_amd_memory_chunk(int is_f32, const void* q, const void* k, const void* v, const void* gate_i, const void* gate_f, int64_t stride,
+                         const float* bias_i, const float* bias_f, float* state, float* norm, const int64_t* slots, const int64_t* positions,
+                         const int32_t* seg_start, const int32_t* seg_len, void* o, int64_t o_stride, int segments, int heads, int key_dim,
+                         int value_dim, float gate_cap, float q_scale, void* stream) {
+  SGL_CLEAR_STALE_ERROR();
+  SGL_CHECK_ARG(q && k && v && gate_i && gate_f && bias_i && bias_f && state && norm && slots && positions && seg_start && seg_len && o,
+                "memory_chunk: null operand");
+  SGL_CHECK_ARG(heads > 0 && value_dim > 0 && key_dim > 0 && key_dim <= 192 && segments <= 65535 && gate_cap > 0.f,
+                "memory_chunk: %d heads of %d x %d (keys at most 192), gate cap %g", heads, key_dim, value_dim, gate_cap);
+  if (segments <= 0) return 0;
+  const size_t al = is_f32 ? 16 : 8;
+  const int vec = key_dim % 4 == 0 && stride % 4 == 0 && aligned_to(q, al) && aligned_to(k, al);
+  MemoryChunkParams p{q, k, v, gate_i, gate_f, stride, bias_i, bias_f, state, norm, slots, positions, seg_start, seg_len, o, o_stride,
+                      heads, key_dim, value_dim, (value_dim + 15) / 16, vec, 0, gate_cap, q_scale};
+  if (is_f32) launch_memory_chunk<float>(p, segments, as_stream(stream));
+  else launch_memory_chunk<uint16_t>(p, segments, as_stream(stream));
+  SGL_CHECK_LAUNCH("memory_chunk");
   return 0;
 }
 

@@ -5,11 +5,13 @@
 //                   The residual row lives in fp32 and is in registers for both norms.
 //   residual_rms    the same step of pre-norm designs with RMS norms:  x <- embedding (+ position row), or x + up to two sublayer
 //                   outputs (rows, split-K partials, or weighted expert rows), then a saved copy, then + rows + vector in front
-//                   of a looped pass, then h = RMS norm(x).  Post-norm designs: x + mult * RMS norm(sum of the outputs), h = x
+//                   of a looped pass, then h = RMS norm(x).  Post-norm designs: x + mult * RMS norm(sum of the outputs), h = x or its norm.
+//                   In decode batches h may leave blended with the row its request left one token ago (token shift)
 //   soft_cap        cap * tanh(z / cap) on logits, fp32 out
 //   gated_rmsnorm   RMS norm of equal column groups with a silu gate, the gate before the norm (Mamba-2) or behind it
-//                   (gated delta rule).
+//                   (gated delta rule), or with a sigmoid gate behind the norm (matrix memory).
 //   gate_mul        act(a) * b for activation types / alignments outside silu_and_mul's bf16 form.
+//   squared_relu    relu(a)^2, in place or not.
 #include "elem_io.hpp"
 #include "glu.hpp"
 #include "sglang_amd.h"
@@ -209,13 +211,18 @@ void launch_residual_norm_t(const ResidualNormParams& p, bool vec, hipStream_t s
 }
 
 // ---------------------------------------------------------------------------------------------------------------
-// One addend of a residual row: the sum over i < n of weight[row, i] * data[row * row_stride + i * item_stride + column].
+// One addend of a residual row: the sum over i < n of weight[row, i] * data[row * row_stride + i * item_stride + column].  An item whose
+// id is negative is the row of `alt` instead (an expert that hands on its input).
 struct RowSource {
   const void* data;
   int f32;                  // element type: fp32, else the activation type
   int n;
   int64_t row_stride, item_stride;
-  const float* weight;      // [rows, n], or null: all ones
+  const float* weight;      // element (row, i) at row * w_row + i * w_item, or null: all ones
+  int64_t w_row, w_item;
+  const int32_t* ids;       // [rows, n], or null
+  const void* alt;          // activation type
+  int64_t alt_stride;
 };
 
 struct ResidualRmsParams {
@@ -232,32 +239,41 @@ struct ResidualRmsParams {
   float* save;              // optional fp32 copy of x as it is here
   const float* extra;       // optional fp32 rows, added behind the copy (the stride of `save` / `extra` is W)
   const float* step;        // optional [W], added last
+  const float* bias;        // optional [W], part of the addends' sum
   const float* post;        // optional [W]: x = x + mult * (RMS norm(a + b) * post)
   float mult;
   const float* w;           // [W]; null: h is the new x itself
   void* h;                  // RMS norm of the new x (may be null)
   int64_t h_stride;
+  const float* shift;       // optional [W]: h = norm + (the row's norm one token ago - norm) * shift; the norm goes to the state
+  void* shift_state;        // [slots, W] activation type
+  const int64_t *shift_slots, *shift_pos;      // [rows]; position 0: nothing in front
   int64_t rows;
   int width;
   float eps;
 };
 
+template <typename T>
+__device__ __forceinline__ const T* source_item(const RowSource& s, int64_t row, int i) {
+  if (s.ids && s.ids[row * s.n + i] < 0) return static_cast<const T*>(s.alt) + row * s.alt_stride;
+  return static_cast<const T*>(s.data) + row * s.row_stride + i * s.item_stride;
+}
+
 template <typename T, int VEC>
 __device__ __forceinline__ void add_source(const RowSource& s, int64_t row, int c, float (&v)[VEC]) {
-  const float* wr = s.weight ? s.weight + row * s.n : nullptr;
-  const int64_t base = row * s.row_stride + c;
+  const float* wr = s.weight ? s.weight + row * s.w_row : nullptr;
   for (int i = 0; i < s.n; i += 4) {                  // four loads in flight, clamped to the last item
     float u[4][VEC];
 #pragma unroll
     for (int q = 0; q < 4; ++q) {
-      const int64_t at = base + static_cast<int64_t>(i + q < s.n ? i + q : s.n - 1) * s.item_stride;
-      if (s.f32) ldv<VEC>(static_cast<const float*>(s.data) + at, u[q]);
-      else ldv<VEC>(static_cast<const T*>(s.data) + at, u[q]);
+      const int item = i + q < s.n ? i + q : s.n - 1;
+      if (s.f32) ldv<VEC>(source_item<float>(s, row, item) + c, u[q]);
+      else ldv<VEC>(source_item<T>(s, row, item) + c, u[q]);
     }
 #pragma unroll
     for (int q = 0; q < 4; ++q)
       if (i + q < s.n) {
-        const float f = wr ? wr[i + q] : 1.0f;
+        const float f = wr ? wr[(i + q) * s.w_item] : 1.0f;
 #pragma unroll
         for (int j = 0; j < VEC; ++j) v[j] += f * u[q][j];
       }
@@ -270,15 +286,14 @@ __device__ __forceinline__ void add_source_row(const RowSource& s, int64_t row, 
   constexpr int kAhead = kItems <= 4 ? 2 : 1;
 #pragma unroll kAhead
   for (int q = 0; q < s.n; ++q) {
-    const int64_t base = row * s.row_stride + q * s.item_stride;
-    const float f = s.weight ? s.weight[row * s.n + q] : 1.0f;
+    const float f = s.weight ? s.weight[row * s.w_row + q * s.w_item] : 1.0f;
     float u[kItems][VEC];
 #pragma unroll
     for (int i = 0; i < kItems; ++i) {
       int c = (i * tpr + lane) * VEC;
       if (c >= W) c = 0;
-      if (s.f32) ldv<VEC>(static_cast<const float*>(s.data) + base + c, u[i]);
-      else ldv<VEC>(static_cast<const T*>(s.data) + base + c, u[i]);
+      if (s.f32) ldv<VEC>(source_item<float>(s, row, q) + c, u[i]);
+      else ldv<VEC>(source_item<T>(s, row, q) + c, u[i]);
     }
 #pragma unroll
     for (int i = 0; i < kItems; ++i)
@@ -343,6 +358,18 @@ __global__ __launch_bounds__(kWaveRow ? 256 : 1024) void residual_rms_kernel(Res
       if (p.a.data) add_source_row<T, VEC, kItems>(p.a, row, lane, tpr, W, v);
       if (p.b.data) add_source_row<T, VEC, kItems>(p.b, row, lane, tpr, W, v);
     }
+    if (p.bias) {
+#pragma unroll
+      for (int i = 0; i < kItems; ++i) {
+        const int c = (i * tpr + lane) * VEC;
+        if (c < W) {
+          float u[VEC];
+          ldv<VEC>(p.bias + c, u);
+#pragma unroll
+          for (int j = 0; j < VEC; ++j) v[i][j] += u[j];
+        }
+      }
+    }
     if (p.post) {
       float sq = 0.f;
 #pragma unroll
@@ -400,6 +427,8 @@ __global__ __launch_bounds__(kWaveRow ? 256 : 1024) void residual_rms_kernel(Res
   }
   ss = kWaveRow ? wave_sum(ss) : block_sum(ss, scratch);
   const float rs = 1.0f / sqrtf(ss / static_cast<float>(W) + p.eps);
+  T* left = p.shift ? static_cast<T*>(p.shift_state) + p.shift_slots[row] * W : nullptr;
+  const bool fresh = p.shift && p.shift_pos[row] <= 0;
 #pragma unroll
   for (int i = 0; i < kItems; ++i) {
     const int c = (i * tpr + lane) * VEC;
@@ -408,6 +437,14 @@ __global__ __launch_bounds__(kWaveRow ? 256 : 1024) void residual_rms_kernel(Res
       ldv<VEC>(p.w + c, wv);
 #pragma unroll
       for (int j = 0; j < VEC; ++j) o[j] = v[i][j] * rs * wv[j];
+      if (p.shift) {
+        float front[VEC], mu[VEC];
+        ldv<VEC>(left + c, front);
+        ldv<VEC>(p.shift + c, mu);
+        stv<VEC>(left + c, o);
+#pragma unroll
+        for (int j = 0; j < VEC; ++j) o[j] += ((fresh ? 0.f : front[j]) - o[j]) * mu[j];
+      }
       stv<VEC>(hr + c, o);
     }
   }
@@ -463,7 +500,7 @@ struct GatedNormParams {
   void* out;
   int64_t out_stride;
   int64_t rows;
-  int groups, size, gate_first, shared_w;
+  int groups, size, gate_first, shared_w, gate_sigmoid;
   float eps;
 };
 
@@ -490,7 +527,7 @@ __global__ void gated_rmsnorm_kernel(GatedNormParams p) {
       ldv<VEC>(gr + c, gt[i]);
 #pragma unroll
       for (int j = 0; j < VEC; ++j) {
-        gt[i][j] = silu_f(gt[i][j]);
+        gt[i][j] = p.gate_sigmoid ? sigmoid_f(gt[i][j]) : silu_f(gt[i][j]);
         if (p.gate_first) v[i][j] *= gt[i][j];
         ss += v[i][j] * v[i][j];
       }
@@ -545,6 +582,37 @@ __global__ __launch_bounds__(256) void gate_mul_kernel(const T* __restrict__ a, 
   if (c < d) st1(out + row * out_stride + c, glu<false>(act, ld1(a + row * in_stride + c), ld1(b + row * in_stride + c)));
 }
 
+// Two vectors a thread.
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void squared_relu_kernel(const T* a, T* out, int d, int64_t in_stride, int64_t out_stride) {
+  const int64_t row = blockIdx.y;
+  const int c0 = (blockIdx.x * 512 + threadIdx.x) * VEC;
+  float v[2][VEC];
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+    if (const int c = c0 + i * 256 * VEC; c < d) ldv<VEC>(a + row * in_stride + c, v[i]);
+#pragma unroll
+  for (int i = 0; i < 2; ++i)
+    if (const int c = c0 + i * 256 * VEC; c < d) {
+#pragma unroll
+      for (int j = 0; j < VEC; ++j) v[i][j] = squared_relu(v[i][j]);
+      stv<VEC>(out + row * out_stride + c, v[i]);
+    }
+}
+
+template <typename T>
+void launch_squared_relu(const void* a, void* out, int64_t rows, int d, int64_t in_stride, int64_t out_stride, hipStream_t st) {
+  const bool vec = d % 8 == 0 && in_stride % 8 == 0 && out_stride % 8 == 0 && aligned_to(a, 16) && aligned_to(out, 16);
+  const int per = 512 * (vec ? 8 : 1);
+  for (int64_t r = 0; r < rows; r += 65535) {
+    const dim3 grid((d + per - 1) / per, static_cast<unsigned>(rows - r < 65535 ? rows - r : 65535));
+    const T* ap = static_cast<const T*>(a) + r * in_stride;
+    T* op = static_cast<T*>(out) + r * out_stride;
+    if (vec) hipLaunchKernelGGL((squared_relu_kernel<T, 8>), grid, dim3(256), 0, st, ap, op, d, in_stride, out_stride);
+    else hipLaunchKernelGGL((squared_relu_kernel<T, 1>), grid, dim3(256), 0, st, ap, op, d, in_stride, out_stride);
+  }
+}
+
 }  // namespace
 
 extern "C" {
@@ -578,24 +646,30 @@ int sgl_amd_residual_rms(int is_f32, const int64_t* ids, const void* table, int6
                          int64_t a_item_stride, const float* a_weight, const void* b, int b_f32, int b_items, int64_t b_row_stride,
                          int64_t b_item_stride, const float* b_weight, float* x, int64_t x_stride, float* save, const float* extra,
                          const float* step, const float* post, float mult, const float* weight, void* h, int64_t h_stride, int64_t rows, int width,
-                         float eps, void* stream) {
+                         float eps, int64_t a_weight_row, int64_t a_weight_item, const int32_t* a_ids, const void* a_alt, int64_t a_alt_stride,
+                         int64_t b_weight_row, int64_t b_weight_item, const float* bias, const float* shift, void* shift_state,
+                         const int64_t* shift_slots, const int64_t* shift_positions, void* stream) {
   SGL_CLEAR_STALE_ERROR();
   SGL_CHECK_ARG(width > 0 && width <= 16384, "residual_rms: width %d outside 1..16384", width);
   SGL_CHECK_ARG(x && (!ids || (table && vocab > 0 && !a && !b)) && (!pos_table || (ids && positions && max_positions > 0)),
                 "residual_rms: missing operand, or an embedding beside sublayer outputs");
   SGL_CHECK_ARG((!a || a_items >= 1) && (!b || b_items >= 1) && (!post || a), "residual_rms: empty source, or a norm behind none");
+  SGL_CHECK_ARG(!a_ids || (a && a_alt && (is_f32 || !a_f32)), "residual_rms: items that are another row need it, in the activation type");
+  SGL_CHECK_ARG(!shift || (shift_state && shift_slots && shift_positions && weight && h), "residual_rms: a shift needs its state, slots, positions and norm");
   SGL_CHECK_ARG(rows <= 0x7fffffffLL, "residual_rms: too many rows");
   if (rows <= 0) return 0;
-  ResidualRmsParams p{ids, table, vocab, scale, positions, pos_table, max_positions, {a, is_f32 || a_f32, a_items, a_row_stride, a_item_stride, a_weight},
-                      {b, is_f32 || b_f32, b_items, b_row_stride, b_item_stride, b_weight}, x, x_stride, save, extra, step, post, mult, weight, h, h_stride, rows,
-                      width, eps};
+  ResidualRmsParams p{ids, table, vocab, scale, positions, pos_table, max_positions, {a, is_f32 || a_f32, a_items, a_row_stride, a_item_stride, a_weight, a_weight_row, a_weight_item, a_ids, a_alt, a_alt_stride},
+                      {b, is_f32 || b_f32, b_items, b_row_stride, b_item_stride, b_weight, b_weight_row, b_weight_item, nullptr, nullptr, 0}, x, x_stride, save, extra,
+                      step, bias, post, mult, weight, h, h_stride, shift, shift_state, shift_slots, shift_positions, rows, width, eps};
   const size_t al = is_f32 ? 16 : 8;
   const bool vec = width % 4 == 0 && x_stride % 4 == 0 && h_stride % 4 == 0 && a_row_stride % 4 == 0 && a_item_stride % 4 == 0 &&
                    b_row_stride % 4 == 0 && b_item_stride % 4 == 0 && aligned_to(table, al) && aligned_to(pos_table, al) &&
                    aligned_to(a, p.a.f32 ? 16 : 8) && aligned_to(b, p.b.f32 ? 16 : 8) && aligned_to(h, al) && aligned_to(x, 16) &&
-                   aligned_to(save, 16) && aligned_to(extra, 16) && aligned_to(step, 16) && aligned_to(post, 16) && aligned_to(weight, 16);
+                   aligned_to(save, 16) && aligned_to(extra, 16) && aligned_to(step, 16) && aligned_to(post, 16) && aligned_to(weight, 16) &&
+                   aligned_to(bias, 16) && aligned_to(shift, 16) && aligned_to(shift_state, al) && a_alt_stride % 4 == 0 && aligned_to(a_alt, al);
   const bool vec8 = vec && width % 8 == 0 && h_stride % 8 == 0 && a_row_stride % 8 == 0 && a_item_stride % 8 == 0 && b_row_stride % 8 == 0 &&
-                    b_item_stride % 8 == 0 && aligned_to(table, 16) && aligned_to(pos_table, 16) && aligned_to(a, 16) && aligned_to(b, 16) && aligned_to(h, 16);
+                    b_item_stride % 8 == 0 && aligned_to(table, 16) && aligned_to(pos_table, 16) && aligned_to(a, 16) && aligned_to(b, 16) && aligned_to(h, 16) &&
+                    a_alt_stride % 8 == 0 && aligned_to(a_alt, 16) && aligned_to(shift_state, 16);
   if (is_f32) launch_residual_rms<float>(p, vec, vec8, as_stream(stream));
   else launch_residual_rms<uint16_t>(p, vec, vec8, as_stream(stream));
   SGL_CHECK_LAUNCH("residual_rms");
@@ -615,12 +689,12 @@ int sgl_amd_soft_cap(int is_f32, const void* z, int64_t z_row_stride, int items,
 
 int sgl_amd_gated_rmsnorm(int is_f32, const void* y, int64_t y_stride, const void* gate, int64_t gate_stride, const float* weight,
                           void* out, int64_t out_stride, int64_t rows, int groups, int group_size, int gate_first, int shared_weight,
-                          float eps, void* stream) {
+                          int gate_sigmoid, float eps, void* stream) {
   SGL_CLEAR_STALE_ERROR();
   SGL_CHECK_ARG(y && gate && weight && out && groups > 0 && group_size > 0 && group_size <= 16384,
                 "gated_rmsnorm: %d groups of %d", groups, group_size);
   if (rows <= 0) return 0;
-  GatedNormParams p{y, y_stride, gate, gate_stride, weight, out, out_stride, rows, groups, group_size, gate_first, shared_weight, eps};
+  GatedNormParams p{y, y_stride, gate, gate_stride, weight, out, out_stride, rows, groups, group_size, gate_first, shared_weight, gate_sigmoid, eps};
   const size_t a = is_f32 ? 16 : 8;
   const bool vec = group_size % 4 == 0 && y_stride % 4 == 0 && gate_stride % 4 == 0 && out_stride % 4 == 0 && aligned_to(y, a) &&
                    aligned_to(gate, a) && aligned_to(out, a) && aligned_to(weight, 16);
@@ -647,6 +721,16 @@ int sgl_amd_gate_mul(int is_f32, const void* gate, const void* up, void* out, in
     hipLaunchKernelGGL((gate_mul_kernel<uint16_t>), grid, dim3(256), 0, as_stream(stream), static_cast<const uint16_t*>(gate),
                        static_cast<const uint16_t*>(up), static_cast<uint16_t*>(out), d, in_stride, out_stride, act);
   SGL_CHECK_LAUNCH("gate_mul");
+  return 0;
+}
+
+int sgl_amd_squared_relu(int is_f32, const void* in, void* out, int64_t rows, int d, int64_t in_stride, int64_t out_stride, void* stream) {
+  SGL_CLEAR_STALE_ERROR();
+  SGL_CHECK_ARG(in && out && d > 0, "squared_relu: null operand or empty rows");
+  if (rows <= 0) return 0;
+  if (is_f32) launch_squared_relu<float>(in, out, rows, d, in_stride, out_stride, as_stream(stream));
+  else launch_squared_relu<uint16_t>(in, out, rows, d, in_stride, out_stride, as_stream(stream));
+  SGL_CHECK_LAUNCH("squared_relu");
   return 0;
 }
 

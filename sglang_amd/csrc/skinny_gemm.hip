@@ -118,6 +118,7 @@ __device__ __forceinline__ void epilogue(const SkinnyParams& p, f32x4_t (&acc)[N
           v = glu<true>(p.glu, acc[0][mt][r], acc[NTW - 1][mt][r]);
         } else {
           v = acc[nt][mt][r] + bias4[r];
+          if (act_pointwise(p.glu.kind)) v = squared_relu(v);
         }
         if (GROUPED && p.row_scale) {
           if (p.round_before_scale) v = rbf(v);
@@ -419,7 +420,7 @@ int sgl_amd_moe_grouped_gemm(const void* a, const void* w, void* c, const int32_
   SGL_CHECK_ARG(top_k_div >= 1 && num_experts >= 1, "moe_grouped_gemm: bad top_k_div / num_experts");
   SGL_CHECK_ARG(!mul_routed_weight || topk_weights, "moe_grouped_gemm: mul_routed_weight needs topk_weights");
   SGL_CHECK_ARG(max_m_blocks <= 65535, "moe_grouped_gemm: too many row blocks (%lld)", (long long)max_m_blocks);
-  SGL_CHECK_ARG(glu_kind >= kGluNone && glu_kind < kGluKinds, "moe_grouped_gemm: no activation %d", glu_kind);
+  SGL_CHECK_ARG(glu_kind >= kGluNone && glu_kind < kActKinds, "moe_grouped_gemm: no activation %d", glu_kind);
   if (max_m_blocks == 0 || num_valid_ids == 0) return 0;
   SkinnyParams p{};
   p.x = static_cast<const uint16_t*>(a);
@@ -433,7 +434,7 @@ int sgl_amd_moe_grouped_gemm(const void* a, const void* w, void* c, const int32_
   p.M = static_cast<int>(num_valid_ids); p.N = static_cast<int>(N); p.K = static_cast<int>(K);
   p.topk_div = top_k_div; p.splits = num_k_splits; p.out_f32 = out_f32; p.round_before_scale = round_before_scale;
   p.glu = GluParams{glu_kind, glu_limit, glu_alpha};
-  dispatch<true>(p, block_m / 16, static_cast<int>(max_m_blocks), glu_kind, tiles_per_wave, as_stream(stream));
+  dispatch<true>(p, block_m / 16, static_cast<int>(max_m_blocks), act_gated(glu_kind), tiles_per_wave, as_stream(stream));
   SGL_CHECK_LAUNCH("moe_grouped_gemm");
   return 0;
 }

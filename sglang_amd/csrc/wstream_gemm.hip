@@ -489,6 +489,10 @@ __global__ __launch_bounds__(64 * NW, 1) void wstream_gemm_kernel(WsParams p) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) o[r] += bf2f(p.bias[nn + r]);
       }
+      if (plain && act_pointwise(p.glu.kind)) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) o[r] = squared_relu(o[r]);
+      }
       if (GROUPED && p.row_scale) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) o[r] = (p.round_before_scale ? rbf(o[r]) : o[r]) * scale;
@@ -587,6 +591,10 @@ __global__ __launch_bounds__(256) void wstream_combine_kernel(CombineParams p) {
   if (p.bias) {
 #pragma unroll
     for (int r = 0; r < 4; ++r) s[r] += bf2f(p.bias[n0 + r]);
+  }
+  if (act_pointwise(p.glu.kind)) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) s[r] = squared_relu(s[r]);
   }
   uint2 w2;
   w2.x = pack_bf2(s[0], s[1]);
@@ -869,8 +877,8 @@ int sgl_amd_wstream_glu_gemm(const void* x, const void* w, const void* bias, voi
                              int64_t x_chunk_stride, int64_t w_row_stride, int64_t y_row_stride, int64_t y_chunk_stride, int glu_kind,
                              float glu_limit, float glu_alpha, int waves_per_group, int tiles_per_wave, int num_k_splits,
                              void* ws_partials, void* stream) {
-  SGL_CHECK_ARG(glu_kind > kGluNone && glu_kind < kGluKinds, "wstream_glu_gemm: no activation %d", glu_kind);
-  return wstream_gemm_impl(x, w, bias, y, M, N, K, x_row_stride, x_chunk_stride, w_row_stride, y_row_stride, y_chunk_stride, 1,
+  SGL_CHECK_ARG(glu_kind > kGluNone && glu_kind < kActKinds, "wstream_glu_gemm: no activation %d", glu_kind);
+  return wstream_gemm_impl(x, w, bias, y, M, N, K, x_row_stride, x_chunk_stride, w_row_stride, y_row_stride, y_chunk_stride, act_gated(glu_kind) ? 1 : 0,
                            GluParams{glu_kind, glu_limit, glu_alpha}, nullptr, 0, nullptr, 0.f, waves_per_group, tiles_per_wave,
                            num_k_splits, ws_partials, stream);
 }
@@ -882,8 +890,8 @@ int sgl_amd_wstream_moe_gemm(const void* a, const void* w, void* c, const int32_
                              int64_t w_expert_stride, int64_t c_row_stride, int block_m, int64_t max_m_blocks,
                              int glu_kind, float glu_limit, float glu_alpha, int out_f32, int waves_per_group, void* stream) {
   SGL_CLEAR_STALE_ERROR();
-  SGL_CHECK_ARG(glu_kind >= kGluNone && glu_kind < kGluKinds, "wstream_moe_gemm: no activation %d", glu_kind);
-  const int fuse_silu = glu_kind != kGluNone;
+  SGL_CHECK_ARG(glu_kind >= kGluNone && glu_kind < kActKinds, "wstream_moe_gemm: no activation %d", glu_kind);
+  const int fuse_silu = act_gated(glu_kind);
   SGL_CHECK_ARG(block_m == 16 || block_m == 32 || block_m == 48 || block_m == 64,
                 "wstream_moe_gemm: block_m=%d (supported: 16/32/48/64, must equal the moe_align block size)", block_m);
   const int64_t wn = fuse_silu ? 2 * N : N;             // weight rows per expert

@@ -5,16 +5,18 @@ import json
 from pathlib import Path
 from typing import Any, Callable, Dict
 
-from . import bulodra, genusun, models, mosurax
+from . import bulodra, dugalix, genusun, models, mosurax
 
 # config.json "architecture" -> reader of the file
 ARCHITECTURES: Dict[str, Callable[[dict, str], Any]] = {"Genusun": genusun.GenusunConfig.from_dict, "Mosurax": mosurax.MosuraxConfig.from_dict,
-                                                        "Bulodra": bulodra.BulodraConfig.from_dict}
+                                                        "Bulodra": bulodra.BulodraConfig.from_dict, "Dugalix": dugalix.DugalixConfig.from_dict}
 _MODELS = {models.ModelConfig: models.CausalLM, genusun.GenusunConfig: genusun.GenusunForCausalLM,
-           mosurax.MosuraxConfig: mosurax.MosuraxForCausalLM, bulodra.BulodraConfig: bulodra.BulodraForCausalLM}
+           mosurax.MosuraxConfig: mosurax.MosuraxForCausalLM, bulodra.BulodraConfig: bulodra.BulodraForCausalLM,
+           dugalix.DugalixConfig: dugalix.DugalixForCausalLM}
 # HIP units (sglang_amd/csrc) a model's path needs; a model that is not listed uses the whole library
-_UNITS = {genusun.GenusunConfig: "hybrid", mosurax.MosuraxConfig: "grouped", bulodra.BulodraConfig: "layered"}
-_NAMED = (models.CONFIGS, genusun.CONFIGS, mosurax.CONFIGS, bulodra.CONFIGS)
+_UNITS = {genusun.GenusunConfig: "hybrid", mosurax.MosuraxConfig: "grouped", bulodra.BulodraConfig: "layered",
+          dugalix.DugalixConfig: "shifted"}
+_NAMED = (models.CONFIGS, genusun.CONFIGS, mosurax.CONFIGS, bulodra.CONFIGS, dugalix.CONFIGS)
 
 
 def model_class(config):

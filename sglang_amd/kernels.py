@@ -110,13 +110,29 @@ class Glu:
     (u' + 1) with g' = min(g, limit) and u' = u clamped to +- limit."""
 
     KINDS = {"silu": 1, "gelu_tanh": 2, "clamped_swish": 3}
+    gated = True
 
     def __init__(self, kind: str = "silu", limit: float = 0.0, alpha: float = 0.0):
         self.kind, self.args = kind, (self.KINDS[kind], float(limit), float(alpha))
 
 
+class Pointwise:
+    """An activation of the up columns alone: 'squared_relu' relu(u)^2."""
+
+    KINDS = {"squared_relu": 4}
+    gated = False
+
+    def __init__(self, kind: str = "squared_relu"):
+        self.kind, self.args = kind, (self.KINDS[kind], 0.0, 0.0)
+
+
 SILU = Glu()
 NO_GLU = (0, 0.0, 0.0)
+
+
+def _act_args(act, fuse_silu: bool):
+    """The activation arguments of a product: of gate and up columns (fuse_silu), of its own columns, or none."""
+    return act.args if fuse_silu or not act.gated else NO_GLU
 
 
 def glu_and_mul(x: torch.Tensor, act: Glu) -> torch.Tensor:
@@ -884,7 +900,7 @@ def wstream_gemm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] 
                  out: Optional[torch.Tensor] = None, waves_per_group: Optional[int] = None,
                  splits: Optional[int] = None, out_blocked: bool = False, tiles_per_wave: Optional[int] = None, act: Glu = SILU) -> torch.Tensor:
     """Decode-batch F.linear(x, w, bias) on the weight-streaming kernel, optionally followed (in the
-    split-K combine kernel) by silu_and_mul or by fused_add_rmsnorm(out, residual, norm_weight, eps).
+    split-K combine kernel) by silu_and_mul, by fused_add_rmsnorm(out, residual, norm_weight, eps) or by a Pointwise activation ("none" with `act`).
     x may be chunk-major (see _x_layout); out_blocked=True returns the result chunk-major.  `act` replaces silu in silu_and_mul."""
     _dev(x, w)
     _need(x.dtype == _BF16 and w.dtype == _BF16 and w.dim() == 2, "wstream_gemm: bf16 x / 2-D bf16 w")
@@ -918,7 +934,8 @@ def wstream_gemm(x: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] 
     # multiple of 16 but not of 32 runs the interleaved one-pass form when the automatic decomposition says one tile per wave
     one_pass = ep == 1 and s == 1 and (N % 16 == 0 if tpw == 1 else N % 32 == 0)
     ws = _gemm_workspace(x.device, native.lib().sgl_amd_wstream_gemm_workspace_floats(M, N, s)) if ((s > 1 or ep) and not one_pass) else None
-    if ep == 1 and act.kind != "silu":
+    if (ep == 1 and act.kind != "silu") or not act.gated:
+        _need(ep == (1 if act.gated else 0), "wstream_gemm: the activation does not fit the epilogue")
         native.call("sgl_amd_wstream_glu_gemm", x.data_ptr(), w.data_ptr(), _ptr(bias), out.data_ptr(), M, N, K, x_rs, x_cs, w.stride(0), y_rs, y_cs,
                     *act.args, nw, tpw, s, _ptr(ws), _stream())
         return out
@@ -1021,7 +1038,7 @@ def moe_wstream_gemm(a: torch.Tensor, w: torch.Tensor, c: torch.Tensor, sorted_t
     native.call("sgl_amd_wstream_moe_gemm", a.data_ptr(), w.data_ptr(), c.data_ptr(), sorted_token_ids.data_ptr(),
                 expert_ids.data_ptr(), num_tokens_post_padded.data_ptr(), _ptr(topk_weights),
                 1 if mul_routed_weight else 0, 1 if round_before_scale else 0, top_k_div, num_valid_ids, N, K,
-                a.stride(0), w.stride(1), w.stride(0), c.stride(0), block_m, max_m_blocks, *(act.args if fuse_silu else NO_GLU),
+                a.stride(0), w.stride(1), w.stride(0), c.stride(0), block_m, max_m_blocks, *_act_args(act, fuse_silu),
                 1 if c.dtype == torch.float32 else 0, waves_per_group, _stream())
     return c
 
@@ -1056,7 +1073,7 @@ def moe_tiled_gemm(a: torch.Tensor, w: torch.Tensor, c: torch.Tensor, sorted_tok
     native.call("sgl_amd_moe_tiled_gemm_ex", a.data_ptr(), w.data_ptr(), c.data_ptr(), sorted_token_ids.data_ptr(),
                 expert_ids.data_ptr(), num_tokens_post_padded.data_ptr(), _ptr(topk_weights), 1 if mul_routed_weight else 0,
                 1 if round_before_scale else 0, top_k_div, num_valid_ids, N, K, a.stride(0), w.stride(1), w.stride(0),
-                c.stride(0), max_m_blocks, *(act.args if fuse_silu else NO_GLU), 1 if c.dtype == torch.float32 else 0, int(block_m), int(tile_rows),
+                c.stride(0), max_m_blocks, *_act_args(act, fuse_silu), 1 if c.dtype == torch.float32 else 0, int(block_m), int(tile_rows),
                 _stream())
     return c
 
@@ -1113,7 +1130,7 @@ def moe_grouped_gemm(a: torch.Tensor, w: torch.Tensor, c: torch.Tensor, sorted_t
     native.call("sgl_amd_moe_grouped_gemm", a.data_ptr(), w.data_ptr(), c.data_ptr(), sorted_token_ids.data_ptr(),
                 expert_ids.data_ptr(), num_tokens_post_padded.data_ptr(), _ptr(topk_weights),
                 1 if mul_routed_weight else 0, 1 if round_before_scale else 0, top_k_div, num_valid_ids, N, K, E,
-                a.stride(0), w.stride(1), w.stride(0), c.stride(0), block_m, max_m_blocks, *(act.args if fuse_silu else NO_GLU),
+                a.stride(0), w.stride(1), w.stride(0), c.stride(0), block_m, max_m_blocks, *_act_args(act, fuse_silu),
                 1 if c.dtype == torch.float32 else 0, ntw, splits, _ptr(slabs), _stream())
     return c
 
@@ -1296,16 +1313,36 @@ def residual_norm(x: torch.Tensor, eps: float, *, embed: Optional[Tuple[torch.Te
 
 
 class ExpertRows:
-    """The routed experts' outputs on their way into the launch that sums them: data [tokens, top, W] and fp32 weights [tokens, top]."""
+    """The routed experts' outputs on their way into the launch that sums them: data [tokens, top, W] and fp32 weights [tokens, top].  With
+    ids [tokens, top], a negative one stands for an expert that hands on its row of `inputs` [tokens, W]."""
 
-    def __init__(self, data: torch.Tensor, weights: torch.Tensor):
-        self.data, self.weights = data, weights
+    def __init__(self, data: torch.Tensor, weights: torch.Tensor, ids: Optional[torch.Tensor] = None, inputs: Optional[torch.Tensor] = None):
+        self.data, self.weights, self.ids, self.inputs = data, weights, ids, inputs
+
+
+class Scaled:
+    """Rows or Partials [tokens, W] times one fp32 factor a row, on their way into the launch that sums them."""
+
+    def __init__(self, rows, weights: torch.Tensor):
+        self.rows, self.weights = rows, weights
+
+
+class TokenShift:
+    """Blend of a row with the one its request left one token ago, h + (left - h) * mu: fp32 mu [W], the state [slots, W] that holds the last
+    rows, and the slots and positions of a batch of single tokens."""
+
+    def __init__(self, mu: torch.Tensor, state: torch.Tensor, slots: torch.Tensor, positions: torch.Tensor):
+        self.mu, self.state, self.slots, self.positions = mu, state, slots, positions
 
 
 def _row_source(who: str, y, rows: int, W: int):
     """(data, fp32?, items, row stride, item stride, weights) of one addend: rows [rows, W], Partials or ExpertRows."""
     if y is None:
         return None, 0, 0, 0, 0, None
+    if isinstance(y, Scaled):
+        data, f32, items, stride, item, weight = _row_source(who, y.rows, rows, W)
+        _need(weight is None and tuple(y.weights.shape) == (rows,) and y.weights.dtype == torch.float32, f"{who}: one fp32 factor a row")
+        return data, f32, items, stride, item, y.weights
     if isinstance(y, Partials):
         _need((y.rows, y.cols) == (rows, W) and y.bias is None, f"{who}: partials are [splits, rows, W] without a bias")
         return y.data, 1, y.splits, W, rows * W, None
@@ -1313,21 +1350,30 @@ def _row_source(who: str, y, rows: int, W: int):
         d = y.data
         _need(d.dim() == 3 and (d.shape[0], d.shape[2]) == (rows, W) and d.stride(2) == 1 and tuple(y.weights.shape) == tuple(d.shape[:2]),
               f"{who}: expert rows are [rows, top, W] with weights [rows, top]")
-        _f32(who, y.weights)
+        _need(y.weights.dtype == torch.float32, f"{who}: fp32 weights")
+        if y.ids is not None:
+            _need(y.ids.dtype == torch.int32 and y.ids.is_contiguous() and y.ids.shape == y.weights.shape and tuple(y.inputs.shape) == (rows, W)
+                  and y.inputs.stride(1) == 1 and y.inputs.dtype == d.dtype, f"{who}: identities take int32 ids [rows, top] and the input rows")
         return d, int(d.dtype == torch.float32), d.shape[1], d.stride(0), d.stride(1), y.weights
     _rows(who, y)
     _need(tuple(y.shape) == (rows, W), f"{who}: row operands are [rows, W]")
     return y, int(y.dtype == torch.float32), 1, y.stride(0), 0, None
 
 
+def _weight_strides(weights: Optional[torch.Tensor]):
+    """(row, item) strides of an addend's weights; one factor a row serves every item."""
+    return (0, 0) if weights is None else (weights.stride(0), weights.stride(1) if weights.dim() == 2 else 0)
+
+
 def residual_rms(x: torch.Tensor, eps: float, *, embed: Optional[Tuple[torch.Tensor, torch.Tensor, float]] = None,
                  pos: Optional[Tuple[torch.Tensor, torch.Tensor]] = None, add: tuple = (), save: Optional[torch.Tensor] = None,
                  extra: Optional[torch.Tensor] = None, step: Optional[torch.Tensor] = None, norm: Optional[torch.Tensor] = None,
-                 h: Optional[torch.Tensor] = None, post: Optional[Tuple[torch.Tensor, float]] = None) -> None:
+                 h: Optional[torch.Tensor] = None, post: Optional[Tuple[torch.Tensor, float]] = None, bias: Optional[torch.Tensor] = None,
+                 shift: Optional[TokenShift] = None) -> None:
     """Update the fp32 residual rows `x` -- embed = (ids, table, scale) with pos = (positions, table): embedding row + position row;
-    else x + the addends `add` (at most two: rows, Partials or ExpertRows) -- copy them to `save`, add the rows `extra` and the
+    else x + the addends `add` (at most two: rows, Partials, Scaled or -- the first -- ExpertRows) and the vector `bias` -- copy them to `save`, add the rows `extra` and the
     vector `step`, then h = RMS norm(x) * norm (no norm: h = x), in one launch.  post = (weight, factor): x + factor * (RMS norm of the
-    addends' sum * weight)."""
+    addends' sum * weight).  shift (single tokens with a norm): h leaves blended with the row in front, its norm stays in the state."""
     _need(x.dtype == torch.float32 and x.dim() == 2 and x.stride(1) == 1, "residual_rms: fp32 residual rows")
     _need(len(add) <= 2 and not (embed is not None and len(add)) and (pos is None or embed is not None), "residual_rms: an embedding, or at most two addends")
     _need(h is not None or norm is None, "residual_rms: a norm without h")
@@ -1349,16 +1395,27 @@ def residual_rms(x: torch.Tensor, eps: float, *, embed: Optional[Tuple[torch.Ten
     _rows("residual_rms", h)
     for t in (save, extra):
         _need(t is None or (t.dtype == torch.float32 and t.is_contiguous() and tuple(t.shape) == (rows, W)), "residual_rms: contiguous fp32 rows")
-    for t in (step, norm, post_w):
+    for t in (step, norm, post_w, bias, shift.mu if shift is not None else None):
         _need(t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == W), "residual_rms: fp32 parameters [W]")
     _need(h is None or tuple(h.shape) == (rows, W), "residual_rms: h [rows, W]")
     _dev(x, ids, table, positions, pos_table, a[0], b[0], save, extra, step, norm, post_w, h)
     acts = [t for t in (table, h, *(s[0] for s in (a, b) if s[0] is not None and not s[1])) if t is not None]
     f32 = _is_f32(*acts) if acts else 1
+    ids_a = alt = None
+    if add and isinstance(add[0], ExpertRows) and add[0].ids is not None:
+        ids_a, alt = add[0].ids, add[0].inputs
+    _need(len(add) < 2 or not isinstance(add[1], ExpertRows) or add[1].ids is None, "residual_rms: identities belong to the first addend")
+    if shift is not None:
+        s = shift
+        _dev(s.mu, s.state, s.slots, s.positions)
+        _i64("residual_rms", s.slots, s.positions)
+        _need(norm is not None and s.slots.numel() == s.positions.numel() == rows and s.state.dim() == 2 and s.state.shape[1] == W
+              and s.state.is_contiguous() and s.state.dtype == h.dtype, "residual_rms: shift state [slots, W] like h, one slot and position a row")
     native.call("sgl_amd_residual_rms", f32, _ptr(ids), _ptr(table), table.shape[0] if table is not None else 0, float(scale), _ptr(positions),
                 _ptr(pos_table), pos_table.shape[0] if pos_table is not None else 0, _ptr(a[0]), *a[1:5], _ptr(a[5]), _ptr(b[0]), *b[1:5], _ptr(b[5]),
                 x.data_ptr(), x.stride(0), _ptr(save), _ptr(extra), _ptr(step), _ptr(post_w), float(mult), _ptr(norm), _ptr(h), h.stride(0) if h is not None else 0, rows, W,
-                float(eps), _stream())
+                float(eps), *_weight_strides(a[5]), _ptr(ids_a), _ptr(alt), alt.stride(0) if alt is not None else 0, *_weight_strides(b[5]), _ptr(bias),
+                *((_ptr(shift.mu), _ptr(shift.state), _ptr(shift.slots), _ptr(shift.positions)) if shift is not None else (None,) * 4), _stream())
 
 
 def soft_cap(z, cap: float) -> torch.Tensor:
@@ -1379,8 +1436,8 @@ def soft_cap(z, cap: float) -> torch.Tensor:
 
 
 def gated_rmsnorm(y: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, groups: int, eps: float, gate_first: bool,
-                  out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """RMS norm of `groups` equal column groups with a silu gate: before the norm (gate_first) or behind it.  `weight` covers
+                  out: Optional[torch.Tensor] = None, sigmoid_gate: bool = False) -> torch.Tensor:
+    """RMS norm of `groups` equal column groups with a silu gate (sigmoid_gate: a sigmoid): before the norm (gate_first) or behind it.  `weight` covers
     all columns, or one group (shared)."""
     _dev(y, gate, weight, out)
     rows, n = y.shape
@@ -1392,7 +1449,7 @@ def gated_rmsnorm(y: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, gro
     _f32("gated_rmsnorm", weight)
     native.call("sgl_amd_gated_rmsnorm", f32, y.data_ptr(), y.stride(0), gate.data_ptr(), gate.stride(0), weight.data_ptr(),
                 out.data_ptr(), out.stride(0), rows, groups, n // groups, 1 if gate_first else 0, 1 if weight.numel() != n else 0,
-                float(eps), _stream())
+                1 if sigmoid_gate else 0, float(eps), _stream())
     return out
 
 
@@ -1408,6 +1465,14 @@ def gate_mul(x: torch.Tensor, act: Glu = SILU) -> torch.Tensor:
         base = x.data_ptr() + r * x.stride(0) * es
         native.call("sgl_amd_gate_mul", f32, base, base + d * es, out.data_ptr() + r * d * es, n, d, x.stride(0), out.stride(0), *act.args, _stream())
     return out
+
+
+def squared_relu_(x: torch.Tensor) -> torch.Tensor:
+    """x <- relu(x)^2 of rows [n, d], in place."""
+    _dev(x)
+    _rows("squared_relu", x)
+    native.call("sgl_amd_squared_relu", _is_f32(x), x.data_ptr(), x.data_ptr(), x.shape[0], x.shape[1], x.stride(0), x.stride(0), _stream())
+    return x
 
 
 # ---------------------------------------------------------------------------- recurrent mixers
@@ -1497,6 +1562,44 @@ def gated_delta_scan(qkv: torch.Tensor, b: torch.Tensor, a: torch.Tensor, A_log:
                 A_log.data_ptr(), dt_bias.data_ptr(), state.data_ptr(), slots.data_ptr(), positions.data_ptr(), _ptr(seg.start), _ptr(seg.len),
                 o.data_ptr(), o.stride(0), B, H, kv_heads, K, V, float(q_scale), _stream())
     return o
+
+
+def memory_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate_i: torch.Tensor, gate_f: torch.Tensor, bias_i: torch.Tensor,
+                bias_f: torch.Tensor, state: torch.Tensor, norm: torch.Tensor, slots: torch.Tensor, positions: torch.Tensor, seg: Segments,
+                gate_cap: float, q_scale: float, form: Optional[str] = None) -> torch.Tensor:
+    """Matrix memory with exponential gates over every segment: q, k [T, heads * K], v [T, heads * V] and the gates [T, heads] are columns of the
+    same rows; state fp32 [slots, heads, K, V], norm fp32 [slots, heads, ceil(V / 16), K + 1]."""
+    _dev(q, k, v, gate_i, gate_f, bias_i, bias_f, state, norm)
+    T = q.shape[0]
+    B = _seg_checks("memory_scan", seg, slots, positions, T)
+    _, H, K, V = state.shape
+    _rows("memory_scan", q, k, v, gate_i, gate_f)
+    _f32("memory_scan", bias_i, bias_f, state, norm)
+    _need(tuple(q.shape) == tuple(k.shape) == (T, H * K) and tuple(v.shape) == (T, H * V) and tuple(gate_i.shape) == tuple(gate_f.shape) == (T, H)
+          and bias_i.numel() == bias_f.numel() == H and tuple(norm.shape) == (state.shape[0], H, (V + 15) // 16, K + 1)
+          and (T <= 1 or len({t.stride(0) for t in (q, k, v, gate_i, gate_f)}) == 1), "memory_scan: shapes")
+    o = torch.empty((T, H * V), dtype=q.dtype, device=q.device)
+    native.call("sgl_amd_memory_chunk" if _chunked(seg, K, form) else "sgl_amd_memory_step", _is_f32(q, k, v, gate_i, gate_f), q.data_ptr(), k.data_ptr(),
+                v.data_ptr(), gate_i.data_ptr(), gate_f.data_ptr(), q.stride(0), bias_i.data_ptr(), bias_f.data_ptr(), state.data_ptr(),
+                norm.data_ptr(), slots.data_ptr(), positions.data_ptr(), _ptr(seg.start), _ptr(seg.len), o.data_ptr(), o.stride(0), B, H, K, V,
+                float(gate_cap), float(q_scale), _stream())
+    return o
+
+
+def token_shift(h: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, slots: torch.Tensor, positions: torch.Tensor, seg: Segments,
+                out: torch.Tensor) -> torch.Tensor:
+    """out = h + (the row in front - h) * mu over every segment; the row in front of a segment's first one is what its slot of `state`
+    [slots, W] holds (zeros at position 0), the last one is left there.  (Single tokens: residual_rms does it on the way, TokenShift.)"""
+    _dev(h, mu, state, out)
+    T, W = h.shape
+    _seg_checks("token_shift", seg, slots, positions, T)
+    _rows("token_shift", h, out)
+    _f32("token_shift", mu)
+    _need(seg.start is not None and mu.numel() == W and state.dim() == 2 and state.shape[1] == W and state.is_contiguous() and out.shape == h.shape
+          and out.data_ptr() != h.data_ptr(), "token_shift: segments, mu [W], state [slots, W], another output")
+    native.call("sgl_amd_token_shift", _is_f32(h, state, out), h.data_ptr(), h.stride(0), mu.data_ptr(), state.data_ptr(), slots.data_ptr(),
+                positions.data_ptr(), seg.tok_seg.data_ptr(), seg.start.data_ptr(), seg.len.data_ptr(), out.data_ptr(), out.stride(0), T, W, _stream())
+    return out
 
 
 # ---------------------------------------------------------------------------- latent attention
@@ -1630,13 +1733,13 @@ def _projection(who: str, p, cols: int):
 
 def head_prepare(p, heads: int, dim: int, kd: int, positions: torch.Tensor, cos_sin: Optional[torch.Tensor], eps: float, *, rot_off: int = 0,
                  norms: Optional[Tuple[torch.Tensor, torch.Tensor]] = None, norm_after: bool = False, gate_cols: int = 0,
-                 kv: Optional[Tuple[int, int, torch.Tensor, torch.Tensor]] = None, plain: bool = False):
+                 kv: Optional[Tuple[int, int, torch.Tensor, torch.Tensor]] = None, value_is_key: bool = False, plain: bool = False):
     """Query heads [T, heads * kd] (and the gate columns [T, gate_cols], or None) of a projection p -- rows, changed in place, or Partials --
     behind an RMS norm a head over `dim` elements (norms = (query weight, key weight) [kd]: in front of the rotation; norm_after: behind it,
     without weights) and the rotation by halves of [rot_off, + cos_sin.shape[1]).  kv = (kv_heads, vd, cache, loc): keys, treated alike, and
-    values go to the cache rows."""
+    values go to the cache rows; value_is_key: the projection has no value columns, the values are its keys."""
     G, vd, cache, loc = kv if kv is not None else (0, 0, None, None)
-    cols = heads * kd + G * (kd + vd)
+    cols = heads * kd + G * (kd if value_is_key else kd + vd)
     rows, stride, part, items, item_stride, bias = _projection("head_prepare", p, cols + gate_cols)
     T = p.rows if part is not None else p.shape[0]
     f32 = 0 if part is not None else _is_f32(p)
@@ -1651,7 +1754,7 @@ def head_prepare(p, heads: int, dim: int, kd: int, positions: torch.Tensor, cos_
                 _ptr(norms[0]) if norms else None, _ptr(norms[1]) if norms else None, 1 if norms else 2 if norm_after else 0, float(eps), _ptr(cos_sin),
                 cos_sin.shape[0] if cos_sin is not None else 0, positions.data_ptr(), rot_off, cos_sin.shape[1] if cos_sin is not None else 0,
                 _ptr(cache), cache.stride(0) if cache is not None else 0, _ptr(loc), T, heads, G, kd, vd, dim, gate_cols if part is not None else 0,
-                1 if plain else 0, _stream())
+                1 if value_is_key else 0, 1 if plain else 0, _stream())
     g0 = heads * kd if part is not None else cols
     return out[:, :heads * kd], out[:, g0:g0 + gate_cols] if gate_cols else None
 
@@ -1718,6 +1821,18 @@ def grouped_kv_store(k: torch.Tensor, v: torch.Tensor, cache: torch.Tensor, loc:
                 cache.stride(0), loc.data_ptr(), k.shape[0], kv_heads, k.shape[1] // kv_heads, v.shape[1] // kv_heads, _stream())
 
 
+def _variant_args(who: str, keep: int, offsets: Optional[torch.Tensor], out_scale: float, heads: int):
+    """(kept first keys, offsets of sigmoid weights, factor on the output) of a launch."""
+    _dev(offsets)
+    _f32(who, offsets)
+    _need(offsets is None or offsets.numel() == heads, f"{who}: one offset a head")
+    return int(keep), _ptr(offsets), float(out_scale)
+
+
+def _output(out: Optional[torch.Tensor], q: torch.Tensor, cols: int) -> torch.Tensor:
+    return torch.empty((q.shape[0], cols), dtype=q.dtype, device=q.device) if out is None else out
+
+
 def _sink_args(who: str, sink, cap: Optional[float], gate: Optional[torch.Tensor], heads: int):
     """(scalar sink, sink of every head, cap, gate a head?) of a launch."""
     per_head = isinstance(sink, torch.Tensor)
@@ -1732,14 +1847,17 @@ def _sink_args(who: str, sink, cap: Optional[float], gate: Optional[torch.Tensor
 def grouped_attention(q: torch.Tensor, cache: torch.Tensor, req_to_token: torch.Tensor, req_pool_indices: torch.Tensor, positions: torch.Tensor,
                       seg: Segments, heads: int, kv_heads: int, kd: int, vd: int, window: int, scale: float, *, sink=None,
                       gate: Optional[torch.Tensor] = None, new: Optional[Tuple[torch.Tensor, torch.Tensor, torch.Tensor]] = None, splits: int = 1,
-                      plain: bool = False, cap: Optional[float] = None) -> torch.Tensor:
+                      plain: bool = False, cap: Optional[float] = None, keep: int = 0, offsets: Optional[torch.Tensor] = None,
+                      out_scale: float = 1.0, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """q [T, heads * kd] over the cached keys of each token's request -> [T, heads * vd], times sigmoid(gate) (one an element, or one a head).
     sink: a float, or fp32 [heads]; cap: scores become cap * tanh(score / cap).  new = (k, v, loc): a
-    decode batch's own keys and values, stored on the way (matrix form).  `plain` forces the form without matrix instructions."""
+    decode batch's own keys and values, stored on the way (matrix form).  keep: first keys that stay visible beside the window.  offsets (fp32
+    [heads]): sigmoid(score + offset) weights instead of the softmax.  out_scale: factor on the result, which goes to the rows `out` if given.
+    `plain` forces the form without matrix instructions."""
     _dev(q, cache, req_to_token, req_pool_indices, positions, gate)
     T = q.shape[0]
     _seg_checks("grouped_attention", seg, req_pool_indices, positions, T)
-    out = torch.empty((T, heads * vd), dtype=q.dtype, device=q.device)
+    out = _output(out, q, heads * vd)
     _grouped_checks("grouped_attention", q, cache, out, gate, heads, kv_heads, kd, vd, req_to_token)
     k = v = loc = None
     if new is not None:
@@ -1757,24 +1875,27 @@ def grouped_attention(q: torch.Tensor, cache: torch.Tensor, req_to_token: torch.
                 k.stride(0) if k is not None else 0, _ptr(v), v.stride(0) if v is not None else 0, _ptr(loc), req_to_token.data_ptr(),
                 req_to_token.stride(0), req_pool_indices.data_ptr(), _ptr(seg.tok_seg), positions.data_ptr(), _ptr(gate),
                 gate.stride(0) if gate is not None else 0, out.data_ptr(), out.stride(0), _ptr(po), _ptr(pml), T, heads, kv_heads, kd, vd, int(window),
-                splits, float(scale), *_sink_args("grouped_attention", sink, cap, gate, heads), 1 if plain else 0, _stream())
+                splits, float(scale), *_sink_args("grouped_attention", sink, cap, gate, heads), 1 if plain else 0,
+                *_variant_args("grouped_attention", keep, offsets, out_scale, heads), _stream())
     return out
 
 
 def grouped_prefill(q: torch.Tensor, cache: torch.Tensor, req_to_token: torch.Tensor, req_pool_indices: torch.Tensor, positions: torch.Tensor,
                     seg: Segments, blocks: QueryBlocks, heads: int, kv_heads: int, kd: int, vd: int, window: int, scale: float, *,
-                    sink=None, gate: Optional[torch.Tensor] = None, cap: Optional[float] = None) -> torch.Tensor:
+                    sink=None, gate: Optional[torch.Tensor] = None, cap: Optional[float] = None, keep: int = 0,
+                    offsets: Optional[torch.Tensor] = None, out_scale: float = 1.0, out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """grouped_attention over long extends whose keys are stored (bf16)."""
     _dev(q, cache, req_to_token, req_pool_indices, positions, gate, blocks.blocks)
     T = q.shape[0]
     _seg_checks("grouped_prefill", seg, req_pool_indices, positions, T)
-    out = torch.empty((T, heads * vd), dtype=q.dtype, device=q.device)
+    out = _output(out, q, heads * vd)
     _grouped_checks("grouped_prefill", q, cache, out, gate, heads, kv_heads, kd, vd, req_to_token)
     _need(_is_f32(q, cache, gate) == 0 and seg.start is not None and blocks.group == heads // kv_heads, "grouped_prefill: bf16 segments, blocks of this group size")
     native.call("sgl_amd_grouped_prefill", q.data_ptr(), q.stride(0), cache.data_ptr(), cache.stride(0), req_to_token.data_ptr(),
                 req_to_token.stride(0), req_pool_indices.data_ptr(), blocks.blocks.data_ptr(), blocks.blocks.shape[0], seg.start.data_ptr(),
                 seg.len.data_ptr(), positions.data_ptr(), _ptr(gate), gate.stride(0) if gate is not None else 0, out.data_ptr(), out.stride(0), heads,
-                kv_heads, kd, vd, int(window), float(scale), *_sink_args("grouped_prefill", sink, cap, gate, heads), _stream())
+                kv_heads, kd, vd, int(window), float(scale), *_sink_args("grouped_prefill", sink, cap, gate, heads),
+                *_variant_args("grouped_prefill", keep, offsets, out_scale, heads), _stream())
     return out
 
 
@@ -1786,33 +1907,44 @@ class SigmoidScores:
     def __init__(self, correction: Optional[torch.Tensor], groups: int = 1, keep: int = 1, scale: float = 1.0):
         self.correction, self.groups, self.keep, self.scale = correction, groups, keep, scale
 
+    KIND, GROUP_BEST = 1, 2
 
-def moe_route(h: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], top: int, scores: Optional[SigmoidScores] = None
-              ) -> Tuple[torch.Tensor, torch.Tensor]:
-    """The `top` largest of w h + bias (fp32) and the softmax over those, or what `scores` picks: fp32 weights, int32 ids [T, top]."""
+
+class SoftmaxScores(SigmoidScores):
+    """The same with the softmax over all experts as the scores; a group counts by its best."""
+
+    KIND, GROUP_BEST = 2, 1
+
+
+def moe_route(h: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], top: int, scores: Optional[SigmoidScores] = None,
+              identities: int = 0, gate_row: bool = False):
+    """The `top` largest of w h + bias (fp32) and the softmax over those, or what `scores` picks: fp32 weights, int32 ids [T, top].  The last
+    `identities` experts have the id -1.  gate_row: w has one more row; its sigmoid [T] is a third result."""
+    E = w.shape[0] - (1 if gate_row else 0)
     c = scores.correction if scores is not None else None
     _dev(h, w, bias, c)
     _rows("moe_route", h)
     _f32("moe_route", bias, c)
-    _need(c is None or c.numel() == w.shape[0], "moe_route: one correction an expert")
+    _need((c is None or c.numel() == E) and 0 <= identities <= E, "moe_route: one correction an expert")
     T, K = h.shape
-    _need(w.dim() == 2 and w.shape[1] == K and w.is_contiguous() and (bias is None or bias.numel() == w.shape[0]), "moe_route: shapes")
-    weights = torch.empty((T, top), dtype=torch.float32, device=h.device)
+    _need(w.dim() == 2 and w.shape[1] == K and w.is_contiguous() and (bias is None or bias.numel() == E), "moe_route: shapes")
+    weights = torch.empty((T, top + (1 if gate_row else 0)), dtype=torch.float32, device=h.device)
     ids = torch.empty((T, top), dtype=torch.int32, device=h.device)
-    f32, E, part, slices, pad = _is_f32(h, w), w.shape[0], None, 0, 0
-    if not f32 and T and E <= 256 and K % 8 == 0 and h.stride(0) % 8 == 0 and h.data_ptr() % 16 == 0:
+    f32, rows, part, slices, pad = _is_f32(h, w), w.shape[0], None, 0, 0
+    if not f32 and T and rows <= 256 and K % 8 == 0 and h.stride(0) % 8 == 0 and h.data_ptr() % 16 == 0:
         # one wave per 64 (32 at most experts, 16 at few) tokens and slice: waves enough for the chip, slices of 64 columns at least
-        pad = next(16 << i for i in range(5) if E <= 16 << i)
+        pad = next(16 << i for i in range(5) if rows <= 16 << i)
         blocks = -(-T // (16 if T <= 16 else 64 if pad <= 128 else 32))
         slices = max(1, min(-(-1024 // blocks), K // 64, 32))
         part = torch.empty((slices, T, pad), dtype=torch.float32, device=h.device)
     native.call("sgl_amd_moe_route", f32, h.data_ptr(), h.stride(0), w.data_ptr(), _ptr(bias), weights.data_ptr(), ids.data_ptr(), _ptr(part), slices,
-                pad, T, K, E, top, *((1, _ptr(c), scores.groups, scores.keep, float(scores.scale)) if scores is not None else (0, None, 1, 1, 1.0)), _stream())
-    return weights, ids
+                pad, T, K, E, top, *((scores.KIND, _ptr(c), scores.groups, scores.keep, scores.GROUP_BEST, float(scores.scale)) if scores is not None
+                                     else (0, None, 1, 1, 1, 1.0)), E - identities, 1 if gate_row else 0, _stream())
+    return (weights[:, :top], ids, weights[:, top]) if gate_row else (weights, ids)
 
 
 def _experts_plain(x: torch.Tensor, w: torch.Tensor, ids: torch.Tensor, up: bool, act: Glu = SILU) -> torch.Tensor:
-    E, N, K = w.shape[0], w.shape[1] // (2 if up else 1), w.shape[2]
+    E, N, K = w.shape[0], w.shape[1] // (2 if up and act.gated else 1), w.shape[2]
     pairs, top = ids.numel(), ids.shape[1]
     _rows("experts", x)
     _need(w.is_contiguous() and ids.dtype == torch.int32 and ids.is_contiguous() and x.shape == (ids.shape[0] if up else pairs, K), "experts: shapes")
@@ -1823,11 +1955,12 @@ def _experts_plain(x: torch.Tensor, w: torch.Tensor, ids: torch.Tensor, up: bool
 
 
 def routed_experts(h: torch.Tensor, w13: torch.Tensor, w2: torch.Tensor, ids: torch.Tensor, plain: bool = False, act: Glu = SILU) -> torch.Tensor:
-    """Every token's chosen experts, act(gate h, up h) and the down projection, unweighted: [T, top, W] in the type of h.  bf16 rows
+    """Every token's chosen experts, act(gate h, up h) -- or a Pointwise act(up h) with w13 [E, N, W] -- and the down projection, unweighted: [T,
+    top, W] in the type of h; rows of negative ids are left as they are.  bf16 rows
     run on the grouped matrix kernels of fused_experts; fp32 rows and sizes they do not take go through a plain form."""
     _dev(h, w13, w2, ids)
     (T, W), (E, N2, _), top = h.shape, w13.shape, ids.shape[1]
-    N, numel = N2 // 2, T * top
+    N, numel = N2 // (2 if act.gated else 1), T * top
     if plain or h.dtype != _BF16 or W % 8 or W < 32 or N % 32:
         return _experts_plain(_experts_plain(h, w13, ids, True, act), w2, ids, False).view(T, top, W)
     inter = torch.empty((numel, N), dtype=_BF16, device=h.device)
@@ -1835,11 +1968,11 @@ def routed_experts(h: torch.Tensor, w13: torch.Tensor, w2: torch.Tensor, ids: to
     if numel // E >= MOE_TILED_MIN_ROWS_PER_EXPERT and W % 64 == 0 and N % 64 == 0:
         block_m, up_rows, down_rows = moe_tile_plan(numel, E, N, W) if MOE_TILE_OVERRIDE is None else MOE_TILE_OVERRIDE
         s = moe_align_block_size(ids, block_m, E)
-        moe_tiled_gemm(h, w13, inter, *s, None, False, top, numel, block_m, fuse_silu=True, tile_rows=up_rows, act=act)
+        moe_tiled_gemm(h, w13, inter, *s, None, False, top, numel, block_m, fuse_silu=act.gated, tile_rows=up_rows, act=act)
         moe_tiled_gemm(inter, w2, down, *s, None, False, 1, numel, block_m, tile_rows=down_rows)
     else:
         block_m = choose_moe_block_m(numel, E)
         s = moe_align_block_size(ids, block_m, E)
-        (moe_wstream_gemm if W % 128 == 0 else moe_grouped_gemm)(h, w13, inter, *s, None, False, top, numel, block_m, fuse_silu=True, act=act)
+        (moe_wstream_gemm if W % 128 == 0 else moe_grouped_gemm)(h, w13, inter, *s, None, False, top, numel, block_m, fuse_silu=act.gated, act=act)
         (moe_wstream_gemm if W % 16 == 0 and N % 128 == 0 else moe_grouped_gemm)(inter, w2, down, *s, None, False, 1, numel, block_m)
     return down.view(T, top, W)

@@ -99,34 +99,37 @@ class HybridAttnBackend(AttentionBackend):
         kernels.grouped_kv_store(k, v, rows, forward_batch.out_cache_loc, layer.kv_heads)
         return self._grouped(layer, q, gate, rows, None, forward_batch)
 
-    def prepared_attention(self, layer, p, run_id: int, forward_batch) -> torch.Tensor:
-        """p: the projection [queries | keys | values | gate], rows or Partials -> gated values [T, heads * vd]; one launch norms, turns and
-        stores in front of attention."""
+    def prepared_attention(self, layer, p, run_id: int, forward_batch, out=None):
+        """p: the projection [queries | keys | values | gate, or columns of a mixer beside], rows or Partials -> gated values [T, heads * vd] (in the
+        rows `out` if given), and the columns beside as rows (or None); one launch norms, turns and stores in front of attention."""
+        tail = layer.gate_cols + layer.beside_cols
         rows = self.token_to_kv_pool.get_kv_rows(run_id)
         q, gate = kernels.head_prepare(p, layer.heads, layer.dim, layer.kd, forward_batch.positions, layer.cos_sin, layer.eps, norms=layer.norms,
-                                       norm_after=layer.norm_after, gate_cols=(layer.gate_cols + 7) // 8 * 8,
+                                       norm_after=layer.norm_after, gate_cols=(tail + 7) // 8 * 8, value_is_key=layer.value_is_key,
                                        kv=(layer.kv_heads, layer.vd, rows, forward_batch.out_cache_loc))
-        return self._grouped(layer, q, gate[:, :layer.gate_cols] if gate is not None else None, rows, None, forward_batch)
+        beside, gate = (gate[:, :tail], None) if layer.beside_cols else (None, gate[:, :tail] if gate is not None else None)
+        return self._grouped(layer, q, gate, rows, None, forward_batch, out), beside
 
-    def _grouped(self, layer, q: torch.Tensor, gate, rows: torch.Tensor, new, forward_batch) -> torch.Tensor:
+    def _grouped(self, layer, q: torch.Tensor, gate, rows: torch.Tensor, new, forward_batch, out=None) -> torch.Tensor:
         """Queries over the stored rows, and over the step's own keys and values `new` of a decode batch that are not stored yet."""
         T, form = q.shape[0], self.grouped_form
         matrix = layer.matrix and form != "plain"
         sizes = (layer.heads, layer.kv_heads, layer.kd, layer.vd, layer.window, layer.scale)
+        variant = dict(sink=layer.sink, gate=gate, cap=layer.cap, keep=layer.keep_first, offsets=layer.offsets, out_scale=layer.out_scale, out=out)
         where = (rows, self.req_to_token_pool.req_to_token, forward_batch.req_pool_indices, forward_batch.positions, self.segments)
         if (matrix and layer.prefill and forward_batch.forward_mode.is_extend()
                 and (max(self._extend[1]) >= self.PREFILL_MIN_TOKENS if form is None else form == "prefill")):
             key = (layer.window, layer.group)
             if key not in self._blocks:
                 self._blocks[key] = kernels.QueryBlocks(*self._extend, layer.window, layer.group, self.device)
-            return kernels.grouped_prefill(q, *where, self._blocks[key], *sizes, sink=layer.sink, gate=gate, cap=layer.cap)
-        return kernels.grouped_attention(q, *where, *sizes, sink=layer.sink, gate=gate, new=new, splits=self._grouped_splits(layer, T, matrix),
-                                         plain=not matrix, cap=layer.cap)
+            return kernels.grouped_prefill(q, *where, self._blocks[key], *sizes, **variant)
+        return kernels.grouped_attention(q, *where, *sizes, new=new, splits=self._grouped_splits(layer, T, matrix),
+                                         plain=not matrix, **variant)
 
     def _grouped_splits(self, layer, tokens: int, matrix: bool) -> int:
         """Workgroups enough for the chip on small batches, never shorter than 128 keys; a function of the batch size and the context
         bound only (fixed inside a captured graph)."""
-        keys = min(layer.window, self.max_context_len) if layer.window > 0 else self.max_context_len
+        keys = min(layer.window + layer.keep_first, self.max_context_len) if layer.window > 0 else self.max_context_len
         groups = layer.kv_heads * ((layer.group + 15) // 16) if matrix else layer.heads
         want = (512 + tokens * groups - 1) // (tokens * groups)
         return max(1, min(want, (keys + 127) // 128, 32))
@@ -171,3 +174,19 @@ class HybridAttnBackend(AttentionBackend):
         qkv = kernels.causal_conv_silu(qkv, layer.conv_weight, None, self.state_pool.conv[run_id], slots, pos, self.segments)
         return kernels.gated_delta_scan(qkv, b, a, layer.A_log, layer.dt_bias, self.state_pool.state[run_id], slots, pos, self.segments,
                                         layer.kv_heads, layer.dim ** -0.5)
+
+    def matrix_memory(self, layer, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, i: torch.Tensor, f: torch.Tensor, run_id: int,
+                      forward_batch) -> torch.Tensor:
+        pool = self.state_pool
+        return kernels.memory_scan(q, k, v, i, f, layer.bias_i, layer.bias_f, pool.state[run_id], pool.norm[run_id], forward_batch.req_pool_indices,
+                                   forward_batch.positions, self.segments, layer.cap, layer.dim ** -0.5)
+
+    def token_shift(self, mu: torch.Tensor, layer_id: int, forward_batch):
+        """What a launch that norms a batch of single tokens needs to shift them on the way (kernels.TokenShift); other batches: None."""
+        if self.segments.start is not None:
+            return None
+        return kernels.TokenShift(mu, self.state_pool.shift[layer_id], forward_batch.req_pool_indices, forward_batch.positions)
+
+    def shift_rows(self, h: torch.Tensor, mu: torch.Tensor, layer_id: int, forward_batch, out: torch.Tensor) -> torch.Tensor:
+        """The token shift of a batch with segments."""
+        return kernels.token_shift(h, mu, self.state_pool.shift[layer_id], forward_batch.req_pool_indices, forward_batch.positions, self.segments, out)

@@ -1,6 +1,5 @@
-"""Token mixers beside RadixAttention: latent attention, grouped-query attention with sizes of its own, the gated delta rule and
-Mamba-2.  A mixer owns its projections and
-constants; caches, states and kernel dispatch belong to the attention backend (layers/attention/hybrid_backend.py).
+"""Token mixers beside RadixAttention: latent attention, grouped-query attention with sizes of its own, the gated delta rule, Mamba-2, a
+matrix memory with exponential gates, and the last beside attention.  A mixer owns its projections and constants; caches, states and kernel dispatch belong to the attention backend (layers/attention/hybrid_backend.py).
 
 Every module takes its tensors from `get(name, shape, init)` (harness/weights.py) and merges the projections that share an
 input into one product, its rows padded to a multiple of 16."""
@@ -13,6 +12,7 @@ import torch
 from torch import nn
 
 from .. import kernels
+from ..mem_cache.memory_pool import StateSpec
 
 
 def merged_rows(parts: List[torch.Tensor]) -> torch.Tensor:
@@ -40,12 +40,19 @@ def yarn_frequencies(f: torch.Tensor, dims: int, base: float, s: dict):
     return f / s["factor"] * ramp + f * (1.0 - ramp), 0.1 * math.log(s["factor"]) + 1.0
 
 
+def scaled_frequencies(f: torch.Tensor, dims: int, base: float, s: dict):
+    """The frequencies under a scaling, and the factor on cos and sin: YaRN, or (no original length) all divided by s['factor']."""
+    if "original" in s:
+        return yarn_frequencies(f, dims, base, s)
+    return f / s["factor"], 1.0
+
+
 def rotary_table(positions: int, dims: int, base: float, device, scaling: Optional[dict] = None) -> torch.Tensor:
     """fp32 cos | sin of p * base^(-2i / dims), evaluated in double so that far positions keep their angle; `scaling` as in
-    yarn_frequencies."""
+    scaled_frequencies."""
     f, factor = float(base) ** (-2.0 * torch.arange(dims // 2, dtype=torch.float64) / dims), 1.0
     if scaling is not None:
-        f, factor = yarn_frequencies(f, dims, float(base), scaling)
+        f, factor = scaled_frequencies(f, dims, float(base), scaling)
     a = torch.arange(positions, dtype=torch.float64)[:, None] * f[None, :]
     return (torch.cat([a.cos(), a.sin()], 1) * factor).to(torch.float32).contiguous().to(device)
 
@@ -108,24 +115,35 @@ def padded_heads(w: torch.Tensor, heads: int, dim: int, to: int, axis: int) -> t
 
 
 class GroupedAttention(nn.Module):
-    """Grouped-query attention: own key and value widths, an optional sliding window (mask.size), an optional soft cap of the scores
+    """Grouped-query attention: own key and value widths, an optional sliding window (mask.size, with mask.keep_first first tokens that stay
+    visible), an optional soft cap of the scores
     (softcap), an optional sink (a score in the softmax denominator that carries no value: a constant, or "learned", one a head), an
     optional sigmoid gate on the heads' outputs ("elements", or "heads": one number each), biases on queries, keys and values,
     rotation by halves (rot), and an RMS norm a head on queries and keys: "before" the rotation, with weights, or "after" it, without.
-    Head vectors are padded with zeros to multiples of 8 elements, in the projections and in the cache."""
+    value_is_key: the values are the keys as projected.  offsets: a learned number a head ("pb") joins the scores, and a key's weight is
+    their sigmoid instead of the softmax.  Head vectors are padded with zeros to multiples of 8 elements, in the projections and in the cache.
+
+    `beside` are weights of another mixer that reads the same input: their columns follow this one's in the projection.  A mixer that is part
+    of another one (out_scale: its factor there) leaves the output projection to it."""
 
     def __init__(self, width: int, m: dict, eps: float, get: Callable, linear: Callable, max_positions: int, device, *,
                  sink: Union[None, float, str] = None, gate: Optional[str] = None, bias: bool = False, rotary: bool = False,
-                 qk_norm: Optional[str] = None):
+                 qk_norm: Optional[str] = None, value_is_key: bool = False, offsets: bool = False, beside: Optional[List[torch.Tensor]] = None,
+                 out_scale: Optional[float] = None):
         super().__init__()
         self.heads, self.kv_heads, dim, vdim = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        self.keep_first = (m.get("mask") or {}).get("keep_first", 0)
+        self.value_is_key, self.out_scale = value_is_key, 1.0 if out_scale is None else float(out_scale)
+        if value_is_key and vdim != dim:
+            raise ValueError(f"grouped attention: values of {vdim} that are keys of {dim}")
         self.window, self.scale, self.cap, self.eps = (m.get("mask") or {}).get("size", 0), float(m["scale"]), m.get("softcap"), eps
         H, G = self.heads, self.kv_heads
         if H % G:
             raise ValueError(f"grouped attention: {H} query heads over {G} key heads")
         self.kd, self.vd, self.group = dim + -dim % 8, vdim + -vdim % 8, H // G
         self.sink = get("sink", (H,)).float() if sink == "learned" else sink
-        heads = (("q", H, dim, self.kd), ("k", G, dim, self.kd), ("v", G, vdim, self.vd))
+        self.offsets = get("pb", (H,)).float() if offsets else None
+        heads = (("q", H, dim, self.kd), ("k", G, dim, self.kd)) + (() if value_is_key else (("v", G, vdim, self.vd),))
         parts = [padded_heads(get(n, (c * d, width)), c, d, to, 0) for n, c, d, to in heads]
         biases = [padded_heads(get(n + ".b", (c * d,), "zeros")[:, None], c, d, to, 0) for n, c, d, to in heads] if bias else []
         self.gate_cols = {None: 0, "heads": H, "elements": H * self.vd}[gate]
@@ -135,17 +153,25 @@ class GroupedAttention(nn.Module):
             parts.append(padded_heads(get("g", (H * vdim, width)), H, vdim, self.vd, 0))
         if bias and gate is not None:
             biases.append(torch.zeros_like(parts[-1][:, :1]))
+        self.beside_cols = sum(w.shape[0] for w in beside or ())
+        if self.beside_cols:
+            if gate is not None:
+                raise ValueError("grouped attention: a gate beside another mixer's columns")
+            parts += beside
+            biases += [torch.zeros_like(w[:, :1]) for w in beside] if bias else []
         self.in_proj = linear(merged_rows(parts), merged_rows(biases)[:, 0].contiguous()) if bias else linear(merged_rows(parts))
         self.dim, self.cos_sin, self.norms, self.norm_after = dim, None, None, qk_norm == "after"
         if rotary:
             rot = m["rot"]
             if rot["dims"] % 2 or rot["dims"] > dim:
                 raise ValueError(f"grouped attention: {rot['dims']} rotated dimensions in heads of {dim}")
-            self.cos_sin = rotary_table(max_positions, rot["dims"], rot["base"], device, rot.get("scaling"))
+            if rot["dims"]:
+                self.cos_sin = rotary_table(max_positions, rot["dims"], rot["base"], device, rot.get("scaling"))
         if qk_norm == "before":
             self.norms = tuple(padded_heads(get(n, (dim,), "ones").float(), 1, dim, self.kd, 0) for n in ("q.norm", "k.norm"))
-        self.prepared = rotary or qk_norm is not None      # a launch between the projection and attention
-        self.o_proj = linear(padded_heads(get("o", (width, H * vdim)), H, vdim, self.vd, 1).contiguous())
+        self.prepared = rotary or qk_norm is not None or value_is_key or self.beside_cols > 0      # a launch between the projection and attention
+        o = padded_heads(get("o", (width, H * vdim)), H, vdim, self.vd, 1).contiguous()
+        self.o_proj, self.out_weight = (linear(o), None) if out_scale is None else (None, o)
         self.matrix = self.in_proj.weight.dtype == torch.bfloat16 and self.scale > 0 and kernels.grouped_attention_matrix_form(self.kd, self.vd)
         self.prefill = self.matrix and kernels.grouped_prefill_supported(self.kd, self.vd, self.group)
 
@@ -155,7 +181,8 @@ class GroupedAttention(nn.Module):
 
     def forward(self, h: torch.Tensor, run_id: int, fb) -> torch.Tensor:
         if self.prepared:
-            return self.o_proj.forward_partials(fb.attn_backend.prepared_attention(self, self.in_proj.forward_partials(h), run_id, fb))
+            o, _ = fb.attn_backend.prepared_attention(self, self.in_proj.forward_partials(h), run_id, fb)
+            return self.o_proj.forward_partials(o)
         p = self.in_proj(h)
         a = self.heads * self.kd
         b = a + self.kv_heads * self.kd
@@ -216,6 +243,70 @@ class Mamba2(nn.Module):
         i, c = self.inner, self.conv_channels
         y = fb.attn_backend.mamba2(self, p[:, i:i + c], p[:, i + c:i + c + self.heads], run_id, fb)
         return self.o_proj.forward_partials(kernels.gated_rmsnorm(y, p[:, :i], self.norm_weight, self.norm_groups, self.eps, gate_first=True))
+
+
+class MatrixMemory(nn.Module):
+    """A matrix memory with exponential gates (mLSTM), read through an RMS norm a head and a sigmoid gate.  It has no projection of its own:
+    `parts` are the rows [q | k | v | gate | input gates | forget gates] of the one it shares, `out_weight` goes into a common output
+    projection.  out_scale: the factor of its output there (it rides on the norm's weights)."""
+
+    def __init__(self, width: int, m: dict, eps: float, get: Callable, out_scale: float = 1.0):
+        super().__init__()
+        self.heads, self.dim, self.vdim, self.cap, self.eps = m["heads"], m["dim"], m["vdim"], float(m["gate_cap"]), eps
+        H, qk, v = self.heads, self.heads * self.dim, self.heads * self.vdim
+        self.parts = [get(n, (rows, width)) for n, rows in (("q", qk), ("k", qk), ("v", v), ("g", v), ("i", H), ("f", H))]
+        self.starts = [0, qk, 2 * qk, 2 * qk + v, 2 * qk + 2 * v, 2 * qk + 2 * v + H, 2 * qk + 2 * v + 2 * H]
+        self.bias_i, self.bias_f = get("i.b", (H,), "zeros").float(), get("f.b", (H,), "zeros").float()
+        self.norm_weight = get("norm", (v,), "ones").float() * out_scale
+        self.out_weight = get("o", (width, v))
+
+    @property
+    def state_spec(self) -> StateSpec:
+        return StateSpec(self.heads, self.dim, self.vdim, norm=True)
+
+    def forward(self, p: torch.Tensor, run_id: int, fb, out: torch.Tensor) -> torch.Tensor:
+        q, k, v, g, i, f = (p[:, a:b] for a, b in zip(self.starts, self.starts[1:]))
+        o = fb.attn_backend.matrix_memory(self, q, k, v, i, f, run_id, fb)
+        return kernels.gated_rmsnorm(o, g, self.norm_weight, self.heads, self.eps, gate_first=False, out=out, sigmoid_gate=True)
+
+
+class Parallel(nn.Module):
+    """Attention and a matrix memory side by side on one input: left_scale * attention + right_scale * memory.  One projection in front of
+    both, one behind both: the factors ride on the heads' outputs, which are rounded behind them.  The bias of the output projection is left
+    to the launch that sums the residual (out_bias)."""
+
+    def __init__(self, width: int, m: dict, eps: float, get: Callable, linear: Callable, max_positions: int, device, **attention):
+        super().__init__()
+
+        def side(name):
+            return lambda n, shape, init=None: get(f"{name}.{n}", shape, init)
+
+        ls = float(m["left_scale"])
+        self.right = MatrixMemory(width, m["right"], eps, side("right"), float(m["right_scale"]))
+        self.left = GroupedAttention(width, m["left"], eps, side("left"), linear, max_positions, device, beside=self.right.parts, out_scale=ls, **attention)
+        self.out_bias = side("left")("o.b", (width,), "zeros").float() * ls
+        self.right.parts = None                            # (they are in the projection)
+        a, b = self.left.out_weight, self.right.out_weight
+        self.split, used = a.shape[1], a.shape[1] + b.shape[1]
+        self.pad = -used % 8
+        self.o_proj = linear(torch.cat([a, b] + ([a.new_zeros((width, self.pad))] if self.pad else []), 1).contiguous())
+        self.left.out_weight = self.right.out_weight = None
+
+    @property
+    def cache_spec(self):
+        return self.left.cache_spec
+
+    @property
+    def state_spec(self):
+        return self.right.state_spec
+
+    def forward(self, h: torch.Tensor, run_id, fb) -> torch.Tensor:
+        """run_id: (of the attention's cache, of the memory's state)."""
+        both = (torch.zeros if self.pad else torch.empty)((h.shape[0], self.o_proj.weight.shape[1]), dtype=h.dtype, device=h.device)
+        a, b = self.split, both.shape[1] - self.pad
+        _, rest = fb.attn_backend.prepared_attention(self.left, self.left.in_proj.forward_partials(h), run_id[0], fb, out=both[:, :a])
+        self.right(rest, run_id[1], fb, both[:, a:b])
+        return self.o_proj.forward_partials(both)
 
 
 MIXERS = {"latent_attention": LatentAttention, "delta": GatedDelta, "mamba2": Mamba2}

@@ -13,7 +13,7 @@ kernels gather with 16-byte lanes.
 from __future__ import annotations
 
 from dataclasses import dataclass
-from typing import List, Optional
+from typing import List, NamedTuple, Optional
 
 import torch
 
@@ -237,25 +237,40 @@ class LayeredTokenToKVPool:
         return self.grouped.get_kv_size_bytes()[0] + self.latent.get_kv_size_bytes()[0] + ids, 0
 
 
+class StateSpec(NamedTuple):
+    """What a recurrent run keeps of a request."""
+
+    heads: int
+    rows: int
+    cols: int
+    taps: int = 0              # of a short convolution, and its channels
+    channels: int = 0
+    norm: bool = False         # a normalizer beside the state: a vector of `rows` and a running maximum a head
+
+
 class RecurrentStatePool:
-    """One slot per request row for every recurrent run: the fp32 state [slots, heads, rows, columns] and the ring of past
-    convolution inputs [slots, taps, channels] in the activation type.  Slot 0 absorbs padded (graph) batch entries.  A
+    """One slot per request row for every recurrent run: the fp32 state [slots, heads, rows, columns], the ring of past
+    convolution inputs [slots, taps, channels] in the activation type, and the normalizer fp32 [slots, heads, column blocks of 16, rows + 1]
+    (or None).  `shift`: per layer the last row [slots, width] of a token shift.  Slot 0 absorbs padded (graph) batch entries.  A
     request that starts at position 0 ignores what its slot holds (the kernels begin from zero), so slots are never cleared."""
 
-    def __init__(self, num_slots: int, specs, dtype: torch.dtype, device):
-        """specs: per run (heads, state rows, state columns, conv taps, conv channels)."""
+    def __init__(self, num_slots: int, specs, dtype: torch.dtype, device, shift_widths=()):
         self.num_slots = num_slots
-        self.state = [torch.zeros((num_slots, h, n, p), dtype=torch.float32, device=device) for h, n, p, _, _ in specs]
-        self.conv = [torch.zeros((num_slots, taps, ch), dtype=dtype, device=device) for _, _, _, taps, ch in specs]
+        specs = [StateSpec(*s) for s in specs]
+        self.state = [torch.zeros((num_slots, s.heads, s.rows, s.cols), dtype=torch.float32, device=device) for s in specs]
+        self.conv = [torch.zeros((num_slots, s.taps, s.channels), dtype=dtype, device=device) for s in specs]
+        self.norm = [torch.zeros((num_slots, s.heads, (s.cols + 15) // 16, s.rows + 1), dtype=torch.float32, device=device) if s.norm else None
+                     for s in specs]
+        self.shift = [torch.zeros((num_slots, w), dtype=dtype, device=device) for w in shift_widths]
 
     def size_bytes(self) -> int:
-        return sum(t.numel() * t.element_size() for t in self.state + self.conv)
+        return sum(t.numel() * t.element_size() for t in self.state + self.conv + self.norm + self.shift if t is not None)
 
 
 class HybridReqToTokenPool(ReqToTokenPool):
     """Request rows of a model with recurrent layers: row i of req_to_token and state slot i belong to the same request, so
     taking and returning a row takes and returns its recurrent state."""
 
-    def __init__(self, size: int, max_context_len: int, device, state_specs, dtype: torch.dtype):
+    def __init__(self, size: int, max_context_len: int, device, state_specs, dtype: torch.dtype, shift_widths=()):
         super().__init__(size, max_context_len, device)
-        self.state_pool = RecurrentStatePool(self._alloc_size, state_specs, dtype, device)
+        self.state_pool = RecurrentStatePool(self._alloc_size, state_specs, dtype, device, shift_widths)

@@ -108,7 +108,8 @@ def test_hybrid_kernels_keep_their_state_in_registers(tmp_path):
     """The chunked recurrences hold the state tile in accumulators over a whole segment and the latent attention kernels hold
     queries and output sums: a spill would sit inside their loops.  (bf16 instances of the sizes real layers have.)"""
     usage = _resource_usage("recurrent_chunk.hip", tmp_path)
-    for kernel in ("mamba2_chunk_kernelItLi8E", "delta_chunk_kernelItLi8E", "mamba2_chunk_kernelItLi4E", "delta_chunk_kernelItLi4E"):
+    for kernel in ("mamba2_chunk_kernelItLi8E", "delta_chunk_kernelItLi8E", "mamba2_chunk_kernelItLi4E", "delta_chunk_kernelItLi4E", "memory_chunk_kernelItLi8E",
+                   "memory_chunk_kernelItLi4E"):
         inst = {k: v for k, v in usage.items() if kernel in k}
         assert len(inst) == 1, sorted(usage)
         for name, u in inst.items():
@@ -128,7 +129,7 @@ def test_grouped_attention_kernels_keep_their_sums_in_registers(tmp_path):
     usage = _resource_usage("grouped_attention.hip", tmp_path)
     decode = {k: v for k, v in usage.items() if "grouped_attention_mfma_kernel" in k}
     prefill = {k: v for k, v in usage.items() if "grouped_prefill_kernel" in k}
-    assert len(decode) == 9 and len(prefill) == 6, sorted(usage)
+    assert len(decode) == 18 and len(prefill) == 12, sorted(usage)      # softmax and sigmoid weights
     for name, u in decode.items():
         assert u["vgpr_spill_count"] <= (20 if "ILi8ELi16E" in name else 0) and u["vgpr_count"] <= 256, (name, u)
     for name, u in prefill.items():
