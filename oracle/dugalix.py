@@ -186,3 +186,103 @@ def forward(cfg: dict, weights: Dict[str, torch.Tensor], tokens: List[int], dtyp
             x = x + m * norm(moe(h, sub, f) if f["kind"] == "moe" else feed_forward(h, sub), w[p + "norm2b"], eps)
         trace.append(x)
     return oh.linear(oh._r(norm(x, w["final.norm"], eps)), w["head"]), trace
+
+
+# ---------------------------------------------------------------------------------------------- random models
+def tensor_shapes(cfg: dict) -> Dict[str, Tuple[int, ...]]:
+    W = cfg["width"]
+    out: Dict[str, Tuple[int, ...]] = {"embed": (cfg["vocab"], W), "head": (cfg["vocab"], W), "final.norm": (W,)}
+
+    def feed(prefix, ff):
+        out.update({prefix + "up": (ff, W), prefix + "down": (W, ff)})
+
+    for i, lay in enumerate(cfg["layers"]):
+        m, f, p = lay["mixer"], lay["mlp"], f"l{i}."
+        out.update({p + "norm1": (W,), p + "norm1b": (W,), p + "shift": (W,)})
+        if lay["type"] == "attention":
+            H, G, D = m["heads"], m["kv_heads"], m["dim"]
+            mix = {"q": (H * D, W), "k": (G * D, W), "pb": (H,), "o": (W, H * D)}
+        else:
+            a, r = m["left"], m["right"]
+            rows = {"q": a["heads"] * a["dim"], "k": a["kv_heads"] * a["dim"], "v": a["kv_heads"] * a["vdim"]}
+            mix = {f"left.{n}": (c, W) for n, c in rows.items()}
+            mix.update({f"left.{n}.b": (c,) for n, c in rows.items()})
+            mix.update({"left.o": (W, a["heads"] * a["vdim"]), "left.o.b": (W,)})
+            H, D, V = r["heads"], r["dim"], r["vdim"]
+            mix.update({f"right.{n}": (c, W) for n, c in (("q", H * D), ("k", H * D), ("v", H * V), ("g", H * V), ("i", H), ("f", H))})
+            mix.update({"right.i.b": (H,), "right.f.b": (H,), "right.norm": (H * V,), "right.o": (W, H * V)})
+        out.update({p + "mix." + n: s for n, s in mix.items()})
+        if f is None:
+            continue
+        out.update({p + "norm2": (W,), p + "norm2b": (W,)})
+        if f["kind"] == "dense":
+            feed(p + "mlp.", f["ff"])
+            continue
+        members = f["router"]["experts"] + f["router"].get("identity", 0)
+        for e in range(f["router"]["experts"]):
+            feed(f"{p}mlp.e{e}.", f["expert"]["ff"])
+        out[p + "mlp.router"], out[p + "mlp.correction"] = (members, W), (members,)
+        if f.get("shared"):
+            feed(p + "mlp.shared.", f["shared"]["ff"])
+            out[p + "mlp.shared.sg"] = (1, W)
+    return out
+
+
+CODE_DIMS, CODES = 8, 12
+
+
+def random_weights(cfg: dict, seed: int) -> Dict[str, torch.Tensor]:
+    """bf16 weights whose every branch matters: matrices keep unit variance, norms make unit rows, offsets, biases and gates are of the size
+    of what they join, memories last for tens of tokens, corrections reach below zero.  No token sits between two experts: the first
+    CODE_DIMS columns of the embedding hold one of CODES sign patterns, nothing else writes to those columns of the residual or reads
+    them, except the routers, which read nothing else and are drawn until the choice of every pattern is clear.  The patterns are large, so
+    that the rest of the residual hardly changes what the norm makes of them."""
+    g = torch.Generator().manual_seed(seed)
+    code = torch.randint(0, 2, (CODES, CODE_DIMS), generator=g) * 2.0 - 1.0
+    amplitude = math.sqrt(6.0 * cfg["width"] / CODE_DIMS)     # the patterns add 6 to the mean square of a row, everything else 1 to 5
+    shapes, out = tensor_shapes(cfg), {}
+    for name, shape in shapes.items():
+        r = torch.randn(shape, generator=g)
+        last = name.split(".")[-1]
+        if last in ("norm1", "norm1b", "norm2", "norm2b", "norm"):
+            t = 0.2 * r + 1.0 if name.endswith("right.norm") else 0.2 * r if last.endswith("b") else 1.9 + 0.5 * r
+        elif last == "shift":
+            t = 0.4 + 0.3 * r
+        elif last in ("embed", "pb"):
+            t = r
+        elif last == "b":
+            t = r * 0.5 + (2.5 if name.endswith("f.b") else 0.0)
+        elif last == "correction":
+            t = r * 0.08 - 0.03
+        else:
+            t = r / math.sqrt(shape[1])
+        if last == "embed":
+            t[:, :CODE_DIMS] = code[torch.arange(shape[0]) % CODES] * amplitude
+        elif last in ("norm1", "norm1b", "norm2b") or name == "final.norm":
+            t[:CODE_DIMS] = -1.0
+        elif last == "norm2":
+            t[:CODE_DIMS] = 5.8 / amplitude - 1.0
+        elif last in ("up", "sg"):
+            t[:, :CODE_DIMS] = 0.0
+        out[name] = t.to(torch.bfloat16)
+    saved = list(margins)
+    seen = torch.cat([code * s for s in (1.66, 1.8, 2.0, 2.25)]).double()
+    for i, lay in enumerate(cfg["layers"]):
+        if lay["mlp"] is None or lay["mlp"]["kind"] != "moe":
+            continue
+        name, best = f"l{i}.mlp.router", None
+        for _ in range(300):
+            w = torch.zeros(shapes[name])
+            w[:, :CODE_DIMS] = torch.randn((shapes[name][0], CODE_DIMS), generator=g) * 0.4
+            w = w.to(torch.bfloat16)
+            margins.clear()
+            picks = [{e for e, _ in t} for t in route(seen, w[:, :CODE_DIMS].double(), out[f"l{i}.mlp.correction"].double(), lay["mlp"]["router"])]
+            changes = sum(p != picks[k % CODES] for k, p in enumerate(picks))
+            gap = min(margins, default=1.0) - changes
+            if best is None or gap > best[0]:
+                best = (gap, w)
+            if gap > 0.01:
+                break
+        out[name] = best[1]
+    margins[:] = saved
+    return out
