@@ -188,7 +188,7 @@ def parse_args():
     ap.add_argument("--cpu-budget-s", type=float, default=30.0)
     ap.add_argument("--hybrid", nargs="*", metavar="NAME", default=None,
                     help="instead of the default workload: throughput and kernel table of layered models (default genusun-1b genusun-8b; also "
-                         "mosurax-1b mosurax-8b bulodra-1b bulodra-8b) beside the closest models of equal size, on one GPU")
+                         "mosurax-1b mosurax-8b bulodra-1b bulodra-8b dugalix-1b dugalix-8b) beside the closest models of equal size, on one GPU")
     ap.add_argument("--hybrid-kernels-only", action="store_true", help="with --hybrid: the kernel table alone")
     return ap.parse_args()
 

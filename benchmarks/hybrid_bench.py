@@ -1,5 +1,5 @@
-"""Throughput of the layered designs (Genusun here, Mosurax with grouped_bench.py, Bulodra with layered_bench.py) beside the closest decoders of this framework at
-equal size, and every kernel of a design against its roofline beside the like kernel of such a decoder.  Run through
+"""Throughput of the layered designs (Genusun here, Mosurax with grouped_bench.py, Bulodra with layered_bench.py, Dugalix with
+shifted_bench.py) beside the closest decoders of this framework at equal size, and every kernel of a design against its roofline beside the like kernel of such a decoder.  Run through
 `bench.py --hybrid`; random weights.
 
 The decoder beside it has the same width, feed-forward width, vocabulary and number of attention heads and as many layers as the
@@ -235,15 +235,17 @@ def kernel_table(cfg, device, T=8192, segs=4, B=64, ctx=1024):
 
 
 def run(names, device, kernels_only=False):
-    from benchmarks import grouped_bench, layered_bench
+    from benchmarks import grouped_bench, layered_bench, shifted_bench
     from sglang_amd.harness.bulodra import BulodraConfig
+    from sglang_amd.harness.dugalix import DugalixConfig
     from sglang_amd.harness.mosurax import MosuraxConfig
     from sglang_amd.harness.registry import named_config
 
     out = {}
     for name in names:
         cfg = named_config(name)
-        key, table, beside = (("design", layered_bench.kernel_table, layered_bench.models_beside) if isinstance(cfg, BulodraConfig) else
+        key, table, beside = (("design", shifted_bench.kernel_table, shifted_bench.models_beside) if isinstance(cfg, DugalixConfig) else
+                              ("design", layered_bench.kernel_table, layered_bench.models_beside) if isinstance(cfg, BulodraConfig) else
                               ("design", grouped_bench.kernel_table, grouped_bench.decoders_beside) if isinstance(cfg, MosuraxConfig) else
                               ("hybrid", kernel_table, lambda c: {"decoder_beside": _llama_beside(c)}))
         shape = dict(prompts=4, length=2048, batch=64, ctx=1024)

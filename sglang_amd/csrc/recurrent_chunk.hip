@@ -506,7 +506,9 @@ __global__ __launch_bounds__(256, NT <= 8 ? 2 : 1) void memory_chunk_kernel(Memo
   __shared__ __attribute__((aligned(16))) float Qs[kQ * LS];
   __shared__ __attribute__((aligned(16))) float Gs[kQ * kSq];
   __shared__ __attribute__((aligned(16))) float ns[NP];
-  __shared__ double cum[kQ], as[kQ], gs[kQ];
+  // what the gates of a chunk make, formed a chunk ahead: a_j, g_i, e^{a_j-g_n}, e^{m0-g_i}, e^{-c_i-g_i}, and the m behind the chunk
+  __shared__ double as[2][kQ], gs[2][kQ];
+  __shared__ float add_w[2][kQ], keep_w[2][kQ], floor_w[2][kQ], m_next[2];
   __shared__ float inv[kQ];
   const int b = blockIdx.y, h = blockIdx.x;
   constexpr int waves = 4;
@@ -529,7 +531,7 @@ __global__ __launch_bounds__(256, NT <= 8 ? 2 : 1) void memory_chunk_kernel(Memo
       s[t][r] = pos0 > 0 && live && n < p.D ? S[static_cast<int64_t>(n) * p.V] : 0.f;
     }
   if (threadIdx.x < NP) ns[threadIdx.x] = pos0 > 0 && static_cast<int>(threadIdx.x) < p.D ? norm[threadIdx.x] : 0.f;
-  double m0 = pos0 > 0 ? norm[p.D] : 0.f;
+  float m0 = pos0 > 0 ? norm[p.D] : 0.f;
   const float bi = p.bi[h], bf = p.bf[h];
   const T* qp = static_cast<const T*>(p.q) + t0 * p.stride + h * p.D;
   const T* kp = static_cast<const T*>(p.k) + t0 * p.stride + h * p.D;
@@ -552,28 +554,46 @@ __global__ __launch_bounds__(256, NT <= 8 ? 2 : 1) void memory_chunk_kernel(Memo
         const int j = 16 * tj + 4 * g + r;
         vr[tj][r] = live && j < len ? vp[row + j * p.stride] : T{};
       }
-    if (wave == 0 && lane < len) {
-      ir = ip[row + lane * p.stride];
-      fr = fp[row + lane * p.stride];
+  };
+  // the last wave, which has no part in the Gram tiles, fetches the gates two chunks ahead and scans them one chunk ahead
+  auto fetch_gates = [&](int c0) __attribute__((always_inline)) {
+    if (c0 + lane < total && lane < kQ) {
+      ir = ip[(c0 + lane) * p.stride];
+      fr = fp[(c0 + lane) * p.stride];
+    }
+  };
+  auto scan_gates = [&](int c0, int to, float from) __attribute__((always_inline)) {
+    const bool in = lane < kQ && c0 + lane < total;
+    const float gi = p.cap * tanhf((ld1(&ir) + bi) / p.cap), gf = -softplus_f(-p.cap * tanhf((ld1(&fr) + bf) / p.cap));
+    const double c = scan32(in ? static_cast<double>(gf) : 0.0, lane), start = from;
+    const double a = in ? static_cast<double>(gi) - c : -INFINITY;
+    double top = a > start ? a : start;
+#pragma unroll
+    for (int off = 1; off < kQ; off <<= 1) {
+      const double u = __shfl_up(top, off, 64);
+      if (lane >= off && u > top) top = u;
+    }
+    const double gn = __shfl(top, kQ - 1, 64);
+    if (lane < kQ) {
+      as[to][lane] = a;
+      gs[to][lane] = top;
+      add_w[to][lane] = expf(static_cast<float>(a - gn));
+      keep_w[to][lane] = expf(static_cast<float>(start - top));
+      floor_w[to][lane] = expf(static_cast<float>(-(c + top)));
+      if (lane == kQ - 1) m_next[to] = static_cast<float>(c + top);      // (what a state of its own would hold)
     }
   };
   fetch(0);
+  if (wave == waves - 1) {
+    fetch_gates(0);
+    scan_gates(0, 0, m0);
+    fetch_gates(kQ);
+  }
   for (int c0 = 0; c0 < total; c0 += kQ) {
     const int len = total - c0 < kQ ? total - c0 : kQ;
     qt.commit(Qs, LS);
     kt.commit(Ks, LS);
-    if (wave == 0) {
-      const float gi = p.cap * tanhf((ld1(&ir) + bi) / p.cap), gf = -softplus_f(-p.cap * tanhf((ld1(&fr) + bf) / p.cap));
-      const double c = scan32(lane < len ? static_cast<double>(gf) : 0.0, lane);
-      const double a = lane < len ? static_cast<double>(gi) - c : -INFINITY;
-      double top = a > m0 ? a : m0;
-#pragma unroll
-      for (int off = 1; off < kQ; off <<= 1) {
-        const double u = __shfl_up(top, off, 64);
-        if (lane >= off && u > top) top = u;
-      }
-      if (lane < kQ) { cum[lane] = c; as[lane] = a; gs[lane] = top; }
-    }
+    const int at = (c0 / kQ) & 1;
     float x[2][4];
 #pragma unroll
     for (int tj = 0; tj < 2; ++tj)
@@ -588,8 +608,12 @@ __global__ __launch_bounds__(256, NT <= 8 ? 2 : 1) void memory_chunk_kernel(Memo
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int i = 16 * ti + 4 * g + r;
-        Gs[i * kSq + j] = j <= i ? gm[r] * p.q_scale * expf(static_cast<float>(as[j] - gs[i])) : 0.f;
+        Gs[i * kSq + j] = j <= i ? gm[r] * p.q_scale * expf(static_cast<float>(as[at][j] - gs[at][i])) : 0.f;
       }
+    }
+    if (wave == waves - 1 && c0 + kQ < total) {
+      scan_gates(c0 + kQ, at ^ 1, m_next[at]);
+      fetch_gates(c0 + 2 * kQ);
     }
     f32x4_t y[2];
 #pragma unroll
@@ -602,7 +626,7 @@ __global__ __launch_bounds__(256, NT <= 8 ? 2 : 1) void memory_chunk_kernel(Memo
         for (int r = 0; r < 4; ++r) y[ti] = mfma4(q[r], s[t][r], y[ti]);
       }
 #pragma unroll
-      for (int r = 0; r < 4; ++r) y[ti][r] *= p.q_scale * expf(static_cast<float>(m0 - gs[16 * ti + 4 * g + r]));
+      for (int r = 0; r < 4; ++r) y[ti][r] *= p.q_scale * keep_w[at][16 * ti + 4 * g + r];
     }
     __syncthreads();
     {                                                  // denominators: eight lanes a token
@@ -612,7 +636,7 @@ __global__ __launch_bounds__(256, NT <= 8 ? 2 : 1) void memory_chunk_kernel(Memo
         const f32x4_t q = *reinterpret_cast<const f32x4_t*>(Qs + i * LS + c), n = *reinterpret_cast<const f32x4_t*>(ns + c);
         d += q[0] * n[0] + q[1] * n[1] + q[2] * n[2] + q[3] * n[3];
       }
-      d *= p.q_scale * expf(static_cast<float>(m0 - gs[i]));
+      d *= p.q_scale * keep_w[at][i];
       if (e < 16 || i >= 16) {                         // (the block above the diagonal is not formed)
         const f32x4_t w = *reinterpret_cast<const f32x4_t*>(Gs + i * kSq + e);
         d += w[0] + w[1] + w[2] + w[3];
@@ -620,7 +644,7 @@ __global__ __launch_bounds__(256, NT <= 8 ? 2 : 1) void memory_chunk_kernel(Memo
       d += __shfl_xor(d, 1, 64);
       d += __shfl_xor(d, 2, 64);
       d += __shfl_xor(d, 4, 64);
-      if (e == 0) inv[i] = 1.0f / (fmaxf(fabsf(d), expf(static_cast<float>(-(cum[i] + gs[i])))) + 1e-6f);
+      if (e == 0) inv[i] = 1.0f / (fmaxf(fabsf(d), floor_w[at][i]) + 1e-6f);
     }
 #pragma unroll
     for (int ti = 0; ti < 2; ++ti)
@@ -630,12 +654,11 @@ __global__ __launch_bounds__(256, NT <= 8 ? 2 : 1) void memory_chunk_kernel(Memo
 #pragma unroll
         for (int r = 0; r < 4; ++r) y[ti] = mfma4(w[r], x[tj][r], y[ti]);
       }
-    const double gn = gs[kQ - 1];
-    const float fix = expf(static_cast<float>(m0 - gn));
+    const float fix = keep_w[at][kQ - 1];
 #pragma unroll
     for (int tj = 0; tj < 2; ++tj)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) x[tj][r] *= expf(static_cast<float>(as[16 * tj + 4 * g + r] - gn));
+      for (int r = 0; r < 4; ++r) x[tj][r] *= add_w[at][16 * tj + 4 * g + r];
 #pragma unroll
     for (int t = 0; t < NT; ++t) {
       s[t] *= fix;
@@ -654,10 +677,11 @@ __global__ __launch_bounds__(256, NT <= 8 ? 2 : 1) void memory_chunk_kernel(Memo
       }
     if (threadIdx.x < NP) {
       float n = ns[threadIdx.x] * fix;
-      for (int j = 0; j < len; ++j) n += Ks[j * LS + threadIdx.x] * expf(static_cast<float>(as[j] - gn));
+#pragma unroll 8
+      for (int j = 0; j < kQ; ++j) n += Ks[j * LS + threadIdx.x] * add_w[at][j];      // (rows behind the last are zero)
       ns[threadIdx.x] = n;
     }
-    m0 = static_cast<float>(cum[kQ - 1] + gn);         // (what a state of its own would hold)
+    m0 = m_next[at];
     __syncthreads();
   }
 #pragma unroll
@@ -669,7 +693,7 @@ __global__ __launch_bounds__(256, NT <= 8 ? 2 : 1) void memory_chunk_kernel(Memo
     }
   for (int w = 0; w < p.col_waves && block + w < p.blocks; ++w) {
     if (static_cast<int>(threadIdx.x) < p.D) norm[w * (p.D + 1) + threadIdx.x] = ns[threadIdx.x];
-    if (threadIdx.x == 0) norm[w * (p.D + 1) + p.D] = static_cast<float>(m0);
+    if (threadIdx.x == 0) norm[w * (p.D + 1) + p.D] = m0;
   }
 }
 
