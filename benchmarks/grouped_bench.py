@@ -85,7 +85,7 @@ def kernel_table(cfg, device, T=8192, segs=4, B=64, ctx=1024):
     proj = [rnd(B, (2 * H + 2 * G) * D) for _ in range(2)]
     a, b, c = H * D, (H + G) * D, (H + 2 * G) * D
     keys, s0, loc = min(ctx, win), K.Segments(), r2t[1:, ctx - 1].long().contiguous()
-    layer = type("L", (), dict(window=win, kv_heads=G, group=H // G, heads=H))
+    layer = type("L", (), dict(window=win, keep_first=0, kv_heads=G, group=H // G, heads=H))
     splits = HybridAttnBackend._grouped_splits(type("B", (), dict(max_context_len=ctx + 128)), layer, B, True)
     dec["grouped_attention"] = _entry(_graph_us([lambda p=p, x=x: K.grouped_attention(p[:, :a], x, r2t, dslots, dpos, s0, H, G, D, D, win, scale, sink=0.0, gate=p[:, c:],
                                                                                      new=(p[:, a:b], p[:, b:c], loc), splits=splits)

@@ -123,7 +123,7 @@ def kernel_table(cfg, device, T=8192, segs=4, B=64, ctx=1024):
     for to, name, v, kw in ((dec, "grouped_attention (sinks)", 0, dict(sink=sinks)), (dec, "grouped_attention (window, cap)", win, dict(cap=cap, gate=gd)),
                             (like_dec, "grouped_attention", 0, dict(sink=0.0)), (like_dec, "grouped_attention (window)", win, dict(sink=0.0))):
         keys = min(ctx, v) if v else ctx
-        layer = type("L", (), dict(window=v, kv_heads=G, group=H // G, heads=H))
+        layer = type("L", (), dict(window=v, keep_first=0, kv_heads=G, group=H // G, heads=H))
         sp = HybridAttnBackend._grouped_splits(backend, layer, B, True)
         to[name] = _entry(_graph_us([lambda x=x: K.grouped_attention(qd, x, r2t, dslots, dpos, s0, H, G, D, D, v, D ** -0.5, splits=sp, **kw) for x in caches * 2]),
                           B * keys * row * 2 + B * H * D * 4, bf16=4 * B * keys * H * D)

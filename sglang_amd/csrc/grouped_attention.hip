@@ -62,18 +62,19 @@ __device__ __forceinline__ void cap_scores(const GroupedParams& p, f32x4_t& s) {
 }
 
 // Visible keys are numbered through: the first `kept` positions, then the window's, `gap` further on.
+template <bool kKeep = true>
 struct KeyMap {
   int kept, gap;
   __device__ __forceinline__ KeyMap(const GroupedParams& p, int window_first) {
-    kept = p.keep < window_first ? p.keep : window_first;
+    kept = kKeep ? (p.keep < window_first ? p.keep : window_first) : 0;
     gap = window_first - kept;
   }
-  __device__ __forceinline__ int operator()(int i) const { return i < kept ? i : i + gap; }
+  __device__ __forceinline__ int operator()(int i) const { return kKeep && i < kept ? i : i + gap; }
 };
 
 __device__ __forceinline__ int window_first(const GroupedParams& p, int pos) { return p.window > 0 && pos + 1 > p.window ? pos + 1 - p.window : 0; }
 
-__device__ __forceinline__ void key_range(const GroupedParams& p, const KeyMap& key, int pos, int split, int& lo, int& hi) {
+__device__ __forceinline__ void key_range(const GroupedParams& p, const KeyMap<>& key, int pos, int split, int& lo, int& hi) {
   const int n = pos + 1 - key.gap, per = (n + p.splits - 1) / p.splits;
   lo = split * per;
   hi = lo + per < n ? lo + per : n;
@@ -136,7 +137,7 @@ __global__ __launch_bounds__(256) void grouped_attention_plain_kernel(GroupedPar
   const int32_t* row = p.req_to_token + p.req[b] * p.r2t_stride;
   const T* cache = static_cast<const T*>(p.cache) + static_cast<int64_t>(kvh) * row_len;
   const int64_t pos = p.positions[t];
-  const KeyMap key(p, window_first(p, static_cast<int>(pos)));
+  const KeyMap<> key(p, window_first(p, static_cast<int>(pos)));
   int lo, hi;
   key_range(p, key, static_cast<int>(pos), split, lo, hi);
   const float offset = p.offsets ? p.offsets[h] : 0.f;
@@ -301,7 +302,7 @@ __global__ __launch_bounds__(256, 2) void grouped_attention_mfma_kernel(GroupedP
   const int64_t head_off = static_cast<int64_t>(kvh) * (p.kd + p.vd);
   const uint16_t* cache = static_cast<const uint16_t*>(p.cache) + head_off;
   const int pos = static_cast<int>(p.positions[t]);
-  const KeyMap key(p, window_first(p, pos));
+  const KeyMap<> key(p, window_first(p, pos));
   const int newest = pos - key.gap;                    // number of the token itself
   int lo, hi;
   key_range(p, key, pos, split, lo, hi);
@@ -459,7 +460,7 @@ __global__ __launch_bounds__(256, 2) void grouped_attention_mfma_kernel(GroupedP
 // needs them for O^T = V^T P^T, so they never touch LDS.
 constexpr int kPfThreads = 256, kPfRows = 128, kPfTile = 64, kPfPass = kPfThreads / 8;
 
-template <int KS, int VT, bool kSigmoid>
+template <int KS, int VT, bool kSigmoid, bool kKeep>
 __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedParams p) {
   constexpr int KLS = KS * 32 + 8, VLS = VT * 16 + 8, KP = KS / 2, VP = VT / 4, NP = kPfTile / kPfPass;
   __shared__ __attribute__((aligned(16))) uint16_t kimg[2][kPfTile * KLS];
@@ -471,7 +472,7 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
   const int left = p.seg_len[b] - q0;
   const int last = (left < p.block_tokens ? left : p.block_tokens) - 1;        // last token of the block, from its first
   const int pos0 = static_cast<int>(p.positions[t0]);
-  const KeyMap key(p, window_first(p, pos0));
+  const KeyMap<kKeep> key(p, window_first(p, pos0));
   const int end = pos0 + last + 1 - key.gap;           // keys the block sees
   const int32_t* row = p.req_to_token + p.req[b] * p.r2t_stride;
   const uint16_t* cache = static_cast<const uint16_t*>(p.cache) + static_cast<int64_t>(kvh) * (p.kd + p.vd);
@@ -551,7 +552,7 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
     }
     // a wave leaves out tiles none of its rows sees
     const int key0 = key(j0), key1 = key(j0 + kPfTile - 1);
-    if (!wave_live || key0 > wave_last || (p.window > 0 && key1 <= wave_first - p.window && key0 >= p.keep)) continue;
+    if (!wave_live || key0 > wave_last || (p.window > 0 && key1 <= wave_first - p.window && (!kKeep || key0 >= p.keep))) continue;
     f32x4_t s[2][4];
 #pragma unroll
     for (int n = 0; n < 4; ++n) {
@@ -579,7 +580,7 @@ __global__ __launch_bounds__(kPfThreads, 2) void grouped_prefill_kernel(GroupedP
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
             const int j = key(j0 + 16 * n + 4 * g + r);
-            if (j > qpos || (p.window > 0 && j <= qpos - p.window && j >= p.keep)) s[c][n][r] = -INFINITY;
+            if (j > qpos || (p.window > 0 && j <= qpos - p.window && (!kKeep || j >= p.keep))) s[c][n][r] = -INFINITY;
           }
       }
     }
@@ -634,17 +635,18 @@ void launch_mfma(const GroupedParams& p, const dim3& grid, hipStream_t st) {
   else launch_mfma<8, kSigmoid>(p, grid, st);
 }
 
-template <int KS, bool kSigmoid>
+template <int KS, bool kSigmoid, bool kKeep>
 void launch_prefill(const GroupedParams& p, const dim3& grid, hipStream_t st) {
-  if (p.vd <= 64) hipLaunchKernelGGL((grouped_prefill_kernel<KS, 4, kSigmoid>), grid, dim3(kPfThreads), 0, st, p);
-  else hipLaunchKernelGGL((grouped_prefill_kernel<KS, 8, kSigmoid>), grid, dim3(kPfThreads), 0, st, p);
+  if (p.vd <= 64) hipLaunchKernelGGL((grouped_prefill_kernel<KS, 4, kSigmoid, kKeep>), grid, dim3(kPfThreads), 0, st, p);
+  else hipLaunchKernelGGL((grouped_prefill_kernel<KS, 8, kSigmoid, kKeep>), grid, dim3(kPfThreads), 0, st, p);
 }
 
-template <bool kSigmoid>
+// (sigmoid weights: one form, with or without kept keys)
+template <bool kSigmoid, bool kKeep>
 void launch_prefill(const GroupedParams& p, const dim3& grid, hipStream_t st) {
-  if (p.kd <= 64) launch_prefill<2, kSigmoid>(p, grid, st);
-  else if (p.kd <= 128) launch_prefill<4, kSigmoid>(p, grid, st);
-  else launch_prefill<8, kSigmoid>(p, grid, st);
+  if (p.kd <= 64) launch_prefill<2, kSigmoid, kKeep>(p, grid, st);
+  else if (p.kd <= 128) launch_prefill<4, kSigmoid, kKeep>(p, grid, st);
+  else launch_prefill<8, kSigmoid, kKeep>(p, grid, st);
 }
 
 // keys the window keeps, weights that are sigmoids, factor on the output
@@ -765,8 +767,9 @@ int sgl_amd_grouped_prefill(const void* q, int64_t q_stride, const void* cache, 
   SGL_CHECK_ARG(whole_vectors(p), "grouped_prefill: rows of whole 16-byte vectors");
   const dim3 grid(kv_heads, num_blocks);
   hipStream_t st = as_stream(stream);
-  if (offsets) launch_prefill<true>(p, grid, st);
-  else launch_prefill<false>(p, grid, st);
+  if (offsets) launch_prefill<true, true>(p, grid, st);
+  else if (p.keep > 0) launch_prefill<false, true>(p, grid, st);
+  else launch_prefill<false, false>(p, grid, st);
   SGL_CHECK_LAUNCH("grouped_prefill");
   return 0;
 }

@@ -253,13 +253,14 @@ struct ResidualRmsParams {
   float eps;
 };
 
-template <typename T>
+// kMore: items may be another row
+template <typename T, bool kMore>
 __device__ __forceinline__ const T* source_item(const RowSource& s, int64_t row, int i) {
-  if (s.ids && s.ids[row * s.n + i] < 0) return static_cast<const T*>(s.alt) + row * s.alt_stride;
+  if (kMore && s.ids && s.ids[row * s.n + i] < 0) return static_cast<const T*>(s.alt) + row * s.alt_stride;
   return static_cast<const T*>(s.data) + row * s.row_stride + i * s.item_stride;
 }
 
-template <typename T, int VEC>
+template <typename T, int VEC, bool kMore>
 __device__ __forceinline__ void add_source(const RowSource& s, int64_t row, int c, float (&v)[VEC]) {
   const float* wr = s.weight ? s.weight + row * s.w_row : nullptr;
   for (int i = 0; i < s.n; i += 4) {                  // four loads in flight, clamped to the last item
@@ -267,8 +268,8 @@ __device__ __forceinline__ void add_source(const RowSource& s, int64_t row, int 
 #pragma unroll
     for (int q = 0; q < 4; ++q) {
       const int item = i + q < s.n ? i + q : s.n - 1;
-      if (s.f32) ldv<VEC>(source_item<float>(s, row, item) + c, u[q]);
-      else ldv<VEC>(source_item<T>(s, row, item) + c, u[q]);
+      if (s.f32) ldv<VEC>(source_item<float, kMore>(s, row, item) + c, u[q]);
+      else ldv<VEC>(source_item<T, kMore>(s, row, item) + c, u[q]);
     }
 #pragma unroll
     for (int q = 0; q < 4; ++q)
@@ -281,19 +282,20 @@ __device__ __forceinline__ void add_source(const RowSource& s, int64_t row, int 
 }
 
 // The same over all the columns of a thread: one item at a time, its pieces in flight together.
-template <typename T, int VEC, int kItems>
+template <typename T, int VEC, int kItems, bool kMore>
 __device__ __forceinline__ void add_source_row(const RowSource& s, int64_t row, int lane, int tpr, int W, float (&v)[kItems][VEC]) {
   constexpr int kAhead = kItems <= 4 ? 2 : 1;
 #pragma unroll kAhead
   for (int q = 0; q < s.n; ++q) {
     const float f = s.weight ? s.weight[row * s.w_row + q * s.w_item] : 1.0f;
+    const void* item = s.f32 ? static_cast<const void*>(source_item<float, kMore>(s, row, q)) : source_item<T, kMore>(s, row, q);
     float u[kItems][VEC];
 #pragma unroll
     for (int i = 0; i < kItems; ++i) {
       int c = (i * tpr + lane) * VEC;
       if (c >= W) c = 0;
-      if (s.f32) ldv<VEC>(source_item<float>(s, row, q) + c, u[i]);
-      else ldv<VEC>(source_item<T>(s, row, q) + c, u[i]);
+      if (s.f32) ldv<VEC>(static_cast<const float*>(item) + c, u[i]);
+      else ldv<VEC>(static_cast<const T*>(item) + c, u[i]);
     }
 #pragma unroll
     for (int i = 0; i < kItems; ++i)
@@ -302,8 +304,9 @@ __device__ __forceinline__ void add_source_row(const RowSource& s, int64_t row, 
   }
 }
 
-// kWaveRow: a wave owns a row (many rows: no barrier), else a workgroup does (decode batches: shortest path to one row).
-template <typename T, int VEC, int kItems, bool kWaveRow>
+// kWaveRow: a wave owns a row (many rows: no barrier), else a workgroup does (decode batches: shortest path to one row).  kMore: with
+// items that are another row, a bias, or a shift.
+template <typename T, int VEC, int kItems, bool kWaveRow, bool kMore>
 __global__ __launch_bounds__(kWaveRow ? 256 : 1024) void residual_rms_kernel(ResidualRmsParams p) {
   __shared__ float scratch[16];
   const int tpr = kWaveRow ? 64 : static_cast<int>(blockDim.x);
@@ -351,14 +354,14 @@ __global__ __launch_bounds__(kWaveRow ? 256 : 1024) void residual_rms_kernel(Res
     }
     if constexpr (kItems == 1) {
       if (lane * VEC < W) {
-        if (p.a.data) add_source<T, VEC>(p.a, row, lane * VEC, v[0]);
-        if (p.b.data) add_source<T, VEC>(p.b, row, lane * VEC, v[0]);
+        if (p.a.data) add_source<T, VEC, kMore>(p.a, row, lane * VEC, v[0]);
+        if (p.b.data) add_source<T, VEC, kMore>(p.b, row, lane * VEC, v[0]);
       }
     } else {
-      if (p.a.data) add_source_row<T, VEC, kItems>(p.a, row, lane, tpr, W, v);
-      if (p.b.data) add_source_row<T, VEC, kItems>(p.b, row, lane, tpr, W, v);
+      if (p.a.data) add_source_row<T, VEC, kItems, kMore>(p.a, row, lane, tpr, W, v);
+      if (p.b.data) add_source_row<T, VEC, kItems, kMore>(p.b, row, lane, tpr, W, v);
     }
-    if (p.bias) {
+    if (kMore && p.bias) {
 #pragma unroll
       for (int i = 0; i < kItems; ++i) {
         const int c = (i * tpr + lane) * VEC;
@@ -427,8 +430,8 @@ __global__ __launch_bounds__(kWaveRow ? 256 : 1024) void residual_rms_kernel(Res
   }
   ss = kWaveRow ? wave_sum(ss) : block_sum(ss, scratch);
   const float rs = 1.0f / sqrtf(ss / static_cast<float>(W) + p.eps);
-  T* left = p.shift ? static_cast<T*>(p.shift_state) + p.shift_slots[row] * W : nullptr;
-  const bool fresh = p.shift && p.shift_pos[row] <= 0;
+  T* left = kMore && p.shift ? static_cast<T*>(p.shift_state) + p.shift_slots[row] * W : nullptr;
+  const bool fresh = kMore && p.shift && p.shift_pos[row] <= 0;
 #pragma unroll
   for (int i = 0; i < kItems; ++i) {
     const int c = (i * tpr + lane) * VEC;
@@ -437,7 +440,7 @@ __global__ __launch_bounds__(kWaveRow ? 256 : 1024) void residual_rms_kernel(Res
       ldv<VEC>(p.w + c, wv);
 #pragma unroll
       for (int j = 0; j < VEC; ++j) o[j] = v[i][j] * rs * wv[j];
-      if (p.shift) {
+      if (kMore && p.shift) {
         float front[VEC], mu[VEC];
         ldv<VEC>(left + c, front);
         ldv<VEC>(p.shift + c, mu);
@@ -450,16 +453,16 @@ __global__ __launch_bounds__(kWaveRow ? 256 : 1024) void residual_rms_kernel(Res
   }
 }
 
-template <typename T>
+template <typename T, bool kMore>
 void launch_residual_rms(const ResidualRmsParams& p, bool vec, bool vec8, hipStream_t st) {
   const unsigned by4 = static_cast<unsigned>((p.rows + 3) / 4), one = static_cast<unsigned>(p.rows);
   const int W = p.width;
-  if (vec8 && p.rows >= 1024 && W <= 1024) hipLaunchKernelGGL((residual_rms_kernel<T, 8, 2, true>), dim3(by4), dim3(256), 0, st, p);
-  else if (vec8 && p.rows >= 1024 && W <= 2048) hipLaunchKernelGGL((residual_rms_kernel<T, 8, 4, true>), dim3(by4), dim3(256), 0, st, p);
-  else if (vec8 && p.rows >= 1024 && W <= 4096) hipLaunchKernelGGL((residual_rms_kernel<T, 8, 8, true>), dim3(by4), dim3(256), 0, st, p);
-  else if (vec && W <= 4096) hipLaunchKernelGGL((residual_rms_kernel<T, 4, 1, false>), dim3(one), dim3((W / 4 + 63) / 64 * 64), 0, st, p);
-  else if (vec) hipLaunchKernelGGL((residual_rms_kernel<T, 4, 4, false>), dim3(one), dim3(1024), 0, st, p);
-  else hipLaunchKernelGGL((residual_rms_kernel<T, 1, 16, false>), dim3(one), dim3(W >= 1024 ? 1024 : (W + 63) / 64 * 64), 0, st, p);
+  if (vec8 && p.rows >= 1024 && W <= 1024) hipLaunchKernelGGL((residual_rms_kernel<T, 8, 2, true, kMore>), dim3(by4), dim3(256), 0, st, p);
+  else if (vec8 && p.rows >= 1024 && W <= 2048) hipLaunchKernelGGL((residual_rms_kernel<T, 8, 4, true, kMore>), dim3(by4), dim3(256), 0, st, p);
+  else if (vec8 && p.rows >= 1024 && W <= 4096) hipLaunchKernelGGL((residual_rms_kernel<T, 8, 8, true, kMore>), dim3(by4), dim3(256), 0, st, p);
+  else if (vec && W <= 4096) hipLaunchKernelGGL((residual_rms_kernel<T, 4, 1, false, kMore>), dim3(one), dim3((W / 4 + 63) / 64 * 64), 0, st, p);
+  else if (vec) hipLaunchKernelGGL((residual_rms_kernel<T, 4, 4, false, kMore>), dim3(one), dim3(1024), 0, st, p);
+  else hipLaunchKernelGGL((residual_rms_kernel<T, 1, 16, false, kMore>), dim3(one), dim3(W >= 1024 ? 1024 : (W + 63) / 64 * 64), 0, st, p);
 }
 
 template <typename T, int VEC>
@@ -670,8 +673,9 @@ int sgl_amd_residual_rms(int is_f32, const int64_t* ids, const void* table, int6
   const bool vec8 = vec && width % 8 == 0 && h_stride % 8 == 0 && a_row_stride % 8 == 0 && a_item_stride % 8 == 0 && b_row_stride % 8 == 0 &&
                     b_item_stride % 8 == 0 && aligned_to(table, 16) && aligned_to(pos_table, 16) && aligned_to(a, 16) && aligned_to(b, 16) && aligned_to(h, 16) &&
                     a_alt_stride % 8 == 0 && aligned_to(a_alt, 16) && aligned_to(shift_state, 16);
-  if (is_f32) launch_residual_rms<float>(p, vec, vec8, as_stream(stream));
-  else launch_residual_rms<uint16_t>(p, vec, vec8, as_stream(stream));
+  const bool more = a_ids || bias || shift;
+  if (is_f32) more ? launch_residual_rms<float, true>(p, vec, vec8, as_stream(stream)) : launch_residual_rms<float, false>(p, vec, vec8, as_stream(stream));
+  else more ? launch_residual_rms<uint16_t, true>(p, vec, vec8, as_stream(stream)) : launch_residual_rms<uint16_t, false>(p, vec, vec8, as_stream(stream));
   SGL_CHECK_LAUNCH("residual_rms");
   return 0;
 }

@@ -129,7 +129,7 @@ def test_grouped_attention_kernels_keep_their_sums_in_registers(tmp_path):
     usage = _resource_usage("grouped_attention.hip", tmp_path)
     decode = {k: v for k, v in usage.items() if "grouped_attention_mfma_kernel" in k}
     prefill = {k: v for k, v in usage.items() if "grouped_prefill_kernel" in k}
-    assert len(decode) == 18 and len(prefill) == 12, sorted(usage)      # softmax and sigmoid weights
+    assert len(decode) == 18 and len(prefill) == 18, sorted(usage)      # softmax (with kept tokens or without) and sigmoid weights
     for name, u in decode.items():
         assert u["vgpr_spill_count"] <= (20 if "ILi8ELi16E" in name else 0) and u["vgpr_count"] <= 256, (name, u)
     for name, u in prefill.items():
